@@ -111,12 +111,13 @@ def host_lib():
         lib.ugh_last_error.restype = C.c_char_p
         lib.ugh_device_name.restype = C.c_char_p
         for f in ("ugh_slice_len", "ugh_lb_rank", "ugh_lb_elem_count", "ugh_schedule_n_items", "ugh_schedule_item_n_args",
-                  "ugh_compiled_n_funcs", "ugh_cache_size"):
+                  "ugh_compiled_n_funcs", "ugh_cache_size", "ugh_decoder_vocab", "ugh_decoder_state_len"):
             getattr(lib, f).restype = C.c_size_t
         for f in ("ugh_cache_new", "ugh_device_raw_hip", "ugh_func_raw_hip", "ugh_compiled_func_raw_hip", "ugh_slice_raw_hip"):
             getattr(lib, f).restype = C.c_void_p
         for f in ("ugh_device_free", "ugh_slice_free", "ugh_func_free", "ugh_ssa_free", "ugh_lb_free", "ugh_schedule_free", "ugh_cache_free",
-                  "ugh_compiled_free", "ugh_llama_ops_free", "ugh_llama_model_free", "ugh_lb_dims", "ugh_ssa_set_launch"):
+                  "ugh_compiled_free", "ugh_llama_ops_free", "ugh_llama_model_free", "ugh_lb_dims", "ugh_ssa_set_launch",
+                  "ugh_decoder_free", "ugh_decoder_state_free"):
             getattr(lib, f).restype = None
         _host = lib
     return _host
@@ -962,6 +963,76 @@ class LlamaModel(_Handle):
         _chk(host_lib().ugh_llama_generate_ex(_p(self.h), prompt.ctypes.data_as(C.c_void_p), C.c_size_t(prompt.size), C.c_size_t(n_steps), fp,
                                               toks.ctypes.data_as(C.c_void_p), C.byref(pre), C.byref(dec), margins.ctypes.data_as(C.c_void_p),
                                               top1.ctypes.data_as(C.c_void_p)))
+        items = host_lib().ugh_llama_last_decode_items
+        items.restype = C.c_size_t
+        return toks, {"prefill_ms": pre.value, "decode_ms": dec.value, "margins": margins, "top1": top1, "decode_items": int(items())}
+
+
+class DecoderState(_Handle):
+    """What one sequence keeps between steps; dropping it gives its memory back."""
+    _free = "ugh_decoder_state_free"
+
+    def __len__(self):
+        return host_lib().ugh_decoder_state_len(_p(self.h))
+
+
+class Decoder(_Handle):
+    """A model of the registry (csrc/host/decoder.cpp), chosen by its config.json."""
+    _free = "ugh_decoder_free"
+
+    @classmethod
+    def load(cls, device, path, bf16=True):
+        """config.json and model.safetensors of a folder; bf16: matrices kept and multiplied as bf16, else everything in f32."""
+        out = C.c_void_p()
+        _chk(host_lib().ugh_decoder_load(_p(device.h), os.fsencode(path), int(bool(bf16)), C.byref(out)))
+        return cls._wrap(out.value, device)
+
+    @classmethod
+    def random(cls, device, config, bf16=True, seed=9, std=0.02, norm_mean=0.0):
+        """The model of `config` (a dict) with random-init weights."""
+        import json
+        out = C.c_void_p()
+        _chk(host_lib().ugh_decoder_random(_p(device.h), json.dumps(config).encode(), int(bool(bf16)), C.c_uint64(seed), C.c_float(std), C.c_float(norm_mean), C.byref(out)))
+        return cls._wrap(out.value, device)
+
+    @classmethod
+    def _wrap(cls, h, device):
+        self = cls(h)
+        self._keep = [device]
+        self.vocab = host_lib().ugh_decoder_vocab(_p(h))
+        return self
+
+    def new_state(self, max_tokens):
+        out = C.c_void_p()
+        _chk(host_lib().ugh_decoder_state_new(_p(self.h), C.c_size_t(max_tokens), C.byref(out)))
+        return DecoderState(out.value)
+
+    def step(self, state, tokens, want=(), hidden=None):
+        """Runs `tokens` behind what `state` holds; logits [len(want), vocab] of those places among them.
+        hidden (layers, width): also returns the residual behind every layer, [layers, len(tokens), width]."""
+        tokens = np.ascontiguousarray(tokens, dtype=np.int32)
+        want = np.ascontiguousarray(want, dtype=np.int32)
+        logits = np.zeros((want.size, self.vocab), np.float32)
+        h = np.zeros((hidden[0], tokens.size, hidden[1]), np.float32) if hidden is not None else None
+        _chk(host_lib().ugh_decoder_step(_p(self.h), _p(state.h), tokens.ctypes.data_as(C.c_void_p), C.c_size_t(tokens.size), want.ctypes.data_as(C.c_void_p),
+                                         C.c_size_t(want.size), logits.ctypes.data_as(C.c_void_p), None if h is None else h.ctypes.data_as(C.c_void_p),
+                                         C.c_size_t(0 if h is None else h.size)))
+        return logits if h is None else (logits, h)
+
+    def generate(self, prompt, n_steps, forced=None):
+        """As LlamaModel.generate."""
+        prompt = np.ascontiguousarray(prompt, dtype=np.int32)
+        toks = np.zeros(n_steps + 1, dtype=np.int32)
+        margins, top1 = np.zeros(n_steps + 1, dtype=np.float32), np.zeros(n_steps + 1, dtype=np.float32)
+        pre, dec, fp = C.c_double(), C.c_double(), None
+        if forced is not None:
+            forced = np.ascontiguousarray(forced, dtype=np.int32)
+            if forced.size != n_steps:
+                raise ValueError(f"forced: expected {n_steps} ids, got {forced.size}")
+            fp = forced.ctypes.data_as(C.c_void_p)
+        _chk(host_lib().ugh_decoder_generate(_p(self.h), prompt.ctypes.data_as(C.c_void_p), C.c_size_t(prompt.size), C.c_size_t(n_steps), fp,
+                                             toks.ctypes.data_as(C.c_void_p), C.byref(pre), C.byref(dec), margins.ctypes.data_as(C.c_void_p),
+                                             top1.ctypes.data_as(C.c_void_p)))
         items = host_lib().ugh_llama_last_decode_items
         items.restype = C.c_size_t
         return toks, {"prefill_ms": pre.value, "decode_ms": dec.value, "margins": margins, "top1": top1, "decode_items": int(items())}

@@ -32,7 +32,8 @@ def _run(cmd):
         raise RuntimeError("build step failed: " + " ".join(cmd))
 
 
-UGHIP_SOURCES = ("runtime.cpp", "lower_hip.cpp", "llama_ops.hip", "matmul.hip", "gemm_tiled.hip", "gemm_dma.hip", "gemm_dma_f32.hip", "rows_x3.hip", "attention.hip", "fused_linear.hip", "convert.hip")
+UGHIP_SOURCES = ("runtime.cpp", "lower_hip.cpp", "llama_ops.hip", "matmul.hip", "gemm_tiled.hip", "gemm_dma.hip", "gemm_dma_f32.hip", "rows_x3.hip", "attention.hip", "fused_linear.hip", "convert.hip",
+                 "rows_product.hip", "row_norms.hip", "latent_attention.hip", "ssm.hip", "moe.hip")
 
 
 def build_ughip(only_changed=False):
@@ -62,7 +63,7 @@ def build_ughip(only_changed=False):
 
 def build_host():
     src = os.path.join(CSRC, "host")
-    files = [os.path.join(src, f) for f in ("ug/lower_op.cpp", "ug/lazy_buffer.cpp", "ug/schedule.cpp", "ug/safetensors.cpp", "hip_device.cpp", "llama.cpp", "capi.cpp")]
+    files = [os.path.join(src, f) for f in ("ug/lower_op.cpp", "ug/lazy_buffer.cpp", "ug/schedule.cpp", "ug/safetensors.cpp", "hip_device.cpp", "llama.cpp", "hybrid.cpp", "decoder.cpp", "capi.cpp")]
     _run(["g++", "-std=c++17", "-O2", "-fPIC", "-shared", "-Wall", "-I" + INC, "-I" + src] + files +
          ["-L" + LIB, "-lughip", "-Wl,-rpath,$ORIGIN", "-lpthread", "-o", os.path.join(LIB, "libug_host.so")])
 
@@ -71,6 +72,13 @@ def build_oracle():
     mk = os.path.join(ROOT, "oracle", "Makefile")
     if os.path.exists(mk):
         _run(["make", "-s", "-C", os.path.join(ROOT, "oracle")])
+
+
+def ensure_built():
+    """Builds what a model needs to run (the two product libraries) where they are missing, e.g. in a fresh checkout."""
+    if not all(os.path.exists(os.path.join(LIB, f)) for f in ("libughip.so", "libug_host.so")):
+        build_ughip()
+        build_host()
 
 
 def build_all():

@@ -9,6 +9,7 @@
 #include <cstring>
 
 #include "hip_device.h"
+#include "decoder.h"
 #include "llama.h"
 #include "ug/lazy_buffer.h"
 #include "ug/samples.h"
@@ -854,6 +855,69 @@ int ugh_llama_generate_ex(void* m, const int32_t* prompt, size_t n_prompt, size_
 }
 // Schedule items (device launches) of the last single-token step of this thread's last ugh_llama_generate_ex.
 size_t ugh_llama_last_decode_items() { return g_last_decode_items; }
+// ---- decoders by configuration ------------------------------------------------------------------------------
+struct DecoderBox {
+  std::unique_ptr<ug_llama::Decoder> model;
+  CompilationCache cache;
+};
+// bf16: matrices kept and multiplied as bf16
+int ugh_decoder_load(void* d, const char* dir, int bf16, void** out) {
+  return guard([&] {
+    auto b = std::make_unique<DecoderBox>();
+    b->model = ug_llama::load_decoder(dir, bf16 ? ug_llama::Precision::BF16 : ug_llama::Precision::F32, dev_of(d));
+    *out = b.release();
+  });
+}
+// The model of a config.json given as text, with random-init weights (ugh_llama_model_new_ex's generator).
+int ugh_decoder_random(void* d, const char* config, int bf16, uint64_t seed, float std, float norm_mean, void** out) {
+  return guard([&] {
+    const std::string text = config;
+    JsonParser jp{text.data(), text.data() + text.size(), "config"};
+    const Json cfg = jp.value(0);
+    auto w = ug_llama::synthetic_weights(seed, std, bf16 != 0, norm_mean);
+    auto b = std::make_unique<DecoderBox>();
+    b->model = ug_llama::build_decoder(cfg, *w, bf16 ? ug_llama::Precision::BF16 : ug_llama::Precision::F32, dev_of(d));
+    *out = b.release();
+  });
+}
+void ugh_decoder_free(void* m) { delete static_cast<DecoderBox*>(m); }
+size_t ugh_decoder_vocab(void* m) { return static_cast<DecoderBox*>(m)->model->vocab_size(); }
+int ugh_decoder_state_new(void* m, size_t max_tokens, void** out) {
+  return guard([&] { *out = static_cast<DecoderBox*>(m)->model->new_state(max_tokens).release(); });
+}
+void ugh_decoder_state_free(void* s) { delete static_cast<ug_llama::DecoderState*>(s); }
+size_t ugh_decoder_state_len(void* s) { return static_cast<ug_llama::DecoderState*>(s)->len; }
+// logits: n_want * vocab floats.  hidden (may be null): hidden_len floats, the residual behind every layer one after the other.
+int ugh_decoder_step(void* m, void* state, const int32_t* tokens, size_t n, const int32_t* want, size_t n_want, float* logits, float* hidden, size_t hidden_len) {
+  return guard([&] {
+    auto* b = static_cast<DecoderBox*>(m);
+    std::vector<std::vector<float>> rows;
+    std::vector<float> out = ug_llama::decoder_step(*b->model, *static_cast<ug_llama::DecoderState*>(state), std::vector<int32_t>(tokens, tokens + n),
+                                                    std::vector<int32_t>(want, want + n_want), b->cache, hidden ? &rows : nullptr);
+    if (!out.empty()) std::memcpy(logits, out.data(), out.size() * sizeof(float));
+    size_t at = 0;
+    for (const auto& r : rows) {
+      if (at + r.size() > hidden_len) throw std::runtime_error("decoder_step: the buffer for the hidden states is too short");
+      std::memcpy(hidden + at, r.data(), r.size() * sizeof(float));
+      at += r.size();
+    }
+  });
+}
+int ugh_decoder_generate(void* m, const int32_t* prompt, size_t n_prompt, size_t n_steps, const int32_t* forced, int32_t* out_tokens, double* prefill_ms, double* decode_ms,
+                         float* margins, float* top1_values) {
+  return guard([&] {
+    ug_llama::GenerateStats st;
+    std::vector<int32_t> p(prompt, prompt + n_prompt), f;
+    if (forced) f.assign(forced, forced + n_steps);
+    std::vector<int32_t> toks = ug_llama::generate_greedy(*static_cast<DecoderBox*>(m)->model, p, n_steps, &st, forced ? &f : nullptr);
+    std::memcpy(out_tokens, toks.data(), toks.size() * sizeof(int32_t));
+    if (prefill_ms) *prefill_ms = st.prefill_ms;
+    if (decode_ms) *decode_ms = st.decode_ms;
+    if (margins) std::memcpy(margins, st.top1_margin.data(), st.top1_margin.size() * sizeof(float));
+    if (top1_values) std::memcpy(top1_values, st.top1_value.data(), st.top1_value.size() * sizeof(float));
+    g_last_decode_items = st.decode_items;
+  });
+}
 int ugh_synthetic_weights(uint64_t seed, float std, int round_bf16, const char* name, size_t n, float* out) {
   return guard([&] {
     auto w = ug_llama::synthetic_weights(seed, std, round_bf16 != 0);

@@ -1082,6 +1082,38 @@ LB Model::fwd(const LB& tokens, const LB& pos, std::vector<Cache>& cache, const 
   return ops_->linear(xs, head_);
 }
 
+// ---- the model as a Decoder -----------------------------------------------------------------------------
+void LlamaState::settle() {
+  for (Cache& c : cache) {
+    c.prev_k.maybe_allocate_uninit();
+    c.prev_v.maybe_allocate_uninit();
+    c.prev_k.detach();
+    c.prev_v.detach();
+  }
+}
+
+std::unique_ptr<DecoderState> Model::new_state(size_t) const {
+  auto s = std::make_unique<LlamaState>();
+  s->cache = new_cache();
+  s->capacity = s->cache.empty() ? 0 : s->cache[0].capacity;
+  return s;
+}
+
+void Model::prepare() const {
+  rope_.cos.realize();
+  rope_.sin.realize();
+}
+
+LB Model::step(const LB& tokens, const LB& pos, DecoderState& state, const LB* rows, const std::function<void(const LB&)>* after_layer) const {
+  LlamaState* s = dynamic_cast<LlamaState*>(&state);
+  if (!s) bail("a llama step needs a llama state");
+  const size_t t = tokens.dims()[1];
+  LB logits = fwd(tokens, pos, s->cache, after_layer, rows == nullptr);
+  s->len += t;
+  if (!rows) return logits;
+  return index_select(logits.reshape(Shape({t, cfg_.vocab_size})), *rows);
+}
+
 // One prefill call over the prompt, then `n_steps` greedy single-token steps (graph rebuilt per
 // step with a shared CompilationCache, as ug-llama/src/main.rs:124-146 does).  Returns the
 // n_steps + 1 argmax ids: one from the prefill logits, one per decode step.
@@ -1109,16 +1141,15 @@ namespace {
 // the launches of step i + 1 are issued while step i still runs.  Inputs that have to come from
 // the host (prompt, positions) are uploaded before the first launch, because an upload waits for
 // the stream.  Ids and the two largest logits of every step are read once at the end.
-std::vector<int32_t> generate_greedy_queued(const Model& model, const std::vector<int32_t>& prompt, size_t n_steps, GenerateStats* stats,
+std::vector<int32_t> generate_greedy_queued(const Decoder& model, const std::vector<int32_t>& prompt, size_t n_steps, GenerateStats* stats,
                                             const std::vector<int32_t>* forced) {
   using clock = std::chrono::steady_clock;
   const DevicePtr& dev = model.device();
   const Ops& ops = model.ops();
-  std::vector<Cache> cache = model.new_cache();
+  std::unique_ptr<DecoderState> state = model.new_state(prompt.size() + n_steps);
   CompilationCache ccache;
   const bool verbose = switch_on(SW_VERBOSE);
-  model.rope().cos.realize();
-  model.rope().sin.realize();
+  model.prepare();
 
   const size_t total = n_steps + 1;
   LB ids = LB::alloc_uninit(DType::I32, Shape({total}), dev), vals = LB::alloc_uninit(DType::F32, Shape({2 * total}), dev);
@@ -1157,7 +1188,7 @@ std::vector<int32_t> generate_greedy_queued(const Model& model, const std::vecto
       st.layers.push_back(std::make_unique<CompiledSchedule>(part.compile_and_run(ccache)));
       st.n_items += part.items().size();
     };
-    LB logits = model.fwd(st.tokens, pos[i], cache, run_now && by_layer ? &realise_layer : nullptr, true);
+    LB logits = model.step(st.tokens, pos[i], *state, nullptr, run_now && by_layer ? &realise_layer : nullptr);
     st.logits = ops.argmax_into(forced ? picked : tokens[i + 1], logits, logits.dims()[logits.rank() - 2] - 1, ids, vals, i);
     auto t1 = clock::now();
     Schedule schedule = Schedule::create_one(st.logits);
@@ -1176,21 +1207,13 @@ std::vector<int32_t> generate_greedy_queued(const Model& model, const std::vecto
 
   PreparedStep cur, done;
   auto t_start = clock::now();
-  for (Cache& c : cache) {
-    c.prev_k.maybe_allocate_uninit();
-    c.prev_v.maybe_allocate_uninit();
-  }
+  state->settle();  // the (empty) caches become buffers
   build(0, cur, true);
   auto t_decode = t_start;
   for (size_t step = 0; step <= n_steps; ++step) {
     const bool more = step < n_steps;
     PreparedStep next;
-    for (Cache& c : cache) {
-      c.prev_k.maybe_allocate_uninit();
-      c.prev_v.maybe_allocate_uninit();
-      c.prev_k.detach();
-      c.prev_v.detach();
-    }
+    state->settle();
     auto t0 = clock::now();
     auto t1 = t0;
     if (more) {
@@ -1253,35 +1276,34 @@ std::vector<int32_t> generate_greedy_queued(const Model& model, const std::vecto
 // known.  Every value computed is the same as in the reference's order.
 // UG_LLAMA_NO_OVERLAP=1 keeps everything on the calling thread.
 // UG_LLAMA_HOST_ARGMAX=1 keeps this read-back loop on a device that could pick the token itself.
-std::vector<int32_t> generate_greedy(const Model& model, const std::vector<int32_t>& prompt, size_t n_steps, GenerateStats* stats,
+std::vector<int32_t> generate_greedy(const Decoder& model, const std::vector<int32_t>& prompt, size_t n_steps, GenerateStats* stats,
                                      const std::vector<int32_t>* forced) {
   using clock = std::chrono::steady_clock;
-  const Config& cfg = model.config();
+  const size_t vocab = model.vocab_size();
   const DevicePtr& dev = model.device();
   if (prompt.empty()) bail("empty prompt");
-  if (prompt.size() + n_steps > cfg.max_position_embeddings) bail("prompt + steps exceed max_position_embeddings");
+  if (prompt.size() + n_steps > model.max_positions()) bail("prompt + steps exceed max_position_embeddings");
   if (forced && forced->size() != n_steps) bail("forced ids: expected one per decode step (" + std::to_string(n_steps) + "), got " + std::to_string(forced->size()));
   // The embedding gather forms its source offset from the id on the device, where nothing can check it
   // (ids picked by the argmax are in range by construction; these come from the caller).
   auto check_ids = [&](const std::vector<int32_t>& ids, const char* what) {
     for (size_t i = 0; i < ids.size(); ++i)
-      if (ids[i] < 0 || (size_t)ids[i] >= cfg.vocab_size)
-        bail(std::string(what) + " id " + std::to_string(ids[i]) + " at index " + std::to_string(i) + " is outside the vocabulary of " + std::to_string(cfg.vocab_size));
+      if (ids[i] < 0 || (size_t)ids[i] >= vocab)
+        bail(std::string(what) + " id " + std::to_string(ids[i]) + " at index " + std::to_string(i) + " is outside the vocabulary of " + std::to_string(vocab));
   };
   check_ids(prompt, "prompt");
   if (forced) check_ids(*forced, "forced");
   if (dev->runs_async() && model.ops().device_argmax() && !switch_on(SW_HOST_ARGMAX) && !switch_on(SW_NO_OVERLAP))
     return generate_greedy_queued(model, prompt, n_steps, stats, forced);
-  std::vector<Cache> cache = model.new_cache();
+  std::unique_ptr<DecoderState> state = model.new_state(prompt.size() + n_steps);
   CompilationCache ccache;
   std::vector<int32_t> out;
   std::vector<float> logits;
   const bool verbose = switch_on(SW_VERBOSE);
   const bool overlap = dev->runs_async() && !switch_on(SW_NO_OVERLAP);
-  // The rotary tables are shared by every step: realise them once, before two steps can be in
+  // What every step shares (the rotary tables) is realised once, before two steps can be in
   // preparation and in flight at the same time.
-  model.rope().cos.realize();
-  model.rope().sin.realize();
+  model.prepare();
 
   auto upload_inputs = [&](const std::vector<int32_t>& ids, size_t pos_v, PreparedStep& st, LB& pos) {
     st.t = ids.size();
@@ -1291,7 +1313,7 @@ std::vector<int32_t> generate_greedy(const Model& model, const std::vector<int32
   };
   auto build = [&](PreparedStep& st, const LB& pos) {
     auto t0 = clock::now();
-    st.logits = model.fwd(st.tokens, pos, cache, nullptr, true);  // read at the last position only, like the queued loop
+    st.logits = model.step(st.tokens, pos, *state, nullptr, nullptr);  // read at the last position only, like the queued loop
     auto t1 = clock::now();
     Schedule schedule = Schedule::create_one(st.logits);
     auto t2 = clock::now();
@@ -1323,12 +1345,7 @@ std::vector<int32_t> generate_greedy(const Model& model, const std::vector<int32
     // The cache buffers this step writes become leaves for the next graph: allocate them now and
     // drop the graph behind them (the compiled schedule keeps what it needs alive), which also
     // keeps the DAG from growing with every step.
-    for (Cache& c : cache) {
-      c.prev_k.maybe_allocate_uninit();
-      c.prev_v.maybe_allocate_uninit();
-      c.prev_k.detach();
-      c.prev_v.detach();
-    }
+    state->settle();
     // The launches go to a second thread; this thread (whose allocator arena holds the graphs)
     // prepares the next step meanwhile.
     auto t0 = clock::now();
@@ -1361,10 +1378,10 @@ std::vector<int32_t> generate_greedy(const Model& model, const std::vector<int32
     logits.resize(cur.logits.elem_count());
     cur.logits.data_vec(logits.data(), DType::F32);
     auto t3 = clock::now();
-    const float* last = logits.data() + (cur.logits.elem_count() / cfg.vocab_size - 1) * cfg.vocab_size;
+    const float* last = logits.data() + (cur.logits.elem_count() / vocab - 1) * vocab;
     size_t best = 0;
     float second = -INFINITY;
-    for (size_t i = 1; i < cfg.vocab_size; ++i) {
+    for (size_t i = 1; i < vocab; ++i) {
       if (last[i] > last[best]) {
         second = last[best];
         best = i;

@@ -7,11 +7,9 @@
 #include <string>
 #include <vector>
 
-#include "ug/lazy_buffer.h"
+#include "decoder.h"
 
 namespace ug_llama {
-
-using LB = ug::LazyBuffer;
 
 // ug-llama/src/main.rs:22-28
 struct Ops {
@@ -174,8 +172,14 @@ struct Cache {
   static std::vector<Cache> create(const Config& cfg, const ug::DevicePtr& dev, size_t capacity = 0);
 };
 
+// The caches of a llama sequence, one per layer.
+struct LlamaState : DecoderState {
+  std::vector<Cache> cache;
+  void settle() override;
+};
+
 // model.rs:299-373
-class Model {
+class Model : public Decoder {
  public:
   Model(const Config& cfg, bool custom_softmax, WeightSource& weights, const ug::DevicePtr& dev, std::shared_ptr<Ops> ops);
   // 0 (default): the reference's op-by-op graph.
@@ -210,9 +214,14 @@ class Model {
   LB fwd(const LB& tokens, const LB& pos, std::vector<Cache>& cache, const std::function<void(const LB&)>* after_layer = nullptr,
          bool last_position_only = false) const;
   const Config& config() const { return cfg_; }
-  const ug::DevicePtr& device() const { return dev_; }
+  const ug::DevicePtr& device() const override { return dev_; }
   const Rope& rope() const { return rope_; }
-  const Ops& ops() const { return *ops_; }
+  const Ops& ops() const override { return *ops_; }
+  std::unique_ptr<DecoderState> new_state(size_t max_tokens) const override;
+  LB step(const LB& tokens, const LB& pos, DecoderState& state, const LB* rows, const std::function<void(const LB&)>* after_layer) const override;
+  size_t vocab_size() const override { return cfg_.vocab_size; }
+  size_t max_positions() const override { return cfg_.max_position_embeddings; }
+  void prepare() const override;
 
  private:
   struct Layer {
@@ -256,7 +265,7 @@ struct GenerateStats {
 // forced != nullptr (n_steps ids): decode step i is fed (*forced)[i - 1] instead of the id picked at step i - 1, so that two
 // devices can be compared position by position on identical inputs; the ids returned are still each step's argmax.
 // Ids outside [0, vocab_size) in `prompt` or `forced` are refused (they would index the embedding table out of bounds).
-std::vector<int32_t> generate_greedy(const Model& model, const std::vector<int32_t>& prompt, size_t n_steps, GenerateStats* stats,
+std::vector<int32_t> generate_greedy(const Decoder& model, const std::vector<int32_t>& prompt, size_t n_steps, GenerateStats* stats,
                                      const std::vector<int32_t>* forced = nullptr);
 
 }  // namespace ug_llama

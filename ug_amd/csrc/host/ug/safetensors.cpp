@@ -1,5 +1,7 @@
 #include "safetensors.h"
 
+#include "json.h"
+
 #include <fcntl.h>
 #include <sys/mman.h>
 #include <sys/stat.h>
@@ -15,156 +17,6 @@
 namespace ug {
 
 namespace {
-
-// ---- a JSON reader for the header: objects, arrays, strings, non-negative integers ----------------
-struct Json {
-  enum Kind { Null, Bool, Num, Str, Arr, Obj } kind = Null;
-  double num = 0;
-  bool is_uint = false;
-  uint64_t uint = 0;
-  std::string str;
-  std::vector<Json> arr;
-  std::vector<std::pair<std::string, Json>> obj;
-};
-
-struct JsonParser {
-  const char* p;
-  const char* end;
-  const std::string& path;
-  [[noreturn]] void fail(const std::string& what) const { bail("invalid safetensors header in " + path + ": " + what); }
-  void ws() {
-    while (p < end && (*p == ' ' || *p == '\n' || *p == '\t' || *p == '\r')) ++p;
-  }
-  char peek() {
-    ws();
-    if (p >= end) fail("unexpected end");
-    return *p;
-  }
-  void expect(char c) {
-    if (peek() != c) fail(std::string("expected '") + c + "'");
-    ++p;
-  }
-  std::string string() {
-    expect('"');
-    std::string out;
-    while (true) {
-      if (p >= end) fail("unterminated string");
-      char c = *p++;
-      if (c == '"') break;
-      if (c != '\\') {
-        out.push_back(c);
-        continue;
-      }
-      if (p >= end) fail("unterminated escape");
-      char e = *p++;
-      switch (e) {
-        case '"': out.push_back('"'); break;
-        case '\\': out.push_back('\\'); break;
-        case '/': out.push_back('/'); break;
-        case 'b': out.push_back('\b'); break;
-        case 'f': out.push_back('\f'); break;
-        case 'n': out.push_back('\n'); break;
-        case 'r': out.push_back('\r'); break;
-        case 't': out.push_back('\t'); break;
-        case 'u': {
-          if (end - p < 4) fail("short \\u escape");
-          unsigned cp = 0;
-          for (int i = 0; i < 4; ++i) {
-            char h = *p++;
-            cp <<= 4;
-            if (h >= '0' && h <= '9') cp |= (unsigned)(h - '0');
-            else if (h >= 'a' && h <= 'f') cp |= (unsigned)(h - 'a' + 10);
-            else if (h >= 'A' && h <= 'F') cp |= (unsigned)(h - 'A' + 10);
-            else fail("bad \\u escape");
-          }
-          // UTF-8 encode the BMP code point (surrogate pairs are kept as two 3-byte sequences)
-          if (cp < 0x80) out.push_back((char)cp);
-          else if (cp < 0x800) {
-            out.push_back((char)(0xC0 | (cp >> 6)));
-            out.push_back((char)(0x80 | (cp & 0x3F)));
-          } else {
-            out.push_back((char)(0xE0 | (cp >> 12)));
-            out.push_back((char)(0x80 | ((cp >> 6) & 0x3F)));
-            out.push_back((char)(0x80 | (cp & 0x3F)));
-          }
-          break;
-        }
-        default: fail("bad escape");
-      }
-    }
-    return out;
-  }
-  Json value(int depth) {
-    if (depth > 16) fail("nesting too deep");
-    Json j;
-    char c = peek();
-    if (c == '{') {
-      ++p;
-      j.kind = Json::Obj;
-      if (peek() == '}') {
-        ++p;
-        return j;
-      }
-      while (true) {
-        std::string k = string();
-        expect(':');
-        j.obj.emplace_back(std::move(k), value(depth + 1));
-        char d = peek();
-        ++p;
-        if (d == '}') break;
-        if (d != ',') fail("expected ',' or '}'");
-        ws();
-      }
-    } else if (c == '[') {
-      ++p;
-      j.kind = Json::Arr;
-      if (peek() == ']') {
-        ++p;
-        return j;
-      }
-      while (true) {
-        j.arr.push_back(value(depth + 1));
-        char d = peek();
-        ++p;
-        if (d == ']') break;
-        if (d != ',') fail("expected ',' or ']'");
-      }
-    } else if (c == '"') {
-      j.kind = Json::Str;
-      j.str = string();
-    } else if (c == 't' && end - p >= 4 && !strncmp(p, "true", 4)) {
-      p += 4;
-      j.kind = Json::Bool;
-      j.num = 1;
-    } else if (c == 'f' && end - p >= 5 && !strncmp(p, "false", 5)) {
-      p += 5;
-      j.kind = Json::Bool;
-    } else if (c == 'n' && end - p >= 4 && !strncmp(p, "null", 4)) {
-      p += 4;
-    } else if (c == '-' || (c >= '0' && c <= '9')) {
-      const char* s = p;
-      bool all_digits = true;
-      uint64_t u = 0;
-      bool overflow = false;
-      while (p < end && (*p == '-' || *p == '+' || *p == '.' || *p == 'e' || *p == 'E' || (*p >= '0' && *p <= '9'))) {
-        if (*p >= '0' && *p <= '9') {
-          if (u > (std::numeric_limits<uint64_t>::max() - (uint64_t)(*p - '0')) / 10) overflow = true;
-          u = u * 10 + (uint64_t)(*p - '0');
-        } else {
-          all_digits = false;
-        }
-        ++p;
-      }
-      j.kind = Json::Num;
-      j.num = strtod(std::string(s, p).c_str(), nullptr);
-      j.is_uint = all_digits && !overflow;
-      j.uint = u;
-    } else {
-      fail(std::string("unexpected character '") + c + "'");
-    }
-    return j;
-  }
-};
 
 size_t st_dtype_size(const std::string& d) {
   if (d == "BOOL" || d == "U8" || d == "I8" || d == "F8_E5M2" || d == "F8_E4M3") return 1;
@@ -225,7 +77,7 @@ std::shared_ptr<MmapedSafetensors::File> MmapedSafetensors::open_file(const std:
   if (n > 100000000ull) bail("safetensors header too large, path: " + path);
   if (n + 8 > f->len) bail("invalid safetensors header length, path: " + path);
   const char* hs = reinterpret_cast<const char*>(base + 8);
-  JsonParser jp{hs, hs + n, path};
+  JsonParser jp{hs, hs + n, "invalid safetensors header in " + path};
   Json root = jp.value(0);
   jp.ws();
   if (jp.p != jp.end) jp.fail("trailing characters");

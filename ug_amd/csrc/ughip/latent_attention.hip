@@ -1,0 +1,578 @@
+// Attention over latents (ughip_layers.h): the cache of a layer is one row per position, [normed latent (rank) | rotated key part
+// (rot)], shared by all heads.
+//
+// Many positions (latent_rows_kernel): keys and values are expanded by products before, and the scores never leave registers.
+//   A wave owns 32 queries, a workgroup 128; keys come in tiles of 64 through LDS.  The scores are computed transposed, S^T = K Q^T
+//   (32 x 32 tiles), which leaves lane l with query l % 32 as its column: the running maximum and sum are one exchange with lane
+//   l ^ 32, and the weights sit where the second product, O^T = V^T P^T, wants its right operand (the order in which keys take
+//   part in it is the order the accumulator layout gives; V is read in the same order).  Values come transposed for that.
+//   bf16 operands: v_mfma_f32_32x32x16_bf16, a weight as two bf16 terms (16 bits of it); f32: v_mfma_f32_32x32x2_f32.
+// Few positions (absorb, split, merge): the up-projection of the keys is folded into the query, that of the values into the
+//   result, so that a head's keys and values are both the cache rows as they are.  16 (position, head) pairs per workgroup against
+//   tiles of 32 cache rows in LDS, v_mfma_f32_16x16x4_f32; the cache is split over workgroups, a last launch adds the parts up.
+#include <hip/hip_runtime.h>
+
+#include "layers.h"
+
+using namespace ughip;
+
+namespace {
+
+typedef float f32x16 __attribute__((ext_vector_type(16)));
+typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
+
+// element e of a rotated part of `rot` elements at a table row: pairs (i, i + rot / 2)
+__device__ __forceinline__ float rotated(const float* part, int e, int rot, const float* cos, const float* sin) {
+  const int half = rot >> 1, i = e < half ? e : e - half;
+  const float u = part[i], v = part[i + half], c = cos[i], s = sin[i];
+  return e < half ? u * c - v * s : v * c + u * s;
+}
+
+__global__ void __launch_bounds__(256) latent_append_kernel(const float* __restrict__ kv, size_t kv_stride, const float* __restrict__ w, float eps,
+                                                            const float* __restrict__ cos, const float* __restrict__ sin, float* __restrict__ cache, size_t pos, int rank,
+                                                            int rot) {
+  __shared__ float red[4];
+  const float* row = kv + (size_t)blockIdx.x * kv_stride;
+  const size_t p = pos + blockIdx.x;
+  float ss = 0.f;
+  for (int c = threadIdx.x; c < rank; c += 256) ss += row[c] * row[c];
+  ss = block_sum<4>(ss, red);
+  const float inv = 1.f / sqrtf(ss / (float)rank + eps);
+  float* out = cache + p * (rank + rot);
+  for (int c = threadIdx.x; c < rank; c += 256) out[c] = row[c] * inv * w[c];
+  for (int e = threadIdx.x; e < rot; e += 256) out[rank + e] = rotated(row + rank, e, rot, cos + p * (rot / 2), sin + p * (rot / 2));
+}
+
+struct RowsArgs {
+  const float* q;
+  const void* k;
+  const void* v;
+  const float* cache;
+  const float* cos;
+  const float* sin;
+  float* dst;
+  size_t q_stride, v_stride, dst_stride;
+  int t, pos, heads, dim, rot, vdim, rank;
+  float scale;
+  bool vec;
+};
+
+template <typename T, int E>
+__device__ __forceinline__ u32x4_t pack_chunk(const float* v) {
+  if constexpr (sizeof(T) == 2) {
+    bf16x8 o;
+#pragma unroll
+    for (int i = 0; i < 8; ++i) o[i] = (__bf16)v[i];
+    return __builtin_bit_cast(u32x4_t, o);
+  } else {
+    return __builtin_bit_cast(u32x4_t, f32x4_t{v[0], v[1], v[2], v[3]});
+  }
+}
+
+template <typename T>
+__device__ __forceinline__ void mfma_chunk(const u32x4_t& a, const u32x4_t& b, f32x16& acc) {
+  if constexpr (sizeof(T) == 2) {
+    acc = __builtin_amdgcn_mfma_f32_32x32x16_bf16(__builtin_bit_cast(bf16x8, a), __builtin_bit_cast(bf16x8, b), acc, 0, 0, 0);
+  } else {
+    const f32x4_t x = __builtin_bit_cast(f32x4_t, a), y = __builtin_bit_cast(f32x4_t, b);
+    acc = __builtin_amdgcn_mfma_f32_32x32x2f32(x.x, y.x, acc, 0, 0, 0);
+    acc = __builtin_amdgcn_mfma_f32_32x32x2f32(x.y, y.y, acc, 0, 0, 0);
+    acc = __builtin_amdgcn_mfma_f32_32x32x2f32(x.z, y.z, acc, 0, 0, 0);
+    acc = __builtin_amdgcn_mfma_f32_32x32x2f32(x.w, y.w, acc, 0, 0, 0);
+  }
+}
+
+constexpr int KT = 64, QT = 128;
+template <typename T, int DQ, int DV>
+constexpr int rows_lds_bytes() {
+  return KT * (DQ * (int)sizeof(T) + 16) + DV * (KT * (int)sizeof(T) + 16);
+}
+
+// DQ >= dim + rot and DV >= vdim, the surplus is zeros.  T: uint16_t (bf16) or float.
+template <typename T, int DQ, int DV>
+__global__ void __launch_bounds__(256) latent_rows_kernel(RowsArgs a) {
+  constexpr int E = 16 / sizeof(T), QC = DQ / E, K_ROW = DQ * sizeof(T) + 16, V_ROW = KT * sizeof(T) + 16, VC = KT / E;
+  extern __shared__ __attribute__((aligned(16))) char lds[];
+  char* Ks = lds;                // [KT][DQ]
+  char* Vs = lds + KT * K_ROW;   // [DV][KT]
+  const int head = blockIdx.x, qb = gridDim.y - 1 - blockIdx.y;  // the longest rows first
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, col = lane & 31, hf = lane >> 5;
+  const int i_mine = qb * QT + wave * 32 + col, iq = i_mine < a.t ? i_mine : a.t - 1;
+  const int p_mine = a.pos + iq;
+  // the wave's queries, rotated, as the right operand of S^T: chunk 2 c + hf of query `col`
+  u32x4_t qf[QC / 2];
+  {
+    const float* qr = a.q + (size_t)iq * a.q_stride + (size_t)head * (a.dim + a.rot);
+    const float* cr = a.cos + (size_t)p_mine * (a.rot / 2);
+    const float* sr = a.sin + (size_t)p_mine * (a.rot / 2);
+#pragma unroll
+    for (int c = 0; c < QC / 2; ++c) {
+      float v[E];
+#pragma unroll
+      for (int e = 0; e < E; ++e) {
+        const int d = (2 * c + hf) * E + e;
+        v[e] = d < a.dim ? qr[d] : d < a.dim + a.rot ? rotated(qr + a.dim, d - a.dim, a.rot, cr, sr) : 0.f;
+      }
+      qf[c] = pack_chunk<T, E>(v);
+    }
+  }
+  f32x16 o[DV / 32];
+#pragma unroll
+  for (int i = 0; i < DV / 32; ++i)
+#pragma unroll
+    for (int e = 0; e < 16; ++e) o[i][e] = 0.f;
+  float mx = -INFINITY, sum = 0.f;
+  const int s_all = a.pos + a.t, last_q = min(a.t, (qb + 1) * QT), keys = a.pos + last_q;
+  const int cache_row = a.rank + a.rot;
+  for (int k0 = 0; k0 < keys; k0 += KT) {
+    __syncthreads();
+    for (int x = threadIdx.x; x < KT * QC; x += 256) {
+      const int key = x / QC, c = x % QC, d0 = c * E, kp = k0 + key;
+      u32x4_t chunk = {0, 0, 0, 0};
+      if (kp < s_all && d0 < a.dim + a.rot) {
+        const T* kr = static_cast<const T*>(a.k) + (size_t)kp * a.heads * a.dim + (size_t)head * a.dim;
+        const float* rr = a.cache + (size_t)kp * cache_row + a.rank;
+        if (a.vec && d0 < a.dim) {
+          chunk = *reinterpret_cast<const u32x4_t*>(kr + d0);
+        } else {
+          float v[E];
+#pragma unroll
+          for (int e = 0; e < E; ++e) {
+            const int d = d0 + e;
+            float f = 0.f;
+            if (d < a.dim) {
+              if constexpr (sizeof(T) == 2) f = bf16_to_f32(kr[d]);
+              else f = kr[d];
+            } else if (d < a.dim + a.rot) {
+              f = rr[d - a.dim];
+            }
+            v[e] = f;
+          }
+          chunk = pack_chunk<T, E>(v);
+        }
+      }
+      *reinterpret_cast<u32x4_t*>(Ks + key * K_ROW + c * 16) = chunk;
+    }
+    for (int x = threadIdx.x; x < DV * VC; x += 256) {
+      const int vc = x / VC, c = x % VC, kp = k0 + c * E;
+      u32x4_t chunk = {0, 0, 0, 0};
+      if (vc < a.vdim && kp < s_all) {
+        const T* vr = static_cast<const T*>(a.v) + ((size_t)head * a.vdim + vc) * a.v_stride;
+        if (kp + E <= s_all) {
+          chunk = *reinterpret_cast<const u32x4_t*>(vr + kp);  // rows are padded to whole tiles and 16-byte aligned
+        } else {  // values past the last position were never written
+          T v[E];
+#pragma unroll
+          for (int e = 0; e < E; ++e) v[e] = kp + e < s_all ? vr[kp + e] : T(0);
+          __builtin_memcpy(&chunk, v, 16);
+        }
+      }
+      *reinterpret_cast<u32x4_t*>(Vs + vc * V_ROW + c * 16) = chunk;
+    }
+    __syncthreads();
+    f32x16 s[2];
+#pragma unroll
+    for (int b = 0; b < 2; ++b) {
+#pragma unroll
+      for (int e = 0; e < 16; ++e) s[b][e] = 0.f;
+      const char* kr = Ks + (b * 32 + col) * K_ROW + hf * 16;
+#pragma unroll
+      for (int c = 0; c < QC / 2; ++c) mfma_chunk<T>(*reinterpret_cast<const u32x4_t*>(kr + c * 32), qf[c], s[b]);
+    }
+    // element e of s[b]: key k0 + 32 b + 8 (e / 4) + 4 hf + e % 4, query `col`
+    float top = mx;
+#pragma unroll
+    for (int b = 0; b < 2; ++b)
+#pragma unroll
+      for (int e = 0; e < 16; ++e) {
+        const int key = k0 + 32 * b + 8 * (e >> 2) + 4 * hf + (e & 3);
+        s[b][e] = key <= p_mine ? s[b][e] * a.scale : -INFINITY;
+        top = fmaxf(top, s[b][e]);
+      }
+    top = fmaxf(top, __shfl_xor(top, 32, 64));
+    const float alpha = expf(mx - top);  // key 0 is visible to everyone: top is finite
+    mx = top;
+    float part = 0.f;
+#pragma unroll
+    for (int b = 0; b < 2; ++b)
+#pragma unroll
+      for (int e = 0; e < 16; ++e) {
+        s[b][e] = expf(s[b][e] - top);
+        part += s[b][e];
+      }
+    sum = sum * alpha + part + __shfl_xor(part, 32, 64);
+#pragma unroll
+    for (int i = 0; i < DV / 32; ++i)
+#pragma unroll
+      for (int e = 0; e < 16; ++e) o[i][e] *= alpha;
+#pragma unroll
+    for (int b = 0; b < 2; ++b) {
+      if constexpr (sizeof(T) == 2) {
+#pragma unroll
+        for (int u = 0; u < 2; ++u) {
+          bf16x8 hi, lo;
+#pragma unroll
+          for (int e = 0; e < 8; ++e) {
+            hi[e] = (__bf16)s[b][8 * u + e];
+            lo[e] = (__bf16)(s[b][8 * u + e] - (float)hi[e]);
+          }
+#pragma unroll
+          for (int i = 0; i < DV / 32; ++i) {
+            const char* vr = Vs + (i * 32 + col) * V_ROW + (b * 32 + 16 * u + 4 * hf) * 2;
+            const uint2 v0 = *reinterpret_cast<const uint2*>(vr), v1 = *reinterpret_cast<const uint2*>(vr + 16);
+            const bf16x8 vf = __builtin_bit_cast(bf16x8, u32x4_t{v0.x, v0.y, v1.x, v1.y});
+            o[i] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(vf, hi, o[i], 0, 0, 0);
+            o[i] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(vf, lo, o[i], 0, 0, 0);
+          }
+        }
+      } else {
+#pragma unroll
+        for (int u = 0; u < 4; ++u)
+#pragma unroll
+          for (int i = 0; i < DV / 32; ++i) {
+            const f32x4_t v = *reinterpret_cast<const f32x4_t*>(Vs + (i * 32 + col) * V_ROW + (b * 32 + 8 * u + 4 * hf) * 4);
+            o[i] = __builtin_amdgcn_mfma_f32_32x32x2f32(v.x, s[b][4 * u], o[i], 0, 0, 0);
+            o[i] = __builtin_amdgcn_mfma_f32_32x32x2f32(v.y, s[b][4 * u + 1], o[i], 0, 0, 0);
+            o[i] = __builtin_amdgcn_mfma_f32_32x32x2f32(v.z, s[b][4 * u + 2], o[i], 0, 0, 0);
+            o[i] = __builtin_amdgcn_mfma_f32_32x32x2f32(v.w, s[b][4 * u + 3], o[i], 0, 0, 0);
+          }
+      }
+    }
+  }
+  if (i_mine >= a.t) return;
+  const float inv = 1.f / sum;
+  float* out = a.dst + (size_t)i_mine * a.dst_stride + (size_t)head * a.vdim;
+#pragma unroll
+  for (int i = 0; i < DV / 32; ++i)
+#pragma unroll
+    for (int e = 0; e < 16; ++e) {
+      const int vc = i * 32 + 8 * (e >> 2) + 4 * hf + (e & 3);
+      if (vc < a.vdim) out[vc] = o[i][e] * inv;
+    }
+}
+
+template <typename T, int DQ, int DV>
+hipError_t launch_rows(hipStream_t st, const RowsArgs& a) {
+  constexpr int bytes = rows_lds_bytes<T, DQ, DV>();
+  static_assert(bytes <= 160 * 1024, "tile does not fit LDS");
+  static const hipError_t attr = hipFuncSetAttribute(reinterpret_cast<const void*>(latent_rows_kernel<T, DQ, DV>), hipFuncAttributeMaxDynamicSharedMemorySize, bytes);
+  if (attr != hipSuccess) return attr;
+  latent_rows_kernel<T, DQ, DV><<<dim3((unsigned)a.heads, (unsigned)((a.t + QT - 1) / QT)), 256, bytes, st>>>(a);
+  return hipGetLastError();
+}
+template <typename T>
+hipError_t launch_rows_any(hipStream_t st, const RowsArgs& a) {
+  const int dq = a.dim + a.rot;
+  if (dq <= 64 && a.vdim <= 64) return launch_rows<T, 64, 64>(st, a);
+  if (dq <= 128 && a.vdim <= 128) return launch_rows<T, 128, 128>(st, a);
+  if (dq <= 192 && a.vdim <= 128) return launch_rows<T, 192, 128>(st, a);
+  return launch_rows<T, 256, 256>(st, a);
+}
+
+// ---- few positions ----------------------------------------------------------------------------------------------------------
+template <typename WT>
+__device__ __forceinline__ float w_f32(WT v) {
+  if constexpr (sizeof(WT) == 2) return bf16_to_f32(v);
+  else return v;
+}
+
+// qa[(i heads + h), 0 .. rank) = scale * sum_d q_h[d] w_uk[h dim + d, :], then the rotated part (scaled too).  A workgroup takes a
+// head and 128 columns; eight groups of 32 threads share d.
+template <typename WT>
+__global__ void __launch_bounds__(256) latent_absorb_kernel(const float* __restrict__ q, size_t q_stride, const WT* __restrict__ w, const float* __restrict__ cos,
+                                                            const float* __restrict__ sin, float* __restrict__ qa, int t, int pos, int heads, int dim, int rot, int rank,
+                                                            float scale) {
+  __shared__ float part[8][128];
+  const int h = blockIdx.x, c0 = blockIdx.y * 128, cg = threadIdx.x & 31, dg = threadIdx.x >> 5, L = rank + rot;
+  const int i = blockIdx.z;
+  const float* qr = q + (size_t)i * q_stride + (size_t)h * (dim + rot);
+  float* out = qa + ((size_t)i * heads + h) * L;
+  float acc[4] = {0.f, 0.f, 0.f, 0.f};
+  const int c = c0 + cg * 4;
+  for (int d = dg; d < dim; d += 8) {
+    const float qv = qr[d];
+    const WT* wr = w + ((size_t)h * dim + d) * rank;
+#pragma unroll
+    for (int e = 0; e < 4; ++e)
+      if (c + e < rank) acc[e] += qv * w_f32(wr[c + e]);
+  }
+#pragma unroll
+  for (int e = 0; e < 4; ++e) part[dg][cg * 4 + e] = acc[e];
+  __syncthreads();
+  if (threadIdx.x < 128 && c0 + (int)threadIdx.x < rank) {
+    float v = 0.f;
+#pragma unroll
+    for (int g = 0; g < 8; ++g) v += part[g][threadIdx.x];
+    out[c0 + threadIdx.x] = v * scale;
+  }
+  if (blockIdx.y == 0) {
+    const size_t p = (size_t)(pos + i) * (rot / 2);
+    for (int e = threadIdx.x; e < rot; e += 256) out[rank + e] = rotated(qr + dim, e, rot, cos + p, sin + p) * scale;
+  }
+}
+
+struct SplitArgs {
+  const float* qa;
+  const float* cache;
+  float* acc;  // [splits, rows, rank]
+  float* ml;   // [splits, rows, 2]
+  int rows, heads, pos, keys, rank, L, tiles_per_split;
+};
+
+constexpr int SK = 32, S_ROW = SK + 4;
+__host__ __device__ inline int split_row(int L) { return ((L + 15) & ~15) + 4; }
+inline size_t split_lds_bytes(int L) { return ((size_t)(SK + 16) * split_row(L) + 3 * 16 * S_ROW + 48) * sizeof(float); }
+
+template <int NT>  // 16-column tiles of the result per wave
+__global__ void __launch_bounds__(256) latent_split_kernel(SplitArgs a) {
+  extern __shared__ __attribute__((aligned(16))) float sl[];
+  const int ld = split_row(a.L), Lp = (a.L + 15) & ~15;
+  float* Ks = sl;                     // [SK][ld]
+  float* Qs = Ks + SK * ld;           // [16][ld]
+  float* Sp = Qs + 16 * ld;           // [2][16][S_ROW] halves of the scores
+  float* Ps = Sp + 2 * 16 * S_ROW;    // [16][S_ROW]
+  float* mrow = Ps + 16 * S_ROW;      // running maximum, sum, and this tile's factor
+  float* lrow = mrow + 16;
+  float* arow = lrow + 16;
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, j = lane & 15, g = lane >> 4;
+  const int r0 = blockIdx.x * 16, split = blockIdx.y;
+  for (int x = threadIdx.x; x < 16 * Lp; x += 256) {
+    const int r = x / Lp, c = x % Lp;
+    Qs[r * ld + c] = r0 + r < a.rows && c < a.L ? a.qa[(size_t)(r0 + r) * a.L + c] : 0.f;
+  }
+  if (threadIdx.x < 16) mrow[threadIdx.x] = -INFINITY, lrow[threadIdx.x] = 0.f;
+  f32x4_t acc[NT];
+#pragma unroll
+  for (int i = 0; i < NT; ++i) acc[i] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+  const int k_begin = split * a.tiles_per_split * SK, k_stop = min(a.keys, k_begin + a.tiles_per_split * SK);
+  for (int k0 = k_begin; k0 < k_stop; k0 += SK) {
+    __syncthreads();
+    if (a.L % 4 == 0) {
+      const int l4 = Lp / 4;
+      for (int x = threadIdx.x; x < SK * l4; x += 256) {
+        const int r = x / l4, c = (x % l4) * 4;
+        *reinterpret_cast<f32x4_t*>(Ks + r * ld + c) =
+            k0 + r < k_stop && c < a.L ? *reinterpret_cast<const f32x4_t*>(a.cache + (size_t)(k0 + r) * a.L + c) : f32x4_t{0.f, 0.f, 0.f, 0.f};
+      }
+    } else {
+      for (int x = threadIdx.x; x < SK * Lp; x += 256) {
+        const int r = x / Lp, c = x % Lp;
+        Ks[r * ld + c] = k0 + r < k_stop && c < a.L ? a.cache[(size_t)(k0 + r) * a.L + c] : 0.f;
+      }
+    }
+    __syncthreads();
+    {  // wave: 16 keys (wave % 2), every other run of 16 elements (wave / 2)
+      f32x4_t s = {0.f, 0.f, 0.f, 0.f};
+      const int kb = (wave & 1) * 16;
+      for (int c = (wave >> 1) * 16; c < Lp; c += 32) {
+        const f32x4_t x = *reinterpret_cast<const f32x4_t*>(Qs + j * ld + c + 4 * g), y = *reinterpret_cast<const f32x4_t*>(Ks + (kb + j) * ld + c + 4 * g);
+        s = __builtin_amdgcn_mfma_f32_16x16x4f32(x.x, y.x, s, 0, 0, 0);
+        s = __builtin_amdgcn_mfma_f32_16x16x4f32(x.y, y.y, s, 0, 0, 0);
+        s = __builtin_amdgcn_mfma_f32_16x16x4f32(x.z, y.z, s, 0, 0, 0);
+        s = __builtin_amdgcn_mfma_f32_16x16x4f32(x.w, y.w, s, 0, 0, 0);
+      }
+#pragma unroll
+      for (int e = 0; e < 4; ++e) Sp[((wave >> 1) * 16 + 4 * g + e) * S_ROW + kb + j] = s[e];
+    }
+    __syncthreads();
+    {  // row 4 wave + g, keys j and j + 16
+      const int r = 4 * wave + g, limit = a.pos + (r0 + r) / a.heads;
+      float s0 = Sp[r * S_ROW + j] + Sp[(16 + r) * S_ROW + j], s1 = Sp[r * S_ROW + j + 16] + Sp[(16 + r) * S_ROW + j + 16];
+      if (k0 + j > limit || k0 + j >= k_stop) s0 = -INFINITY;
+      if (k0 + j + 16 > limit || k0 + j + 16 >= k_stop) s1 = -INFINITY;
+      float top = fmaxf(s0, s1);
+      for (int d = 8; d; d >>= 1) top = fmaxf(top, __shfl_xor(top, d, 64));
+      const float before = mrow[r];
+      top = fmaxf(top, before);
+      const float base = top == -INFINITY ? 0.f : top;  // nothing of this split is visible to the row so far
+      const float p0 = expf(s0 - base), p1 = expf(s1 - base), alpha = expf(before - base);
+      float part = p0 + p1;
+      for (int d = 8; d; d >>= 1) part += __shfl_xor(part, d, 64);
+      Ps[r * S_ROW + j] = p0;
+      Ps[r * S_ROW + j + 16] = p1;
+      if (j == 0) {
+        mrow[r] = top;
+        lrow[r] = lrow[r] * alpha + part;
+        arow[r] = alpha;
+      }
+    }
+    __syncthreads();
+    float al[4];
+#pragma unroll
+    for (int e = 0; e < 4; ++e) al[e] = arow[4 * g + e];
+    float pf[SK / 4];
+#pragma unroll
+    for (int kk = 0; kk < SK / 4; ++kk) pf[kk] = Ps[j * S_ROW + 4 * kk + g];
+#pragma unroll
+    for (int i = 0; i < NT; ++i) {
+      const int c0 = (wave + 4 * i) * 16;
+      if (c0 >= a.rank) continue;  // uniform over the wave (columns up to Lp exist in LDS)
+#pragma unroll
+      for (int e = 0; e < 4; ++e) acc[i][e] *= al[e];
+#pragma unroll
+      for (int kk = 0; kk < SK / 4; ++kk) acc[i] = __builtin_amdgcn_mfma_f32_16x16x4f32(pf[kk], Ks[(4 * kk + g) * ld + c0 + j], acc[i], 0, 0, 0);
+    }
+  }
+  __syncthreads();
+#pragma unroll
+  for (int i = 0; i < NT; ++i) {
+    const int c = (wave + 4 * i) * 16 + j;
+    if (c >= a.rank) continue;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      const int r = r0 + 4 * g + e;
+      if (r < a.rows) a.acc[((size_t)split * a.rows + r) * a.rank + c] = acc[i][e];
+    }
+  }
+  if (threadIdx.x < 16 && r0 + (int)threadIdx.x < a.rows) {
+    float* o = a.ml + ((size_t)split * a.rows + r0 + threadIdx.x) * 2;
+    o[0] = mrow[threadIdx.x];
+    o[1] = lrow[threadIdx.x];
+  }
+}
+
+// The parts of one (position, head) added up, then 16 elements of the head's result through the values' up-projection.
+constexpr int MERGE_V = 16;
+template <typename WT>
+__global__ void __launch_bounds__(256) latent_merge_kernel(const float* __restrict__ acc, const float* __restrict__ ml, const WT* __restrict__ w, float* __restrict__ dst,
+                                                           size_t dst_stride, int rows, int splits, int heads, int rank, int vdim) {
+  extern __shared__ __attribute__((aligned(16))) float sl[];
+  float* lat = sl;              // [rank]
+  float* fac = sl + ((rank + 3) & ~3);  // [splits]
+  const int h = blockIdx.x, i = blockIdx.y, v0 = blockIdx.z * MERGE_V, row = i * heads + h;
+  float top = -INFINITY;
+  for (int s = 0; s < splits; ++s) top = fmaxf(top, ml[((size_t)s * rows + row) * 2]);
+  float sum = 0.f;
+  for (int s = 0; s < splits; ++s) sum += expf(ml[((size_t)s * rows + row) * 2] - top) * ml[((size_t)s * rows + row) * 2 + 1];
+  for (int s = threadIdx.x; s < splits; s += 256) fac[s] = expf(ml[((size_t)s * rows + row) * 2] - top) / sum;
+  __syncthreads();
+  for (int c = threadIdx.x; c < rank; c += 256) {
+    float v = 0.f;
+    for (int s = 0; s < splits; ++s) v += fac[s] * acc[((size_t)s * rows + row) * rank + c];
+    lat[c] = v;
+  }
+  __syncthreads();
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  for (int v = v0 + wave; v < min(vdim, v0 + MERGE_V); v += 4) {
+    const WT* wr = w + ((size_t)h * vdim + v) * rank;
+    float s = 0.f;
+    for (int c = lane; c < rank; c += 64) s += w_f32(wr[c]) * lat[c];
+    for (int d = 32; d; d >>= 1) s += __shfl_xor(s, d, 64);
+    if (lane == 0) dst[(size_t)i * dst_stride + (size_t)h * vdim + v] = s;
+  }
+}
+
+int check_tables(const ughip_device* dev, const ughip_slice* cos, const ughip_slice* sin, size_t table_rows, size_t pos, size_t t, size_t rot, const char* what) {
+  if (rot == 0 || rot % 2 != 0) return set_error(UGHIP_ERR_INVALID, "%s: a rotated part of %zu elements", what, rot);
+  if (pos + t > table_rows) return set_error(UGHIP_ERR_BOUNDS, "%s: positions up to %zu, tables for %zu", what, pos + t, table_rows);
+  for (const ughip_slice* s : {cos, sin})
+    if (int rc = check_buf(dev, s, table_rows * (rot / 2), UGHIP_F32, what)) return rc;
+  return UGHIP_OK;
+}
+
+}  // namespace
+
+extern "C" int ughip_latent_append(ughip_device* dev, ughip_view kv, const ughip_slice* w, float eps, const ughip_slice* cos, const ughip_slice* sin, size_t table_rows,
+                                   ughip_slice* cache, size_t cap, size_t pos, size_t t, size_t rank, size_t rot) {
+  const char* what = "latent_append";
+  if (!dev) return set_error(UGHIP_ERR_INVALID, "%s: null device", what);
+  if (rank == 0 || rank > 65536) return set_error(UGHIP_ERR_INVALID, "%s: rank %zu", what, rank);
+  if (int rc = check_view(dev, kv, t, rank + rot, UGHIP_F32, what)) return rc;
+  if (int rc = check_buf(dev, w, rank, UGHIP_F32, what)) return rc;
+  if (int rc = check_tables(dev, cos, sin, table_rows, pos, t, rot, what)) return rc;
+  if (pos + t > cap) return set_error(UGHIP_ERR_BOUNDS, "%s: %zu rows exceed the cache's %zu", what, pos + t, cap);
+  if (int rc = check_buf(dev, cache, cap * (rank + rot), UGHIP_F32, what)) return rc;
+  if (t == 0) return UGHIP_OK;
+  if (int rc = device_activate(dev)) return rc;
+  latent_append_kernel<<<(unsigned)t, 256, 0, dev->stream>>>(view_ptr<float>(kv), kv.stride, buf_ptr<float>(w), eps, buf_ptr<float>(cos), buf_ptr<float>(sin),
+                                                             static_cast<float*>(cache->ptr), pos, (int)rank, (int)rot);
+  UGHIP_HIPCHK(hipGetLastError());
+  return UGHIP_OK;
+}
+
+extern "C" int ughip_latent_attention_rows(ughip_device* dev, ughip_view q, const ughip_slice* k, const ughip_slice* v_t, size_t v_stride, const ughip_slice* cache,
+                                           const ughip_slice* cos, const ughip_slice* sin, size_t table_rows, ughip_view dst, size_t t, size_t pos, size_t heads, size_t dim,
+                                           size_t rot, size_t vdim, size_t rank, float scale) {
+  const char* what = "latent_attention_rows";
+  if (!dev || !k || !v_t) return set_error(UGHIP_ERR_INVALID, "%s: null argument", what);
+  if (heads == 0 || dim == 0 || vdim == 0 || rank == 0 || dim + rot > 256 || vdim > 256 || heads > 65535)
+    return set_error(UGHIP_ERR_UNSUPPORTED, "%s: heads %zu of %zu + %zu and %zu elements (built for up to 256)", what, heads, dim, rot, vdim);
+  const size_t s = pos + t;
+  if (s > 0x3fffffffull || v_stride % 64 != 0 || v_stride < s) return set_error(UGHIP_ERR_INVALID, "%s: %zu positions, value rows of %zu (whole tiles of 64)", what, s, v_stride);
+  if (k->dtype != v_t->dtype || (k->dtype != UGHIP_F32 && k->dtype != UGHIP_BF16)) return set_error(UGHIP_ERR_UNSUPPORTED, "%s: keys and values are both F32 or both BF16", what);
+  if (int rc = check_view(dev, q, t, heads * (dim + rot), UGHIP_F32, what)) return rc;
+  if (int rc = check_buf(dev, k, s * heads * dim, -1, what)) return rc;
+  if (int rc = check_buf(dev, v_t, heads * vdim * v_stride, -1, what)) return rc;
+  if (int rc = check_buf(dev, cache, s * (rank + rot), UGHIP_F32, what)) return rc;
+  if (int rc = check_tables(dev, cos, sin, table_rows, pos, t, rot, what)) return rc;
+  if (int rc = check_view(dev, dst, t, heads * vdim, UGHIP_F32, what)) return rc;
+  if (t == 0) return UGHIP_OK;
+  if ((t + QT - 1) / QT > 65535) return set_error(UGHIP_ERR_UNSUPPORTED, "%s: too many positions", what);
+  if (int rc = device_activate(dev)) return rc;
+  RowsArgs a{view_ptr<float>(q), k->ptr, v_t->ptr, buf_ptr<float>(cache), buf_ptr<float>(cos), buf_ptr<float>(sin), view_ptr<float>(dst), q.stride, v_stride, dst.stride,
+             (int)t, (int)pos, (int)heads, (int)dim, (int)rot, (int)vdim, (int)rank, scale, dim % 8 == 0};
+  UGHIP_HIPCHK(k->dtype == UGHIP_BF16 ? launch_rows_any<uint16_t>(dev->stream, a) : launch_rows_any<float>(dev->stream, a));
+  return UGHIP_OK;
+}
+
+extern "C" int ughip_latent_attention_absorbed(ughip_device* dev, ughip_view q, const ughip_slice* w_uk, const ughip_slice* w_uv, const ughip_slice* cache,
+                                               const ughip_slice* cos, const ughip_slice* sin, size_t table_rows, ughip_view dst, size_t t, size_t pos, size_t heads,
+                                               size_t dim, size_t rot, size_t vdim, size_t rank, float scale) {
+  const char* what = "latent_attention_absorbed";
+  if (!dev || !w_uk || !w_uv) return set_error(UGHIP_ERR_INVALID, "%s: null argument", what);
+  if (heads == 0 || dim == 0 || vdim == 0 || rank == 0 || heads > 65535 || t > 65535) return set_error(UGHIP_ERR_INVALID, "%s: bad shape", what);
+  const size_t s = pos + t, L = rank + rot, rows = t * heads;
+  if (s > 0x3fffffffull || rows > 0x3fffffffull) return set_error(UGHIP_ERR_INVALID, "%s: %zu positions", what, s);
+  if (rank > 1024 || split_lds_bytes((int)L) > 160 * 1024) return set_error(UGHIP_ERR_UNSUPPORTED, "%s: latents of %zu + %zu elements", what, rank, rot);
+  if (w_uk->dtype != w_uv->dtype || (w_uk->dtype != UGHIP_F32 && w_uk->dtype != UGHIP_BF16)) return set_error(UGHIP_ERR_UNSUPPORTED, "%s: matrices are both F32 or both BF16", what);
+  if (int rc = check_view(dev, q, t, heads * (dim + rot), UGHIP_F32, what)) return rc;
+  if (int rc = check_buf(dev, w_uk, heads * dim * rank, -1, what)) return rc;
+  if (int rc = check_buf(dev, w_uv, heads * vdim * rank, -1, what)) return rc;
+  if (int rc = check_buf(dev, cache, s * L, UGHIP_F32, what)) return rc;
+  if (int rc = check_tables(dev, cos, sin, table_rows, pos, t, rot, what)) return rc;
+  if (int rc = check_view(dev, dst, t, heads * vdim, UGHIP_F32, what)) return rc;
+  if (t == 0) return UGHIP_OK;
+  if (int rc = device_activate(dev)) return rc;
+  const size_t tiles = (s + SK - 1) / SK, row_blocks = (rows + 15) / 16;
+  size_t splits = row_blocks >= 256 ? 1 : 256 / row_blocks;
+  if (splits > 64) splits = 64;
+  if (splits > tiles) splits = tiles;
+  const size_t per = (tiles + splits - 1) / splits;
+  splits = (tiles + per - 1) / per;
+  auto up = [](size_t v) { return (v + 63) & ~(size_t)63; };
+  const size_t n_qa = up(rows * L), n_ml = up(splits * rows * 2), n_acc = splits * rows * rank;
+  void* ws = nullptr;
+  if (int rc = rows_scratch(dev, (n_qa + n_ml + n_acc) * sizeof(float), &ws)) return rc;
+  float* qa = static_cast<float*>(ws);
+  SplitArgs a{qa, buf_ptr<float>(cache), qa + n_qa + n_ml, qa + n_qa, (int)rows, (int)heads, (int)pos, (int)s, (int)rank, (int)L, (int)per};
+  const dim3 g1((unsigned)heads, (unsigned)((rank + 127) / 128), (unsigned)t);
+  const bool bf = w_uk->dtype == UGHIP_BF16;
+  if (bf) latent_absorb_kernel<uint16_t><<<g1, 256, 0, dev->stream>>>(view_ptr<float>(q), q.stride, buf_ptr<uint16_t>(w_uk), buf_ptr<float>(cos), buf_ptr<float>(sin), qa, (int)t,
+                                                                     (int)pos, (int)heads, (int)dim, (int)rot, (int)rank, scale);
+  else latent_absorb_kernel<float><<<g1, 256, 0, dev->stream>>>(view_ptr<float>(q), q.stride, buf_ptr<float>(w_uk), buf_ptr<float>(cos), buf_ptr<float>(sin), qa, (int)t,
+                                                               (int)pos, (int)heads, (int)dim, (int)rot, (int)rank, scale);
+  UGHIP_HIPCHK(hipGetLastError());
+  const dim3 g2((unsigned)row_blocks, (unsigned)splits);
+  const size_t lds = split_lds_bytes((int)L);
+  static const hipError_t attr = [] {
+    hipError_t e = hipSuccess;
+    for (const void* f : {reinterpret_cast<const void*>(latent_split_kernel<2>), reinterpret_cast<const void*>(latent_split_kernel<4>),
+                          reinterpret_cast<const void*>(latent_split_kernel<8>), reinterpret_cast<const void*>(latent_split_kernel<16>)})
+      if (e == hipSuccess) e = hipFuncSetAttribute(f, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
+    return e;
+  }();
+  UGHIP_HIPCHK(attr);
+  if (rank <= 128) latent_split_kernel<2><<<g2, 256, lds, dev->stream>>>(a);
+  else if (rank <= 256) latent_split_kernel<4><<<g2, 256, lds, dev->stream>>>(a);
+  else if (rank <= 512) latent_split_kernel<8><<<g2, 256, lds, dev->stream>>>(a);
+  else latent_split_kernel<16><<<g2, 256, lds, dev->stream>>>(a);
+  UGHIP_HIPCHK(hipGetLastError());
+  const dim3 g3((unsigned)heads, (unsigned)t, (unsigned)((vdim + MERGE_V - 1) / MERGE_V));
+  const size_t lds3 = (((rank + 3) & ~(size_t)3) + splits) * sizeof(float);
+  if (bf) latent_merge_kernel<uint16_t><<<g3, 256, lds3, dev->stream>>>(a.acc, a.ml, buf_ptr<uint16_t>(w_uv), view_ptr<float>(dst), dst.stride, (int)rows, (int)splits, (int)heads,
+                                                                       (int)rank, (int)vdim);
+  else latent_merge_kernel<float><<<g3, 256, lds3, dev->stream>>>(a.acc, a.ml, buf_ptr<float>(w_uv), view_ptr<float>(dst), dst.stride, (int)rows, (int)splits, (int)heads,
+                                                                 (int)rank, (int)vdim);
+  UGHIP_HIPCHK(hipGetLastError());
+  return UGHIP_OK;
+}

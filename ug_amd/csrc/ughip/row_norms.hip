@@ -1,0 +1,150 @@
+// Lookups and RMS norms over rows (ughip_layers.h): a workgroup per row (or per part of a row), the row in LDS between the
+// pass that sums its squares and the pass that scales it.
+#include <hip/hip_runtime.h>
+
+#include "bf16_split.h"
+#include "layers.h"
+
+using namespace ughip;
+
+namespace {
+
+template <typename T>
+__global__ void __launch_bounds__(256) gather_rows_kernel(const T* __restrict__ table, int table_rows, size_t stride, size_t col, int cols, const int* __restrict__ ids,
+                                                          float* __restrict__ dst, size_t dst_stride) {
+  const int row = blockIdx.y, id = ids[row];
+  const int c = blockIdx.x * 256 + threadIdx.x;
+  if (c >= cols) return;
+  float v = __uint_as_float(0x7fc00000u);
+  if (id >= 0 && id < table_rows) {
+    const T e = table[(size_t)id * stride + col + c];
+    if constexpr (sizeof(T) == 2) v = bf16_to_f32(e);
+    else v = e;
+  }
+  dst[(size_t)row * dst_stride + c] = v;
+}
+
+struct AddNormArgs {
+  const float* x;
+  const float* y;
+  const float* w;
+  float* dst;
+  size_t x_stride, y_stride, dst_stride;
+  const int* slots;
+  const float* weights;
+  int top, y_rows, n;
+  float eps;
+};
+
+__global__ void __launch_bounds__(256) add_rms_norm_kernel(AddNormArgs a) {
+  extern __shared__ float row[];
+  __shared__ float red[4];
+  const size_t i = blockIdx.x;
+  float ss = 0.f;
+  if (a.slots) {
+    for (int c = threadIdx.x; c < a.n; c += 256) {
+      float v = 0.f;
+      for (int j = 0; j < a.top; ++j) {
+        const int r = a.slots[i * a.top + j];
+        if (r >= 0 && r < a.y_rows) v += a.weights[i * a.top + j] * a.y[(size_t)r * a.y_stride + c];
+      }
+      row[c] = v;
+      ss += v * v;
+    }
+  } else {
+    for (int c = threadIdx.x; c < a.n; c += 256) {
+      const float v = a.y[i * a.y_stride + c];
+      row[c] = v;
+      ss += v * v;
+    }
+  }
+  ss = block_sum<4>(ss, red);
+  const float inv = 1.f / sqrtf(ss / (float)a.n + a.eps);
+  for (int c = threadIdx.x; c < a.n; c += 256) {
+    const float v = row[c] * inv * a.w[c];  // every thread reads back its own elements
+    a.dst[i * a.dst_stride + c] = a.x ? a.x[i * a.x_stride + c] + v : v;
+  }
+}
+
+__global__ void __launch_bounds__(256) gated_rms_norm_kernel(const float* __restrict__ y, size_t y_stride, const float* __restrict__ z, size_t z_stride,
+                                                             const float* __restrict__ w, float eps, float* __restrict__ dst, size_t dst_stride, int part) {
+  extern __shared__ float row[];
+  __shared__ float red[4];
+  const size_t i = blockIdx.x, c0 = (size_t)blockIdx.y * part;
+  float ss = 0.f;
+  for (int c = threadIdx.x; c < part; c += 256) {
+    float g = y[i * y_stride + c0 + c];
+    if (z) g *= silu_f(z[i * z_stride + c0 + c]);
+    row[c] = g;
+    ss += g * g;
+  }
+  ss = block_sum<4>(ss, red);
+  const float inv = 1.f / sqrtf(ss / (float)part + eps);
+  for (int c = threadIdx.x; c < part; c += 256) dst[i * dst_stride + c0 + c] = row[c] * inv * w[c0 + c];
+}
+
+constexpr size_t ROW_MAX = 16000;  // the row and the reduction fit the 64 KiB a launch gets without asking
+
+}  // namespace
+
+extern "C" int ughip_gather_rows(ughip_device* dev, const ughip_slice* table, size_t table_rows, size_t stride, size_t col, size_t cols, const ughip_slice* ids, size_t m,
+                                 ughip_view dst) {
+  if (!dev || !table) return set_error(UGHIP_ERR_INVALID, "gather_rows: null argument");
+  if (table->dtype != UGHIP_F32 && table->dtype != UGHIP_BF16) return set_error(UGHIP_ERR_UNSUPPORTED, "gather_rows: a table is F32 or BF16");
+  if (int rc = check_view(dev, ughip_view{const_cast<ughip_slice*>(table), 0, stride}, table_rows, stride, -1, "gather_rows table")) return rc;
+  if (col > stride || cols > stride - col) return set_error(UGHIP_ERR_BOUNDS, "gather_rows: columns %zu + %zu of rows of %zu", col, cols, stride);
+  if (int rc = check_buf(dev, ids, m, UGHIP_I32, "gather_rows ids")) return rc;
+  if (int rc = check_view(dev, dst, m, cols, UGHIP_F32, "gather_rows dst")) return rc;
+  if (m == 0 || cols == 0) return UGHIP_OK;
+  if (m > 65535) return set_error(UGHIP_ERR_UNSUPPORTED, "gather_rows: up to 65535 rows");
+  if (int rc = device_activate(dev)) return rc;
+  const dim3 grid((unsigned)((cols + 255) / 256), (unsigned)m);
+  float* d = view_ptr<float>(dst);
+  if (table->dtype == UGHIP_F32)
+    gather_rows_kernel<float><<<grid, 256, 0, dev->stream>>>(buf_ptr<float>(table), (int)table_rows, stride, col, (int)cols, buf_ptr<int>(ids), d, dst.stride);
+  else
+    gather_rows_kernel<uint16_t><<<grid, 256, 0, dev->stream>>>(buf_ptr<uint16_t>(table), (int)table_rows, stride, col, (int)cols, buf_ptr<int>(ids), d, dst.stride);
+  UGHIP_HIPCHK(hipGetLastError());
+  return UGHIP_OK;
+}
+
+extern "C" int ughip_add_rms_norm_rows(ughip_device* dev, ughip_view x, ughip_view y, const ughip_slice* slots, const ughip_slice* weights, size_t top, size_t y_rows,
+                                       const ughip_slice* w, float eps, ughip_view dst, size_t m, size_t n) {
+  if (!dev) return set_error(UGHIP_ERR_INVALID, "add_rms_norm_rows: null device");
+  if (n > ROW_MAX) return set_error(UGHIP_ERR_UNSUPPORTED, "add_rms_norm_rows: rows of %zu elements, up to %zu are supported", n, ROW_MAX);
+  if (x.s)
+    if (int rc = check_view(dev, x, m, n, UGHIP_F32, "add_rms_norm_rows x")) return rc;
+  if (int rc = check_view(dev, y, slots ? y_rows : m, n, UGHIP_F32, "add_rms_norm_rows y")) return rc;
+  if (slots) {
+    if (top == 0 || top > 4096) return set_error(UGHIP_ERR_INVALID, "add_rms_norm_rows: top %zu", top);
+    if (int rc = check_buf(dev, slots, m * top, UGHIP_I32, "add_rms_norm_rows slots")) return rc;
+    if (int rc = check_buf(dev, weights, m * top, UGHIP_F32, "add_rms_norm_rows weights")) return rc;
+  }
+  if (int rc = check_buf(dev, w, n, UGHIP_F32, "add_rms_norm_rows w")) return rc;
+  if (int rc = check_view(dev, dst, m, n, UGHIP_F32, "add_rms_norm_rows dst")) return rc;
+  if (m == 0 || n == 0) return UGHIP_OK;
+  if (int rc = device_activate(dev)) return rc;
+  AddNormArgs a{view_ptr<float>(x), view_ptr<float>(y), buf_ptr<float>(w), view_ptr<float>(dst), x.stride, y.stride, dst.stride, buf_ptr<int>(slots), buf_ptr<float>(weights),
+                (int)top, (int)y_rows, (int)n, eps};
+  add_rms_norm_kernel<<<(unsigned)m, 256, n * sizeof(float), dev->stream>>>(a);
+  UGHIP_HIPCHK(hipGetLastError());
+  return UGHIP_OK;
+}
+
+extern "C" int ughip_gated_rms_norm_rows(ughip_device* dev, ughip_view y, ughip_view z, const ughip_slice* w, float eps, size_t groups, ughip_view dst, size_t m, size_t n) {
+  if (!dev) return set_error(UGHIP_ERR_INVALID, "gated_rms_norm_rows: null device");
+  if (groups == 0 || n % groups != 0 || groups > 65535) return set_error(UGHIP_ERR_INVALID, "gated_rms_norm_rows: %zu elements in %zu groups", n, groups);
+  if (n / groups > ROW_MAX) return set_error(UGHIP_ERR_UNSUPPORTED, "gated_rms_norm_rows: groups of up to %zu elements", ROW_MAX);
+  if (int rc = check_view(dev, y, m, n, UGHIP_F32, "gated_rms_norm_rows y")) return rc;
+  if (z.s)
+    if (int rc = check_view(dev, z, m, n, UGHIP_F32, "gated_rms_norm_rows z")) return rc;
+  if (int rc = check_buf(dev, w, n, UGHIP_F32, "gated_rms_norm_rows w")) return rc;
+  if (int rc = check_view(dev, dst, m, n, UGHIP_F32, "gated_rms_norm_rows dst")) return rc;
+  if (m == 0 || n == 0) return UGHIP_OK;
+  if (int rc = device_activate(dev)) return rc;
+  const size_t part = n / groups;
+  gated_rms_norm_kernel<<<dim3((unsigned)m, (unsigned)groups), 256, part * sizeof(float), dev->stream>>>(view_ptr<float>(y), y.stride, view_ptr<float>(z), z.stride,
+                                                                                                        buf_ptr<float>(w), eps, view_ptr<float>(dst), dst.stride, (int)part);
+  UGHIP_HIPCHK(hipGetLastError());
+  return UGHIP_OK;
+}

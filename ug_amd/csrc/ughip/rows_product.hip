@@ -1,0 +1,348 @@
+// Products of rows of any size with their neighbours folded in (ughip_product_rows): y = x w^T for m >= 1 rows, any n and k,
+// x / w / result as F32 or BF16, bias, SwiGLU or gated-lookup epilogues, and the grouped form (rows sorted by expert, a
+// matrix per group, rows of x gathered on their way in).
+//
+// A workgroup of four waves (2 x 2) takes a 64 MI x 64 NI tile.  A K step is 128 bytes of every row in LDS: 64 bf16 or 32
+// floats, in eight 16-byte chunks; rows are 144 bytes apart, which spreads the 16-byte reads of 32 consecutive rows over all
+// banks.  Two LDS buffers: while one step is multiplied the next one's elements are in flight to registers.  Whatever type
+// the operands are stored in, they are converted between registers and LDS; the products are v_mfma_f32_32x32x16_bf16 or, for
+// F32, four v_mfma_f32_32x32x2_f32 per chunk (k taken chunk by chunk: lanes 0-31 the even, lanes 32-63 the odd one).
+#include <hip/hip_runtime.h>
+
+#include "bf16_split.h"
+#include "layers.h"
+
+using namespace ughip;
+
+namespace {
+
+typedef float f32x16 __attribute__((ext_vector_type(16)));
+typedef float f32x8 __attribute__((ext_vector_type(8)));
+typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
+typedef __bf16 bf16x4 __attribute__((ext_vector_type(4)));
+
+struct ProductArgs {
+  const void* x;
+  const void* w;
+  const void* w_up;
+  const float* bias;
+  const float* bias_up;
+  void* dst;
+  size_t x_stride, w_stride, dst_stride, w_group;  // elements; w_group: from one group's matrix to the next
+  int m, n, k;
+  bool dst_bf16;
+  const void* table;
+  const int* ids;
+  size_t table_stride, table_col;
+  int table_rows;
+  bool table_bf16;
+  const int* row_index;
+  const int* group_end;
+  int groups, x_rows;
+};
+
+constexpr int ROW_BYTES = 144, CHUNKS = 8;
+
+// One 16-byte LDS chunk's worth of a row, as it is stored: 8 elements for bf16 products, 4 for f32 ones.
+template <typename CT, typename ST>
+struct Raw;
+template <>
+struct Raw<__bf16, float> {
+  f32x4_t a, b;
+  __device__ u32x4_t pack() const {
+    const f32x8 v = {a.x, a.y, a.z, a.w, b.x, b.y, b.z, b.w};
+    return __builtin_bit_cast(u32x4_t, __builtin_convertvector(v, bf16x8));
+  }
+};
+template <>
+struct Raw<__bf16, uint16_t> {
+  u32x4_t a;
+  __device__ u32x4_t pack() const { return a; }
+};
+template <>
+struct Raw<float, float> {
+  f32x4_t a;
+  __device__ u32x4_t pack() const { return __builtin_bit_cast(u32x4_t, a); }
+};
+
+template <typename CT, typename ST, bool VEC>
+__device__ __forceinline__ Raw<CT, ST> load_chunk(const ST* row, int k0, int k, bool ok) {
+  constexpr int E = sizeof(CT) == 2 ? 8 : 4;
+  Raw<CT, ST> r;
+  if constexpr (VEC) {  // k is a multiple of 8 and rows are 16-byte aligned: a chunk is inside or outside as a whole
+    ok = ok && k0 < k;
+    if constexpr (sizeof(CT) == 2 && sizeof(ST) == 4) {
+      r.a = ok ? *reinterpret_cast<const f32x4_t*>(row + k0) : f32x4_t{0.f, 0.f, 0.f, 0.f};
+      r.b = ok ? *reinterpret_cast<const f32x4_t*>(row + k0 + 4) : f32x4_t{0.f, 0.f, 0.f, 0.f};
+    } else if constexpr (sizeof(ST) == 4) {
+      r.a = ok ? *reinterpret_cast<const f32x4_t*>(row + k0) : f32x4_t{0.f, 0.f, 0.f, 0.f};
+    } else {
+      r.a = ok ? *reinterpret_cast<const u32x4_t*>(row + k0) : u32x4_t{0, 0, 0, 0};
+    }
+  } else {
+    ST v[E];
+#pragma unroll
+    for (int i = 0; i < E; ++i) v[i] = ok && k0 + i < k ? row[k0 + i] : ST(0);
+    if constexpr (sizeof(CT) == 2 && sizeof(ST) == 4) {
+      r.a = f32x4_t{v[0], v[1], v[2], v[3]};
+      r.b = f32x4_t{v[4], v[5], v[6], v[7]};
+    } else if constexpr (sizeof(ST) == 4) {
+      r.a = f32x4_t{v[0], v[1], v[2], v[3]};
+    } else {
+      r.a = u32x4_t{v[0] | (uint32_t)v[1] << 16, v[2] | (uint32_t)v[3] << 16, v[4] | (uint32_t)v[5] << 16, v[6] | (uint32_t)v[7] << 16};
+    }
+  }
+  return r;
+}
+
+template <typename CT>
+__device__ __forceinline__ void mfma_chunk(const u32x4_t& a, const u32x4_t& b, f32x16& acc) {
+  if constexpr (sizeof(CT) == 2) {
+    acc = __builtin_amdgcn_mfma_f32_32x32x16_bf16(__builtin_bit_cast(bf16x8, a), __builtin_bit_cast(bf16x8, b), acc, 0, 0, 0);
+  } else {
+    const f32x4_t fa = __builtin_bit_cast(f32x4_t, a), fb = __builtin_bit_cast(f32x4_t, b);
+    acc = __builtin_amdgcn_mfma_f32_32x32x2f32(fa.x, fb.x, acc, 0, 0, 0);
+    acc = __builtin_amdgcn_mfma_f32_32x32x2f32(fa.y, fb.y, acc, 0, 0, 0);
+    acc = __builtin_amdgcn_mfma_f32_32x32x2f32(fa.z, fb.z, acc, 0, 0, 0);
+    acc = __builtin_amdgcn_mfma_f32_32x32x2f32(fa.w, fb.w, acc, 0, 0, 0);
+  }
+}
+
+template <typename CT, typename XT, typename WT, int MI, int NI, int ACT, bool VEC>
+__global__ void __launch_bounds__(256) rows_product_kernel(ProductArgs a) {
+  constexpr int BM = 64 * MI, BN = 64 * NI, XC = BM / 32, WC = BN / 32, KE = sizeof(CT) == 2 ? 64 : 32, CE = KE / CHUNKS;
+  constexpr int COLS = ACT == UGHIP_ACT_SWIGLU ? BN / 2 : BN;  // result columns of a tile
+  __shared__ __attribute__((aligned(16))) char lds[2][(BM + BN) * ROW_BYTES];
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, wm = wave >> 1, wn = wave & 1;
+  const int n0 = blockIdx.x * COLS;
+  int m0 = blockIdx.y * BM, m_end = a.m, group = 0;
+  if (a.groups) {
+    // which group this tile of rows belongs to: groups take ceil(rows / BM) tiles each, in order
+    int tile = blockIdx.y, begin = 0;
+    bool found = false;
+    for (int g = 0; g < a.groups; ++g) {
+      int end = a.group_end[g];
+      end = end < begin ? begin : end > a.m ? a.m : end;
+      const int tiles = (end - begin + BM - 1) / BM;
+      if (tile < tiles) {
+        group = g, m0 = begin + tile * BM, m_end = end, found = true;
+        break;
+      }
+      tile -= tiles;
+      begin = end;
+    }
+    if (!found) return;  // the same for the whole workgroup
+  }
+  const XT* xrow[XC];
+  bool xok[XC];
+  const WT* wrow[WC];
+  bool wok[WC];
+#pragma unroll
+  for (int i = 0; i < XC; ++i) {
+    const int r = m0 + (tid >> 3) + 32 * i;
+    xok[i] = r < m_end;
+    int src = xok[i] ? r : 0;
+    if (a.row_index && xok[i]) {
+      src = a.row_index[r];
+      xok[i] = src >= 0 && src < a.x_rows;
+      if (!xok[i]) src = 0;
+    }
+    xrow[i] = static_cast<const XT*>(a.x) + (size_t)src * a.x_stride;
+  }
+#pragma unroll
+  for (int i = 0; i < WC; ++i) {
+    const int rb = (tid >> 3) + 32 * i;
+    int col;
+    const void* base = a.w;
+    if (ACT == UGHIP_ACT_SWIGLU) {  // LDS rows: 32 gate columns, the same 32 of up, the next 32 gate columns, ...
+      col = n0 + (rb >> 6) * 32 + (rb & 31);
+      if (rb & 32) base = a.w_up;
+    } else {
+      col = n0 + rb;
+    }
+    wok[i] = col < a.n;
+    wrow[i] = static_cast<const WT*>(base) + (size_t)group * a.w_group + (size_t)(wok[i] ? col : 0) * a.w_stride;
+  }
+  f32x16 acc[MI][NI];
+#pragma unroll
+  for (int i = 0; i < MI; ++i)
+#pragma unroll
+    for (int j = 0; j < NI; ++j)
+#pragma unroll
+      for (int e = 0; e < 16; ++e) acc[i][j][e] = 0.f;
+
+  Raw<CT, XT> xr[XC];
+  Raw<CT, WT> wr[WC];
+  const int ck = (tid & 7) * CE;
+  auto fetch = [&](int k0) {
+#pragma unroll
+    for (int i = 0; i < XC; ++i) xr[i] = load_chunk<CT, XT, VEC>(xrow[i], k0 + ck, a.k, xok[i]);
+#pragma unroll
+    for (int i = 0; i < WC; ++i) wr[i] = load_chunk<CT, WT, VEC>(wrow[i], k0 + ck, a.k, wok[i]);
+  };
+  fetch(0);
+  const int steps = (a.k + KE - 1) / KE;
+  for (int s = 0; s < steps; ++s) {
+    char* buf = lds[s & 1];
+#pragma unroll
+    for (int i = 0; i < XC; ++i) *reinterpret_cast<u32x4_t*>(buf + ((tid >> 3) + 32 * i) * ROW_BYTES + (tid & 7) * 16) = xr[i].pack();
+#pragma unroll
+    for (int i = 0; i < WC; ++i) *reinterpret_cast<u32x4_t*>(buf + (BM + (tid >> 3) + 32 * i) * ROW_BYTES + (tid & 7) * 16) = wr[i].pack();
+    if (s + 1 < steps) fetch((s + 1) * KE);
+    __syncthreads();  // (one barrier a step: the buffer written two steps from now is read before the next barrier)
+    const char* xa = buf + (wm * 32 * MI + (lane & 31)) * ROW_BYTES + (lane >> 5) * 16;
+    const char* wa = buf + (BM + wn * 32 * NI + (lane & 31)) * ROW_BYTES + (lane >> 5) * 16;
+#pragma unroll
+    for (int c = 0; c < CHUNKS / 2; ++c) {
+      u32x4_t fx[MI], fw[NI];
+#pragma unroll
+      for (int i = 0; i < MI; ++i) fx[i] = *reinterpret_cast<const u32x4_t*>(xa + i * 32 * ROW_BYTES + c * 32);
+#pragma unroll
+      for (int j = 0; j < NI; ++j) fw[j] = *reinterpret_cast<const u32x4_t*>(wa + j * 32 * ROW_BYTES + c * 32);
+#pragma unroll
+      for (int i = 0; i < MI; ++i)
+#pragma unroll
+        for (int j = 0; j < NI; ++j) mfma_chunk<CT>(fx[i], fw[j], acc[i][j]);
+    }
+  }
+
+  // element e of an accumulator: row 8 (e / 4) + 4 (lane / 32) + e % 4, column lane % 32
+#pragma unroll
+  for (int i = 0; i < MI; ++i)
+#pragma unroll
+    for (int e = 0; e < 16; ++e) {
+      const int r = m0 + wm * 32 * MI + i * 32 + 8 * (e >> 2) + 4 * (lane >> 5) + (e & 3);
+      if (r >= m_end) continue;
+#pragma unroll
+      for (int j = 0; j < (ACT == UGHIP_ACT_SWIGLU ? 1 : NI); ++j) {
+        const int col = ACT == UGHIP_ACT_SWIGLU ? n0 + wn * 32 + (lane & 31) : n0 + wn * 32 * NI + j * 32 + (lane & 31);
+        if (col >= a.n) continue;
+        float v = acc[i][j][e];
+        if (a.bias) v += a.bias[col];
+        if constexpr (ACT == UGHIP_ACT_SWIGLU) {
+          float u = acc[i][1][e];
+          if (a.bias_up) u += a.bias_up[col];
+          v = silu_f(v) * u;
+        }
+        if constexpr (ACT == UGHIP_ACT_GELU_MUL) {
+          const int id = a.ids[r];
+          float t = __uint_as_float(0x7fc00000u);
+          if (id >= 0 && id < a.table_rows) {
+            const size_t at = (size_t)id * a.table_stride + a.table_col + col;
+            t = a.table_bf16 ? bf16_to_f32(static_cast<const uint16_t*>(a.table)[at]) : static_cast<const float*>(a.table)[at];
+          }
+          v = gelu_tanh_f(v) * t;
+        }
+        const size_t at = (size_t)r * a.dst_stride + col;
+        if (a.dst_bf16) static_cast<uint16_t*>(a.dst)[at] = bf16_rne(v);
+        else static_cast<float*>(a.dst)[at] = v;
+      }
+    }
+}
+
+template <typename CT, typename XT, typename WT, int MI, int NI, int ACT>
+hipError_t launch_tile(hipStream_t st, const ProductArgs& a, bool vec) {
+  constexpr int BM = 64 * MI, COLS = ACT == UGHIP_ACT_SWIGLU ? 32 * NI : 64 * NI;
+  const dim3 grid((unsigned)((a.n + COLS - 1) / COLS), (unsigned)((a.m + BM - 1) / BM + (a.groups ? a.groups : 0)));
+  if (grid.y > 65535) return hipErrorInvalidValue;
+  if (vec) rows_product_kernel<CT, XT, WT, MI, NI, ACT, true><<<grid, 256, 0, st>>>(a);
+  else rows_product_kernel<CT, XT, WT, MI, NI, ACT, false><<<grid, 256, 0, st>>>(a);
+  return hipGetLastError();
+}
+
+template <typename CT, typename XT, typename WT, int ACT>
+hipError_t launch_act(hipStream_t st, const ProductArgs& a, bool vec) {
+  const int rows = a.groups ? (a.m + a.groups - 1) / a.groups : a.m;
+  if constexpr (ACT == UGHIP_ACT_SWIGLU) {  // a tile's columns come in gate / up pairs
+    return rows > 64 ? launch_tile<CT, XT, WT, 2, 2, ACT>(st, a, vec) : launch_tile<CT, XT, WT, 1, 2, ACT>(st, a, vec);
+  } else {
+    const long long big = (long long)((a.m + 127) / 128) * ((a.n + 127) / 128);
+    if (rows > 64 && big >= 192) return launch_tile<CT, XT, WT, 2, 2, ACT>(st, a, vec);
+    return launch_tile<CT, XT, WT, 1, 1, ACT>(st, a, vec);
+  }
+}
+
+template <typename CT, typename XT, typename WT>
+hipError_t launch_types(hipStream_t st, const ProductArgs& a, int act, bool vec) {
+  if (act == UGHIP_ACT_SWIGLU) return launch_act<CT, XT, WT, UGHIP_ACT_SWIGLU>(st, a, vec);
+  if (act == UGHIP_ACT_GELU_MUL) return launch_act<CT, XT, WT, UGHIP_ACT_GELU_MUL>(st, a, vec);
+  return launch_act<CT, XT, WT, UGHIP_ACT_NONE>(st, a, vec);
+}
+
+bool aligned16(const void* p) { return (reinterpret_cast<uintptr_t>(p) & 15) == 0; }
+
+}  // namespace
+
+extern "C" int ughip_product_rows(ughip_device* dev, const ughip_product* p) {
+  const char* what = "product_rows";
+  if (!dev || !p || !p->w) return set_error(UGHIP_ERR_INVALID, "%s: null argument", what);
+  if (p->product != UGHIP_PRODUCT_F32 && p->product != UGHIP_PRODUCT_BF16) return set_error(UGHIP_ERR_INVALID, "%s: unknown product %d", what, p->product);
+  if (p->act < UGHIP_ACT_NONE || p->act > UGHIP_ACT_GELU_MUL) return set_error(UGHIP_ERR_INVALID, "%s: unknown act %d", what, p->act);
+  if (p->m == 0 || p->n == 0) return UGHIP_OK;
+  if (p->k == 0) return set_error(UGHIP_ERR_INVALID, "%s: k == 0", what);
+  const bool f32 = p->product == UGHIP_PRODUCT_F32;
+  const size_t mats = p->groups ? p->groups : 1;
+  if (p->groups > 16384 || p->n > 0x7fffffffull / p->k) return set_error(UGHIP_ERR_INVALID, "%s: shape too large", what);
+  const size_t x_rows = p->row_index ? p->x_rows : p->m;
+  if (p->row_index && !p->groups) return set_error(UGHIP_ERR_INVALID, "%s: row_index belongs to the grouped form", what);
+  if (x_rows == 0) return set_error(UGHIP_ERR_INVALID, "%s: no rows of x", what);
+  if (int rc = check_view(dev, p->x, x_rows, p->k, f32 ? UGHIP_F32 : -1, "product_rows x")) return rc;
+  const size_t w_stride = p->w_stride ? p->w_stride : p->k;
+  if (w_stride != p->k && (p->groups || p->w_up)) return set_error(UGHIP_ERR_UNSUPPORTED, "%s: rows of w %zu elements apart belong to the plain form", what, w_stride);
+  if (p->groups) {
+    if (int rc = check_buf(dev, p->w, mats * p->n * p->k, f32 ? UGHIP_F32 : -1, "product_rows w")) return rc;
+  } else if (int rc = check_view(dev, ughip_view{const_cast<ughip_slice*>(p->w), 0, w_stride}, p->n, p->k, f32 ? UGHIP_F32 : -1, "product_rows w")) {
+    return rc;
+  }
+  if (p->act == UGHIP_ACT_SWIGLU) {
+    if (int rc = check_buf(dev, p->w_up, mats * p->n * p->k, p->w->dtype, "product_rows w_up")) return rc;
+  }
+  if (int rc = check_view(dev, p->dst, p->m, p->n, f32 ? UGHIP_F32 : -1, "product_rows dst")) return rc;
+  auto f_or_b = [](const ughip_slice* s) { return s->dtype == UGHIP_F32 || s->dtype == UGHIP_BF16; };
+  if (!f_or_b(p->x.s) || !f_or_b(p->w) || !f_or_b(p->dst.s)) return set_error(UGHIP_ERR_UNSUPPORTED, "%s: operands are F32 or BF16", what);
+  if ((p->bias || p->bias_up) && p->groups) return set_error(UGHIP_ERR_UNSUPPORTED, "%s: the grouped form takes no bias", what);
+  if (p->bias)
+    if (int rc = check_buf(dev, p->bias, p->n, UGHIP_F32, "product_rows bias")) return rc;
+  if (p->bias_up)
+    if (int rc = check_buf(dev, p->bias_up, p->n, UGHIP_F32, "product_rows bias_up")) return rc;
+  if (p->act == UGHIP_ACT_GELU_MUL) {
+    if (!p->table || !f_or_b(p->table)) return set_error(UGHIP_ERR_INVALID, "%s: a gate's table is F32 or BF16", what);
+    if (int rc = check_buf(dev, p->table, p->table_rows * p->table_stride, p->table->dtype, "product_rows table")) return rc;
+    if (p->table_col > p->table_stride || p->n > p->table_stride - p->table_col) return set_error(UGHIP_ERR_BOUNDS, "%s: table columns %zu + %zu of %zu", what, p->table_col, p->n, p->table_stride);
+    if (int rc = check_buf(dev, p->ids, p->m, UGHIP_I32, "product_rows ids")) return rc;
+  }
+  if (p->groups) {
+    if (int rc = check_buf(dev, p->group_end, p->groups, UGHIP_I32, "product_rows group_end")) return rc;
+    if (p->row_index)
+      if (int rc = check_buf(dev, p->row_index, p->m, UGHIP_I32, "product_rows row_index")) return rc;
+  }
+  if (p->dst.s == p->x.s && p->dst.s->ptr && p->act != UGHIP_ACT_NONE) return set_error(UGHIP_ERR_INVALID, "%s: dst aliases x", what);
+  if (int rc = device_activate(dev)) return rc;
+  ProductArgs a{};
+  const size_t xs = p->x.s->dtype == UGHIP_BF16 ? 2 : 4;
+  a.x = static_cast<const char*>(p->x.s->ptr) + p->x.offset * xs;
+  a.w = p->w->ptr;
+  a.w_up = p->w_up ? p->w_up->ptr : nullptr;
+  a.bias = buf_ptr<float>(p->bias), a.bias_up = buf_ptr<float>(p->bias_up);
+  a.dst_bf16 = p->dst.s->dtype == UGHIP_BF16;
+  a.dst = static_cast<char*>(p->dst.s->ptr) + p->dst.offset * (a.dst_bf16 ? 2 : 4);
+  a.x_stride = p->x.stride, a.w_stride = w_stride, a.dst_stride = p->dst.stride, a.w_group = p->n * p->k;
+  a.m = (int)p->m, a.n = (int)p->n, a.k = (int)p->k;
+  if (p->act == UGHIP_ACT_GELU_MUL) {
+    a.table = p->table->ptr, a.table_bf16 = p->table->dtype == UGHIP_BF16, a.table_rows = (int)p->table_rows;
+    a.table_stride = p->table_stride, a.table_col = p->table_col, a.ids = buf_ptr<int>(p->ids);
+  }
+  a.row_index = buf_ptr<int>(p->row_index), a.group_end = buf_ptr<int>(p->group_end), a.groups = (int)p->groups, a.x_rows = (int)x_rows;
+  const bool vec = p->k % 8 == 0 && (p->x.stride * xs) % 16 == 0 && (w_stride * (p->w->dtype == UGHIP_BF16 ? 2 : 4)) % 16 == 0 && aligned16(a.x) && aligned16(a.w) && (!a.w_up || aligned16(a.w_up));
+  const bool xb = p->x.s->dtype == UGHIP_BF16, wb = p->w->dtype == UGHIP_BF16;
+  hipError_t e;
+  if (f32) e = launch_types<float, float, float>(dev->stream, a, p->act, vec);
+  else if (xb && wb) e = launch_types<__bf16, uint16_t, uint16_t>(dev->stream, a, p->act, vec);
+  else if (wb) e = launch_types<__bf16, float, uint16_t>(dev->stream, a, p->act, vec);
+  else if (p->act == UGHIP_ACT_NONE && xb) e = launch_act<__bf16, uint16_t, float, UGHIP_ACT_NONE>(dev->stream, a, vec);
+  else if (p->act == UGHIP_ACT_NONE) e = launch_act<__bf16, float, float, UGHIP_ACT_NONE>(dev->stream, a, vec);
+  else return set_error(UGHIP_ERR_UNSUPPORTED, "%s: bf16 products with an activation take a BF16 matrix", what);
+  UGHIP_HIPCHK(e);
+  note_kernel("rows_product<%s,%s%s>", f32 ? "f32" : "bf16", p->act == UGHIP_ACT_SWIGLU ? "swiglu" : p->act == UGHIP_ACT_GELU_MUL ? "gelu_mul" : "none", p->groups ? ",grouped" : "");
+  return UGHIP_OK;
+}
