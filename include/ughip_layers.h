@@ -80,10 +80,11 @@ int ughip_latent_attention_rows(ughip_device* dev, ughip_view q, const ughip_sli
                                 const ughip_slice* cos, const ughip_slice* sin, size_t table_rows, ughip_view dst, size_t t, size_t pos, size_t heads, size_t dim,
                                 size_t rot, size_t vdim, size_t rank, float scale);
 /* The same for few positions without expanding anything: the heads' up-projections are folded into the query and the result
- * (w_uk [heads dim, rank], w_uv [heads vdim, rank]), every head attends to the latents themselves.  All in f32. */
-int ughip_latent_attention_absorbed(ughip_device* dev, ughip_view q, const ughip_slice* w_uk, const ughip_slice* w_uv, const ughip_slice* cache,
-                                    const ughip_slice* cos, const ughip_slice* sin, size_t table_rows, ughip_view dst, size_t t, size_t pos, size_t heads,
-                                    size_t dim, size_t rot, size_t vdim, size_t rank, float scale);
+ * (w_uk [heads dim, rank], w_uv [heads vdim, rank]), every head attends to the latents themselves.  All in f32.
+ * kv given: the step's rows are appended to the cache (cap rows) on the way, as ughip_latent_append does with (kv, kv_norm, eps). */
+int ughip_latent_attention_absorbed(ughip_device* dev, ughip_view q, ughip_view kv, const ughip_slice* kv_norm, float eps, const ughip_slice* w_uk,
+                                    const ughip_slice* w_uv, ughip_slice* cache, size_t cap, const ughip_slice* cos, const ughip_slice* sin, size_t table_rows,
+                                    ughip_view dst, size_t t, size_t pos, size_t heads, size_t dim, size_t rot, size_t vdim, size_t rank, float scale);
 
 /* ---- a state-space recurrence behind a causal convolution ------------------------------------------------------------------
  * ughip_conv_silu_rows: dst[i, c] = silu(bias[c] + sum_j taps[c, j] x[i - (n_taps - 1) + j, c]) for t positions from `pos` on;
@@ -109,6 +110,45 @@ int ughip_route_rows(ughip_device* dev, ughip_view x, const ughip_slice* router,
  * group_end[e] = number of pairs with an expert <= e. */
 int ughip_group_rows(ughip_device* dev, const ughip_slice* ids, size_t m, size_t top, size_t experts, ughip_slice* row_index, ughip_slice* slots,
                      ughip_slice* group_end);
+
+/* ---- one position ---------------------------------------------------------------------------------------------------------
+ * A product of one row with what stands in front of it folded into the launch.  The row the matrix meets is made in every
+ * workgroup while the matrix is on its way:
+ *   v = x                                                     (k values)
+ *   v = x + y / sqrt(mean(y^2) + eps) * y_norm                y given: a sublayer's output joins the residual; v also goes to
+ *                                                             dst at x_out (keep_x)
+ *   v = x * silu(gate)                                        gate given
+ *   v = v / sqrt(mean(v^2) + eps) * norm                      norm given, the mean over each of norm_groups equal parts
+ * Then dst[dst_offset ..] = act(v w^T + bias) as in ughip_product_rows (n columns, w F32 or BF16, sums in f32).
+ * Routed experts: route != 0, w (and w_up) hold `experts` matrices [n, k].
+ *   route == 1: the choice is made from router logits (in every workgroup; the first one leaves ids and weights), and the
+ *     result is one run of n columns per chosen expert, top n in all;
+ *   route == 2: ids and weights are read, x holds one row of k per chosen expert (top k values), and the result is the weighted
+ *     sum of the experts' products: n columns.
+ * k (route 2: top k) <= 16000. */
+typedef struct ughip_row_step {
+  const ughip_slice* x;
+  size_t x_offset;
+  const ughip_slice *y, *y_norm, *gate, *norm;
+  size_t y_offset, gate_offset, norm_groups;
+  float eps;
+  int act, route, keep_x;
+  const ughip_slice *w, *w_up, *bias, *bias_up;
+  size_t n, k;
+  const ughip_slice *table, *ids; /* UGHIP_ACT_GELU_MUL: ids[0] is the row's token */
+  size_t table_rows, table_stride, table_col;
+  const ughip_slice *logits, *correction;
+  size_t logits_offset, experts, groups, keep, top;
+  ughip_slice *route_ids, *route_weights;
+  ughip_slice* dst;
+  size_t dst_offset, x_out;
+} ughip_row_step;
+int ughip_product_row(ughip_device* dev, const ughip_row_step* p);
+/* One position of the state-space mixer from the projected row p = [.. | x | B | C (at xbc_offset) | dt (at dt_offset)]:
+ * ughip_conv_silu_rows, ughip_conv_ring_store and ughip_ssm_rows for t = 1 in one launch. */
+int ughip_ssm_step(ughip_device* dev, const ughip_slice* p, size_t xbc_offset, size_t dt_offset, const ughip_slice* taps, const ughip_slice* conv_bias,
+                   size_t n_taps, ughip_slice* ring, const ughip_slice* dt_bias, const ughip_slice* a_log, const ughip_slice* skip, ughip_slice* s, size_t pos,
+                   size_t heads, size_t vdim, size_t groups, size_t state, ughip_view dst);
 
 #ifdef __cplusplus
 }

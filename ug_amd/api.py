@@ -367,7 +367,7 @@ def tuning(**switches):
 
 def set_llama_switch(name, on=True):
     """A switch of the host-side llama loops and hooks (NO_FOLD_EPILOGUES, NO_APPEND_PAIR, VERBOSE, NO_LAYER_STEPS,
-    HOST_ARGMAX, NO_OVERLAP); like the backend's table, read from the environment (UG_LLAMA_<NAME>) once per process."""
+    HOST_ARGMAX, NO_OVERLAP, NO_FUSED_STEP); like the backend's table, read from the environment (UG_LLAMA_<NAME>) once per process."""
     _chk(host_lib().ugh_llama_set_switch(name.encode(), int(bool(on))))
 
 

@@ -33,7 +33,7 @@ def _run(cmd):
 
 
 UGHIP_SOURCES = ("runtime.cpp", "lower_hip.cpp", "llama_ops.hip", "matmul.hip", "gemm_tiled.hip", "gemm_dma.hip", "gemm_dma_f32.hip", "rows_x3.hip", "attention.hip", "fused_linear.hip", "convert.hip",
-                 "rows_product.hip", "row_norms.hip", "latent_attention.hip", "ssm.hip", "moe.hip")
+                 "rows_product.hip", "row_step.hip", "row_norms.hip", "latent_attention.hip", "ssm.hip", "moe.hip")
 
 
 def build_ughip(only_changed=False):

@@ -54,7 +54,7 @@ struct Product {
   LB table, ids;
   size_t table_rows = 0, table_stride = 0, table_col = 0;
 };
-int product_mode(const LB& w) { return w.dtype() == DType::BF16 ? UGHIP_PRODUCT_BF16 : UGHIP_PRODUCT_F32; }
+int product_mode(const LB& w) { return w.dtype() == DType::BF16 ? (int)UGHIP_PRODUCT_BF16 : (int)UGHIP_PRODUCT_F32; }
 
 LB product_rows(const Rows& x, size_t m, const Product& p) {
   std::vector<LB> args = {x.lb, p.w};
@@ -111,6 +111,62 @@ void settle(StepContext& c, Stream& s) {
   s.norm = LB();
   s.slots = s.weights = LB();
   s.top = s.y_rows = 0;
+}
+
+// One position: a product of one row with what stands in front of it folded in (ughip_product_row).
+struct RowStep {
+  Product p;
+  LB norm, gate;  // v = x * silu(gate), then normed over `norm_groups` parts
+  size_t norm_groups = 1, gate_offset = 0;
+  float eps = 0;
+};
+constexpr size_t kRowStepMax = 16000;  // elements of the row a folded product meets
+
+// `pending` joins x first; keep_x: the joined row lies in front of the result (which starts at *at).
+LB row_step(const Rows& x, const Stream* pending, size_t width, const RowStep& r, size_t* at, bool keep_x = true) {
+  const bool join = pending && pending->norm.valid();
+  std::vector<LB> args = {x.lb, r.p.w};
+  auto add = [&](const LB& lb) {
+    if (!lb.valid()) return (size_t)0;
+    args.push_back(lb);
+    return args.size() - 1;
+  };
+  const size_t up = add(r.p.w_up), b = add(r.p.bias), bu = add(r.p.bias_up), tb = add(r.p.table), ids = add(r.p.ids), nm = add(r.norm), gt = add(r.gate);
+  const size_t y = join ? add(pending->y.lb) : 0, yn = join ? add(pending->norm) : 0, y_off = join ? pending->y.offset : 0, off = x.offset;
+  const Product pr = r.p;  // (the buffers inside keep their owners alive as the arguments do)
+  const size_t ng = r.norm_groups, g_off = r.gate_offset, base = join && keep_x ? width : 0;
+  const float eps = r.eps;
+  const size_t n = pr.n, k = pr.k, trows = pr.table_rows, tstride = pr.table_stride, tcol = pr.table_col;
+  const int act = pr.act;
+  *at = base;
+  return hip_op("row_step", args, {1, base + n}, [=](ughip_device* d, const std::vector<ughip_slice*>& in, ughip_slice* out) {
+    ughip_row_step q{};
+    q.x = in[0], q.x_offset = off, q.w = in[1];
+    if (y) q.y = in[y], q.y_offset = y_off, q.y_norm = in[yn], q.keep_x = base != 0;
+    if (up) q.w_up = in[up];
+    if (b) q.bias = in[b];
+    if (bu) q.bias_up = in[bu];
+    if (tb) q.table = in[tb], q.ids = in[ids];
+    if (nm) q.norm = in[nm], q.norm_groups = ng;
+    if (gt) q.gate = in[gt], q.gate_offset = g_off;
+    q.eps = eps, q.act = act, q.n = n, q.k = k;
+    q.table_rows = trows, q.table_stride = tstride, q.table_col = tcol;
+    q.dst = out, q.dst_offset = base, q.x_out = 0;
+    return ughip_product_row(d, &q);
+  });
+}
+
+// A product of the stream's row; what was pending joins the residual on the way, which then lies in front of the result.
+LB stream_step(StepContext& c, Stream& s, RowStep r, size_t* at) {
+  if (s.top) settle(c, s);
+  r.eps = c.eps;
+  LB out = row_step(s.x, &s, c.width, r, at);
+  if (s.norm.valid()) {
+    s.x = {out, 0, c.width};
+    s.y = Rows();
+    s.norm = LB();
+  }
+  return out;
 }
 
 // ---- loading --------------------------------------------------------------------------------------------------------------
@@ -185,32 +241,37 @@ struct LatentAttention : Mixer {
   }
 
   void run(StepContext& c, Stream& s, size_t layer) const override {
-    settle(c, s);
     const bool own = kv_from < 0;
     const size_t t = c.t, pos = c.pos, cap = c.capacity, H = heads, d = dim, r = rot, v = vdim, rk = rank, qr = q_rank, all = pos + t;
     const size_t wide = qr + (own ? rk + r : 0), trows = rope->rows;
     const float e = eps, sc = scale;
     const LB cache = c.state->layers[own ? layer : (size_t)kv_from].buffers[0];
-    LB low = product_rows(s.x, t, {down, LB(), LB(), LB(), wide, width});
-    LB cq = norm_rows({low, 0, wide}, t, qr, dq_norm, e);
-    LB q = product_rows({cq, 0, qr}, t, {uq, LB(), LB(), LB(), H * (d + r), qr});
+    const bool fused = c.fused && t <= absorb_up_to && std::max({width, qr, H * v}) <= kRowStepMax;
+    LB low, q;
+    size_t low_at = 0, none;
+    if (fused) {
+      low = stream_step(c, s, {{down, LB(), LB(), LB(), wide, width}}, &low_at);
+      RowStep up{{uq, LB(), LB(), LB(), H * (d + r), qr}};
+      up.norm = dq_norm, up.eps = e;
+      q = row_step({low, low_at, qr}, nullptr, 0, up, &none);
+    } else {
+      settle(c, s);
+      low = product_rows(s.x, t, {down, LB(), LB(), LB(), wide, width});
+      LB cq = norm_rows({low, 0, wide}, t, qr, dq_norm, e);
+      q = product_rows({cq, 0, qr}, t, {uq, LB(), LB(), LB(), H * (d + r), qr});
+    }
     // `low` is the first to know this step's rows: an op that reads the cache takes it as an argument, and the first one of
     // the layer that owns the cache writes the rows
     std::vector<LB> head_args = {low, cache, rope->cos, rope->sin};
     if (own) head_args.push_back(kv_norm);
-    auto append = [=](ughip_device* dev, const std::vector<ughip_slice*>& in) {
-      if (!own) return (int)UGHIP_OK;
-      return ughip_latent_append(dev, {in[0], qr, wide}, in[4], e, in[2], in[3], trows, in[1], cap, pos, t, rk, r);
-    };
     const size_t n_head = head_args.size();
     LB a;
     if (t <= absorb_up_to) {
       std::vector<LB> args = head_args;
       args.insert(args.end(), {q, uk, uv});
       a = hip_op("latent_attention_absorbed", args, {t, H * v}, [=](ughip_device* dev, const std::vector<ughip_slice*>& in, ughip_slice* out) {
-        if (int rc = append(dev, in)) return rc;
-        return ughip_latent_attention_absorbed(dev, {in[n_head], 0, H * (d + r)}, in[n_head + 1], in[n_head + 2], in[1], in[2], in[3], trows, {out, 0, H * v}, t, pos, H, d, r,
-                                               v, rk, sc);
+        return ughip_latent_attention_absorbed(dev, {in[n_head], 0, H * (d + r)}, {own ? in[0] : nullptr, low_at + qr, wide}, own ? in[4] : nullptr, e, in[n_head + 1],
+                                               in[n_head + 2], in[1], cap, in[2], in[3], trows, {out, 0, H * v}, t, pos, H, d, r, v, rk, sc);
       });
     } else {
       const int mode = product_mode(uk);
@@ -219,7 +280,8 @@ struct LatentAttention : Mixer {
       args.push_back(uk);
       LB k = hip_op("latent_keys", args, {all, H * d},
                     [=](ughip_device* dev, const std::vector<ughip_slice*>& in, ughip_slice* out) {
-                      if (int rc = append(dev, in)) return rc;
+                      if (own)
+                        if (int rc = ughip_latent_append(dev, {in[0], qr, wide}, in[4], e, in[2], in[3], trows, in[1], cap, pos, t, rk, r)) return rc;
                       ughip_product p{};
                       p.x = {in[1], 0, rk + r}, p.dst = {out, 0, H * d}, p.w = in[n_head];
                       p.m = all, p.n = H * d, p.k = rk, p.product = mode;
@@ -240,7 +302,8 @@ struct LatentAttention : Mixer {
         return ughip_latent_attention_rows(dev, {in[0], 0, H * (d + r)}, in[1], in[2], v_stride, in[3], in[4], in[5], trows, {out, 0, H * v}, t, pos, H, d, r, v, rk, sc);
       });
     }
-    s.y = {product_rows({a, 0, H * v}, t, {o, LB(), LB(), LB(), width, H * v}), 0, width};
+    if (fused) s.y = {row_step({a, 0, H * v}, nullptr, 0, {{o, LB(), LB(), LB(), width, H * v}}, &none), 0, width};
+    else s.y = {product_rows({a, 0, H * v}, t, {o, LB(), LB(), LB(), width, H * v}), 0, width};
   }
 
 };
@@ -272,10 +335,21 @@ struct Mamba2 : Mixer {
   }
 
   void run(StepContext& c, Stream& s, size_t layer) const override {
-    settle(c, s);
     const size_t t = c.t, pos = c.pos, I = inner(), ch = channels(), H = heads, vd = vdim, N = state, G = groups, nt = taps, wide = I + ch + H, ng = norm_groups;
     const float e = eps;
     const LB S = c.state->layers[layer].buffers[0], ring = c.state->layers[layer].buffers[1];
+    if (c.fused && std::max(width, I) <= kRowStepMax && N <= 4096) {
+      size_t at, none;
+      LB p = stream_step(c, s, {{in, LB(), LB(), LB(), wide, width}}, &at);
+      LB y = hip_op("ssm_step", {p, conv, conv_b, dt_bias, a_log, skip, S, ring}, {1, I}, [=](ughip_device* dev, const std::vector<ughip_slice*>& a, ughip_slice* out) {
+        return ughip_ssm_step(dev, a[0], at + I, at + I + ch, a[1], a[2], nt, a[7], a[3], a[4], a[5], a[6], pos, H, vd, G, N, {out, 0, I});
+      });
+      RowStep last{{o, LB(), LB(), LB(), width, I}};
+      last.gate = p, last.gate_offset = at, last.norm = norm, last.norm_groups = ng, last.eps = e;
+      s.y = {row_step({y, 0, I}, nullptr, 0, last, &none), 0, width};
+      return;
+    }
+    settle(c, s);
     LB p = product_rows(s.x, t, {in, LB(), LB(), LB(), wide, width});
     LB xbc = hip_op("conv_silu", {p, conv, conv_b, ring}, {t, ch}, [=](ughip_device* dev, const std::vector<ughip_slice*>& a, ughip_slice* out) {
       return ughip_conv_silu_rows(dev, {a[0], I, wide}, a[1], a[2], nt, a[3], pos, t, ch, {out, 0, ch});
@@ -302,6 +376,12 @@ struct DenseFeedForward : FeedForward {
     down = ld.matrix(p + "down", {width, ff}), down_b = ld.vec(p + "down.b", width);
   }
   void run(StepContext& c, Stream& s) const override {
+    if (c.fused && std::max(width, ff) <= kRowStepMax) {
+      size_t at, none;
+      LB a = stream_step(c, s, {{gate, up, gate_b, up_b, ff, width, UGHIP_ACT_SWIGLU}}, &at);
+      s.y = {row_step({a, at, ff}, nullptr, 0, {{down, LB(), down_b, LB(), width, ff}}, &none), 0, width};
+      return;
+    }
     settle(c, s);
     LB a = product_rows(s.x, c.t, {gate, up, gate_b, up_b, ff, width, UGHIP_ACT_SWIGLU});
     s.y = {product_rows({a, 0, ff}, c.t, {down, LB(), down_b, LB(), width, ff}), 0, width};
@@ -329,6 +409,7 @@ struct MoeFeedForward : FeedForward {
     gate = ld.stacked(gs, width), up = ld.stacked(us, width), down = ld.stacked(ds, ff);
   }
   void run(StepContext& c, Stream& s) const override {
+    if (c.fused && std::max(width, top * ff) <= kRowStepMax && top <= 64) return run_step(c, s);
     settle(c, s);
     const size_t t = c.t, E = experts, tp = top, w = width, f = ff, gc = count, kp = keep, pairs = t * tp;
     const int mode = product_mode(gate);
@@ -355,6 +436,34 @@ struct MoeFeedForward : FeedForward {
     });
     s.y = {y, 0, w};
     s.slots = slots, s.weights = weights, s.top = tp, s.y_rows = pairs;
+  }
+
+ private:
+  void run_step(StepContext& c, Stream& s) const {
+    const size_t E = experts, tp = top, w = width, f = ff, gc = count, kp = keep;
+    size_t at;
+    LB logits = stream_step(c, s, {{router, LB(), LB(), LB(), E, w}}, &at);
+    const Rows x = s.x;
+    LB ids = scratch(DType::I32, tp, c.dev), weights = scratch(DType::F32, tp, c.dev);
+    auto routed = [=](const std::vector<ughip_slice*>& in, size_t first) {
+      ughip_row_step q{};
+      q.route_ids = in[first], q.route_weights = in[first + 1];
+      q.experts = E, q.groups = gc, q.keep = kp, q.top = tp;
+      return q;
+    };
+    LB a = hip_op("experts_gate_up_step", {x.lb, logits, correction, gate, up, ids, weights}, {1, tp * f},
+                  [=](ughip_device* dev, const std::vector<ughip_slice*>& in, ughip_slice* out) {
+                    ughip_row_step q = routed(in, 5);
+                    q.x = in[0], q.x_offset = x.offset, q.logits = in[1], q.logits_offset = at, q.correction = in[2];
+                    q.w = in[3], q.w_up = in[4], q.act = UGHIP_ACT_SWIGLU, q.route = 1, q.n = f, q.k = w, q.dst = out;
+                    return ughip_product_row(dev, &q);
+                  });
+    LB y = hip_op("experts_down_step", {a, down, ids, weights}, {1, w}, [=](ughip_device* dev, const std::vector<ughip_slice*>& in, ughip_slice* out) {
+      ughip_row_step q = routed(in, 2);
+      q.x = in[0], q.w = in[1], q.route = 2, q.n = w, q.k = f, q.dst = out;
+      return ughip_product_row(dev, &q);
+    });
+    s.y = {y, 0, w};
   }
 };
 
@@ -443,12 +552,19 @@ std::unique_ptr<DecoderState> HybridModel::new_state(size_t max_tokens) const {
 }
 
 void HybridModel::side(StepContext& c, Stream& s, const Layer& l, size_t index) const {
-  settle(c, s);
   Product p{l.side_gate, LB(), LB(), LB(), side_dim_, width_, UGHIP_ACT_GELU_MUL};
   p.table = side_embed_, p.ids = c.tokens;
   p.table_rows = vocab_, p.table_stride = layers_.size() * side_dim_, p.table_col = index * side_dim_;
-  LB g = product_rows(s.x, c.t, p);
-  s.y = {product_rows({g, 0, side_dim_}, c.t, {l.side_proj, LB(), LB(), LB(), width_, side_dim_}), 0, width_};
+  const Product proj{l.side_proj, LB(), LB(), LB(), width_, side_dim_};
+  if (c.fused && std::max(width_, side_dim_) <= kRowStepMax) {
+    size_t at, none;
+    LB g = stream_step(c, s, {p}, &at);
+    s.y = {row_step({g, at, side_dim_}, nullptr, 0, {proj}, &none), 0, width_};
+  } else {
+    settle(c, s);
+    LB g = product_rows(s.x, c.t, p);
+    s.y = {product_rows({g, 0, side_dim_}, c.t, proj), 0, width_};
+  }
   s.norm = l.side_norm;
 }
 
@@ -458,7 +574,7 @@ LB HybridModel::step(const LB& tokens, const LB&, DecoderState& state, const LB*
   const size_t t = tokens.elem_count();
   if (t == 0) bail("a step without tokens");
   if (st->len + t > st->capacity) bail("a sequence of " + std::to_string(st->len) + " + " + std::to_string(t) + " positions exceeds its capacity of " + std::to_string(st->capacity));
-  StepContext c{dev_, tokens, t, st->len, st->capacity, width_, eps_, st, false};
+  StepContext c{dev_, tokens, t, st->len, st->capacity, width_, eps_, st, t == 1 && !switch_on(SW_NO_FUSED_STEP)};
   Stream s;
   s.x = {gather_rows(embed_, vocab_, width_, 0, width_, tokens, t), 0, width_};
   for (size_t i = 0; i < layers_.size(); ++i) {
@@ -476,6 +592,14 @@ LB HybridModel::step(const LB& tokens, const LB&, DecoderState& state, const LB*
     }
   }
   st->len += t;
+  const Product head{head_, LB(), LB(), LB(), vocab_, width_};
+  if (c.fused && width_ <= kRowStepMax && (!rows || rows->elem_count() == 1)) {
+    size_t at;
+    if (s.top) settle(c, s);
+    RowStep r{head};
+    r.norm = final_norm_, r.eps = eps_;
+    return row_step(s.x, &s, width_, r, &at, false);
+  }
   settle(c, s);
   Rows x = s.x;
   size_t r = 1;
@@ -486,7 +610,7 @@ LB HybridModel::step(const LB& tokens, const LB&, DecoderState& state, const LB*
     x.offset += (t - 1) * x.stride;
   }
   LB xn = norm_rows(x, r, width_, final_norm_, eps_);
-  return product_rows({xn, 0, width_}, r, {head_, LB(), LB(), LB(), vocab_, width_});
+  return product_rows({xn, 0, width_}, r, head);
 }
 
 }  // namespace ug_llama

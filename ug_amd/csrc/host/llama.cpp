@@ -16,7 +16,7 @@
 namespace ug_llama {
 
 namespace {
-const char* const kSwitchNames[SW_COUNT] = {"NO_FOLD_EPILOGUES", "NO_APPEND_PAIR", "VERBOSE", "NO_LAYER_STEPS", "HOST_ARGMAX", "NO_OVERLAP"};
+const char* const kSwitchNames[SW_COUNT] = {"NO_FOLD_EPILOGUES", "NO_APPEND_PAIR", "VERBOSE", "NO_LAYER_STEPS", "HOST_ARGMAX", "NO_OVERLAP", "NO_FUSED_STEP"};
 std::atomic<int> g_switch[SW_COUNT];
 std::once_flag g_switch_once;
 void switches_init() {

@@ -251,7 +251,7 @@ class Model : public Decoder {
 // Switches of the host-side loops and hooks (measurements, tests): read once per process from the environment
 // (UG_LLAMA_<NAME>) and changed afterwards only through set_switch, so that the hooks running on the preparing
 // thread never call getenv next to a caller that changes the environment.
-enum Switch { SW_NO_FOLD_EPILOGUES, SW_NO_APPEND_PAIR, SW_VERBOSE, SW_NO_LAYER_STEPS, SW_HOST_ARGMAX, SW_NO_OVERLAP, SW_COUNT };
+enum Switch { SW_NO_FOLD_EPILOGUES, SW_NO_APPEND_PAIR, SW_VERBOSE, SW_NO_LAYER_STEPS, SW_HOST_ARGMAX, SW_NO_OVERLAP, SW_NO_FUSED_STEP, SW_COUNT };
 bool switch_on(Switch s);
 bool set_switch(const std::string& name, bool on);  // false: no switch of that name ("NO_OVERLAP", "UG_LLAMA_NO_OVERLAP")
 

@@ -12,6 +12,8 @@
 //   tiles of 32 cache rows in LDS, v_mfma_f32_16x16x4_f32; the cache is split over workgroups, a last launch adds the parts up.
 #include <hip/hip_runtime.h>
 
+#include <type_traits>
+
 #include "layers.h"
 
 using namespace ughip;
@@ -28,19 +30,33 @@ __device__ __forceinline__ float rotated(const float* part, int e, int rot, cons
   return e < half ? u * c - v * s : v * c + u * s;
 }
 
-__global__ void __launch_bounds__(256) latent_append_kernel(const float* __restrict__ kv, size_t kv_stride, const float* __restrict__ w, float eps,
-                                                            const float* __restrict__ cos, const float* __restrict__ sin, float* __restrict__ cache, size_t pos, int rank,
-                                                            int rot) {
-  __shared__ float red[4];
-  const float* row = kv + (size_t)blockIdx.x * kv_stride;
-  const size_t p = pos + blockIdx.x;
+struct AppendArgs {
+  const float* kv;  // null: nothing to append
+  size_t kv_stride;
+  const float* w;
+  float eps;
+  const float* cos;
+  const float* sin;
+  float* cache;
+  size_t pos;
+  int rank, rot;
+};
+
+__device__ __forceinline__ void append_row(const AppendArgs& a, int i, float* red) {
+  const float* row = a.kv + (size_t)i * a.kv_stride;
+  const size_t p = a.pos + i;
   float ss = 0.f;
-  for (int c = threadIdx.x; c < rank; c += 256) ss += row[c] * row[c];
+  for (int c = threadIdx.x; c < a.rank; c += 256) ss += row[c] * row[c];
   ss = block_sum<4>(ss, red);
-  const float inv = 1.f / sqrtf(ss / (float)rank + eps);
-  float* out = cache + p * (rank + rot);
-  for (int c = threadIdx.x; c < rank; c += 256) out[c] = row[c] * inv * w[c];
-  for (int e = threadIdx.x; e < rot; e += 256) out[rank + e] = rotated(row + rank, e, rot, cos + p * (rot / 2), sin + p * (rot / 2));
+  const float inv = 1.f / sqrtf(ss / (float)a.rank + a.eps);
+  float* out = a.cache + p * (a.rank + a.rot);
+  for (int c = threadIdx.x; c < a.rank; c += 256) out[c] = row[c] * inv * a.w[c];
+  for (int e = threadIdx.x; e < a.rot; e += 256) out[a.rank + e] = rotated(row + a.rank, e, a.rot, a.cos + p * (a.rot / 2), a.sin + p * (a.rot / 2));
+}
+
+__global__ void __launch_bounds__(256) latent_append_kernel(AppendArgs a) {
+  __shared__ float red[4];
+  append_row(a, blockIdx.x, red);
 }
 
 struct RowsArgs {
@@ -270,31 +286,57 @@ hipError_t launch_rows_any(hipStream_t st, const RowsArgs& a) {
 }
 
 // ---- few positions ----------------------------------------------------------------------------------------------------------
-template <typename WT>
-__device__ __forceinline__ float w_f32(WT v) {
-  if constexpr (sizeof(WT) == 2) return bf16_to_f32(v);
-  else return v;
+// Four consecutive elements of a matrix row (V4: they are there and aligned).
+template <bool V4>
+__device__ __forceinline__ f32x4_t load4(const float* p, int left) {
+  if constexpr (V4) return *reinterpret_cast<const f32x4_t*>(p);
+  f32x4_t v = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+  for (int i = 0; i < 4; ++i)
+    if (i < left) v[i] = p[i];
+  return v;
+}
+template <bool V4>
+__device__ __forceinline__ f32x4_t load4(const uint16_t* p, int left) {
+  if constexpr (V4) {
+    const uint2 v = *reinterpret_cast<const uint2*>(p);
+    return f32x4_t{__uint_as_float(v.x << 16), __uint_as_float(v.x & 0xffff0000u), __uint_as_float(v.y << 16), __uint_as_float(v.y & 0xffff0000u)};
+  }
+  f32x4_t v = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+  for (int i = 0; i < 4; ++i)
+    if (i < left) v[i] = bf16_to_f32(p[i]);
+  return v;
 }
 
 // qa[(i heads + h), 0 .. rank) = scale * sum_d q_h[d] w_uk[h dim + d, :], then the rotated part (scaled too).  A workgroup takes a
-// head and 128 columns; eight groups of 32 threads share d.
-template <typename WT>
-__global__ void __launch_bounds__(256) latent_absorb_kernel(const float* __restrict__ q, size_t q_stride, const WT* __restrict__ w, const float* __restrict__ cos,
-                                                            const float* __restrict__ sin, float* __restrict__ qa, int t, int pos, int heads, int dim, int rot, int rank,
-                                                            float scale) {
+// head and 128 columns; eight groups of 32 threads share d.  One workgroup more than there are heads appends the step's row.
+template <typename WT, bool V4>
+__global__ void __launch_bounds__(256) latent_absorb_kernel(const float* __restrict__ q, size_t q_stride, const WT* __restrict__ w, AppendArgs ap, float* __restrict__ qa,
+                                                            int heads, int dim, float scale) {
   __shared__ float part[8][128];
-  const int h = blockIdx.x, c0 = blockIdx.y * 128, cg = threadIdx.x & 31, dg = threadIdx.x >> 5, L = rank + rot;
+  __shared__ float red[4];
+  const int h = blockIdx.x, c0 = blockIdx.y * 128, cg = threadIdx.x & 31, dg = threadIdx.x >> 5, rank = ap.rank, rot = ap.rot, L = rank + rot;
   const int i = blockIdx.z;
+  if (h == heads) {
+    if (blockIdx.y == 0) append_row(ap, i, red);
+    return;
+  }
   const float* qr = q + (size_t)i * q_stride + (size_t)h * (dim + rot);
   float* out = qa + ((size_t)i * heads + h) * L;
-  float acc[4] = {0.f, 0.f, 0.f, 0.f};
+  f32x4_t acc = {0.f, 0.f, 0.f, 0.f};
   const int c = c0 + cg * 4;
-  for (int d = dg; d < dim; d += 8) {
-    const float qv = qr[d];
-    const WT* wr = w + ((size_t)h * dim + d) * rank;
-#pragma unroll
-    for (int e = 0; e < 4; ++e)
-      if (c + e < rank) acc[e] += qv * w_f32(wr[c + e]);
+  if (c < rank) {
+    const WT* wr = w + (size_t)h * dim * rank + c;
+#pragma unroll 8
+    for (int d = dg; d < dim; d += 8) {
+      const float qv = qr[d];
+      const f32x4_t v = load4<V4>(wr + (size_t)d * rank, rank - c);
+      acc.x += qv * v.x;
+      acc.y += qv * v.y;
+      acc.z += qv * v.z;
+      acc.w += qv * v.w;
+    }
   }
 #pragma unroll
   for (int e = 0; e < 4; ++e) part[dg][cg * 4 + e] = acc[e];
@@ -306,8 +348,8 @@ __global__ void __launch_bounds__(256) latent_absorb_kernel(const float* __restr
     out[c0 + threadIdx.x] = v * scale;
   }
   if (blockIdx.y == 0) {
-    const size_t p = (size_t)(pos + i) * (rot / 2);
-    for (int e = threadIdx.x; e < rot; e += 256) out[rank + e] = rotated(qr + dim, e, rot, cos + p, sin + p) * scale;
+    const size_t p = (ap.pos + i) * (rot / 2);
+    for (int e = threadIdx.x; e < rot; e += 256) out[rank + e] = rotated(qr + dim, e, rot, ap.cos + p, ap.sin + p) * scale;
   }
 }
 
@@ -432,31 +474,46 @@ __global__ void __launch_bounds__(256) latent_split_kernel(SplitArgs a) {
 }
 
 // The parts of one (position, head) added up, then 16 elements of the head's result through the values' up-projection.
-constexpr int MERGE_V = 16;
-template <typename WT>
+constexpr int MERGE_V = 16, SPLITS_MAX = 64;
+template <typename WT, bool V4>
 __global__ void __launch_bounds__(256) latent_merge_kernel(const float* __restrict__ acc, const float* __restrict__ ml, const WT* __restrict__ w, float* __restrict__ dst,
                                                            size_t dst_stride, int rows, int splits, int heads, int rank, int vdim) {
-  extern __shared__ __attribute__((aligned(16))) float sl[];
-  float* lat = sl;              // [rank]
-  float* fac = sl + ((rank + 3) & ~3);  // [splits]
+  extern __shared__ __attribute__((aligned(16))) float lat[];  // [rank], zeros up to a multiple of 256
+  __shared__ float fac[SPLITS_MAX];
   const int h = blockIdx.x, i = blockIdx.y, v0 = blockIdx.z * MERGE_V, row = i * heads + h;
-  float top = -INFINITY;
-  for (int s = 0; s < splits; ++s) top = fmaxf(top, ml[((size_t)s * rows + row) * 2]);
-  float sum = 0.f;
-  for (int s = 0; s < splits; ++s) sum += expf(ml[((size_t)s * rows + row) * 2] - top) * ml[((size_t)s * rows + row) * 2 + 1];
-  for (int s = threadIdx.x; s < splits; s += 256) fac[s] = expf(ml[((size_t)s * rows + row) * 2] - top) / sum;
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  if (wave == 0) {
+    const float m = lane < splits ? ml[((size_t)lane * rows + row) * 2] : -INFINITY, l = lane < splits ? ml[((size_t)lane * rows + row) * 2 + 1] : 0.f;
+    float top = m;
+    for (int d = 32; d; d >>= 1) top = fmaxf(top, __shfl_xor(top, d, 64));
+    const float f = expf(m - top);
+    float sum = f * l;
+    for (int d = 32; d; d >>= 1) sum += __shfl_xor(sum, d, 64);
+    fac[lane] = f / sum;
+  }
   __syncthreads();
-  for (int c = threadIdx.x; c < rank; c += 256) {
+  for (int c = threadIdx.x; c < ((rank + 255) & ~255); c += 256) {
     float v = 0.f;
-    for (int s = 0; s < splits; ++s) v += fac[s] * acc[((size_t)s * rows + row) * rank + c];
+    if (c < rank) {
+#pragma unroll 8
+      for (int s = 0; s < splits; ++s) v += fac[s] * acc[((size_t)s * rows + row) * rank + c];
+    }
     lat[c] = v;
   }
   __syncthreads();
-  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
-  for (int v = v0 + wave; v < min(vdim, v0 + MERGE_V); v += 4) {
+#pragma unroll
+  for (int u = 0; u < MERGE_V / 4; ++u) {
+    const int v = v0 + wave + 4 * u;
+    if (v >= vdim) break;
     const WT* wr = w + ((size_t)h * vdim + v) * rank;
     float s = 0.f;
-    for (int c = lane; c < rank; c += 64) s += w_f32(wr[c]) * lat[c];
+    for (int c = lane * 4; c < rank; c += 256) {
+      const f32x4_t a = load4<V4>(wr + c, rank - c), b = *reinterpret_cast<const f32x4_t*>(lat + c);
+      s += a.x * b.x;
+      s += a.y * b.y;
+      s += a.z * b.z;
+      s += a.w * b.w;
+    }
     for (int d = 32; d; d >>= 1) s += __shfl_xor(s, d, 64);
     if (lane == 0) dst[(size_t)i * dst_stride + (size_t)h * vdim + v] = s;
   }
@@ -484,8 +541,8 @@ extern "C" int ughip_latent_append(ughip_device* dev, ughip_view kv, const ughip
   if (int rc = check_buf(dev, cache, cap * (rank + rot), UGHIP_F32, what)) return rc;
   if (t == 0) return UGHIP_OK;
   if (int rc = device_activate(dev)) return rc;
-  latent_append_kernel<<<(unsigned)t, 256, 0, dev->stream>>>(view_ptr<float>(kv), kv.stride, buf_ptr<float>(w), eps, buf_ptr<float>(cos), buf_ptr<float>(sin),
-                                                             static_cast<float*>(cache->ptr), pos, (int)rank, (int)rot);
+  latent_append_kernel<<<(unsigned)t, 256, 0, dev->stream>>>(
+      AppendArgs{view_ptr<float>(kv), kv.stride, buf_ptr<float>(w), eps, buf_ptr<float>(cos), buf_ptr<float>(sin), static_cast<float*>(cache->ptr), pos, (int)rank, (int)rot});
   UGHIP_HIPCHK(hipGetLastError());
   return UGHIP_OK;
 }
@@ -515,9 +572,9 @@ extern "C" int ughip_latent_attention_rows(ughip_device* dev, ughip_view q, cons
   return UGHIP_OK;
 }
 
-extern "C" int ughip_latent_attention_absorbed(ughip_device* dev, ughip_view q, const ughip_slice* w_uk, const ughip_slice* w_uv, const ughip_slice* cache,
-                                               const ughip_slice* cos, const ughip_slice* sin, size_t table_rows, ughip_view dst, size_t t, size_t pos, size_t heads,
-                                               size_t dim, size_t rot, size_t vdim, size_t rank, float scale) {
+extern "C" int ughip_latent_attention_absorbed(ughip_device* dev, ughip_view q, ughip_view kv, const ughip_slice* kv_norm, float eps, const ughip_slice* w_uk,
+                                               const ughip_slice* w_uv, ughip_slice* cache, size_t cap, const ughip_slice* cos, const ughip_slice* sin, size_t table_rows,
+                                               ughip_view dst, size_t t, size_t pos, size_t heads, size_t dim, size_t rot, size_t vdim, size_t rank, float scale) {
   const char* what = "latent_attention_absorbed";
   if (!dev || !w_uk || !w_uv) return set_error(UGHIP_ERR_INVALID, "%s: null argument", what);
   if (heads == 0 || dim == 0 || vdim == 0 || rank == 0 || heads > 65535 || t > 65535) return set_error(UGHIP_ERR_INVALID, "%s: bad shape", what);
@@ -528,14 +585,19 @@ extern "C" int ughip_latent_attention_absorbed(ughip_device* dev, ughip_view q, 
   if (int rc = check_view(dev, q, t, heads * (dim + rot), UGHIP_F32, what)) return rc;
   if (int rc = check_buf(dev, w_uk, heads * dim * rank, -1, what)) return rc;
   if (int rc = check_buf(dev, w_uv, heads * vdim * rank, -1, what)) return rc;
-  if (int rc = check_buf(dev, cache, s * L, UGHIP_F32, what)) return rc;
+  if (s > cap) return set_error(UGHIP_ERR_BOUNDS, "%s: %zu rows exceed the cache's %zu", what, s, cap);
+  if (int rc = check_buf(dev, cache, cap * L, UGHIP_F32, what)) return rc;
+  if (kv.s) {
+    if (int rc = check_view(dev, kv, t, L, UGHIP_F32, what)) return rc;
+    if (int rc = check_buf(dev, kv_norm, rank, UGHIP_F32, what)) return rc;
+  }
   if (int rc = check_tables(dev, cos, sin, table_rows, pos, t, rot, what)) return rc;
   if (int rc = check_view(dev, dst, t, heads * vdim, UGHIP_F32, what)) return rc;
   if (t == 0) return UGHIP_OK;
   if (int rc = device_activate(dev)) return rc;
   const size_t tiles = (s + SK - 1) / SK, row_blocks = (rows + 15) / 16;
   size_t splits = row_blocks >= 256 ? 1 : 256 / row_blocks;
-  if (splits > 64) splits = 64;
+  if (splits > SPLITS_MAX) splits = SPLITS_MAX;
   if (splits > tiles) splits = tiles;
   const size_t per = (tiles + splits - 1) / splits;
   splits = (tiles + per - 1) / per;
@@ -545,12 +607,17 @@ extern "C" int ughip_latent_attention_absorbed(ughip_device* dev, ughip_view q, 
   if (int rc = rows_scratch(dev, (n_qa + n_ml + n_acc) * sizeof(float), &ws)) return rc;
   float* qa = static_cast<float*>(ws);
   SplitArgs a{qa, buf_ptr<float>(cache), qa + n_qa + n_ml, qa + n_qa, (int)rows, (int)heads, (int)pos, (int)s, (int)rank, (int)L, (int)per};
-  const dim3 g1((unsigned)heads, (unsigned)((rank + 127) / 128), (unsigned)t);
-  const bool bf = w_uk->dtype == UGHIP_BF16;
-  if (bf) latent_absorb_kernel<uint16_t><<<g1, 256, 0, dev->stream>>>(view_ptr<float>(q), q.stride, buf_ptr<uint16_t>(w_uk), buf_ptr<float>(cos), buf_ptr<float>(sin), qa, (int)t,
-                                                                     (int)pos, (int)heads, (int)dim, (int)rot, (int)rank, scale);
-  else latent_absorb_kernel<float><<<g1, 256, 0, dev->stream>>>(view_ptr<float>(q), q.stride, buf_ptr<float>(w_uk), buf_ptr<float>(cos), buf_ptr<float>(sin), qa, (int)t,
-                                                               (int)pos, (int)heads, (int)dim, (int)rot, (int)rank, scale);
+  const AppendArgs ap{view_ptr<float>(kv), kv.stride, buf_ptr<float>(kv_norm), eps, buf_ptr<float>(cos), buf_ptr<float>(sin), static_cast<float*>(cache->ptr), pos, (int)rank, (int)rot};
+  const dim3 g1((unsigned)(heads + (kv.s ? 1 : 0)), (unsigned)((rank + 127) / 128), (unsigned)t);
+  const bool bf = w_uk->dtype == UGHIP_BF16, v4 = rank % 4 == 0;
+  auto absorb = [&](auto* w, auto vec) {
+    latent_absorb_kernel<std::remove_const_t<std::remove_pointer_t<decltype(w)>>, decltype(vec)::value>
+        <<<g1, 256, 0, dev->stream>>>(view_ptr<float>(q), q.stride, w, ap, qa, (int)heads, (int)dim, scale);
+  };
+  if (bf && v4) absorb(buf_ptr<uint16_t>(w_uk), std::true_type{});
+  else if (bf) absorb(buf_ptr<uint16_t>(w_uk), std::false_type{});
+  else if (v4) absorb(buf_ptr<float>(w_uk), std::true_type{});
+  else absorb(buf_ptr<float>(w_uk), std::false_type{});
   UGHIP_HIPCHK(hipGetLastError());
   const dim3 g2((unsigned)row_blocks, (unsigned)splits);
   const size_t lds = split_lds_bytes((int)L);
@@ -568,11 +635,15 @@ extern "C" int ughip_latent_attention_absorbed(ughip_device* dev, ughip_view q, 
   else latent_split_kernel<16><<<g2, 256, lds, dev->stream>>>(a);
   UGHIP_HIPCHK(hipGetLastError());
   const dim3 g3((unsigned)heads, (unsigned)t, (unsigned)((vdim + MERGE_V - 1) / MERGE_V));
-  const size_t lds3 = (((rank + 3) & ~(size_t)3) + splits) * sizeof(float);
-  if (bf) latent_merge_kernel<uint16_t><<<g3, 256, lds3, dev->stream>>>(a.acc, a.ml, buf_ptr<uint16_t>(w_uv), view_ptr<float>(dst), dst.stride, (int)rows, (int)splits, (int)heads,
-                                                                       (int)rank, (int)vdim);
-  else latent_merge_kernel<float><<<g3, 256, lds3, dev->stream>>>(a.acc, a.ml, buf_ptr<float>(w_uv), view_ptr<float>(dst), dst.stride, (int)rows, (int)splits, (int)heads,
-                                                                 (int)rank, (int)vdim);
+  const size_t lds3 = ((rank + 255) & ~(size_t)255) * sizeof(float);
+  auto merge = [&](auto* w, auto vec) {
+    latent_merge_kernel<std::remove_const_t<std::remove_pointer_t<decltype(w)>>, decltype(vec)::value>
+        <<<g3, 256, lds3, dev->stream>>>(a.acc, a.ml, w, view_ptr<float>(dst), dst.stride, (int)rows, (int)splits, (int)heads, (int)rank, (int)vdim);
+  };
+  if (bf && v4) merge(buf_ptr<uint16_t>(w_uv), std::true_type{});
+  else if (bf) merge(buf_ptr<uint16_t>(w_uv), std::false_type{});
+  else if (v4) merge(buf_ptr<float>(w_uv), std::true_type{});
+  else merge(buf_ptr<float>(w_uv), std::false_type{});
   UGHIP_HIPCHK(hipGetLastError());
   return UGHIP_OK;
 }

@@ -192,6 +192,76 @@ __global__ void __launch_bounds__(256) ssm_chunk_out_kernel(SsmArgs a) {
   }
 }
 
+// One position in one launch.  A workgroup takes a head and 16 of its columns: it convolves those columns and the head's B and
+// C rows (again in every workgroup: a few hundred channels), then 16 threads per column walk the state.  The ring's slot of this
+// position is one no tap of this position reads, so the rows go in while other workgroups still convolve.
+constexpr int STEP_COLS = 16;
+struct SsmStepArgs {
+  const float* xbc;  // this position's inputs of the convolution
+  const float* dt;
+  const float* taps;
+  const float* conv_bias;
+  float* ring;
+  const float* dt_bias;
+  const float* a_log;
+  const float* skip;
+  float* s;
+  float* dst;
+  long long pos;
+  int n_taps, heads, vdim, groups, state, channels;
+};
+
+__device__ __forceinline__ float conv_one(const SsmStepArgs& a, int c) {
+  float v = a.conv_bias ? a.conv_bias[c] : 0.f;
+  for (int j = 0; j + 1 < a.n_taps; ++j) {
+    const long long p = a.pos - (a.n_taps - 1) + j;
+    if (p >= 0) v += a.taps[(size_t)c * a.n_taps + j] * a.ring[(size_t)(p % a.n_taps) * a.channels + c];
+  }
+  return silu_f(v + a.taps[(size_t)c * a.n_taps + a.n_taps - 1] * a.xbc[c]);
+}
+
+__global__ void __launch_bounds__(256) ssm_step_kernel(SsmStepArgs a) {
+  extern __shared__ float lds[];
+  float* B = lds;
+  float* C = lds + a.state;
+  __shared__ float xs[STEP_COLS], part[16][STEP_COLS + 1];
+  const int h = blockIdx.x, p0 = blockIdx.y * STEP_COLS, inner = a.heads * a.vdim, N = a.state, per = a.heads / a.groups, g = h / per;
+  const bool first = h % per == 0 && blockIdx.y == 0;  // stores the group's B and C rows
+  float* slot = a.ring + (size_t)(a.pos % a.n_taps) * a.channels;
+  for (int i = threadIdx.x; i < 2 * N; i += 256) {
+    const int c = inner + (i < N ? 0 : a.groups * N) + g * N + (i < N ? i : i - N);
+    lds[i] = conv_one(a, c);
+    if (first) slot[c] = a.xbc[c];
+  }
+  if (threadIdx.x < STEP_COLS && p0 + (int)threadIdx.x < a.vdim) {
+    const int c = h * a.vdim + p0 + threadIdx.x;
+    xs[threadIdx.x] = conv_one(a, c);
+    slot[c] = a.xbc[c];
+  }
+  __syncthreads();
+  const int col = threadIdx.x & 15, ng = threadIdx.x >> 4, p = p0 + col;
+  const float d = softplus_f(a.dt[h] + a.dt_bias[h]), keep = expf(-expf(a.a_log[h]) * d);
+  float y = 0.f;
+  if (p < a.vdim) {
+    const float dx = d * xs[col];
+    float* S = a.s + (size_t)h * N * a.vdim + p;
+    for (int n = ng; n < N; n += 16) {
+      float v = dx * B[n];
+      if (a.pos) v += keep * S[(size_t)n * a.vdim];
+      S[(size_t)n * a.vdim] = v;
+      y += v * C[n];
+    }
+  }
+  part[ng][col] = y;
+  __syncthreads();
+  if (ng == 0 && p < a.vdim) {
+    float v = 0.f;
+#pragma unroll
+    for (int i = 0; i < 16; ++i) v += part[i][col];
+    a.dst[h * a.vdim + p] = v + a.skip[h] * xs[col];
+  }
+}
+
 size_t chunk_lds_bytes(int q, int state) { return (size_t)(128 + 2 * q * row_n(state) + q * (PB + 4) + q * (q + 4)) * sizeof(float); }
 
 }  // namespace
@@ -260,6 +330,34 @@ extern "C" int ughip_ssm_rows(ughip_device* dev, ughip_view xbc, ughip_view dt, 
   ssm_chunk_state_kernel<<<grid, 256, lds, dev->stream>>>(a);
   ssm_chunk_scan_kernel<<<dim3((unsigned)((per + 255) / 256), (unsigned)heads), 256, 0, dev->stream>>>(a);
   ssm_chunk_out_kernel<<<grid, 256, lds, dev->stream>>>(a);
+  UGHIP_HIPCHK(hipGetLastError());
+  return UGHIP_OK;
+}
+
+extern "C" int ughip_ssm_step(ughip_device* dev, const ughip_slice* p, size_t xbc_offset, size_t dt_offset, const ughip_slice* taps, const ughip_slice* conv_bias,
+                              size_t n_taps, ughip_slice* ring, const ughip_slice* dt_bias, const ughip_slice* a_log, const ughip_slice* skip, ughip_slice* s, size_t pos,
+                              size_t heads, size_t vdim, size_t groups, size_t state, ughip_view dst) {
+  if (!dev) return set_error(UGHIP_ERR_INVALID, "ssm_step: null device");
+  if (heads == 0 || vdim == 0 || groups == 0 || state == 0 || heads % groups != 0 || heads > 65535 || vdim > 65535 || state > 4096)
+    return set_error(UGHIP_ERR_INVALID, "ssm_step: heads %zu, vdim %zu, groups %zu, state %zu", heads, vdim, groups, state);
+  if (n_taps == 0 || n_taps > 1024) return set_error(UGHIP_ERR_INVALID, "ssm_step: %zu taps", n_taps);
+  const size_t ch = heads * vdim + 2 * groups * state;
+  ughip_view in{const_cast<ughip_slice*>(p), xbc_offset, ch}, dt{const_cast<ughip_slice*>(p), dt_offset, heads};
+  if (int rc = check_view(dev, in, 1, ch, UGHIP_F32, "ssm_step p")) return rc;
+  if (int rc = check_view(dev, dt, 1, heads, UGHIP_F32, "ssm_step p")) return rc;
+  if (int rc = check_buf(dev, taps, ch * n_taps, UGHIP_F32, "ssm_step taps")) return rc;
+  if (conv_bias)
+    if (int rc = check_buf(dev, conv_bias, ch, UGHIP_F32, "ssm_step conv bias")) return rc;
+  if (int rc = check_buf(dev, ring, n_taps * ch, UGHIP_F32, "ssm_step ring")) return rc;
+  for (const ughip_slice* v : {dt_bias, a_log, skip})
+    if (int rc = check_buf(dev, v, heads, UGHIP_F32, "ssm_step per-head vector")) return rc;
+  if (int rc = check_buf(dev, s, heads * state * vdim, UGHIP_F32, "ssm_step state")) return rc;
+  if (int rc = check_view(dev, dst, 1, heads * vdim, UGHIP_F32, "ssm_step dst")) return rc;
+  if (int rc = device_activate(dev)) return rc;
+  SsmStepArgs a{view_ptr<float>(in), view_ptr<float>(dt), buf_ptr<float>(taps), buf_ptr<float>(conv_bias), static_cast<float*>(ring->ptr), buf_ptr<float>(dt_bias),
+                buf_ptr<float>(a_log), buf_ptr<float>(skip), static_cast<float*>(s->ptr), view_ptr<float>(dst), (long long)pos, (int)n_taps, (int)heads, (int)vdim,
+                (int)groups, (int)state, (int)ch};
+  ssm_step_kernel<<<dim3((unsigned)heads, (unsigned)((vdim + STEP_COLS - 1) / STEP_COLS)), 256, 2 * state * sizeof(float), dev->stream>>>(a);
   UGHIP_HIPCHK(hipGetLastError());
   return UGHIP_OK;
 }
