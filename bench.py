@@ -989,6 +989,72 @@ def llama_decode(dev, n_prompt=128, n_steps=128, fused_attention=0, bf16_matrice
             **({"prefill_ms_warm": warm_ms} if warm_ms is not None else {}), **({"prefill_ms_by_prompt_tokens": by_length} if by_length else {})}
 
 
+def hybrid_config(width, layers, heads, q_rank, kv_rank, ssm_heads, ssm_groups, ff, experts, top, expert_ff, side):
+    """A Tanolorn of the size a real model's layers have: latent attention in front (dense feed-forward), then two state-space
+    layers to every attention layer (routed experts), the second attention layer reading the first one's latents."""
+    attn = {"type": "latent_attention", "mixer": {"heads": heads, "dim": 128, "rot_dim": 64, "vdim": 128, "q_rank": q_rank, "kv_rank": kv_rank, "scale": 192 ** -0.5,
+                                                  "rot": {"base": 10000.0, "dims": 64}}}
+    ssm = {"type": "mamba2", "mixer": {"heads": ssm_heads, "vdim": 64, "state": 128, "groups": ssm_groups, "norm_groups": ssm_groups, "conv": 4}}
+    moe = {"kind": "moe", "expert": {"ff": expert_ff}, "router": {"experts": experts, "top": top, "groups": {"count": 4, "keep": 2}}}
+    out, first = [], None
+    for i in range(layers):
+        if i % 3 == 0:
+            m = dict(attn["mixer"])
+            if first is None:
+                first = i
+            elif i == 3:
+                m["kv_from"] = first
+            out.append({"type": attn["type"], "mixer": m, "mlp": {"kind": "dense", "ff": ff} if i == 0 else moe})
+        else:
+            out.append({**ssm, "mlp": moe})
+    return {"architecture": "Tanolorn", "vocab": 32000, "width": width, "norm": {"eps": 1e-5}, "token_side": {"dim": side}, "layers": out}
+
+
+def llama_config(width, layers, heads, kv_heads, ff):
+    return {"model_type": "llama", "hidden_size": width, "intermediate_size": ff, "max_position_embeddings": 4096, "num_attention_heads": heads, "num_key_value_heads": kv_heads,
+            "num_hidden_layers": layers, "rms_norm_eps": 1e-5, "vocab_size": 32000}
+
+
+# width -> the two designs at equal width, depth and (active) feed-forward size
+DECODER_SIZES = {
+    "1024": (hybrid_config(1024, 6, 8, 512, 256, 32, 4, 2816, 16, 4, 704, 128), llama_config(1024, 6, 16, 4, 2816)),
+    "2048": (hybrid_config(2048, 6, 16, 768, 512, 64, 8, 5632, 16, 4, 1408, 256), llama_config(2048, 6, 32, 4, 5632)),
+    "4096": (hybrid_config(4096, 3, 32, 1536, 512, 128, 8, 11008, 8, 2, 5504, 256), llama_config(4096, 3, 32, 8, 11008)),
+}
+
+
+def decoder_throughput(dev, config, prompts=(128, 512, 2048), n_steps=64):
+    """Prefill and decode throughput of a registered decoder with random-init bf16 matrices: prompts of several lengths (best of
+    five back to back), greedy steps behind the shortest and the longest of them."""
+    import ug_amd
+    from ug_amd import rng
+    model = ug_amd.Decoder.random(dev, config, bf16=True, seed=9, std=0.02)
+    out = {"prefill_ms": {}, "prefill_tok/s": {}, "decode_ms_per_token": {}, "decode_tok/s": {}}
+    for t in prompts:
+        prompt = rng.token_ids(10, t, model.vocab)
+        model.generate(prompt, 1)
+        ms = min(model.generate(prompt, 0)[1]["prefill_ms"] for _ in range(5))
+        out["prefill_ms"][str(t)], out["prefill_tok/s"][str(t)] = round(ms, 3), round(t / ms * 1e3)
+        if t in (prompts[0], prompts[-1]):
+            model.generate(prompt, 4)
+            st = min((model.generate(prompt, n_steps)[1] for _ in range(2)), key=lambda s: s["decode_ms"])
+            out["decode_ms_per_token"][str(t)], out["decode_tok/s"][str(t)] = round(st["decode_ms"] / n_steps, 4), round(n_steps / st["decode_ms"] * 1e3, 1)
+            out["launch_items_per_token"] = st["decode_items"]
+    return out
+
+
+def decoders(dev, sizes=tuple(DECODER_SIZES)):
+    """Tanolorn beside llama at equal width and depth (random weights, bf16 matrices)."""
+    dev.set_zero_fill(False)
+    out = {}
+    for size in sizes:
+        hybrid, llama = DECODER_SIZES[size]
+        out[f"width {size}, {len(hybrid['layers'])} layers"] = {"tanolorn": decoder_throughput(dev, hybrid), "llama": decoder_throughput(dev, llama)}
+        print(f"decoders: width {size} done", file=sys.stderr, flush=True)
+    dev.set_zero_fill(True)
+    return out
+
+
 def config_summary(line):
     """BASELINE.json's five configs in one compact block (value, unit, fraction of the roofline that bounds it, kernel, whether
     the device result was checked): what the long `extras` hold, short enough to read at a glance."""
@@ -1077,7 +1143,8 @@ def main():
     ap.add_argument("--no-extras", action="store_true")
     ap.add_argument("--no-llama", action="store_true")
     ap.add_argument("--headline-only", action="store_true", help="only the config-2 kernel: no extras, no llama, no CPU baseline")
-    ap.add_argument("--only", choices=["softmax", "bmm", "llama_pieces", "hbm_large", "floors", "safetensors", "cpu", "llama"], help="besides the headline, run just this group (profiler runs)")
+    ap.add_argument("--only", choices=["softmax", "bmm", "llama_pieces", "hbm_large", "floors", "safetensors", "cpu", "llama", "decoders"], help="besides the headline, run just this group (profiler runs)")
+    ap.add_argument("--decoder-size", action="append", choices=list(DECODER_SIZES), help="with --only decoders: this width only (may be given several times)")
     ap.add_argument("--no-cpu-baseline", action="store_true")
     ap.add_argument("--sustained-trace", type=float, default=0.0, metavar="SECONDS",
                     help="also run the headline step without a pause for this long and report its rate per 50 ms of elapsed time")
@@ -1139,7 +1206,7 @@ def main():
                               "GB/s": round(8.0 * N * args.steps / (cms * 1e-3) / 1e9, 1)}
     if args.only:
         args.no_cpu_baseline = True
-        args.no_extras = args.only == "llama"
+        args.no_extras = args.only in ("llama", "decoders")
         args.no_llama = args.only != "llama"
     if not (args.no_cpu_baseline or args.headline_only):
         line["cpu_baseline"] = cpu_baseline(a, b, truth)
@@ -1150,6 +1217,11 @@ def main():
             line["extras"] = extras(dev, max(20, args.steps // 4), args.warmup, None if args.only in (None, "llama") else args.only)
         except Exception as e:  # noqa: BLE001
             line["extras"] = {"error": f"{type(e).__name__}: {e}"}
+    if args.only == "decoders":
+        try:
+            line.setdefault("extras", {})["decoders"] = decoders(dev, args.decoder_size or tuple(DECODER_SIZES))
+        except Exception as e:  # noqa: BLE001
+            line.setdefault("extras", {})["decoders"] = {"error": f"{type(e).__name__}: {e}"}
     if not (args.no_llama or args.headline_only):
         # the last entry: the same model decoding behind a 1900-token prompt (caches near their 2048 rows)
         # the x3 entries: the prompt's products as three bf16 terms per row element on the bf16 matrix pipe (decode steps are unchanged)

@@ -308,7 +308,7 @@ extern "C" int ughip_product_row(ughip_device* dev, const ughip_row_step* p) {
   if (p->n == 0) return UGHIP_OK;
   const size_t segs = p->route == 2 ? p->top : 1, total = segs * p->k;
   if (p->k == 0 || p->k > ROW_MAX || segs == 0 || segs > 64 || total > ROW_MAX) return set_error(UGHIP_ERR_UNSUPPORTED, "%s: rows of %zu elements, up to %zu are supported", what, total, ROW_MAX);
-  if (p->n > 0x7fffffffull / p->k / 64) return set_error(UGHIP_ERR_INVALID, "%s: shape too large", what);
+  if (p->n > 0x7fffffffull / 128) return set_error(UGHIP_ERR_INVALID, "%s: shape too large", what);
   if (p->w->dtype != UGHIP_F32 && p->w->dtype != UGHIP_BF16) return set_error(UGHIP_ERR_UNSUPPORTED, "%s: matrices are F32 or BF16", what);
   const size_t mats = p->route ? p->experts : 1;
   if (p->route) {
