@@ -22,8 +22,10 @@ typedef struct ughip_view {
   size_t offset, stride;
 } ughip_view;
 
-/* dst[i, :] = table[ids[i], col .. col + cols), table F32 or BF16 with rows of `stride` elements (an embedding lookup, or the
- * part of one that belongs to a layer).  Ids outside [0, table_rows) give NaN rows and read nothing. */
+/* (Results called F32 or BF16 below take the dtype of their slice.)
+ * dst[i, :] = table[ids[i], col .. col + cols), table F32 or BF16 with rows of `stride` elements (an embedding lookup, or the
+ * part of one that belongs to a layer).  Ids outside [0, table_rows) give NaN rows and read nothing.
+ * dst F32 or BF16. */
 int ughip_gather_rows(ughip_device* dev, const ughip_slice* table, size_t table_rows, size_t stride, size_t col, size_t cols,
                       const ughip_slice* ids, size_t m, ughip_view dst);
 
@@ -31,20 +33,21 @@ int ughip_gather_rows(ughip_device* dev, const ughip_slice* table, size_t table_
  * dst = act(x w^T + bias), any m, n, k.  `product`:
  *   UGHIP_PRODUCT_F32   x and w F32, the f32 matrix pipe;
  *   UGHIP_PRODUCT_BF16  x and w rounded to (or stored as) bf16, the bf16 matrix pipe, f32 accumulation.
- * x, w and dst may each be F32 or BF16 (F32 only for UGHIP_PRODUCT_F32).
+ * x, w and dst may each be F32 or BF16 (F32 only for UGHIP_PRODUCT_F32).  BF16 rows and matrices of regular sizes take the
+ * one-wave-per-SIMD kernel of ughip_matmul, the rest one that takes any size (ughip_last_kernel names it).
  * `act`:
  *   UGHIP_ACT_NONE      dst[m, n] = y;
- *   UGHIP_ACT_SWIGLU    a second matrix w_up [n, k]: dst = silu(y) * y_up;
+ *   UGHIP_ACT_SWIGLU    w is [2 n, k], gate rows then up rows (and bias 2 n values): dst = silu(y_gate) * y_up;
  *   UGHIP_ACT_GELU_MUL  dst[i, c] = gelu_tanh(y[i, c]) * table[ids[i], table_col + c]: a gate whose other factor is a table row
  *                       chosen by the row's token.
- * groups > 0: w (and w_up) hold `groups` matrices one after the other and the m rows come sorted by group: rows
+ * groups > 0: w holds `groups` matrices one after the other and the m rows come sorted by group: rows
  * group_end[g - 1] .. group_end[g] - 1 meet matrix g, and row r reads x row row_index[r] (NULL: r); what ughip_group_rows
  * writes.  No bias then. */
 enum { UGHIP_PRODUCT_BF16 = 2 };
 enum { UGHIP_ACT_NONE = 0, UGHIP_ACT_SWIGLU = 1, UGHIP_ACT_GELU_MUL = 2 };
 typedef struct ughip_product {
   ughip_view x, dst;
-  const ughip_slice *w, *w_up, *bias, *bias_up;
+  const ughip_slice *w, *bias;
   size_t w_stride; /* elements from one row of w to the next, 0: k (plain form only) */
   size_t m, n, k;
   int product, act;
@@ -58,11 +61,11 @@ int ughip_product_rows(ughip_device* dev, const ughip_product* p);
 /* ---- norms --------------------------------------------------------------------------------------------------------------
  * dst[i] = x[i] + y[i] / sqrt(mean(y[i]^2) + eps) * w: a sublayer's normed output joins the residual (x.s NULL: the norm
  * alone).  y may be the sum of `top` rows: y[i] = sum_j weights[i top + j] * y.row(slots[i top + j]) (routed experts, summed
- * in the order j).  dst may be x.  n <= 16000. */
+ * in the order j).  dst may be x, and may be BF16; dst_bf16 (may be NULL): the rows once more as dense BF16 [m, n].  n <= 16000. */
 int ughip_add_rms_norm_rows(ughip_device* dev, ughip_view x, ughip_view y, const ughip_slice* slots, const ughip_slice* weights, size_t top, size_t y_rows,
-                            const ughip_slice* w, float eps, ughip_view dst, size_t m, size_t n);
+                            const ughip_slice* w, float eps, ughip_view dst, ughip_slice* dst_bf16, size_t m, size_t n);
 /* dst[i] = g / sqrt(mean(g^2) + eps) * w with g = y[i] * silu(z[i]), the mean taken over each of `groups` equal parts of the
- * row on its own.  z.s NULL: g = y. */
+ * row on its own.  z.s NULL: g = y.  dst F32 or BF16. */
 int ughip_gated_rms_norm_rows(ughip_device* dev, ughip_view y, ughip_view z, const ughip_slice* w, float eps, size_t groups, ughip_view dst, size_t m, size_t n);
 
 /* ---- latent attention -----------------------------------------------------------------------------------------------------
@@ -74,7 +77,7 @@ int ughip_latent_append(ughip_device* dev, ughip_view kv, const ughip_slice* w, 
                         ughip_slice* cache, size_t cap, size_t pos, size_t t, size_t rank, size_t rot);
 /* Causal attention of t positions pos .. pos + t - 1 over cache rows 0 .. pos + t - 1 with keys and values expanded from the
  * latents: q rows [t, heads (dim + rot)] (not yet rotated), k [pos + t, heads dim], v_t [heads vdim, v_stride] (values
- * transposed: one row per value element, position along it), both F32 or both BF16; dst [t, heads vdim] F32.  With BF16
+ * transposed: one row per value element, position along it), both F32 or both BF16; dst [t, heads vdim] F32 or BF16.  With BF16
  * operands q is rounded to bf16, scores and weights stay f32 (a weight meets v as two bf16 terms). */
 int ughip_latent_attention_rows(ughip_device* dev, ughip_view q, const ughip_slice* k, const ughip_slice* v_t, size_t v_stride, const ughip_slice* cache,
                                 const ughip_slice* cos, const ughip_slice* sin, size_t table_rows, ughip_view dst, size_t t, size_t pos, size_t heads, size_t dim,
@@ -120,7 +123,7 @@ int ughip_group_rows(ughip_device* dev, const ughip_slice* ids, size_t m, size_t
  *   v = x * silu(gate)                                        gate given
  *   v = v / sqrt(mean(v^2) + eps) * norm                      norm given, the mean over each of norm_groups equal parts
  * Then dst[dst_offset ..] = act(v w^T + bias) as in ughip_product_rows (n columns, w F32 or BF16, sums in f32).
- * Routed experts: route != 0, w (and w_up) hold `experts` matrices [n, k].
+ * Routed experts: route != 0, w holds `experts` matrices one after the other.
  *   route == 1: the choice is made from router logits (in every workgroup; the first one leaves ids and weights), and the
  *     result is one run of n columns per chosen expert, top n in all;
  *   route == 2: ids and weights are read, x holds one row of k per chosen expert (top k values), and the result is the weighted
@@ -133,7 +136,7 @@ typedef struct ughip_row_step {
   size_t y_offset, gate_offset, norm_groups;
   float eps;
   int act, route, keep_x;
-  const ughip_slice *w, *w_up, *bias, *bias_up;
+  const ughip_slice *w, *bias;
   size_t n, k;
   const ughip_slice *table, *ids; /* UGHIP_ACT_GELU_MUL: ids[0] is the row's token */
   size_t table_rows, table_stride, table_col;

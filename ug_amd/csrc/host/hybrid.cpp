@@ -48,7 +48,7 @@ LB scratch(DType dtype, size_t n, const DevicePtr& dev) {
 }
 
 struct Product {
-  LB w, w_up, bias, bias_up;
+  LB w, bias;  // UGHIP_ACT_SWIGLU: gate rows then up rows
   size_t n = 0, k = 0;
   int act = UGHIP_ACT_NONE;
   LB table, ids;
@@ -56,14 +56,16 @@ struct Product {
 };
 int product_mode(const LB& w) { return w.dtype() == DType::BF16 ? (int)UGHIP_PRODUCT_BF16 : (int)UGHIP_PRODUCT_F32; }
 
-LB product_rows(const Rows& x, size_t m, const Product& p) {
+// `after`: a buffer whose op has to run first (x is scratch that it wrote).
+LB product_rows(const Rows& x, size_t m, const Product& p, const LB& after = LB(), DType out_type = DType::F32) {
   std::vector<LB> args = {x.lb, p.w};
   auto add = [&](const LB& lb) {
     if (!lb.valid()) return (size_t)0;
     args.push_back(lb);
     return args.size() - 1;
   };
-  const size_t up = add(p.w_up), b = add(p.bias), bu = add(p.bias_up), tb = add(p.table), ids = add(p.ids);
+  const size_t b = add(p.bias), tb = add(p.table), ids = add(p.ids);
+  add(after);
   const size_t off = x.offset, stride = x.stride, n = p.n, k = p.k, trows = p.table_rows, tstride = p.table_stride, tcol = p.table_col;
   const int act = p.act, mode = product_mode(p.w);
   return hip_op("product_rows", args, {m, n}, [=](ughip_device* d, const std::vector<ughip_slice*>& in, ughip_slice* out) {
@@ -71,25 +73,29 @@ LB product_rows(const Rows& x, size_t m, const Product& p) {
     q.x = {in[0], off, stride};
     q.dst = {out, 0, n};
     q.w = in[1];
-    if (up) q.w_up = in[up];
     if (b) q.bias = in[b];
-    if (bu) q.bias_up = in[bu];
     if (tb) q.table = in[tb], q.ids = in[ids];
     q.m = m, q.n = n, q.k = k, q.product = mode, q.act = act;
     q.table_rows = trows, q.table_stride = tstride, q.table_col = tcol;
     return ughip_product_rows(d, &q);
-  });
+  }, out_type);
 }
 
-LB norm_rows(const Rows& y, size_t m, size_t n, const LB& w, float eps) {
+LB norm_rows(const Rows& y, size_t m, size_t n, const LB& w, float eps, DType out_type = DType::F32) {
   const size_t off = y.offset, stride = y.stride;
   return hip_op("norm_rows", {y.lb, w}, {m, n}, [=](ughip_device* d, const std::vector<ughip_slice*>& in, ughip_slice* out) {
-    return ughip_add_rms_norm_rows(d, {nullptr, 0, 0}, {in[0], off, stride}, nullptr, nullptr, 0, 0, in[1], eps, {out, 0, n}, m, n);
-  });
+    return ughip_add_rms_norm_rows(d, {nullptr, 0, 0}, {in[0], off, stride}, nullptr, nullptr, 0, 0, in[1], eps, {out, 0, n}, nullptr, m, n);
+  }, out_type);
 }
 
-LB gather_rows(const LB& table, size_t rows, size_t stride, size_t col, size_t cols, const LB& ids, size_t m) {
-  return hip_op("gather_rows", {table, ids}, {m, cols}, [=](ughip_device* d, const std::vector<ughip_slice*>& in, ughip_slice* out) {
+// copy (may be invalid): scratch that receives the rows as bf16
+LB gather_rows(const LB& table, size_t rows, size_t stride, size_t col, size_t cols, const LB& ids, size_t m, const LB& copy = LB()) {
+  std::vector<LB> args = {table, ids};
+  const bool twice = copy.valid();
+  if (twice) args.push_back(copy);
+  return hip_op("gather_rows", args, {m, cols}, [=](ughip_device* d, const std::vector<ughip_slice*>& in, ughip_slice* out) {
+    if (twice)
+      if (int rc = ughip_gather_rows(d, in[0], rows, stride, col, cols, in[1], m, {in[2], 0, cols})) return rc;
     return ughip_gather_rows(d, in[0], rows, stride, col, cols, in[1], m, {out, 0, cols});
   });
 }
@@ -102,9 +108,12 @@ void settle(StepContext& c, Stream& s) {
   const float eps = c.eps;
   std::vector<LB> args = {x.lb, y.lb, s.norm};
   if (top) args.push_back(s.slots), args.push_back(s.weights);
+  s.x16 = c.half_rows ? scratch(DType::BF16, t * n, c.dev) : LB();
+  const size_t copy = s.x16.valid() ? args.size() : 0;
+  if (copy) args.push_back(s.x16);
   LB out = hip_op("add_norm", args, {t, n}, [=](ughip_device* d, const std::vector<ughip_slice*>& in, ughip_slice* dst) {
     return ughip_add_rms_norm_rows(d, {in[0], x.offset, x.stride}, {in[1], y.offset, y.stride}, top ? in[3] : nullptr, top ? in[4] : nullptr, top, y_rows, in[2], eps,
-                                   {dst, 0, n}, t, n);
+                                   {dst, 0, n}, copy ? in[copy] : nullptr, t, n);
   });
   s.x = {out, 0, n};
   s.y = Rows();
@@ -112,6 +121,13 @@ void settle(StepContext& c, Stream& s) {
   s.slots = s.weights = LB();
   s.top = s.y_rows = 0;
 }
+
+// A product of the (settled) stream's rows, in the form the step's products read.
+LB stream_product(const StepContext& c, const Stream& s, const Product& p, DType out_type = DType::F32) {
+  if (s.x16.valid()) return product_rows({s.x16, 0, c.width}, c.t, p, s.x.lb, out_type);
+  return product_rows(s.x, c.t, p, LB(), out_type);
+}
+DType half_type(const StepContext& c) { return c.half_rows ? DType::BF16 : DType::F32; }
 
 // One position: a product of one row with what stands in front of it folded in (ughip_product_row).
 struct RowStep {
@@ -131,7 +147,7 @@ LB row_step(const Rows& x, const Stream* pending, size_t width, const RowStep& r
     args.push_back(lb);
     return args.size() - 1;
   };
-  const size_t up = add(r.p.w_up), b = add(r.p.bias), bu = add(r.p.bias_up), tb = add(r.p.table), ids = add(r.p.ids), nm = add(r.norm), gt = add(r.gate);
+  const size_t b = add(r.p.bias), tb = add(r.p.table), ids = add(r.p.ids), nm = add(r.norm), gt = add(r.gate);
   const size_t y = join ? add(pending->y.lb) : 0, yn = join ? add(pending->norm) : 0, y_off = join ? pending->y.offset : 0, off = x.offset;
   const Product pr = r.p;  // (the buffers inside keep their owners alive as the arguments do)
   const size_t ng = r.norm_groups, g_off = r.gate_offset, base = join && keep_x ? width : 0;
@@ -143,9 +159,7 @@ LB row_step(const Rows& x, const Stream* pending, size_t width, const RowStep& r
     ughip_row_step q{};
     q.x = in[0], q.x_offset = off, q.w = in[1];
     if (y) q.y = in[y], q.y_offset = y_off, q.y_norm = in[yn], q.keep_x = base != 0;
-    if (up) q.w_up = in[up];
     if (b) q.bias = in[b];
-    if (bu) q.bias_up = in[bu];
     if (tb) q.table = in[tb], q.ids = in[ids];
     if (nm) q.norm = in[nm], q.norm_groups = ng;
     if (gt) q.gate = in[gt], q.gate_offset = g_off;
@@ -169,6 +183,9 @@ LB stream_step(StepContext& c, Stream& s, RowStep r, size_t* at) {
   return out;
 }
 
+// From this many positions on, products of bf16 matrices read rows that their producers wrote as bf16.
+constexpr size_t kHalfRows = 96;
+
 // ---- loading --------------------------------------------------------------------------------------------------------------
 struct Loader {
   WeightSource& w;
@@ -179,6 +196,14 @@ struct Loader {
     if (plus != 0.f)
       for (float& e : v) e += plus;
     return LB::copy(v.data(), DType::F32, n, Shape({n}), dev);
+  }
+  LB stacked_vec(const std::vector<std::pair<std::string, size_t>>& parts) const {
+    std::vector<float> all;
+    for (const auto& p : parts) {
+      std::vector<float> v = w.get(p.first, {p.second});
+      all.insert(all.end(), v.begin(), v.end());
+    }
+    return LB::copy(all.data(), DType::F32, all.size(), Shape({all.size()}), dev);
   }
   LB f32(const std::string& name, const std::vector<size_t>& shape) const { return w.load(name, shape, dev); }
   // a matrix (or several by rows) in the dtype the products of this model read
@@ -250,15 +275,15 @@ struct LatentAttention : Mixer {
     LB low, q;
     size_t low_at = 0, none;
     if (fused) {
-      low = stream_step(c, s, {{down, LB(), LB(), LB(), wide, width}}, &low_at);
-      RowStep up{{uq, LB(), LB(), LB(), H * (d + r), qr}};
+      low = stream_step(c, s, {{down, LB(), wide, width}}, &low_at);
+      RowStep up{{uq, LB(), H * (d + r), qr}};
       up.norm = dq_norm, up.eps = e;
       q = row_step({low, low_at, qr}, nullptr, 0, up, &none);
     } else {
       settle(c, s);
-      low = product_rows(s.x, t, {down, LB(), LB(), LB(), wide, width});
-      LB cq = norm_rows({low, 0, wide}, t, qr, dq_norm, e);
-      q = product_rows({cq, 0, qr}, t, {uq, LB(), LB(), LB(), H * (d + r), qr});
+      low = stream_product(c, s, {down, LB(), wide, width});
+      LB cq = norm_rows({low, 0, wide}, t, qr, dq_norm, e, half_type(c));
+      q = product_rows({cq, 0, qr}, t, {uq, LB(), H * (d + r), qr});
     }
     // `low` is the first to know this step's rows: an op that reads the cache takes it as an argument, and the first one of
     // the layer that owns the cache writes the rows
@@ -300,10 +325,10 @@ struct LatentAttention : Mixer {
                      kv_type);
       a = hip_op("latent_attention", {q, k, vt, cache, rope->cos, rope->sin}, {t, H * v}, [=](ughip_device* dev, const std::vector<ughip_slice*>& in, ughip_slice* out) {
         return ughip_latent_attention_rows(dev, {in[0], 0, H * (d + r)}, in[1], in[2], v_stride, in[3], in[4], in[5], trows, {out, 0, H * v}, t, pos, H, d, r, v, rk, sc);
-      });
+      }, half_type(c));
     }
-    if (fused) s.y = {row_step({a, 0, H * v}, nullptr, 0, {{o, LB(), LB(), LB(), width, H * v}}, &none), 0, width};
-    else s.y = {product_rows({a, 0, H * v}, t, {o, LB(), LB(), LB(), width, H * v}), 0, width};
+    if (fused) s.y = {row_step({a, 0, H * v}, nullptr, 0, {{o, LB(), width, H * v}}, &none), 0, width};
+    else s.y = {product_rows({a, 0, H * v}, t, {o, LB(), width, H * v}), 0, width};
   }
 
 };
@@ -340,17 +365,17 @@ struct Mamba2 : Mixer {
     const LB S = c.state->layers[layer].buffers[0], ring = c.state->layers[layer].buffers[1];
     if (c.fused && std::max(width, I) <= kRowStepMax && N <= 4096) {
       size_t at, none;
-      LB p = stream_step(c, s, {{in, LB(), LB(), LB(), wide, width}}, &at);
+      LB p = stream_step(c, s, {{in, LB(), wide, width}}, &at);
       LB y = hip_op("ssm_step", {p, conv, conv_b, dt_bias, a_log, skip, S, ring}, {1, I}, [=](ughip_device* dev, const std::vector<ughip_slice*>& a, ughip_slice* out) {
         return ughip_ssm_step(dev, a[0], at + I, at + I + ch, a[1], a[2], nt, a[7], a[3], a[4], a[5], a[6], pos, H, vd, G, N, {out, 0, I});
       });
-      RowStep last{{o, LB(), LB(), LB(), width, I}};
+      RowStep last{{o, LB(), width, I}};
       last.gate = p, last.gate_offset = at, last.norm = norm, last.norm_groups = ng, last.eps = e;
       s.y = {row_step({y, 0, I}, nullptr, 0, last, &none), 0, width};
       return;
     }
     settle(c, s);
-    LB p = product_rows(s.x, t, {in, LB(), LB(), LB(), wide, width});
+    LB p = stream_product(c, s, {in, LB(), wide, width});
     LB xbc = hip_op("conv_silu", {p, conv, conv_b, ring}, {t, ch}, [=](ughip_device* dev, const std::vector<ughip_slice*>& a, ughip_slice* out) {
       return ughip_conv_silu_rows(dev, {a[0], I, wide}, a[1], a[2], nt, a[3], pos, t, ch, {out, 0, ch});
     });
@@ -360,37 +385,37 @@ struct Mamba2 : Mixer {
     });
     LB yn = hip_op("gated_norm", {y, p, norm}, {t, I}, [=](ughip_device* dev, const std::vector<ughip_slice*>& a, ughip_slice* out) {
       return ughip_gated_rms_norm_rows(dev, {a[0], 0, I}, {a[1], 0, wide}, a[2], e, ng, {out, 0, I}, t, I);
-    });
-    s.y = {product_rows({yn, 0, I}, t, {o, LB(), LB(), LB(), width, I}), 0, width};
+    }, half_type(c));
+    s.y = {product_rows({yn, 0, I}, t, {o, LB(), width, I}), 0, width};
   }
 };
 
 // ---- feed-forward ---------------------------------------------------------------------------------------------------------
 struct DenseFeedForward : FeedForward {
   size_t ff, width;
-  LB gate, gate_b, up, up_b, down, down_b;
+  LB gate_up, gate_up_b, down, down_b;
   DenseFeedForward(const Json& m, const std::string& p, const Loader& ld, size_t width_) : width(width_) {
     ff = m.size_at("ff");
-    gate = ld.matrix(p + "gate", {ff, width}), gate_b = ld.vec(p + "gate.b", ff);
-    up = ld.matrix(p + "up", {ff, width}), up_b = ld.vec(p + "up.b", ff);
+    gate_up = ld.stacked({{p + "gate", ff}, {p + "up", ff}}, width), gate_up_b = ld.stacked_vec({{p + "gate.b", ff}, {p + "up.b", ff}});
     down = ld.matrix(p + "down", {width, ff}), down_b = ld.vec(p + "down.b", width);
   }
   void run(StepContext& c, Stream& s) const override {
+    const Product first{gate_up, gate_up_b, ff, width, UGHIP_ACT_SWIGLU}, second{down, down_b, width, ff};
     if (c.fused && std::max(width, ff) <= kRowStepMax) {
       size_t at, none;
-      LB a = stream_step(c, s, {{gate, up, gate_b, up_b, ff, width, UGHIP_ACT_SWIGLU}}, &at);
-      s.y = {row_step({a, at, ff}, nullptr, 0, {{down, LB(), down_b, LB(), width, ff}}, &none), 0, width};
+      LB a = stream_step(c, s, {first}, &at);
+      s.y = {row_step({a, at, ff}, nullptr, 0, {second}, &none), 0, width};
       return;
     }
     settle(c, s);
-    LB a = product_rows(s.x, c.t, {gate, up, gate_b, up_b, ff, width, UGHIP_ACT_SWIGLU});
-    s.y = {product_rows({a, 0, ff}, c.t, {down, LB(), down_b, LB(), width, ff}), 0, width};
+    LB a = stream_product(c, s, first, half_type(c));
+    s.y = {product_rows({a, 0, ff}, c.t, second), 0, width};
   }
 };
 
 struct MoeFeedForward : FeedForward {
   size_t experts, top, count, keep, ff, width;
-  LB router, correction, gate, up, down;  // the experts' matrices one after the other
+  LB router, correction, gate_up, down;  // the experts' matrices one after the other, every gate in front of its up
   MoeFeedForward(const Json& m, const std::string& p, const Loader& ld, size_t width_) : width(width_) {
     const Json& r = m.at("router");
     experts = r.size_at("experts"), top = r.size_at("top");
@@ -401,30 +426,33 @@ struct MoeFeedForward : FeedForward {
       bail("configuration: a router of " + std::to_string(top) + " of " + std::to_string(experts) + " experts in " + std::to_string(keep) + " of " + std::to_string(count) + " groups");
     router = ld.f32(p + "router", {experts, width});
     correction = ld.vec(p + "correction", experts);
-    std::vector<std::pair<std::string, size_t>> gs, us, ds;
+    std::vector<std::pair<std::string, size_t>> gs, ds;
     for (size_t e = 0; e < experts; ++e) {
       const std::string q = p + "e" + std::to_string(e);
-      gs.push_back({q + ".gate", ff}), us.push_back({q + ".up", ff}), ds.push_back({q + ".down", width});
+      gs.push_back({q + ".gate", ff}), gs.push_back({q + ".up", ff}), ds.push_back({q + ".down", width});
     }
-    gate = ld.stacked(gs, width), up = ld.stacked(us, width), down = ld.stacked(ds, ff);
+    gate_up = ld.stacked(gs, width), down = ld.stacked(ds, ff);
   }
   void run(StepContext& c, Stream& s) const override {
     if (c.fused && std::max(width, top * ff) <= kRowStepMax && top <= 64) return run_step(c, s);
     settle(c, s);
     const size_t t = c.t, E = experts, tp = top, w = width, f = ff, gc = count, kp = keep, pairs = t * tp;
-    const int mode = product_mode(gate);
+    const int mode = product_mode(gate_up);
     const Rows x = s.x;
+    const bool half = s.x16.valid();
     LB ids = scratch(DType::I32, pairs, c.dev), weights = scratch(DType::F32, pairs, c.dev), row_index = scratch(DType::I32, pairs, c.dev);
     LB slots = scratch(DType::I32, pairs, c.dev), group_end = scratch(DType::I32, E, c.dev);
-    const DType act_type = gate.dtype();
-    LB a = hip_op("route_gate_up", {x.lb, router, correction, gate, up, ids, weights, row_index, slots, group_end}, {pairs, f},
+    const DType act_type = gate_up.dtype();
+    std::vector<LB> args = {x.lb, router, correction, gate_up, ids, weights, row_index, slots, group_end};
+    if (half) args.push_back(s.x16);
+    LB a = hip_op("route_gate_up", args, {pairs, f},
                   [=](ughip_device* dev, const std::vector<ughip_slice*>& in, ughip_slice* out) {
-                    if (int rc = ughip_route_rows(dev, {in[0], x.offset, x.stride}, in[1], in[2], t, w, E, gc, kp, tp, in[5], in[6])) return rc;
-                    if (int rc = ughip_group_rows(dev, in[5], t, tp, E, in[7], in[8], in[9])) return rc;
+                    if (int rc = ughip_route_rows(dev, {in[0], x.offset, x.stride}, in[1], in[2], t, w, E, gc, kp, tp, in[4], in[5])) return rc;
+                    if (int rc = ughip_group_rows(dev, in[4], t, tp, E, in[6], in[7], in[8])) return rc;
                     ughip_product p{};
-                    p.x = {in[0], x.offset, x.stride}, p.dst = {out, 0, f}, p.w = in[3], p.w_up = in[4];
+                    p.x = half ? ughip_view{in[9], 0, w} : ughip_view{in[0], x.offset, x.stride}, p.dst = {out, 0, f}, p.w = in[3];
                     p.m = pairs, p.n = f, p.k = w, p.product = mode, p.act = UGHIP_ACT_SWIGLU;
-                    p.row_index = in[7], p.group_end = in[9], p.groups = E, p.x_rows = t;
+                    p.row_index = in[6], p.group_end = in[8], p.groups = E, p.x_rows = t;
                     return ughip_product_rows(dev, &p);
                   },
                   act_type);
@@ -442,7 +470,7 @@ struct MoeFeedForward : FeedForward {
   void run_step(StepContext& c, Stream& s) const {
     const size_t E = experts, tp = top, w = width, f = ff, gc = count, kp = keep;
     size_t at;
-    LB logits = stream_step(c, s, {{router, LB(), LB(), LB(), E, w}}, &at);
+    LB logits = stream_step(c, s, {{router, LB(), E, w}}, &at);
     const Rows x = s.x;
     LB ids = scratch(DType::I32, tp, c.dev), weights = scratch(DType::F32, tp, c.dev);
     auto routed = [=](const std::vector<ughip_slice*>& in, size_t first) {
@@ -451,11 +479,11 @@ struct MoeFeedForward : FeedForward {
       q.experts = E, q.groups = gc, q.keep = kp, q.top = tp;
       return q;
     };
-    LB a = hip_op("experts_gate_up_step", {x.lb, logits, correction, gate, up, ids, weights}, {1, tp * f},
+    LB a = hip_op("experts_gate_up_step", {x.lb, logits, correction, gate_up, ids, weights}, {1, tp * f},
                   [=](ughip_device* dev, const std::vector<ughip_slice*>& in, ughip_slice* out) {
-                    ughip_row_step q = routed(in, 5);
+                    ughip_row_step q = routed(in, 4);
                     q.x = in[0], q.x_offset = x.offset, q.logits = in[1], q.logits_offset = at, q.correction = in[2];
-                    q.w = in[3], q.w_up = in[4], q.act = UGHIP_ACT_SWIGLU, q.route = 1, q.n = f, q.k = w, q.dst = out;
+                    q.w = in[3], q.act = UGHIP_ACT_SWIGLU, q.route = 1, q.n = f, q.k = w, q.dst = out;
                     return ughip_product_row(dev, &q);
                   });
     LB y = hip_op("experts_down_step", {a, down, ids, weights}, {1, w}, [=](ughip_device* dev, const std::vector<ughip_slice*>& in, ughip_slice* out) {
@@ -552,17 +580,17 @@ std::unique_ptr<DecoderState> HybridModel::new_state(size_t max_tokens) const {
 }
 
 void HybridModel::side(StepContext& c, Stream& s, const Layer& l, size_t index) const {
-  Product p{l.side_gate, LB(), LB(), LB(), side_dim_, width_, UGHIP_ACT_GELU_MUL};
+  Product p{l.side_gate, LB(), side_dim_, width_, UGHIP_ACT_GELU_MUL};
   p.table = side_embed_, p.ids = c.tokens;
   p.table_rows = vocab_, p.table_stride = layers_.size() * side_dim_, p.table_col = index * side_dim_;
-  const Product proj{l.side_proj, LB(), LB(), LB(), width_, side_dim_};
+  const Product proj{l.side_proj, LB(), width_, side_dim_};
   if (c.fused && std::max(width_, side_dim_) <= kRowStepMax) {
     size_t at, none;
     LB g = stream_step(c, s, {p}, &at);
     s.y = {row_step({g, at, side_dim_}, nullptr, 0, {proj}, &none), 0, width_};
   } else {
     settle(c, s);
-    LB g = product_rows(s.x, c.t, p);
+    LB g = stream_product(c, s, p, half_type(c));
     s.y = {product_rows({g, 0, side_dim_}, c.t, proj), 0, width_};
   }
   s.norm = l.side_norm;
@@ -574,9 +602,10 @@ LB HybridModel::step(const LB& tokens, const LB&, DecoderState& state, const LB*
   const size_t t = tokens.elem_count();
   if (t == 0) bail("a step without tokens");
   if (st->len + t > st->capacity) bail("a sequence of " + std::to_string(st->len) + " + " + std::to_string(t) + " positions exceeds its capacity of " + std::to_string(st->capacity));
-  StepContext c{dev_, tokens, t, st->len, st->capacity, width_, eps_, st, t == 1 && !switch_on(SW_NO_FUSED_STEP)};
+  StepContext c{dev_, tokens, t, st->len, st->capacity, width_, eps_, st, precision_ == Precision::BF16 && t >= kHalfRows, t == 1 && !switch_on(SW_NO_FUSED_STEP)};
   Stream s;
-  s.x = {gather_rows(embed_, vocab_, width_, 0, width_, tokens, t), 0, width_};
+  if (c.half_rows) s.x16 = scratch(DType::BF16, t * width_, dev_);
+  s.x = {gather_rows(embed_, vocab_, width_, 0, width_, tokens, t, s.x16), 0, width_};
   for (size_t i = 0; i < layers_.size(); ++i) {
     const Layer& l = layers_[i];
     l.mixer->run(c, s, i);
@@ -592,15 +621,22 @@ LB HybridModel::step(const LB& tokens, const LB&, DecoderState& state, const LB*
     }
   }
   st->len += t;
-  const Product head{head_, LB(), LB(), LB(), vocab_, width_};
-  if (c.fused && width_ <= kRowStepMax && (!rows || rows->elem_count() == 1)) {
+  const Product head{head_, LB(), vocab_, width_};
+  const bool one = width_ <= kRowStepMax && (c.fused ? !rows || rows->elem_count() == 1 : !rows && !switch_on(SW_NO_FUSED_STEP));
+  if (one && c.t == 1 && s.top == 0) {
     size_t at;
-    if (s.top) settle(c, s);
     RowStep r{head};
     r.norm = final_norm_, r.eps = eps_;
     return row_step(s.x, &s, width_, r, &at, false);
   }
   settle(c, s);
+  if (one) {
+    // a prompt whose logits are read at the last position only
+    size_t at;
+    RowStep r{head};
+    r.norm = final_norm_, r.eps = eps_;
+    return row_step({s.x.lb, s.x.offset + (t - 1) * s.x.stride, width_}, nullptr, width_, r, &at);
+  }
   Rows x = s.x;
   size_t r = 1;
   if (rows) {

@@ -44,6 +44,7 @@ struct HybridState : DecoderState {
 // reads the stream next either folds that in or settles it with an op of its own.
 struct Stream {
   Rows x, y;
+  LB x16;  // the rows of x once more as bf16, where the step's products read that (valid only while nothing is pending)
   LB norm;  // weight of the pending norm; invalid: nothing is pending
   LB slots, weights;  // y is a weighted sum of `top` rows of y_rows (routed experts)
   size_t top = 0, y_rows = 0;
@@ -57,6 +58,7 @@ struct StepContext {
   size_t width = 0;
   float eps = 0;
   HybridState* state = nullptr;
+  bool half_rows = false;  // products read bf16 rows (bf16 matrices and enough positions)
   bool fused = false;  // one position, with the neighbours of every product folded into its launch
 };
 
@@ -88,7 +90,7 @@ class HybridModel : public Decoder {
   struct Layer {
     std::unique_ptr<Mixer> mixer;
     std::unique_ptr<FeedForward> mlp;
-    LB norm1, norm2;
+    LB norm1, norm2;  // (1 + the stored weight)
     LB side_gate, side_proj, side_norm;
   };
   void side(StepContext& c, Stream& s, const Layer& l, size_t index) const;

@@ -70,6 +70,23 @@ double gemm_dma_cost_us(const MMArgs& p, size_t batch, int tile);
 void gemm_dma_name(int dtype, const MMArgs& p, int tile, char* out, size_t out_len);
 void gemm_tiled_name(int dtype, const MMArgs& p, size_t batch, bool rhs_bf16, const GemmEpilogue* epi, char* out, size_t out_len);
 
+// The same kernel for rows that meet a matrix per group and leave through an epilogue (ughip_product_rows): bf16 rows (gathered by
+// row_index when given) against [n, k]-major bf16 matrices, `groups` of them w_group elements apart with the rows sorted by group
+// (group_end), or one (groups 0).  swiglu: the matrices are [2 n_out, k], gate rows then up rows, the result silu(gate) * up.
+// p: a, a_rs, b, b_cs (k), M rows, N matrix rows (2 n_out with swiglu), K; p.c is not used.
+struct DmaRows {
+  const int* row_index = nullptr;
+  const int* group_end = nullptr;
+  const float* bias = nullptr;  // N values
+  void* dst = nullptr;
+  long long w_group = 0, dst_stride = 0;
+  int groups = 0, x_rows = 0, n_out = 0;
+  bool dst_bf16 = false;
+};
+bool gemm_dma_rows_supported(const MMArgs& p, const DmaRows& r, bool swiglu, int tile);
+int gemm_dma_rows_pick(const MMArgs& p, const DmaRows& r, bool swiglu);  // a tile code, 0: no tile takes it
+hipError_t gemm_dma_launch_rows(hipStream_t stream, const MMArgs& p, const DmaRows& r, bool swiglu, int tile);
+
 // f32, one wave per SIMD: 256 x 128 tiles of v_mfma_f32_32x32x2_f32, loads that write LDS directly, rhs [n, k]- or [k, n]-major
 // (gemm_dma_f32.hip).  Any M, N % 4 == 0, K % 32 == 0 and K >= 64, 16-byte aligned rows, contiguous [batch, M, N] result.
 // _pick: whether this kernel should take the problem ([k, n]-major rhs, whole rounds of 256 tiles or nearly, K >= 512;

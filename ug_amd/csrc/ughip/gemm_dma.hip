@@ -96,8 +96,10 @@ __device__ __forceinline__ int kn_byte(int k, int n) {
 // by side, and K tile t of the loop is term t % 6 of k tile t / 6 of an f32 product taken as six bf16 ones -- (hi, lo),
 // (lo, hi), (mid, mid), (hi, mid), (mid, hi), (hi, hi), the small ones first; (mid, lo), (lo, mid) and (lo, lo) stay below
 // 2^-24 of the product and are left out.
-template <typename T, int BM, int BN, bool B_KN, bool TWO, bool F32OUT = false, int BDIV = 1>
-__global__ void __launch_bounds__(256) gemm_dma4(MMArgs p, int tiles_m, int tiles_n, const float* __restrict__ residual) {
+// ROWS (1, or 2 with SwiGLU): the lhs rows, the matrix and the result are those of DmaRows.
+template <typename T, int BM, int BN, bool B_KN, bool TWO, bool F32OUT = false, int BDIV = 1, int ROWS = 0>
+__global__ void __launch_bounds__(256) gemm_dma4(MMArgs p, int tiles_m, int tiles_n, const float* __restrict__ residual, DmaRows rw) {
+  static_assert(ROWS == 0 || (BDIV == 1 && !B_KN && !F32OUT), "rows: one plane against an [n, k]-major rhs");
   static_assert(BDIV == 1 || BDIV == 6 || !B_KN, "planes of the lhs alone: against an [n, k]-major rhs only");
   extern __shared__ u32x4 lds[];
   constexpr int NI = BM / 32, NJ = BN / 32;            // 16-row and 16-column fragments per wave
@@ -125,10 +127,27 @@ __global__ void __launch_bounds__(256) gemm_dma4(MMArgs p, int tiles_m, int tile
     tm = t_in / tiles_n;
     tn = t_in - tm * tiles_n;
   }
-  const int m0 = tm * BM, n0 = tn * BN;
+  int m0 = tm * BM, m_end = p.M, group = 0;
+  const int n0 = tn * BN;
+  if constexpr (ROWS != 0) {
+    if (rw.groups) {
+      // groups take ceil(rows / BM) tile rows each, in order
+      int t = tm, begin = 0;
+      bool found = false;
+      for (int g = 0; g < rw.groups && !found; ++g) {
+        int end = rw.group_end[g];
+        end = end < begin ? begin : end > p.M ? p.M : end;
+        const int tiles = (end - begin + BM - 1) / BM;
+        if (t < tiles) group = g, m0 = begin + t * BM, m_end = end, found = true;
+        else t -= tiles, begin = end;
+      }
+      if (!found) return;  // the same for the whole workgroup
+    }
+  }
   const long long lda = p.a_rs, ldb = B_KN ? p.b_rs : p.b_cs;
-  const char* Ab = reinterpret_cast<const char*>(static_cast<const T*>(p.a) + (size_t)batch * p.a_bs + (size_t)m0 * lda);
-  const char* Bb = reinterpret_cast<const char*>(static_cast<const T*>(p.b) + (size_t)batch * p.b_bs + (B_KN ? (size_t)n0 : (size_t)n0 * ldb));
+  const char* Ab = reinterpret_cast<const char*>(static_cast<const T*>(p.a) + (size_t)batch * p.a_bs + (ROWS ? 0 : (size_t)m0 * lda));
+  const char* Bb = reinterpret_cast<const char*>(static_cast<const T*>(p.b) + (size_t)batch * p.b_bs + (ROWS ? (size_t)group * rw.w_group : 0) +
+                                                 (ROWS == 2 ? 0 : B_KN ? (size_t)n0 : (size_t)n0 * ldb));
   const int KT = p.K / BK;
   const int wm = (wave >> 1) * (BM / 2), wn = (wave & 1) * (BN / 2);
   const unsigned lds_addr = (unsigned)(size_t)(__attribute__((address_space(3))) char*)lds;
@@ -136,18 +155,28 @@ __global__ void __launch_bounds__(256) gemm_dma4(MMArgs p, int tiles_m, int tile
   unsigned voff[ND];
   // a last tile may hang over the end of M or N: rows past the end fetch the last row again (their results are not
   // stored), so every address stays inside the operands
-  const int m_last = p.M - 1 - m0, n_left = p.N - n0;
+  const int m_last = m_end - 1 - m0, n_left = p.N - n0;
 #pragma unroll
   for (int i = 0; i < NDA; ++i) {
     const int row = (i * 4 + wave) * 8 + (lane >> 3), cp = lane & 7;
-    voff[i] = (unsigned)(min(row, m_last) * lda * 2 + ((cp ^ ((row >> 1) & 7)) << 4));
+    int src = min(row, m_last);
+    if constexpr (ROWS != 0) {
+      src += m0;
+      if (rw.row_index) src = max(0, min(rw.row_index[src], rw.x_rows - 1));
+    }
+    voff[i] = (unsigned)(src * lda * 2 + ((cp ^ ((row >> 1) & 7)) << 4));
   }
 #pragma unroll
   for (int i = 0; i < NDB; ++i) {
     const int g = i * 4 + wave;
     if (!B_KN) {
       const int row = g * 8 + (lane >> 3), cp = lane & 7;
-      voff[NDA + i] = (unsigned)(min(row, n_left - 1) * ldb * 2 + ((cp ^ ((row >> 1) & 7)) << 4));
+      int src = min(row, n_left - 1);
+      if constexpr (ROWS == 2) {  // a wave's half of the tile: BN / 4 gate columns, then the same columns of up
+        const int q = row % (BN / 2);
+        src = min(tn * (BN / 2) + row / (BN / 2) * (BN / 4) + q % (BN / 4), rw.n_out - 1) + (q >= BN / 4 ? rw.n_out : 0);
+      }
+      voff[NDA + i] = (unsigned)(src * ldb * 2 + ((cp ^ ((row >> 1) & 7)) << 4));
     } else {
       // one instruction fills 1 KB = 512 / BN rows of k; the lane at LDS position (k, 16-byte chunk cpos) fetches the
       // chunk that the swizzle of the row's 32-byte pieces maps there
@@ -352,6 +381,35 @@ __global__ void __launch_bounds__(256) gemm_dma4(MMArgs p, int tiles_m, int tile
   tile(KT - 1, N_(), N_());
 
   // Register e of lane l of block (i, j): row wm + 16 i + l % 16, column wn + 16 j + 4 (l / 16) + e.
+  if constexpr (ROWS != 0) {
+    typedef __bf16 bf16x4 __attribute__((ext_vector_type(4)));
+    constexpr int NC = ROWS == 2 ? NJ / 2 : NJ;
+#pragma unroll
+    for (int j = 0; j < NC; ++j) {
+      const int col = ROWS == 2 ? tn * (BN / 2) + (wave & 1) * (BN / 4) + j * 16 + (lane >> 4) * 4 : n0 + wn + j * 16 + (lane >> 4) * 4;
+      if (col >= rw.n_out) continue;  // n_out % 4 == 0: a group of 4 columns exists whole or not at all
+      floatx4 b = {0.f, 0.f, 0.f, 0.f}, bu = {0.f, 0.f, 0.f, 0.f};
+      if (rw.bias) {
+        b = *reinterpret_cast<const floatx4*>(rw.bias + col);
+        if (ROWS == 2) bu = *reinterpret_cast<const floatx4*>(rw.bias + rw.n_out + col);
+      }
+#pragma unroll
+      for (int i = 0; i < NI; ++i) {
+        const int row = wm + i * 16 + (lane & 15);
+        if (row > m_last) continue;
+        floatx4 v = acc[i][j] + b;
+        if constexpr (ROWS == 2) {
+          const floatx4 u = acc[i][j + NC] + bu;
+#pragma unroll
+          for (int e = 0; e < 4; ++e) v[e] = v[e] / (1.f + __expf(-v[e])) * u[e];
+        }
+        const size_t at = (size_t)(m0 + row) * rw.dst_stride + col;
+        if (rw.dst_bf16) *reinterpret_cast<u32x2*>(static_cast<T*>(rw.dst) + at) = __builtin_bit_cast(u32x2, __builtin_convertvector(v, bf16x4));
+        else *reinterpret_cast<floatx4*>(static_cast<float*>(rw.dst) + at) = v;
+      }
+    }
+    return;
+  }
   if constexpr (F32OUT) {
     // four consecutive f32 per lane: 16-byte stores, 64 contiguous bytes per row and instruction
     float* __restrict__ C = static_cast<float*>(p.c) + (size_t)batch * p.c_bs + (size_t)m0 * p.N + n0;
@@ -398,15 +456,15 @@ __global__ void __launch_bounds__(256) gemm_dma4(MMArgs p, int tiles_m, int tile
   }
 }
 
-template <typename T, int BM, int BN, bool B_KN, bool F32OUT = false, int BDIV = 1>
-hipError_t launch(hipStream_t stream, const MMArgs& p, size_t batch, const float* residual = nullptr) {
-  constexpr int STAGES = 2 * (BM + BN) * BK * 2, EPI = F32OUT ? 0 : BM * (BN * 2 + 8);
+template <typename T, int BM, int BN, bool B_KN, bool F32OUT = false, int BDIV = 1, int ROWS = 0>
+hipError_t launch(hipStream_t stream, const MMArgs& p, size_t batch, const float* residual = nullptr, const DmaRows& rw = DmaRows()) {
+  constexpr int STAGES = 2 * (BM + BN) * BK * 2, EPI = F32OUT || ROWS ? 0 : BM * (BN * 2 + 8);
   constexpr int LDS_BYTES = STAGES > EPI ? STAGES : EPI;
   static std::atomic<unsigned long long> configured{0};  // one bit per device: the attribute is per device
   // the schedule with two barriers, except where it does not fit the registers (the transposing reads of the
   // largest tile need pairs of temporaries: 256 registers and spills)
   constexpr bool TWO = !(B_KN && BM == 256 && BN == 256);
-  auto kernel = gemm_dma4<T, BM, BN, B_KN, TWO, F32OUT, BDIV>;
+  auto kernel = gemm_dma4<T, BM, BN, B_KN, TWO, F32OUT, BDIV, ROWS>;
   int dev = 0;
   if (hipError_t e = hipGetDevice(&dev)) return e;
   const unsigned long long bit = dev < 64 ? 1ull << dev : 0;
@@ -414,9 +472,9 @@ hipError_t launch(hipStream_t stream, const MMArgs& p, size_t batch, const float
     if (hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(kernel), hipFuncAttributeMaxDynamicSharedMemorySize, LDS_BYTES)) return e;
     configured.fetch_or(bit, std::memory_order_relaxed);
   }
-  const int tiles_m = (p.M + BM - 1) / BM, tiles_n = (p.N + BN - 1) / BN;
+  const int tiles_m = (p.M + BM - 1) / BM + rw.groups, tiles_n = (p.N + BN - 1) / BN;
   const size_t total = batch * (size_t)tiles_m * tiles_n;
-  kernel<<<dim3((unsigned)total), dim3(256), LDS_BYTES, stream>>>(p, tiles_m, tiles_n, residual);
+  kernel<<<dim3((unsigned)total), dim3(256), LDS_BYTES, stream>>>(p, tiles_m, tiles_n, residual, rw);
   return hipGetLastError();
 }
 
@@ -565,6 +623,47 @@ hipError_t gemm_dma_launch_planes3(hipStream_t stream, const MMArgs& p, int tile
   return launch<__bf16, 128, 128, false, true, 3>(stream, q, (size_t)nsplit, residual);
 }
 
+
+bool gemm_dma_rows_supported(const MMArgs& p, const DmaRows& r, bool swiglu, int tile) {
+  int bm, bn;
+  if (!tile_dims(tile, &bm, &bn)) return false;
+  if (p.M <= 0 || p.N <= 0 || p.N % 8 || p.K % BK || p.K < 4 * BK || p.a_cs != 1 || p.a_rs % 8 || p.b_rs != 1 || p.b_cs % 8) return false;
+  if (r.n_out <= 0 || r.n_out % 4 || p.N != (swiglu ? 2 * r.n_out : r.n_out) || r.dst_stride % 4 || r.w_group % 8) return false;
+  // per-lane offsets are 32-bit: rows of x anywhere, matrix rows of a tile (of the whole matrix with SwiGLU)
+  const unsigned long long x_rows = r.row_index ? r.x_rows : p.M;
+  if (x_rows * p.a_rs * 2 >= (1ull << 31) || (unsigned long long)p.b_cs * 2 * (swiglu ? p.N : bn) >= (1ull << 31)) return false;
+  if (!aligned16(p.a) || !aligned16(p.b) || !aligned16(r.dst) || (r.bias && !aligned16(r.bias))) return false;
+  return ((size_t)(p.M + bm - 1) / bm + r.groups) * (size_t)((p.N + bn - 1) / bn) < (1u << 24);
+}
+
+int gemm_dma_rows_pick(const MMArgs& p, const DmaRows& r, bool swiglu) {
+  int best = 0;
+  double best_us = 0;
+  MMArgs q = p;
+  const size_t groups = r.groups ? r.groups : 1;
+  q.M = (int)((p.M + groups - 1) / groups);  // rows as if they were spread evenly
+  for (int tile : {256, 128, 64}) {
+    if (!gemm_dma_rows_supported(p, r, swiglu, tile)) continue;
+    const double us = gemm_dma_cost_us(q, groups, tile);
+    if (!best || us < best_us * 0.97) best = tile, best_us = us;
+  }
+  return best;
+}
+
+hipError_t gemm_dma_launch_rows(hipStream_t stream, const MMArgs& p, const DmaRows& r, bool swiglu, int tile) {
+  if (!gemm_dma_rows_supported(p, r, swiglu, tile)) return hipErrorInvalidValue;
+  int bm = 0, bn = 0;
+  tile_dims(tile, &bm, &bn);
+  note_kernel("gemm_dma4<bf16,NT,%dx%d,256t,rows%s%s>", bm, bn, swiglu ? ",swiglu" : "", r.groups ? ",grouped" : "");
+  if (swiglu) {
+    if (tile == 256) return launch<__bf16, 256, 256, false, false, 1, 2>(stream, p, 1, nullptr, r);
+    if (tile == 128) return launch<__bf16, 256, 128, false, false, 1, 2>(stream, p, 1, nullptr, r);
+    return launch<__bf16, 128, 128, false, false, 1, 2>(stream, p, 1, nullptr, r);
+  }
+  if (tile == 256) return launch<__bf16, 256, 256, false, false, 1, 1>(stream, p, 1, nullptr, r);
+  if (tile == 128) return launch<__bf16, 256, 128, false, false, 1, 1>(stream, p, 1, nullptr, r);
+  return launch<__bf16, 128, 128, false, false, 1, 1>(stream, p, 1, nullptr, r);
+}
 
 // Both operands as three bf16 planes per 64 elements of k (p.K = 6 k, rows of 3 k elements), f32 result: see BDIV == 6.
 bool gemm_dma_planes6_supported(const MMArgs& p, size_t batch, int tile) { return p.K % (6 * BK) == 0 && gemm_dma_supported(UGHIP_BF16, p, batch, tile); }

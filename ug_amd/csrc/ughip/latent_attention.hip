@@ -14,6 +14,7 @@
 
 #include <type_traits>
 
+#include "bf16_split.h"
 #include "layers.h"
 
 using namespace ughip;
@@ -66,11 +67,11 @@ struct RowsArgs {
   const float* cache;
   const float* cos;
   const float* sin;
-  float* dst;
+  void* dst;
   size_t q_stride, v_stride, dst_stride;
   int t, pos, heads, dim, rot, vdim, rank;
   float scale;
-  bool vec;
+  bool vec, dst_bf16;
 };
 
 template <typename T, int E>
@@ -257,13 +258,16 @@ __global__ void __launch_bounds__(256) latent_rows_kernel(RowsArgs a) {
   }
   if (i_mine >= a.t) return;
   const float inv = 1.f / sum;
-  float* out = a.dst + (size_t)i_mine * a.dst_stride + (size_t)head * a.vdim;
+  const size_t at = (size_t)i_mine * a.dst_stride + (size_t)head * a.vdim;
 #pragma unroll
   for (int i = 0; i < DV / 32; ++i)
 #pragma unroll
     for (int e = 0; e < 16; ++e) {
       const int vc = i * 32 + 8 * (e >> 2) + 4 * hf + (e & 3);
-      if (vc < a.vdim) out[vc] = o[i][e] * inv;
+      if (vc < a.vdim) {
+        if (a.dst_bf16) static_cast<uint16_t*>(a.dst)[at + vc] = bf16_rne(o[i][e] * inv);
+        else static_cast<float*>(a.dst)[at + vc] = o[i][e] * inv;
+      }
     }
 }
 
@@ -562,12 +566,14 @@ extern "C" int ughip_latent_attention_rows(ughip_device* dev, ughip_view q, cons
   if (int rc = check_buf(dev, v_t, heads * vdim * v_stride, -1, what)) return rc;
   if (int rc = check_buf(dev, cache, s * (rank + rot), UGHIP_F32, what)) return rc;
   if (int rc = check_tables(dev, cos, sin, table_rows, pos, t, rot, what)) return rc;
-  if (int rc = check_view(dev, dst, t, heads * vdim, UGHIP_F32, what)) return rc;
+  if (int rc = check_view(dev, dst, t, heads * vdim, -1, what)) return rc;
+  const bool bf16 = dst.s->dtype == UGHIP_BF16;
+  if (!bf16 && dst.s->dtype != UGHIP_F32) return set_error(UGHIP_ERR_UNSUPPORTED, "%s: the result is F32 or BF16", what);
   if (t == 0) return UGHIP_OK;
   if ((t + QT - 1) / QT > 65535) return set_error(UGHIP_ERR_UNSUPPORTED, "%s: too many positions", what);
   if (int rc = device_activate(dev)) return rc;
-  RowsArgs a{view_ptr<float>(q), k->ptr, v_t->ptr, buf_ptr<float>(cache), buf_ptr<float>(cos), buf_ptr<float>(sin), view_ptr<float>(dst), q.stride, v_stride, dst.stride,
-             (int)t, (int)pos, (int)heads, (int)dim, (int)rot, (int)vdim, (int)rank, scale, dim % 8 == 0};
+  RowsArgs a{view_ptr<float>(q), k->ptr, v_t->ptr, buf_ptr<float>(cache), buf_ptr<float>(cos), buf_ptr<float>(sin), static_cast<char*>(dst.s->ptr) + dst.offset * (bf16 ? 2 : 4), q.stride, v_stride, dst.stride,
+             (int)t, (int)pos, (int)heads, (int)dim, (int)rot, (int)vdim, (int)rank, scale, dim % 8 == 0, bf16};
   UGHIP_HIPCHK(k->dtype == UGHIP_BF16 ? launch_rows_any<uint16_t>(dev->stream, a) : launch_rows_any<float>(dev->stream, a));
   return UGHIP_OK;
 }

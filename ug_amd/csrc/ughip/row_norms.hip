@@ -9,9 +9,15 @@ using namespace ughip;
 
 namespace {
 
+// An element of a result that is F32 or BF16.
+__device__ __forceinline__ void put(void* dst, bool bf16, size_t at, float v) {
+  if (bf16) static_cast<uint16_t*>(dst)[at] = bf16_rne(v);
+  else static_cast<float*>(dst)[at] = v;
+}
+
 template <typename T>
 __global__ void __launch_bounds__(256) gather_rows_kernel(const T* __restrict__ table, int table_rows, size_t stride, size_t col, int cols, const int* __restrict__ ids,
-                                                          float* __restrict__ dst, size_t dst_stride) {
+                                                          void* __restrict__ dst, size_t dst_stride, bool dst_bf16) {
   const int row = blockIdx.y, id = ids[row];
   const int c = blockIdx.x * 256 + threadIdx.x;
   if (c >= cols) return;
@@ -21,19 +27,21 @@ __global__ void __launch_bounds__(256) gather_rows_kernel(const T* __restrict__ 
     if constexpr (sizeof(T) == 2) v = bf16_to_f32(e);
     else v = e;
   }
-  dst[(size_t)row * dst_stride + c] = v;
+  put(dst, dst_bf16, (size_t)row * dst_stride + c, v);
 }
 
 struct AddNormArgs {
   const float* x;
   const float* y;
   const float* w;
-  float* dst;
+  void* dst;
+  uint16_t* dst16;
   size_t x_stride, y_stride, dst_stride;
   const int* slots;
   const float* weights;
   int top, y_rows, n;
   float eps;
+  bool dst_bf16;
 };
 
 __global__ void __launch_bounds__(256) add_rms_norm_kernel(AddNormArgs a) {
@@ -61,13 +69,15 @@ __global__ void __launch_bounds__(256) add_rms_norm_kernel(AddNormArgs a) {
   ss = block_sum<4>(ss, red);
   const float inv = 1.f / sqrtf(ss / (float)a.n + a.eps);
   for (int c = threadIdx.x; c < a.n; c += 256) {
-    const float v = row[c] * inv * a.w[c];  // every thread reads back its own elements
-    a.dst[i * a.dst_stride + c] = a.x ? a.x[i * a.x_stride + c] + v : v;
+    float v = row[c] * inv * a.w[c];  // every thread reads back its own elements
+    if (a.x) v += a.x[i * a.x_stride + c];
+    put(a.dst, a.dst_bf16, i * a.dst_stride + c, v);
+    if (a.dst16) a.dst16[i * a.n + c] = bf16_rne(v);
   }
 }
 
 __global__ void __launch_bounds__(256) gated_rms_norm_kernel(const float* __restrict__ y, size_t y_stride, const float* __restrict__ z, size_t z_stride,
-                                                             const float* __restrict__ w, float eps, float* __restrict__ dst, size_t dst_stride, int part) {
+                                                             const float* __restrict__ w, float eps, void* __restrict__ dst, size_t dst_stride, bool dst_bf16, int part) {
   extern __shared__ float row[];
   __shared__ float red[4];
   const size_t i = blockIdx.x, c0 = (size_t)blockIdx.y * part;
@@ -80,7 +90,16 @@ __global__ void __launch_bounds__(256) gated_rms_norm_kernel(const float* __rest
   }
   ss = block_sum<4>(ss, red);
   const float inv = 1.f / sqrtf(ss / (float)part + eps);
-  for (int c = threadIdx.x; c < part; c += 256) dst[i * dst_stride + c0 + c] = row[c] * inv * w[c0 + c];
+  for (int c = threadIdx.x; c < part; c += 256) put(dst, dst_bf16, i * dst_stride + c0 + c, row[c] * inv * w[c0 + c]);
+}
+
+// Checks a result that may be F32 or BF16; *at: its first element.
+int check_result(const ughip_device* dev, const ughip_view& v, size_t m, size_t n, const char* what, void** at, bool* bf16) {
+  if (int rc = check_view(dev, v, m, n, -1, what)) return rc;
+  if (v.s->dtype != UGHIP_F32 && v.s->dtype != UGHIP_BF16) return set_error(UGHIP_ERR_UNSUPPORTED, "%s: dtype %s, F32 or BF16 expected", what, dtype_name(v.s->dtype));
+  *bf16 = v.s->dtype == UGHIP_BF16;
+  *at = static_cast<char*>(v.s->ptr) + v.offset * (*bf16 ? 2 : 4);
+  return UGHIP_OK;
 }
 
 constexpr size_t ROW_MAX = 16000;  // the row and the reduction fit the 64 KiB a launch gets without asking
@@ -94,22 +113,23 @@ extern "C" int ughip_gather_rows(ughip_device* dev, const ughip_slice* table, si
   if (int rc = check_view(dev, ughip_view{const_cast<ughip_slice*>(table), 0, stride}, table_rows, stride, -1, "gather_rows table")) return rc;
   if (col > stride || cols > stride - col) return set_error(UGHIP_ERR_BOUNDS, "gather_rows: columns %zu + %zu of rows of %zu", col, cols, stride);
   if (int rc = check_buf(dev, ids, m, UGHIP_I32, "gather_rows ids")) return rc;
-  if (int rc = check_view(dev, dst, m, cols, UGHIP_F32, "gather_rows dst")) return rc;
+  void* d;
+  bool bf16;
+  if (int rc = check_result(dev, dst, m, cols, "gather_rows dst", &d, &bf16)) return rc;
   if (m == 0 || cols == 0) return UGHIP_OK;
   if (m > 65535) return set_error(UGHIP_ERR_UNSUPPORTED, "gather_rows: up to 65535 rows");
   if (int rc = device_activate(dev)) return rc;
   const dim3 grid((unsigned)((cols + 255) / 256), (unsigned)m);
-  float* d = view_ptr<float>(dst);
   if (table->dtype == UGHIP_F32)
-    gather_rows_kernel<float><<<grid, 256, 0, dev->stream>>>(buf_ptr<float>(table), (int)table_rows, stride, col, (int)cols, buf_ptr<int>(ids), d, dst.stride);
+    gather_rows_kernel<float><<<grid, 256, 0, dev->stream>>>(buf_ptr<float>(table), (int)table_rows, stride, col, (int)cols, buf_ptr<int>(ids), d, dst.stride, bf16);
   else
-    gather_rows_kernel<uint16_t><<<grid, 256, 0, dev->stream>>>(buf_ptr<uint16_t>(table), (int)table_rows, stride, col, (int)cols, buf_ptr<int>(ids), d, dst.stride);
+    gather_rows_kernel<uint16_t><<<grid, 256, 0, dev->stream>>>(buf_ptr<uint16_t>(table), (int)table_rows, stride, col, (int)cols, buf_ptr<int>(ids), d, dst.stride, bf16);
   UGHIP_HIPCHK(hipGetLastError());
   return UGHIP_OK;
 }
 
 extern "C" int ughip_add_rms_norm_rows(ughip_device* dev, ughip_view x, ughip_view y, const ughip_slice* slots, const ughip_slice* weights, size_t top, size_t y_rows,
-                                       const ughip_slice* w, float eps, ughip_view dst, size_t m, size_t n) {
+                                       const ughip_slice* w, float eps, ughip_view dst, ughip_slice* dst_bf16, size_t m, size_t n) {
   if (!dev) return set_error(UGHIP_ERR_INVALID, "add_rms_norm_rows: null device");
   if (n > ROW_MAX) return set_error(UGHIP_ERR_UNSUPPORTED, "add_rms_norm_rows: rows of %zu elements, up to %zu are supported", n, ROW_MAX);
   if (x.s)
@@ -121,11 +141,15 @@ extern "C" int ughip_add_rms_norm_rows(ughip_device* dev, ughip_view x, ughip_vi
     if (int rc = check_buf(dev, weights, m * top, UGHIP_F32, "add_rms_norm_rows weights")) return rc;
   }
   if (int rc = check_buf(dev, w, n, UGHIP_F32, "add_rms_norm_rows w")) return rc;
-  if (int rc = check_view(dev, dst, m, n, UGHIP_F32, "add_rms_norm_rows dst")) return rc;
+  void* d;
+  bool bf16;
+  if (int rc = check_result(dev, dst, m, n, "add_rms_norm_rows dst", &d, &bf16)) return rc;
+  if (dst_bf16)
+    if (int rc = check_buf(dev, dst_bf16, m * n, UGHIP_BF16, "add_rms_norm_rows bf16 rows")) return rc;
   if (m == 0 || n == 0) return UGHIP_OK;
   if (int rc = device_activate(dev)) return rc;
-  AddNormArgs a{view_ptr<float>(x), view_ptr<float>(y), buf_ptr<float>(w), view_ptr<float>(dst), x.stride, y.stride, dst.stride, buf_ptr<int>(slots), buf_ptr<float>(weights),
-                (int)top, (int)y_rows, (int)n, eps};
+  AddNormArgs a{view_ptr<float>(x), view_ptr<float>(y), buf_ptr<float>(w), d, dst_bf16 ? static_cast<uint16_t*>(dst_bf16->ptr) : nullptr, x.stride, y.stride, dst.stride, buf_ptr<int>(slots), buf_ptr<float>(weights),
+                (int)top, (int)y_rows, (int)n, eps, bf16};
   add_rms_norm_kernel<<<(unsigned)m, 256, n * sizeof(float), dev->stream>>>(a);
   UGHIP_HIPCHK(hipGetLastError());
   return UGHIP_OK;
@@ -139,12 +163,14 @@ extern "C" int ughip_gated_rms_norm_rows(ughip_device* dev, ughip_view y, ughip_
   if (z.s)
     if (int rc = check_view(dev, z, m, n, UGHIP_F32, "gated_rms_norm_rows z")) return rc;
   if (int rc = check_buf(dev, w, n, UGHIP_F32, "gated_rms_norm_rows w")) return rc;
-  if (int rc = check_view(dev, dst, m, n, UGHIP_F32, "gated_rms_norm_rows dst")) return rc;
+  void* d;
+  bool bf16;
+  if (int rc = check_result(dev, dst, m, n, "gated_rms_norm_rows dst", &d, &bf16)) return rc;
   if (m == 0 || n == 0) return UGHIP_OK;
   if (int rc = device_activate(dev)) return rc;
   const size_t part = n / groups;
   gated_rms_norm_kernel<<<dim3((unsigned)m, (unsigned)groups), 256, part * sizeof(float), dev->stream>>>(view_ptr<float>(y), y.stride, view_ptr<float>(z), z.stride,
-                                                                                                        buf_ptr<float>(w), eps, view_ptr<float>(dst), dst.stride, (int)part);
+                                                                                                        buf_ptr<float>(w), eps, d, dst.stride, bf16, (int)part);
   UGHIP_HIPCHK(hipGetLastError());
   return UGHIP_OK;
 }

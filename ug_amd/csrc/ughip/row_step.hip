@@ -22,9 +22,7 @@ struct RowArgs {
   float* x_out;  // null: not kept
   float* dst;
   const void* w;
-  const void* w_up;
   const float* bias;
-  const float* bias_up;
   const void* table;
   const int* ids;
   size_t table_stride, table_col, w_group;
@@ -135,7 +133,7 @@ __global__ void __launch_bounds__(256) row_step_kernel(RowArgs a) {
       at = (size_t)s_ids[j] * a.w_group + (size_t)((live[r] ? col : 0) - j * a.n) * a.k;
     }
     rows[0][r] = static_cast<const WT*>(a.w) + at;
-    if (NM == 2) rows[NM - 1][r] = static_cast<const WT*>(a.w_up) + at;
+    if (NM == 2) rows[NM - 1][r] = static_cast<const WT*>(a.w) + at + (size_t)a.n * a.k;  // gate rows, then up rows
   }
   // eight elements from `kk` on of a row (ROUTE 2: of the segments' rows one after the other)
   auto fetch = [&](Eight<WT>& e, const WT* row, bool ok, int kk) {
@@ -253,7 +251,7 @@ __global__ void __launch_bounds__(256) row_step_kernel(RowArgs a) {
     if (a.bias) v += a.bias[col];
     if (NM == 2) {
       float u = acc[NM - 1][r];
-      if (a.bias_up) u += a.bias_up[col];
+      if (a.bias) u += a.bias[a.n + col];
       v = silu_f(v) * u;
     } else if (a.table) {
       const int id = a.ids[0];
@@ -310,11 +308,11 @@ extern "C" int ughip_product_row(ughip_device* dev, const ughip_row_step* p) {
   if (p->k == 0 || p->k > ROW_MAX || segs == 0 || segs > 64 || total > ROW_MAX) return set_error(UGHIP_ERR_UNSUPPORTED, "%s: rows of %zu elements, up to %zu are supported", what, total, ROW_MAX);
   if (p->n > 0x7fffffffull / 128) return set_error(UGHIP_ERR_INVALID, "%s: shape too large", what);
   if (p->w->dtype != UGHIP_F32 && p->w->dtype != UGHIP_BF16) return set_error(UGHIP_ERR_UNSUPPORTED, "%s: matrices are F32 or BF16", what);
-  const size_t mats = p->route ? p->experts : 1;
+  const size_t mats = p->route ? p->experts : 1, w_rows = p->act == UGHIP_ACT_SWIGLU ? 2 * p->n : p->n;
   if (p->route) {
     if (int rc = route_check(p->experts, p->groups, p->keep, p->top, what)) return rc;
     if (p->top > 64) return set_error(UGHIP_ERR_UNSUPPORTED, "%s: up to 64 experts per row", what);
-    if (p->bias || p->bias_up || (p->route == 1) != (p->act == UGHIP_ACT_SWIGLU) || (p->route == 2 && p->act != UGHIP_ACT_NONE) || p->y || p->norm || p->gate)
+    if (p->bias || (p->route == 1) != (p->act == UGHIP_ACT_SWIGLU) || (p->route == 2 && p->act != UGHIP_ACT_NONE) || p->y || p->norm || p->gate)
       return set_error(UGHIP_ERR_UNSUPPORTED, "%s: routed products are SwiGLU (1) or plain (2), on x as it is", what);
     if (int rc = check_buf(dev, p->route_ids, p->top, UGHIP_I32, "product_row ids")) return rc;
     if (int rc = check_buf(dev, p->route_weights, p->top, UGHIP_F32, "product_row weights")) return rc;
@@ -333,13 +331,9 @@ extern "C" int ughip_product_row(ughip_device* dev, const ughip_row_step* p) {
     if (p->k % norm_groups) return set_error(UGHIP_ERR_INVALID, "%s: %zu elements in %zu groups", what, p->k, norm_groups);
     if (int rc = row(p->norm, 0, p->k, UGHIP_F32)) return rc;
   }
-  if (int rc = row(p->w, 0, mats * p->n * p->k, -1)) return rc;
-  if (p->act == UGHIP_ACT_SWIGLU)
-    if (int rc = row(p->w_up, 0, mats * p->n * p->k, p->w->dtype)) return rc;
+  if (int rc = row(p->w, 0, mats * w_rows * p->k, -1)) return rc;
   if (p->bias)
-    if (int rc = row(p->bias, 0, p->n, UGHIP_F32)) return rc;
-  if (p->bias_up)
-    if (int rc = row(p->bias_up, 0, p->n, UGHIP_F32)) return rc;
+    if (int rc = row(p->bias, 0, w_rows, UGHIP_F32)) return rc;
   const size_t cols = p->route == 1 ? p->top * p->n : p->n;
   if (int rc = row(p->dst, p->dst_offset, cols, UGHIP_F32)) return rc;
   if (p->keep_x) {
@@ -367,13 +361,13 @@ extern "C" int ughip_product_row(ughip_device* dev, const ughip_row_step* p) {
   float* d = static_cast<float*>(p->dst->ptr);
   a.x_out = p->keep_x ? d + p->x_out : nullptr;
   a.dst = d + p->dst_offset;
-  a.w = p->w->ptr, a.w_up = p->act == UGHIP_ACT_SWIGLU ? p->w_up->ptr : nullptr;
-  a.bias = buf_ptr<float>(p->bias), a.bias_up = buf_ptr<float>(p->bias_up);
+  a.w = p->w->ptr;
+  a.bias = buf_ptr<float>(p->bias);
   if (p->act == UGHIP_ACT_GELU_MUL) {
     a.table = p->table->ptr, a.table_bf16 = p->table->dtype == UGHIP_BF16, a.table_rows = (int)p->table_rows;
     a.table_stride = p->table_stride, a.table_col = p->table_col, a.ids = buf_ptr<int>(p->ids);
   }
-  a.w_group = p->n * p->k, a.eps = p->eps, a.n = (int)p->n, a.k = (int)p->k, a.cols = (int)cols, a.segs = (int)segs;
+  a.w_group = w_rows * p->k, a.eps = p->eps, a.n = (int)p->n, a.k = (int)p->k, a.cols = (int)cols, a.segs = (int)segs;
   size_t lds = (total + RUN - 1) / RUN * RUN * sizeof(float);
   if (p->route) {
     a.route = RouteArgs{buf_ptr<float>(p->correction), (int)p->experts, (int)p->groups, (int)p->keep, (int)p->top};
@@ -383,8 +377,8 @@ extern "C" int ughip_product_row(ughip_device* dev, const ughip_row_step* p) {
       lds += (p->experts + (size_t)route_lds_floats(a.route.experts, a.route.groups) + 2 * p->top) * sizeof(float);
     }
   }
-  const bool vec = p->k % 8 == 0 && (reinterpret_cast<uintptr_t>(a.w) & 15) == 0 && (reinterpret_cast<uintptr_t>(a.w_up) & 15) == 0;
-  UGHIP_HIPCHK(p->w->dtype == UGHIP_BF16 ? launch_any<uint16_t>(dev->stream, a, p->route, a.w_up != nullptr, lds, vec)
-                                         : launch_any<float>(dev->stream, a, p->route, a.w_up != nullptr, lds, vec));
+  const bool vec = p->k % 8 == 0 && (reinterpret_cast<uintptr_t>(a.w) & 15) == 0;
+  UGHIP_HIPCHK(p->w->dtype == UGHIP_BF16 ? launch_any<uint16_t>(dev->stream, a, p->route, p->act == UGHIP_ACT_SWIGLU, lds, vec)
+                                         : launch_any<float>(dev->stream, a, p->route, p->act == UGHIP_ACT_SWIGLU, lds, vec));
   return UGHIP_OK;
 }

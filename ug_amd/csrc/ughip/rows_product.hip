@@ -10,6 +10,7 @@
 #include <hip/hip_runtime.h>
 
 #include "bf16_split.h"
+#include "gemm.h"
 #include "layers.h"
 
 using namespace ughip;
@@ -24,9 +25,7 @@ typedef __bf16 bf16x4 __attribute__((ext_vector_type(4)));
 struct ProductArgs {
   const void* x;
   const void* w;
-  const void* w_up;
   const float* bias;
-  const float* bias_up;
   void* dst;
   size_t x_stride, w_stride, dst_stride, w_group;  // elements; w_group: from one group's matrix to the next
   int m, n, k;
@@ -152,16 +151,15 @@ __global__ void __launch_bounds__(256) rows_product_kernel(ProductArgs a) {
 #pragma unroll
   for (int i = 0; i < WC; ++i) {
     const int rb = (tid >> 3) + 32 * i;
-    int col;
-    const void* base = a.w;
+    int col, up = 0;
     if (ACT == UGHIP_ACT_SWIGLU) {  // LDS rows: 32 gate columns, the same 32 of up, the next 32 gate columns, ...
       col = n0 + (rb >> 6) * 32 + (rb & 31);
-      if (rb & 32) base = a.w_up;
+      up = rb & 32 ? a.n : 0;
     } else {
       col = n0 + rb;
     }
     wok[i] = col < a.n;
-    wrow[i] = static_cast<const WT*>(base) + (size_t)group * a.w_group + (size_t)(wok[i] ? col : 0) * a.w_stride;
+    wrow[i] = static_cast<const WT*>(a.w) + (size_t)group * a.w_group + (size_t)(wok[i] ? up + col : 0) * a.w_stride;
   }
   f32x16 acc[MI][NI];
 #pragma unroll
@@ -221,7 +219,7 @@ __global__ void __launch_bounds__(256) rows_product_kernel(ProductArgs a) {
         if (a.bias) v += a.bias[col];
         if constexpr (ACT == UGHIP_ACT_SWIGLU) {
           float u = acc[i][1][e];
-          if (a.bias_up) u += a.bias_up[col];
+          if (a.bias) u += a.bias[a.n + col];
           v = silu_f(v) * u;
         }
         if constexpr (ACT == UGHIP_ACT_GELU_MUL) {
@@ -269,6 +267,8 @@ hipError_t launch_types(hipStream_t st, const ProductArgs& a, int act, bool vec)
   return launch_act<CT, XT, WT, UGHIP_ACT_NONE>(st, a, vec);
 }
 
+constexpr size_t DMA_ROWS_MIN = 96;  // below that a 128-row tile is mostly padding
+
 bool aligned16(const void* p) { return (reinterpret_cast<uintptr_t>(p) & 15) == 0; }
 
 }  // namespace
@@ -288,23 +288,19 @@ extern "C" int ughip_product_rows(ughip_device* dev, const ughip_product* p) {
   if (x_rows == 0) return set_error(UGHIP_ERR_INVALID, "%s: no rows of x", what);
   if (int rc = check_view(dev, p->x, x_rows, p->k, f32 ? UGHIP_F32 : -1, "product_rows x")) return rc;
   const size_t w_stride = p->w_stride ? p->w_stride : p->k;
-  if (w_stride != p->k && (p->groups || p->w_up)) return set_error(UGHIP_ERR_UNSUPPORTED, "%s: rows of w %zu elements apart belong to the plain form", what, w_stride);
+  const size_t w_rows = p->act == UGHIP_ACT_SWIGLU ? 2 * p->n : p->n;
+  if (w_stride != p->k && p->groups) return set_error(UGHIP_ERR_UNSUPPORTED, "%s: rows of w %zu elements apart belong to the plain form", what, w_stride);
   if (p->groups) {
-    if (int rc = check_buf(dev, p->w, mats * p->n * p->k, f32 ? UGHIP_F32 : -1, "product_rows w")) return rc;
-  } else if (int rc = check_view(dev, ughip_view{const_cast<ughip_slice*>(p->w), 0, w_stride}, p->n, p->k, f32 ? UGHIP_F32 : -1, "product_rows w")) {
+    if (int rc = check_buf(dev, p->w, mats * w_rows * p->k, f32 ? UGHIP_F32 : -1, "product_rows w")) return rc;
+  } else if (int rc = check_view(dev, ughip_view{const_cast<ughip_slice*>(p->w), 0, w_stride}, w_rows, p->k, f32 ? UGHIP_F32 : -1, "product_rows w")) {
     return rc;
-  }
-  if (p->act == UGHIP_ACT_SWIGLU) {
-    if (int rc = check_buf(dev, p->w_up, mats * p->n * p->k, p->w->dtype, "product_rows w_up")) return rc;
   }
   if (int rc = check_view(dev, p->dst, p->m, p->n, f32 ? UGHIP_F32 : -1, "product_rows dst")) return rc;
   auto f_or_b = [](const ughip_slice* s) { return s->dtype == UGHIP_F32 || s->dtype == UGHIP_BF16; };
   if (!f_or_b(p->x.s) || !f_or_b(p->w) || !f_or_b(p->dst.s)) return set_error(UGHIP_ERR_UNSUPPORTED, "%s: operands are F32 or BF16", what);
-  if ((p->bias || p->bias_up) && p->groups) return set_error(UGHIP_ERR_UNSUPPORTED, "%s: the grouped form takes no bias", what);
+  if (p->bias && p->groups) return set_error(UGHIP_ERR_UNSUPPORTED, "%s: the grouped form takes no bias", what);
   if (p->bias)
-    if (int rc = check_buf(dev, p->bias, p->n, UGHIP_F32, "product_rows bias")) return rc;
-  if (p->bias_up)
-    if (int rc = check_buf(dev, p->bias_up, p->n, UGHIP_F32, "product_rows bias_up")) return rc;
+    if (int rc = check_buf(dev, p->bias, w_rows, UGHIP_F32, "product_rows bias")) return rc;
   if (p->act == UGHIP_ACT_GELU_MUL) {
     if (!p->table || !f_or_b(p->table)) return set_error(UGHIP_ERR_INVALID, "%s: a gate's table is F32 or BF16", what);
     if (int rc = check_buf(dev, p->table, p->table_rows * p->table_stride, p->table->dtype, "product_rows table")) return rc;
@@ -322,19 +318,33 @@ extern "C" int ughip_product_rows(ughip_device* dev, const ughip_product* p) {
   const size_t xs = p->x.s->dtype == UGHIP_BF16 ? 2 : 4;
   a.x = static_cast<const char*>(p->x.s->ptr) + p->x.offset * xs;
   a.w = p->w->ptr;
-  a.w_up = p->w_up ? p->w_up->ptr : nullptr;
-  a.bias = buf_ptr<float>(p->bias), a.bias_up = buf_ptr<float>(p->bias_up);
+  a.bias = buf_ptr<float>(p->bias);
   a.dst_bf16 = p->dst.s->dtype == UGHIP_BF16;
   a.dst = static_cast<char*>(p->dst.s->ptr) + p->dst.offset * (a.dst_bf16 ? 2 : 4);
-  a.x_stride = p->x.stride, a.w_stride = w_stride, a.dst_stride = p->dst.stride, a.w_group = p->n * p->k;
+  a.x_stride = p->x.stride, a.w_stride = w_stride, a.dst_stride = p->dst.stride, a.w_group = w_rows * p->k;
   a.m = (int)p->m, a.n = (int)p->n, a.k = (int)p->k;
   if (p->act == UGHIP_ACT_GELU_MUL) {
     a.table = p->table->ptr, a.table_bf16 = p->table->dtype == UGHIP_BF16, a.table_rows = (int)p->table_rows;
     a.table_stride = p->table_stride, a.table_col = p->table_col, a.ids = buf_ptr<int>(p->ids);
   }
   a.row_index = buf_ptr<int>(p->row_index), a.group_end = buf_ptr<int>(p->group_end), a.groups = (int)p->groups, a.x_rows = (int)x_rows;
-  const bool vec = p->k % 8 == 0 && (p->x.stride * xs) % 16 == 0 && (w_stride * (p->w->dtype == UGHIP_BF16 ? 2 : 4)) % 16 == 0 && aligned16(a.x) && aligned16(a.w) && (!a.w_up || aligned16(a.w_up));
+  const bool vec = p->k % 8 == 0 && (p->x.stride * xs) % 16 == 0 && (w_stride * (p->w->dtype == UGHIP_BF16 ? 2 : 4)) % 16 == 0 && aligned16(a.x) && aligned16(a.w);
   const bool xb = p->x.s->dtype == UGHIP_BF16, wb = p->w->dtype == UGHIP_BF16;
+  if (xb && wb && p->act != UGHIP_ACT_GELU_MUL && p->m >= DMA_ROWS_MIN) {
+    MMArgs q;
+    q.a = a.x, q.b = a.w, q.c = nullptr;
+    q.M = a.m, q.N = (int)w_rows, q.K = a.k;
+    q.a_rs = (long long)a.x_stride, q.a_cs = 1, q.b_rs = 1, q.b_cs = (long long)a.w_stride;
+    q.a_bs = q.b_bs = q.c_bs = 0;
+    DmaRows r;
+    r.row_index = a.row_index, r.group_end = a.group_end, r.bias = a.bias, r.dst = a.dst, r.w_group = (long long)a.w_group, r.dst_stride = (long long)a.dst_stride;
+    r.groups = a.groups, r.x_rows = a.x_rows, r.n_out = a.n, r.dst_bf16 = a.dst_bf16;
+    const bool swiglu = p->act == UGHIP_ACT_SWIGLU;
+    if (const int tile = gemm_dma_rows_pick(q, r, swiglu)) {
+      UGHIP_HIPCHK(gemm_dma_launch_rows(dev->stream, q, r, swiglu, tile));
+      return UGHIP_OK;
+    }
+  }
   hipError_t e;
   if (f32) e = launch_types<float, float, float>(dev->stream, a, p->act, vec);
   else if (xb && wb) e = launch_types<__bf16, uint16_t, uint16_t>(dev->stream, a, p->act, vec);
