@@ -114,7 +114,25 @@ __global__ void __launch_bounds__(256) gemm_dma4(MMArgs p, int tiles_m, int tile
   // tiles, and tiles are numbered in super-rows of 4 tile rows, column by column inside, so that such a run is a 4-row
   // block: its workgroups share few A and B panels in their XCD's L2.
   int bid = blockIdx.x;
-  if ((gridDim.x & 7) == 0) bid = (bid & 7) * (int)(gridDim.x >> 3) + (bid >> 3);
+  if constexpr (ROWS != 0) {
+    if (rw.groups) {
+      // how many tile rows there are is known here only: the workgroups past them leave before the runs are dealt
+      int rows = 0, begin = 0;
+      for (int g = 0; g < rw.groups; ++g) {
+        int end = rw.group_end[g];
+        end = end < begin ? begin : end > p.M ? p.M : end;
+        rows += (end - begin + BM - 1) / BM;
+        begin = end;
+      }
+      const int tiles = rows * tiles_n, per = (tiles + 7) >> 3;
+      if (bid >= 8 * per) return;
+      bid = (bid & 7) * per + (bid >> 3);
+      if (bid >= tiles) return;
+      tiles_m = rows;
+    } else if ((gridDim.x & 7) == 0) {
+      bid = (bid & 7) * (int)(gridDim.x >> 3) + (bid >> 3);
+    }
+  } else if ((gridDim.x & 7) == 0) bid = (bid & 7) * (int)(gridDim.x >> 3) + (bid >> 3);
   const int tpb = tiles_m * tiles_n;
   const int batch = bid / tpb;
   const int t_in = bid - batch * tpb;
@@ -473,7 +491,8 @@ hipError_t launch(hipStream_t stream, const MMArgs& p, size_t batch, const float
     configured.fetch_or(bit, std::memory_order_relaxed);
   }
   const int tiles_m = (p.M + BM - 1) / BM + rw.groups, tiles_n = (p.N + BN - 1) / BN;
-  const size_t total = batch * (size_t)tiles_m * tiles_n;
+  // (8 more for groups: the kernel deals the tiles that exist in 8 equal runs)
+  const size_t total = batch * (size_t)tiles_m * tiles_n + (rw.groups ? 8 : 0);
   kernel<<<dim3((unsigned)total), dim3(256), LDS_BYTES, stream>>>(p, tiles_m, tiles_n, residual, rw);
   return hipGetLastError();
 }

@@ -60,31 +60,67 @@ __global__ void __launch_bounds__(256) latent_append_kernel(AppendArgs a) {
   append_row(a, blockIdx.x, red);
 }
 
-struct RowsArgs {
+struct PackArgs {
   const float* q;
   const void* k;
-  const void* v;
   const float* cache;
   const float* cos;
   const float* sin;
-  void* dst;
-  size_t q_stride, v_stride, dst_stride;
-  int t, pos, heads, dim, rot, vdim, rank;
-  float scale;
-  bool vec, dst_bf16;
+  void* qp;
+  void* kp;
+  size_t q_stride;
+  int t, pos, heads, dim, rot, rank, q_rows, k_rows;
 };
 
-template <typename T, int E>
-__device__ __forceinline__ u32x4_t pack_chunk(const float* v) {
-  if constexpr (sizeof(T) == 2) {
-    bf16x8 o;
-#pragma unroll
-    for (int i = 0; i < 8; ++i) o[i] = (__bf16)v[i];
-    return __builtin_bit_cast(u32x4_t, o);
-  } else {
-    return __builtin_bit_cast(u32x4_t, f32x4_t{v[0], v[1], v[2], v[3]});
-  }
+template <typename T>
+__device__ __forceinline__ T to_elem(float v) {
+  if constexpr (sizeof(T) == 2) return bf16_rne(v);
+  else return v;
 }
+
+// The operands of the scores as the kernel below reads them: [heads][rows][DQ], queries rotated, keys with the shared rotated part
+// behind each head's own, zeros past the last element and the last position.  A thread makes 16 bytes.
+template <typename T, int DQ>
+__global__ void __launch_bounds__(256) latent_pack_kernel(PackArgs a) {
+  constexpr int E = 16 / sizeof(T), CH = DQ / E;
+  const size_t e0 = (size_t)blockIdx.x * 256 + threadIdx.x, all = (size_t)(a.q_rows + a.k_rows) * CH;
+  if (e0 >= all) return;
+  const int head = blockIdx.y, row = (int)(e0 / CH), c = (int)(e0 % CH) * E;
+  const bool is_q = row < a.q_rows;
+  const int r = is_q ? row : row - a.q_rows, p = is_q ? a.pos + r : r;
+  T v[E];
+  if (is_q ? r < a.t : r < a.pos + a.t) {
+    const float* qr = is_q ? a.q + (size_t)r * a.q_stride + (size_t)head * (a.dim + a.rot) : nullptr;
+    const T* kr = static_cast<const T*>(a.k) + (size_t)r * a.heads * a.dim + (size_t)head * a.dim;
+    const float* rr = a.cache + (size_t)r * (a.rank + a.rot) + a.rank;
+#pragma unroll
+    for (int e = 0; e < E; ++e) {
+      const int d = c + e;
+      if (d < a.dim) v[e] = is_q ? to_elem<T>(qr[d]) : kr[d];
+      else if (d < a.dim + a.rot)
+        v[e] = to_elem<T>(is_q ? rotated(qr + a.dim, d - a.dim, a.rot, a.cos + (size_t)p * (a.rot / 2), a.sin + (size_t)p * (a.rot / 2)) : rr[d - a.dim]);
+      else v[e] = T(0);
+    }
+  } else {
+#pragma unroll
+    for (int e = 0; e < E; ++e) v[e] = T(0);
+  }
+  T* out = static_cast<T*>(is_q ? a.qp : a.kp) + ((size_t)head * (is_q ? a.q_rows : a.k_rows) + r) * DQ + c;
+  u32x4_t chunk;
+  __builtin_memcpy(&chunk, v, 16);
+  *reinterpret_cast<u32x4_t*>(out) = chunk;
+}
+
+struct RowsArgs {
+  const void* q;  // packed
+  const void* k;
+  const void* v;
+  void* dst;
+  size_t v_stride, dst_stride;
+  int t, pos, vdim, q_rows, k_rows;
+  float scale2;  // scale * log2(e): the weights are powers of two
+  bool dst_bf16;
+};
 
 template <typename T>
 __device__ __forceinline__ void mfma_chunk(const u32x4_t& a, const u32x4_t& b, f32x16& acc) {
@@ -109,29 +145,21 @@ constexpr int rows_lds_bytes() {
 template <typename T, int DQ, int DV>
 __global__ void __launch_bounds__(256) latent_rows_kernel(RowsArgs a) {
   constexpr int E = 16 / sizeof(T), QC = DQ / E, K_ROW = DQ * sizeof(T) + 16, V_ROW = KT * sizeof(T) + 16, VC = KT / E;
+  constexpr int NK = KT * QC / 256, NV = DV * VC / 256;  // 16-byte pieces of a tile per thread
+  constexpr bool AHEAD = NK + NV <= 16;                   // the next tile waits in registers while this one is multiplied
+  static_assert(KT * QC % 256 == 0 && DV * VC % 256 == 0, "whole pieces per thread");
   extern __shared__ __attribute__((aligned(16))) char lds[];
   char* Ks = lds;                // [KT][DQ]
   char* Vs = lds + KT * K_ROW;   // [DV][KT]
   const int head = blockIdx.x, qb = gridDim.y - 1 - blockIdx.y;  // the longest rows first
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, col = lane & 31, hf = lane >> 5;
-  const int i_mine = qb * QT + wave * 32 + col, iq = i_mine < a.t ? i_mine : a.t - 1;
-  const int p_mine = a.pos + iq;
-  // the wave's queries, rotated, as the right operand of S^T: chunk 2 c + hf of query `col`
+  const int i_mine = qb * QT + wave * 32 + col, p_mine = a.pos + min(i_mine, a.t - 1);
+  // the wave's queries as the right operand of S^T: chunk 2 c + hf of query `col` (rows up to q_rows exist, zeros past t)
   u32x4_t qf[QC / 2];
   {
-    const float* qr = a.q + (size_t)iq * a.q_stride + (size_t)head * (a.dim + a.rot);
-    const float* cr = a.cos + (size_t)p_mine * (a.rot / 2);
-    const float* sr = a.sin + (size_t)p_mine * (a.rot / 2);
+    const char* qr = static_cast<const char*>(a.q) + ((size_t)head * a.q_rows + i_mine) * DQ * sizeof(T) + hf * 16;
 #pragma unroll
-    for (int c = 0; c < QC / 2; ++c) {
-      float v[E];
-#pragma unroll
-      for (int e = 0; e < E; ++e) {
-        const int d = (2 * c + hf) * E + e;
-        v[e] = d < a.dim ? qr[d] : d < a.dim + a.rot ? rotated(qr + a.dim, d - a.dim, a.rot, cr, sr) : 0.f;
-      }
-      qf[c] = pack_chunk<T, E>(v);
-    }
+    for (int c = 0; c < QC / 2; ++c) qf[c] = *reinterpret_cast<const u32x4_t*>(qr + c * 32);
   }
   f32x16 o[DV / 32];
 #pragma unroll
@@ -139,89 +167,96 @@ __global__ void __launch_bounds__(256) latent_rows_kernel(RowsArgs a) {
 #pragma unroll
     for (int e = 0; e < 16; ++e) o[i][e] = 0.f;
   float mx = -INFINITY, sum = 0.f;
-  const int s_all = a.pos + a.t, last_q = min(a.t, (qb + 1) * QT), keys = a.pos + last_q;
-  const int cache_row = a.rank + a.rot;
-  for (int k0 = 0; k0 < keys; k0 += KT) {
-    __syncthreads();
-    for (int x = threadIdx.x; x < KT * QC; x += 256) {
-      const int key = x / QC, c = x % QC, d0 = c * E, kp = k0 + key;
-      u32x4_t chunk = {0, 0, 0, 0};
-      if (kp < s_all && d0 < a.dim + a.rot) {
-        const T* kr = static_cast<const T*>(a.k) + (size_t)kp * a.heads * a.dim + (size_t)head * a.dim;
-        const float* rr = a.cache + (size_t)kp * cache_row + a.rank;
-        if (a.vec && d0 < a.dim) {
-          chunk = *reinterpret_cast<const u32x4_t*>(kr + d0);
-        } else {
-          float v[E];
+  const int s_all = a.pos + a.t, last_q = min(a.t, (qb + 1) * QT), keys = a.pos + last_q, first_p = a.pos + qb * QT + wave * 32;
+  const char* k_head = static_cast<const char*>(a.k) + (size_t)head * a.k_rows * DQ * sizeof(T);
+  const T* v_head = static_cast<const T*>(a.v) + (size_t)head * a.vdim * a.v_stride;
+  u32x4_t kr[NK], vr[NV];
+  auto fetch = [&](int k0) {
 #pragma unroll
-          for (int e = 0; e < E; ++e) {
-            const int d = d0 + e;
-            float f = 0.f;
-            if (d < a.dim) {
-              if constexpr (sizeof(T) == 2) f = bf16_to_f32(kr[d]);
-              else f = kr[d];
-            } else if (d < a.dim + a.rot) {
-              f = rr[d - a.dim];
-            }
-            v[e] = f;
-          }
-          chunk = pack_chunk<T, E>(v);
-        }
-      }
-      *reinterpret_cast<u32x4_t*>(Ks + key * K_ROW + c * 16) = chunk;
-    }
-    for (int x = threadIdx.x; x < DV * VC; x += 256) {
-      const int vc = x / VC, c = x % VC, kp = k0 + c * E;
+    for (int u = 0; u < NK; ++u) kr[u] = *reinterpret_cast<const u32x4_t*>(k_head + (size_t)k0 * DQ * sizeof(T) + (threadIdx.x + u * 256) * 16);
+#pragma unroll
+    for (int u = 0; u < NV; ++u) {
+      const int x = threadIdx.x + u * 256, vc = x / VC, kp = k0 + x % VC * E;
       u32x4_t chunk = {0, 0, 0, 0};
       if (vc < a.vdim && kp < s_all) {
-        const T* vr = static_cast<const T*>(a.v) + ((size_t)head * a.vdim + vc) * a.v_stride;
+        const T* p = v_head + (size_t)vc * a.v_stride + kp;
         if (kp + E <= s_all) {
-          chunk = *reinterpret_cast<const u32x4_t*>(vr + kp);  // rows are padded to whole tiles and 16-byte aligned
+          chunk = *reinterpret_cast<const u32x4_t*>(p);  // rows are padded to whole tiles and 16-byte aligned
         } else {  // values past the last position were never written
           T v[E];
 #pragma unroll
-          for (int e = 0; e < E; ++e) v[e] = kp + e < s_all ? vr[kp + e] : T(0);
+          for (int e = 0; e < E; ++e) v[e] = kp + e < s_all ? p[e] : T(0);
           __builtin_memcpy(&chunk, v, 16);
         }
       }
-      *reinterpret_cast<u32x4_t*>(Vs + vc * V_ROW + c * 16) = chunk;
+      vr[u] = chunk;
+    }
+  };
+  if (AHEAD) fetch(0);
+  for (int k0 = 0; k0 < keys; k0 += KT) {
+    __syncthreads();
+    if (!AHEAD) fetch(k0);
+#pragma unroll
+    for (int u = 0; u < NK; ++u) {
+      const int x = threadIdx.x + u * 256;
+      *reinterpret_cast<u32x4_t*>(Ks + x / QC * K_ROW + x % QC * 16) = kr[u];
+    }
+#pragma unroll
+    for (int u = 0; u < NV; ++u) {
+      const int x = threadIdx.x + u * 256;
+      *reinterpret_cast<u32x4_t*>(Vs + x / VC * V_ROW + x % VC * 16) = vr[u];
     }
     __syncthreads();
+    if (AHEAD && k0 + KT < keys) fetch(k0 + KT);
+    if (k0 > first_p + 31) continue;  // nothing in this tile is visible to the wave's queries
     f32x16 s[2];
-#pragma unroll
-    for (int b = 0; b < 2; ++b) {
-#pragma unroll
-      for (int e = 0; e < 16; ++e) s[b][e] = 0.f;
-      const char* kr = Ks + (b * 32 + col) * K_ROW + hf * 16;
-#pragma unroll
-      for (int c = 0; c < QC / 2; ++c) mfma_chunk<T>(*reinterpret_cast<const u32x4_t*>(kr + c * 32), qf[c], s[b]);
-    }
-    // element e of s[b]: key k0 + 32 b + 8 (e / 4) + 4 hf + e % 4, query `col`
-    float top = mx;
 #pragma unroll
     for (int b = 0; b < 2; ++b)
 #pragma unroll
-      for (int e = 0; e < 16; ++e) {
-        const int key = k0 + 32 * b + 8 * (e >> 2) + 4 * hf + (e & 3);
-        s[b][e] = key <= p_mine ? s[b][e] * a.scale : -INFINITY;
-        top = fmaxf(top, s[b][e]);
-      }
+      for (int e = 0; e < 16; ++e) s[b][e] = 0.f;
+#pragma unroll
+    for (int c = 0; c < QC / 2; ++c)
+#pragma unroll
+      for (int b = 0; b < 2; ++b) mfma_chunk<T>(*reinterpret_cast<const u32x4_t*>(Ks + (b * 32 + col) * K_ROW + hf * 16 + c * 32), qf[c], s[b]);
+    // element e of s[b]: key k0 + 32 b + 8 (e / 4) + 4 hf + e % 4, query `col`
+    float top = mx;
+    if (k0 + KT - 1 > first_p) {  // some keys of the tile lie behind some of the wave's queries
+#pragma unroll
+      for (int b = 0; b < 2; ++b)
+#pragma unroll
+        for (int e = 0; e < 16; ++e) {
+          const int key = k0 + 32 * b + 8 * (e >> 2) + 4 * hf + (e & 3);
+          s[b][e] = key <= p_mine ? s[b][e] * a.scale2 : -INFINITY;
+        }
+    } else {
+#pragma unroll
+      for (int b = 0; b < 2; ++b)
+#pragma unroll
+        for (int e = 0; e < 16; ++e) s[b][e] *= a.scale2;
+    }
+#pragma unroll
+    for (int b = 0; b < 2; ++b)
+#pragma unroll
+      for (int e = 0; e < 16; ++e) top = fmaxf(top, s[b][e]);
     top = fmaxf(top, __shfl_xor(top, 32, 64));
-    const float alpha = expf(mx - top);  // key 0 is visible to everyone: top is finite
-    mx = top;
+    if (__any(top > mx)) {  // (key 0 is visible to everyone: after the first tile top is finite)
+      const float alpha = exp2f(mx - top);
+      sum *= alpha;
+#pragma unroll
+      for (int i = 0; i < DV / 32; ++i)
+#pragma unroll
+        for (int e = 0; e < 16; ++e) o[i][e] *= alpha;
+      mx = top;
+    }
     float part = 0.f;
 #pragma unroll
     for (int b = 0; b < 2; ++b)
 #pragma unroll
       for (int e = 0; e < 16; ++e) {
-        s[b][e] = expf(s[b][e] - top);
+        s[b][e] = __builtin_amdgcn_exp2f(s[b][e] - mx);
         part += s[b][e];
       }
-    sum = sum * alpha + part + __shfl_xor(part, 32, 64);
-#pragma unroll
-    for (int i = 0; i < DV / 32; ++i)
-#pragma unroll
-      for (int e = 0; e < 16; ++e) o[i][e] *= alpha;
+    sum += part + __shfl_xor(part, 32, 64);
 #pragma unroll
     for (int b = 0; b < 2; ++b) {
       if constexpr (sizeof(T) == 2) {
@@ -233,14 +268,17 @@ __global__ void __launch_bounds__(256) latent_rows_kernel(RowsArgs a) {
             hi[e] = (__bf16)s[b][8 * u + e];
             lo[e] = (__bf16)(s[b][8 * u + e] - (float)hi[e]);
           }
+          bf16x8 vf[DV / 32];
 #pragma unroll
           for (int i = 0; i < DV / 32; ++i) {
-            const char* vr = Vs + (i * 32 + col) * V_ROW + (b * 32 + 16 * u + 4 * hf) * 2;
-            const uint2 v0 = *reinterpret_cast<const uint2*>(vr), v1 = *reinterpret_cast<const uint2*>(vr + 16);
-            const bf16x8 vf = __builtin_bit_cast(bf16x8, u32x4_t{v0.x, v0.y, v1.x, v1.y});
-            o[i] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(vf, hi, o[i], 0, 0, 0);
-            o[i] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(vf, lo, o[i], 0, 0, 0);
+            const char* p = Vs + (i * 32 + col) * V_ROW + (b * 32 + 16 * u + 4 * hf) * 2;
+            const uint2 v0 = *reinterpret_cast<const uint2*>(p), v1 = *reinterpret_cast<const uint2*>(p + 16);
+            vf[i] = __builtin_bit_cast(bf16x8, u32x4_t{v0.x, v0.y, v1.x, v1.y});
           }
+#pragma unroll
+          for (int i = 0; i < DV / 32; ++i) o[i] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(vf[i], hi, o[i], 0, 0, 0);
+#pragma unroll
+          for (int i = 0; i < DV / 32; ++i) o[i] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(vf[i], lo, o[i], 0, 0, 0);
         }
       } else {
 #pragma unroll
@@ -272,21 +310,32 @@ __global__ void __launch_bounds__(256) latent_rows_kernel(RowsArgs a) {
 }
 
 template <typename T, int DQ, int DV>
-hipError_t launch_rows(hipStream_t st, const RowsArgs& a) {
+int launch_rows(ughip_device* dev, RowsArgs a, PackArgs pk) {
   constexpr int bytes = rows_lds_bytes<T, DQ, DV>();
   static_assert(bytes <= 160 * 1024, "tile does not fit LDS");
   static const hipError_t attr = hipFuncSetAttribute(reinterpret_cast<const void*>(latent_rows_kernel<T, DQ, DV>), hipFuncAttributeMaxDynamicSharedMemorySize, bytes);
-  if (attr != hipSuccess) return attr;
-  latent_rows_kernel<T, DQ, DV><<<dim3((unsigned)a.heads, (unsigned)((a.t + QT - 1) / QT)), 256, bytes, st>>>(a);
-  return hipGetLastError();
+  UGHIP_HIPCHK(attr);
+  pk.q_rows = (pk.t + QT - 1) / QT * QT, pk.k_rows = (pk.pos + pk.t + KT - 1) / KT * KT;
+  const size_t q_bytes = (size_t)pk.heads * pk.q_rows * DQ * sizeof(T), k_bytes = (size_t)pk.heads * pk.k_rows * DQ * sizeof(T);
+  void* ws = nullptr;
+  if (int rc = rows_scratch(dev, q_bytes + k_bytes, &ws)) return rc;
+  pk.qp = ws, pk.kp = static_cast<char*>(ws) + q_bytes;
+  a.q = pk.qp, a.k = pk.kp, a.q_rows = pk.q_rows, a.k_rows = pk.k_rows;
+  constexpr int CH = DQ * (int)sizeof(T) / 16;
+  const size_t pieces = (size_t)(pk.q_rows + pk.k_rows) * CH;
+  latent_pack_kernel<T, DQ><<<dim3((unsigned)((pieces + 255) / 256), (unsigned)pk.heads), 256, 0, dev->stream>>>(pk);
+  UGHIP_HIPCHK(hipGetLastError());
+  latent_rows_kernel<T, DQ, DV><<<dim3((unsigned)pk.heads, (unsigned)(pk.q_rows / QT)), 256, bytes, dev->stream>>>(a);
+  UGHIP_HIPCHK(hipGetLastError());
+  return UGHIP_OK;
 }
 template <typename T>
-hipError_t launch_rows_any(hipStream_t st, const RowsArgs& a) {
-  const int dq = a.dim + a.rot;
-  if (dq <= 64 && a.vdim <= 64) return launch_rows<T, 64, 64>(st, a);
-  if (dq <= 128 && a.vdim <= 128) return launch_rows<T, 128, 128>(st, a);
-  if (dq <= 192 && a.vdim <= 128) return launch_rows<T, 192, 128>(st, a);
-  return launch_rows<T, 256, 256>(st, a);
+int launch_rows_any(ughip_device* dev, const RowsArgs& a, const PackArgs& pk) {
+  const int dq = pk.dim + pk.rot;
+  if (dq <= 64 && a.vdim <= 64) return launch_rows<T, 64, 64>(dev, a, pk);
+  if (dq <= 128 && a.vdim <= 128) return launch_rows<T, 128, 128>(dev, a, pk);
+  if (dq <= 192 && a.vdim <= 128) return launch_rows<T, 192, 128>(dev, a, pk);
+  return launch_rows<T, 256, 256>(dev, a, pk);
 }
 
 // ---- few positions ----------------------------------------------------------------------------------------------------------
@@ -369,6 +418,31 @@ constexpr int SK = 32, S_ROW = SK + 4;
 __host__ __device__ inline int split_row(int L) { return ((L + 15) & ~15) + 4; }
 inline size_t split_lds_bytes(int L) { return ((size_t)(SK + 16) * split_row(L) + 3 * 16 * S_ROW + 48) * sizeof(float); }
 
+// n rows of L floats (rows from `left` on and columns from L on are zeros) to LDS, eight 16-byte loads per thread on their way at once.
+__device__ __forceinline__ void load_rows(float* lds, int ld, int Lp, int n, const float* src, int L, int left) {
+  if (L % 4 == 0) {
+    const int l4 = Lp / 4, total = n * l4;
+    for (int base = 0; base < total; base += 8 * 256) {
+      f32x4_t v[8];
+#pragma unroll
+      for (int u = 0; u < 8; ++u) {
+        const int x = base + threadIdx.x + u * 256, r = x / l4, c = (x - r * l4) * 4;
+        v[u] = x < total && r < left && c < L ? *reinterpret_cast<const f32x4_t*>(src + (size_t)r * L + c) : f32x4_t{0.f, 0.f, 0.f, 0.f};
+      }
+#pragma unroll
+      for (int u = 0; u < 8; ++u) {
+        const int x = base + threadIdx.x + u * 256, r = x / l4, c = (x - r * l4) * 4;
+        if (x < total) *reinterpret_cast<f32x4_t*>(lds + r * ld + c) = v[u];
+      }
+    }
+  } else {
+    for (int x = threadIdx.x; x < n * Lp; x += 256) {
+      const int r = x / Lp, c = x % Lp;
+      lds[r * ld + c] = r < left && c < L ? src[(size_t)r * L + c] : 0.f;
+    }
+  }
+}
+
 template <int NT>  // 16-column tiles of the result per wave
 __global__ void __launch_bounds__(256) latent_split_kernel(SplitArgs a) {
   extern __shared__ __attribute__((aligned(16))) float sl[];
@@ -382,10 +456,7 @@ __global__ void __launch_bounds__(256) latent_split_kernel(SplitArgs a) {
   float* arow = lrow + 16;
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, j = lane & 15, g = lane >> 4;
   const int r0 = blockIdx.x * 16, split = blockIdx.y;
-  for (int x = threadIdx.x; x < 16 * Lp; x += 256) {
-    const int r = x / Lp, c = x % Lp;
-    Qs[r * ld + c] = r0 + r < a.rows && c < a.L ? a.qa[(size_t)(r0 + r) * a.L + c] : 0.f;
-  }
+  load_rows(Qs, ld, Lp, 16, a.qa + (size_t)r0 * a.L, a.L, a.rows - r0);
   if (threadIdx.x < 16) mrow[threadIdx.x] = -INFINITY, lrow[threadIdx.x] = 0.f;
   f32x4_t acc[NT];
 #pragma unroll
@@ -393,19 +464,7 @@ __global__ void __launch_bounds__(256) latent_split_kernel(SplitArgs a) {
   const int k_begin = split * a.tiles_per_split * SK, k_stop = min(a.keys, k_begin + a.tiles_per_split * SK);
   for (int k0 = k_begin; k0 < k_stop; k0 += SK) {
     __syncthreads();
-    if (a.L % 4 == 0) {
-      const int l4 = Lp / 4;
-      for (int x = threadIdx.x; x < SK * l4; x += 256) {
-        const int r = x / l4, c = (x % l4) * 4;
-        *reinterpret_cast<f32x4_t*>(Ks + r * ld + c) =
-            k0 + r < k_stop && c < a.L ? *reinterpret_cast<const f32x4_t*>(a.cache + (size_t)(k0 + r) * a.L + c) : f32x4_t{0.f, 0.f, 0.f, 0.f};
-      }
-    } else {
-      for (int x = threadIdx.x; x < SK * Lp; x += 256) {
-        const int r = x / Lp, c = x % Lp;
-        Ks[r * ld + c] = k0 + r < k_stop && c < a.L ? a.cache[(size_t)(k0 + r) * a.L + c] : 0.f;
-      }
-    }
+    load_rows(Ks, ld, Lp, SK, a.cache + (size_t)k0 * a.L, a.L, k_stop - k0);
     __syncthreads();
     {  // wave: 16 keys (wave % 2), every other run of 16 elements (wave / 2)
       f32x4_t s = {0.f, 0.f, 0.f, 0.f};
@@ -572,10 +631,13 @@ extern "C" int ughip_latent_attention_rows(ughip_device* dev, ughip_view q, cons
   if (t == 0) return UGHIP_OK;
   if ((t + QT - 1) / QT > 65535) return set_error(UGHIP_ERR_UNSUPPORTED, "%s: too many positions", what);
   if (int rc = device_activate(dev)) return rc;
-  RowsArgs a{view_ptr<float>(q), k->ptr, v_t->ptr, buf_ptr<float>(cache), buf_ptr<float>(cos), buf_ptr<float>(sin), static_cast<char*>(dst.s->ptr) + dst.offset * (bf16 ? 2 : 4), q.stride, v_stride, dst.stride,
-             (int)t, (int)pos, (int)heads, (int)dim, (int)rot, (int)vdim, (int)rank, scale, dim % 8 == 0, bf16};
-  UGHIP_HIPCHK(k->dtype == UGHIP_BF16 ? launch_rows_any<uint16_t>(dev->stream, a) : launch_rows_any<float>(dev->stream, a));
-  return UGHIP_OK;
+  RowsArgs a{};
+  a.v = v_t->ptr, a.dst = static_cast<char*>(dst.s->ptr) + dst.offset * (bf16 ? 2 : 4), a.v_stride = v_stride, a.dst_stride = dst.stride;
+  a.t = (int)t, a.pos = (int)pos, a.vdim = (int)vdim, a.scale2 = scale * 1.4426950408889634f, a.dst_bf16 = bf16;
+  PackArgs pk{};
+  pk.q = view_ptr<float>(q), pk.k = k->ptr, pk.cache = buf_ptr<float>(cache), pk.cos = buf_ptr<float>(cos), pk.sin = buf_ptr<float>(sin), pk.q_stride = q.stride;
+  pk.t = (int)t, pk.pos = (int)pos, pk.heads = (int)heads, pk.dim = (int)dim, pk.rot = (int)rot, pk.rank = (int)rank;
+  return k->dtype == UGHIP_BF16 ? launch_rows_any<uint16_t>(dev, a, pk) : launch_rows_any<float>(dev, a, pk);
 }
 
 extern "C" int ughip_latent_attention_absorbed(ughip_device* dev, ughip_view q, ughip_view kv, const ughip_slice* kv_norm, float eps, const ughip_slice* w_uk,

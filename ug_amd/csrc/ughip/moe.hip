@@ -9,12 +9,27 @@ using namespace ughip;
 
 namespace {
 
-// 16 rows per workgroup.  The four waves share k: each multiplies every fourth run of 16 elements (v_mfma_f32_16x16x4_f32, k
-// taken four elements per lane so that rows are read 16 bytes at a time), their partial logits meet in LDS in wave order;
-// then each wave chooses for four of the rows.
+// 16 rows per workgroup.  The eight waves share k: each multiplies every eighth run of 16 elements (v_mfma_f32_16x16x4_f32, k
+// taken four elements per lane so that rows are read 16 bytes at a time), AHEAD runs asked for before the first is used; their
+// partial logits meet in LDS in wave order; then each wave chooses for two of the rows.
+constexpr int ROUTE_WAVES = 8, AHEAD = 4;
+
 template <bool VEC>
-__global__ void __launch_bounds__(256) route_rows_kernel(const float* __restrict__ x, size_t x_stride, const float* __restrict__ router, RouteArgs r, int m, int k,
-                                                         int* __restrict__ ids, float* __restrict__ weights) {
+__device__ __forceinline__ f32x4_t run4(const float* row, bool ok, int kk, int k) {
+  f32x4_t v = {0.f, 0.f, 0.f, 0.f};
+  if (VEC) {
+    if (ok && kk < k) v = *reinterpret_cast<const f32x4_t*>(row + kk);
+  } else {
+#pragma unroll
+    for (int c = 0; c < 4; ++c)
+      if (ok && kk + c < k) v[c] = row[kk + c];
+  }
+  return v;
+}
+
+template <bool VEC, int NT>  // NT tiles of 16 experts at a time
+__global__ void __launch_bounds__(64 * ROUTE_WAVES) route_rows_kernel(const float* __restrict__ x, size_t x_stride, const float* __restrict__ router, RouteArgs r, int m, int k,
+                                                                      int* __restrict__ ids, float* __restrict__ weights) {
   extern __shared__ float smem[];
   const int E = r.experts, per_wave = route_lds_floats(E, r.groups);
   float* logits = smem;  // [16][E]
@@ -23,40 +38,37 @@ __global__ void __launch_bounds__(256) route_rows_kernel(const float* __restrict
   const int row0 = blockIdx.x * 16;
   const bool row_ok = row0 + j < m;
   const float* xr = x + (size_t)(row_ok ? row0 + j : row0) * x_stride;
-  for (int e0 = 0; e0 < E; e0 += 64) {
-    f32x4_t acc[4];
+  for (int e0 = 0; e0 < E; e0 += 16 * NT) {
+    f32x4_t acc[NT];
+    const float* wr[NT];
+    bool ok[NT];
 #pragma unroll
-    for (int i = 0; i < 4; ++i) acc[i] = f32x4_t{0.f, 0.f, 0.f, 0.f};
-    for (int k0 = wave * 16; k0 < k; k0 += 64) {
-      const int kk = k0 + 4 * g;
-      float xv[4], wv[4];
-      if (VEC) {
-        const f32x4_t v = row_ok && kk < k ? *reinterpret_cast<const f32x4_t*>(xr + kk) : f32x4_t{0.f, 0.f, 0.f, 0.f};
-        xv[0] = v.x, xv[1] = v.y, xv[2] = v.z, xv[3] = v.w;
-      } else {
-#pragma unroll
-        for (int c = 0; c < 4; ++c) xv[c] = row_ok && kk + c < k ? xr[kk + c] : 0.f;
-      }
-#pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        if (e0 + 16 * i >= E) continue;  // uniform over the wave
-        const int e = e0 + 16 * i + j;
-        const float* wr = router + (size_t)(e < E ? e : 0) * k;
-        if (VEC) {
-          const f32x4_t v = e < E && kk < k ? *reinterpret_cast<const f32x4_t*>(wr + kk) : f32x4_t{0.f, 0.f, 0.f, 0.f};
-          wv[0] = v.x, wv[1] = v.y, wv[2] = v.z, wv[3] = v.w;
-        } else {
-#pragma unroll
-          for (int c = 0; c < 4; ++c) wv[c] = e < E && kk + c < k ? wr[kk + c] : 0.f;
-        }
-#pragma unroll
-        for (int c = 0; c < 4; ++c) acc[i] = __builtin_amdgcn_mfma_f32_16x16x4f32(xv[c], wv[c], acc[i], 0, 0, 0);
-      }
+    for (int i = 0; i < NT; ++i) {
+      acc[i] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+      const int e = e0 + 16 * i + j;
+      ok[i] = e < E;
+      wr[i] = router + (size_t)(ok[i] ? e : 0) * k;
     }
-    for (int wv = 0; wv < 4; ++wv) {
+    for (int k0 = wave * 16; k0 < k; k0 += 16 * ROUTE_WAVES * AHEAD) {
+      f32x4_t xv[AHEAD], wv[AHEAD][NT];
+#pragma unroll
+      for (int u = 0; u < AHEAD; ++u) {
+        const int kk = k0 + 16 * ROUTE_WAVES * u + 4 * g;
+        xv[u] = run4<VEC>(xr, row_ok, kk, k);
+#pragma unroll
+        for (int i = 0; i < NT; ++i) wv[u][i] = run4<VEC>(wr[i], ok[i], kk, k);
+      }
+#pragma unroll
+      for (int u = 0; u < AHEAD; ++u)
+#pragma unroll
+        for (int i = 0; i < NT; ++i)
+#pragma unroll
+          for (int c = 0; c < 4; ++c) acc[i] = __builtin_amdgcn_mfma_f32_16x16x4f32(xv[u][c], wv[u][i][c], acc[i], 0, 0, 0);
+    }
+    for (int wv = 0; wv < ROUTE_WAVES; ++wv) {
       if (wave == wv) {
 #pragma unroll
-        for (int i = 0; i < 4; ++i) {
+        for (int i = 0; i < NT; ++i) {
           const int e = e0 + 16 * i + j;
           if (e >= E) continue;
 #pragma unroll
@@ -69,38 +81,46 @@ __global__ void __launch_bounds__(256) route_rows_kernel(const float* __restrict
       __syncthreads();
     }
   }
-  for (int t = 0; t < 4; ++t) {
-    const int rr = wave * 4 + t;
+  for (int t = 0; t < 16 / ROUTE_WAVES; ++t) {
+    const int rr = wave * (16 / ROUTE_WAVES) + t;
     if (row0 + rr >= m) break;  // uniform over the wave
     const size_t at = (size_t)(row0 + rr) * r.top;
     route_choose(logits + rr * E, r, work + wave * per_wave, ids + at, weights + at);
   }
 }
 
-// A workgroup (one wave) per expert: it counts the pairs of lower experts and its own, then writes its own in row order.
-__global__ void __launch_bounds__(64) group_rows_kernel(const int* __restrict__ ids, int pairs, int top, int* __restrict__ row_index, int* __restrict__ slots,
-                                                        int* __restrict__ group_end) {
-  const int e = blockIdx.x, lane = threadIdx.x;
+// A workgroup per expert: every thread takes a run of the pairs and counts the lower experts' and its expert's own, a scan over the
+// threads says where its own go (in row order).
+__global__ void __launch_bounds__(256) group_rows_kernel(const int* __restrict__ ids, int pairs, int top, int* __restrict__ row_index, int* __restrict__ slots,
+                                                         int* __restrict__ group_end) {
+  __shared__ int s_own[256], s_low[4];
+  const int e = blockIdx.x, tid = threadIdx.x, lane = tid & 63, per = (pairs + 255) / 256, p0 = min(pairs, tid * per), p1 = min(pairs, p0 + per);
   int lower = 0, own = 0;
-  for (int p = lane; p < pairs; p += 64) {
+#pragma unroll 8
+  for (int p = p0; p < p1; ++p) {
     const int id = ids[p];
     lower += id < e;
     own += id == e;
   }
-  for (int d = 32; d; d >>= 1) lower += __shfl_xor(lower, d, 64), own += __shfl_xor(own, d, 64);
-  if (lane == 0) group_end[e] = lower + own;
-  int at = lower;
-  for (int p0 = 0; p0 < pairs; p0 += 64) {
-    const int p = p0 + lane;
-    const bool mine = p < pairs && ids[p] == e;
-    const unsigned long long mask = __ballot(mine);
-    if (mine) {
-      const int r = at + __popcll(mask & ((1ull << lane) - 1));
-      row_index[r] = p / top;
-      slots[p] = r;
-    }
-    at += __popcll(mask);
+  for (int d = 32; d; d >>= 1) lower += __shfl_xor(lower, d, 64);
+  if (lane == 0) s_low[tid >> 6] = lower;
+  s_own[tid] = own;
+  __syncthreads();
+  lower = s_low[0] + s_low[1] + s_low[2] + s_low[3];
+  for (int d = 1; d < 256; d <<= 1) {  // inclusive scan
+    const int o = tid >= d ? s_own[tid - d] : 0;
+    __syncthreads();
+    s_own[tid] += o;
+    __syncthreads();
   }
+  if (tid == 255) group_end[e] = lower + s_own[255];
+  int at = lower + s_own[tid] - own;
+  if (own == 0) return;
+  for (int p = p0; p < p1; ++p)
+    if (ids[p] == e) {
+      row_index[at] = p / top;
+      slots[p] = at++;
+    }
 }
 
 }  // namespace
@@ -119,13 +139,19 @@ extern "C" int ughip_route_rows(ughip_device* dev, ughip_view x, const ughip_sli
   if (m == 0) return UGHIP_OK;
   if (int rc = device_activate(dev)) return rc;
   const RouteArgs r{buf_ptr<float>(correction), (int)experts, (int)groups, (int)keep, (int)top};
-  const size_t lds = (16 * experts + 4 * (size_t)route_lds_floats((int)experts, (int)groups)) * sizeof(float);
+  const size_t lds = (16 * experts + ROUTE_WAVES * (size_t)route_lds_floats((int)experts, (int)groups)) * sizeof(float);
   const float* xp = view_ptr<float>(x);
   const float* rp = buf_ptr<float>(router);
   const unsigned grid = (unsigned)((m + 15) / 16);
   const bool vec = k % 4 == 0 && x.stride % 4 == 0 && (reinterpret_cast<uintptr_t>(xp) & 15) == 0;
-  if (vec) route_rows_kernel<true><<<grid, 256, lds, dev->stream>>>(xp, x.stride, rp, r, (int)m, (int)k, static_cast<int*>(ids->ptr), static_cast<float*>(weights->ptr));
-  else route_rows_kernel<false><<<grid, 256, lds, dev->stream>>>(xp, x.stride, rp, r, (int)m, (int)k, static_cast<int*>(ids->ptr), static_cast<float*>(weights->ptr));
+  auto go = [&](auto kernel) {
+    if (lds > 64 * 1024)
+      if (hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(kernel), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds); e != hipSuccess) return e;
+    kernel<<<grid, 64 * ROUTE_WAVES, lds, dev->stream>>>(xp, x.stride, rp, r, (int)m, (int)k, static_cast<int*>(ids->ptr), static_cast<float*>(weights->ptr));
+    return hipSuccess;
+  };
+  if (experts <= 16) UGHIP_HIPCHK(vec ? go(route_rows_kernel<true, 1>) : go(route_rows_kernel<false, 1>));
+  else UGHIP_HIPCHK(vec ? go(route_rows_kernel<true, 4>) : go(route_rows_kernel<false, 4>));
   UGHIP_HIPCHK(hipGetLastError());
   return UGHIP_OK;
 }
@@ -139,7 +165,7 @@ extern "C" int ughip_group_rows(ughip_device* dev, const ughip_slice* ids, size_
   if (int rc = check_buf(dev, slots, m * top, UGHIP_I32, "group_rows slots")) return rc;
   if (int rc = check_buf(dev, group_end, experts, UGHIP_I32, "group_rows group_end")) return rc;
   if (int rc = device_activate(dev)) return rc;
-  group_rows_kernel<<<(unsigned)experts, 64, 0, dev->stream>>>(buf_ptr<int>(ids), (int)(m * top), (int)top, static_cast<int*>(row_index->ptr), static_cast<int*>(slots->ptr),
+  group_rows_kernel<<<(unsigned)experts, 256, 0, dev->stream>>>(buf_ptr<int>(ids), (int)(m * top), (int)top, static_cast<int*>(row_index->ptr), static_cast<int*>(slots->ptr),
                                                                static_cast<int*>(group_end->ptr));
   UGHIP_HIPCHK(hipGetLastError());
   return UGHIP_OK;

@@ -41,7 +41,39 @@ __device__ __forceinline__ void route_fence() {
   __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "workgroup");
   __builtin_amdgcn_wave_barrier();
 }
+// Up to 64 experts: one per lane.  An expert's place among the chosen is the number of experts in front of it, which every lane
+// counts for its own.
+__device__ __forceinline__ void route_choose64(const float* logits, const RouteArgs& r, int* ids, float* weights) {
+  const int lane = threadIdx.x & 63, size = r.experts / r.groups, E = r.experts;
+  const float s = lane < E ? 1.f / (1.f + expf(-logits[lane])) : 0.f;
+  float v = lane < E ? s + (r.correction ? r.correction[lane] : 0.f) : -INFINITY;
+  const int g = lane / size;
+  float a = -INFINITY, b = -INFINITY;
+  for (int i = 0; i < size; ++i) {
+    const float c = __shfl(v, min(g * size + i, 63), 64);
+    b = fmaxf(b, fminf(a, c));
+    a = fmaxf(a, c);
+  }
+  const float score = size > 1 ? a + b : a;
+  int front = 0;
+  for (int h = 0; h < r.groups; ++h) {
+    const float o = __uint_as_float(__builtin_amdgcn_readlane(__float_as_uint(score), h * size));
+    front += o > score || (o == score && h < g);
+  }
+  if (front >= r.keep) v = -INFINITY;
+  front = 0;
+  for (int e = 0; e < E; ++e) {
+    const float o = __uint_as_float(__builtin_amdgcn_readlane(__float_as_uint(v), e));
+    front += o > v || (o == v && e < lane);
+  }
+  for (int i = lane; i < r.top; i += 64) ids[i] = i, weights[i] = 0.f;  // (scores that are not numbers leave places empty)
+  route_fence();
+  if (lane < E && front < r.top) ids[front] = lane, weights[front] = s;
+  route_fence();
+}
+
 __device__ __forceinline__ void route_choose(const float* logits, const RouteArgs& r, float* work, int* ids, float* weights) {
+  if (r.experts <= 64) return route_choose64(logits, r, ids, weights);
   const int lane = threadIdx.x & 63, size = r.experts / r.groups;
   float* choice = work;
   float* score = work + r.experts;

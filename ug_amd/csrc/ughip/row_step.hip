@@ -1,9 +1,10 @@
 // Products of one row with their neighbours folded in (ughip_product_row): a decode step of the layers in ughip_layers.h.
 //
-// A workgroup of four waves takes 4 R columns, R per wave.  A wave asks for the first PRE runs of 512 elements of its matrix rows
-// (eight elements per lane and run), then the workgroup makes the input row in LDS -- residual add with the norm of the sublayer
-// in front, gate, norm -- in the shadow of those loads, and every wave multiplies.  The input row costs a few cache reads per
-// workgroup and spares the launches that would make it; the first workgroup stores the new residual.
+// A workgroup of four waves takes 4 R columns, R per wave.  It asks for everything the input row is made of (PV 16-byte pieces per
+// thread and vector), then every wave for the first PRE runs of 512 elements of its matrix rows (eight elements per lane and run);
+// the row -- residual add with the norm of the sublayer in front, gate, norm -- is made in LDS in the shadow of the matrix, and
+// every wave multiplies.  The input row costs a few cache reads per workgroup and spares the launches that would make it; the
+// first workgroup stores the new residual.  PV = 0: rows of any length and alignment, element by element.
 #include <hip/hip_runtime.h>
 
 #include "layers.h"
@@ -35,7 +36,7 @@ struct RowArgs {
   float* route_weights;
 };
 
-constexpr int RUN = 512, PRE = 4;
+constexpr int RUN = 512;
 
 template <typename WT>
 struct Eight;
@@ -90,7 +91,7 @@ struct Eight<float> {
 };
 
 // R columns of NM matrices per wave; VEC: rows are 16-byte aligned and a multiple of 8 long.  ROUTE as in ughip_row_step.
-template <typename WT, int R, int NM, int ROUTE, bool VEC>
+template <typename WT, int R, int NM, int ROUTE, bool VEC, int PRE, int PV>
 __global__ void __launch_bounds__(256) row_step_kernel(RowArgs a) {
   extern __shared__ __attribute__((aligned(16))) float in[];  // the row, then ROUTE 1: logits and the choice's work space
   __shared__ float red[4][4];
@@ -99,6 +100,20 @@ __global__ void __launch_bounds__(256) row_step_kernel(RowArgs a) {
   const int total = ROUTE == 2 ? a.segs * a.k : a.k;  // elements of the input row
   const int padded = (total + RUN - 1) / RUN * RUN;
   const int col0 = (blockIdx.x * 4 + wave) * R;
+  constexpr int NP = PV ? PV : 1;
+  const f32x4_t zero = {0.f, 0.f, 0.f, 0.f};
+  f32x4_t px[NP], py[NP], pyn[NP], pn[NP];  // x, y or the gate, and the two norms' weights
+  if constexpr (PV != 0) {
+#pragma unroll
+    for (int u = 0; u < PV; ++u) {
+      const int i = (u * 256 + (int)threadIdx.x) * 4;
+      const bool ok = i < total;  // a multiple of 4
+      px[u] = ok ? *reinterpret_cast<const f32x4_t*>(a.x + i) : zero;
+      py[u] = ok && (a.y || a.gate) ? *reinterpret_cast<const f32x4_t*>((a.y ? a.y : a.gate) + i) : zero;
+      pyn[u] = ok && a.y ? *reinterpret_cast<const f32x4_t*>(a.y_norm + i) : zero;
+      pn[u] = ok && a.norm ? *reinterpret_cast<const f32x4_t*>(a.norm + i) : zero;
+    }
+  }
   if constexpr (ROUTE == 1) {  // which experts' matrices: before anything of them can be asked for
     float* lg = in + padded;
     for (int e = threadIdx.x; e < a.route.experts; e += 256) lg[e] = a.logits[e];
@@ -168,42 +183,83 @@ __global__ void __launch_bounds__(256) row_step_kernel(RowArgs a) {
 
   // the input row
   float ss = 0.f;
-  for (int i = threadIdx.x; i < padded; i += 256) {
-    float v = 0.f;
-    if (i < total) {
-      v = a.y ? a.y[i] : a.x[i];
-      if (a.gate) v *= silu_f(a.gate[i]);
-      if (ROUTE == 2) v *= a.route_weights[i / a.k];
+  if constexpr (PV != 0) {
+    auto square = [](const f32x4_t& v) { return v.x * v.x + v.y * v.y + v.z * v.z + v.w * v.w; };
+    if (a.y) {
+#pragma unroll
+      for (int u = 0; u < PV; ++u) ss += square(py[u]);
+      ss = block_sum<4>(ss, red[0]);
+      const float inv = 1.f / sqrtf(ss / (float)a.k + a.eps);
+#pragma unroll
+      for (int u = 0; u < PV; ++u) {
+        px[u] = px[u] + py[u] * inv * pyn[u];
+        const int i = (u * 256 + (int)threadIdx.x) * 4;
+        if (a.x_out && blockIdx.x == 0 && i < total) *reinterpret_cast<f32x4_t*>(a.x_out + i) = px[u];
+      }
+    } else if (a.gate) {
+#pragma unroll
+      for (int u = 0; u < PV; ++u)
+#pragma unroll
+        for (int e = 0; e < 4; ++e) px[u][e] *= silu_f(py[u][e]);
     }
-    in[i] = v;  // read back by the same thread until the last barrier
-    ss += v * v;
-  }
-  if (a.y) {
-    ss = block_sum<4>(ss, red[0]);
-    const float inv = 1.f / sqrtf(ss / (float)a.k + a.eps);
-    ss = 0.f;
-    for (int i = threadIdx.x; i < total; i += 256) {
-      const float v = a.x[i] + in[i] * inv * a.y_norm[i];
-      in[i] = v;
+    if (ROUTE == 2) {
+#pragma unroll
+      for (int u = 0; u < PV; ++u) {
+        const int i = (u * 256 + (int)threadIdx.x) * 4;
+        if (i < total) px[u] *= a.route_weights[i / a.k];  // a.k is a multiple of 4
+      }
+    }
+    if (a.norm && a.norm_groups == 1) {
+      ss = 0.f;
+#pragma unroll
+      for (int u = 0; u < PV; ++u) ss += square(px[u]);
+      ss = block_sum<4>(ss, red[1]);
+      const float inv = 1.f / sqrtf(ss / (float)a.k + a.eps);
+#pragma unroll
+      for (int u = 0; u < PV; ++u) px[u] = px[u] * inv * pn[u];
+    }
+#pragma unroll
+    for (int u = 0; u < PV; ++u) {
+      const int i = (u * 256 + (int)threadIdx.x) * 4;
+      if (i < padded) *reinterpret_cast<f32x4_t*>(in + i) = px[u];
+    }
+  } else {
+    for (int i = threadIdx.x; i < padded; i += 256) {
+      float v = 0.f;
+      if (i < total) {
+        v = a.y ? a.y[i] : a.x[i];
+        if (a.gate) v *= silu_f(a.gate[i]);
+        if (ROUTE == 2) v *= a.route_weights[i / a.k];
+      }
+      in[i] = v;  // read back by the same thread until the last barrier
       ss += v * v;
-      if (a.x_out && blockIdx.x == 0) a.x_out[i] = v;
     }
-  }
-  if (a.norm) {
-    if (a.norm_groups == 1) {
+    if (a.y) {
+      ss = block_sum<4>(ss, red[0]);
+      const float inv = 1.f / sqrtf(ss / (float)a.k + a.eps);
+      ss = 0.f;
+      for (int i = threadIdx.x; i < total; i += 256) {
+        const float v = a.x[i] + in[i] * inv * a.y_norm[i];
+        in[i] = v;
+        ss += v * v;
+        if (a.x_out && blockIdx.x == 0) a.x_out[i] = v;
+      }
+    }
+    if (a.norm && a.norm_groups == 1) {
       ss = block_sum<4>(ss, red[1]);
       const float inv = 1.f / sqrtf(ss / (float)a.k + a.eps);
       for (int i = threadIdx.x; i < total; i += 256) in[i] *= inv * a.norm[i];
-    } else {
-      const int part = a.k / a.norm_groups;
-      __syncthreads();  // a part is summed by one wave
-      for (int g = wave; g < a.norm_groups; g += 4) {
-        float s = 0.f;
-        for (int i = lane; i < part; i += 64) s += in[g * part + i] * in[g * part + i];
-        for (int d = 32; d; d >>= 1) s += __shfl_xor(s, d, 64);
-        const float inv = 1.f / sqrtf(s / (float)part + a.eps);
-        for (int i = lane; i < part; i += 64) in[g * part + i] *= inv * a.norm[g * part + i];
-      }
+    }
+  }
+  if (a.norm && a.norm_groups > 1) {
+    const int part = a.k / a.norm_groups;
+    __syncthreads();  // a part is summed by one wave
+    for (int g = wave; g < a.norm_groups; g += 4) {
+      float s = 0.f;
+      for (int i = lane; i < part; i += 64) s += in[g * part + i] * in[g * part + i];
+      for (int d = 32; d; d >>= 1) s += __shfl_xor(s, d, 64);
+      const float inv = 1.f / sqrtf(s / (float)part + a.eps);
+      for (int i = lane; i < part; i += 64) in[g * part + i] *= inv * a.norm[g * part + i];
     }
   }
   __syncthreads();
@@ -266,33 +322,42 @@ __global__ void __launch_bounds__(256) row_step_kernel(RowArgs a) {
   }
 }
 
-template <typename WT, int R, int NM, int ROUTE>
-hipError_t launch_vec(hipStream_t st, const RowArgs& a, size_t lds, bool vec) {
+template <typename WT, int R, int NM, int ROUTE, bool VEC, int PRE, int PV>
+hipError_t launch_one(hipStream_t st, const RowArgs& a, size_t lds) {
   const unsigned grid = (unsigned)((a.cols + 4 * R - 1) / (4 * R));
-  auto go = [&](auto kernel) {
-    if (lds > 64 * 1024) {
-      if (hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(kernel), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds); e != hipSuccess) return e;
-    }
-    kernel<<<grid, 256, lds, st>>>(a);
-    return hipGetLastError();
-  };
-  return vec ? go(row_step_kernel<WT, R, NM, ROUTE, true>) : go(row_step_kernel<WT, R, NM, ROUTE, false>);
+  auto kernel = row_step_kernel<WT, R, NM, ROUTE, VEC, PRE, PV>;
+  if (lds > 64 * 1024)
+    if (hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(kernel), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds); e != hipSuccess) return e;
+  kernel<<<grid, 256, lds, st>>>(a);
+  return hipGetLastError();
+}
+
+// pieces: the input row is read 16 bytes at a time
+template <typename WT, int R, int NM, int ROUTE>
+hipError_t launch_vec(hipStream_t st, const RowArgs& a, size_t lds, bool vec, bool pieces) {
+  const int total = (ROUTE == 2 ? a.segs : 1) * a.k;
+  if (!vec) return launch_one<WT, R, NM, ROUTE, false, 4, 0>(st, a, lds);
+  if (!pieces || total > 8192) return launch_one<WT, R, NM, ROUTE, true, 4, 0>(st, a, lds);
+  constexpr bool ROOM = R * NM * sizeof(WT) <= 4;  // registers for twelve runs of every row
+  if (total <= 2048) return launch_one<WT, R, NM, ROUTE, true, 4, 2>(st, a, lds);
+  if (total <= 4096) return launch_one<WT, R, NM, ROUTE, true, ROOM ? 8 : 4, 4>(st, a, lds);
+  return launch_one<WT, R, NM, ROUTE, true, ROOM ? 12 : 4, 8>(st, a, lds);
 }
 
 template <typename WT, int NM, int ROUTE>
-hipError_t launch_rows(hipStream_t st, const RowArgs& a, size_t lds, bool vec) {
+hipError_t launch_rows(hipStream_t st, const RowArgs& a, size_t lds, bool vec, bool pieces) {
   // enough workgroups for the chip first, then more columns for each of them to share the input row
   const int r = a.cols >= 8192 && NM == 1 ? 4 : a.cols >= 2048 ? 2 : 1;
   if constexpr (NM == 1)
-    if (r == 4) return launch_vec<WT, 4, NM, ROUTE>(st, a, lds, vec);
-  return r >= 2 ? launch_vec<WT, 2, NM, ROUTE>(st, a, lds, vec) : launch_vec<WT, 1, NM, ROUTE>(st, a, lds, vec);
+    if (r == 4) return launch_vec<WT, 4, NM, ROUTE>(st, a, lds, vec, pieces);
+  return r >= 2 ? launch_vec<WT, 2, NM, ROUTE>(st, a, lds, vec, pieces) : launch_vec<WT, 1, NM, ROUTE>(st, a, lds, vec, pieces);
 }
 
 template <typename WT>
-hipError_t launch_any(hipStream_t st, const RowArgs& a, int route, bool up, size_t lds, bool vec) {
-  if (route == 1) return up ? launch_rows<WT, 2, 1>(st, a, lds, vec) : hipErrorInvalidValue;
-  if (route == 2) return launch_rows<WT, 1, 2>(st, a, lds, vec);
-  return up ? launch_rows<WT, 2, 0>(st, a, lds, vec) : launch_rows<WT, 1, 0>(st, a, lds, vec);
+hipError_t launch_any(hipStream_t st, const RowArgs& a, int route, bool up, size_t lds, bool vec, bool pieces) {
+  if (route == 1) return up ? launch_rows<WT, 2, 1>(st, a, lds, vec, pieces) : hipErrorInvalidValue;
+  if (route == 2) return launch_rows<WT, 1, 2>(st, a, lds, vec, pieces);
+  return up ? launch_rows<WT, 2, 0>(st, a, lds, vec, pieces) : launch_rows<WT, 1, 0>(st, a, lds, vec, pieces);
 }
 
 constexpr size_t ROW_MAX = 16000;
@@ -378,7 +443,9 @@ extern "C" int ughip_product_row(ughip_device* dev, const ughip_row_step* p) {
     }
   }
   const bool vec = p->k % 8 == 0 && (reinterpret_cast<uintptr_t>(a.w) & 15) == 0;
-  UGHIP_HIPCHK(p->w->dtype == UGHIP_BF16 ? launch_any<uint16_t>(dev->stream, a, p->route, p->act == UGHIP_ACT_SWIGLU, lds, vec)
-                                         : launch_any<float>(dev->stream, a, p->route, p->act == UGHIP_ACT_SWIGLU, lds, vec));
+  auto a16 = [](const void* q) { return (reinterpret_cast<uintptr_t>(q) & 15) == 0; };
+  const bool pieces = p->k % 4 == 0 && a16(a.x) && a16(a.y) && a16(a.gate) && a16(a.x_out);
+  UGHIP_HIPCHK(p->w->dtype == UGHIP_BF16 ? launch_any<uint16_t>(dev->stream, a, p->route, p->act == UGHIP_ACT_SWIGLU, lds, vec, pieces)
+                                         : launch_any<float>(dev->stream, a, p->route, p->act == UGHIP_ACT_SWIGLU, lds, vec, pieces));
   return UGHIP_OK;
 }

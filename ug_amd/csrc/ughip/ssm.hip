@@ -3,11 +3,13 @@
 //   S_t = exp(a_t) S_{t-1} + d_t B_t x_t^T,   y_t = S_t^T C_t + skip x_t,   a_t = -exp(a_log) d_t, d_t = softplus(dt_t + bias)
 //
 // Several positions run in chunks of Q.  With A_i = a_1 + .. + a_i inside a chunk:
-//   ssm_chunk_state   what a chunk adds to the state: sum_j exp(A_Q - A_j) d_j B_j x_j^T              (one workgroup per chunk and head)
+//   ssm_chunk_state   what a chunk adds to the state: sum_j B_j (exp(A_Q - A_j) d_j x_j)^T
 //   ssm_chunk_scan    the state in front of every chunk, S <- exp(A_Q) S + that, in place              (elementwise, chunks in order)
 //   ssm_chunk_out     y_i = sum_{j <= i} exp(A_i - A_j) d_j (C_i . B_j) x_j + exp(A_i) S^T C_i + skip x_i
-// Every exponent is <= 0.  The products are v_mfma_f32_16x16x4_f32 on f32 tiles in LDS (lane l: row or column l % 16, k = l / 16;
-// result element e: row 4 (l / 16) + e, column l % 16).
+// Every exponent is <= 0.  A workgroup takes a chunk and some heads of one group: B, C and the products C_i . B_j are the group's
+// and are made once, then the heads follow one after the other, the next head's x (and state) on their way to registers while
+// this one is multiplied.  The products are v_mfma_f32_16x16x4_f32 on f32 tiles in LDS (lane l: row or column l % 16, k = l / 16;
+// result element e: row 4 (l / 16) + e, column l % 16), four independent column tiles at a time.
 #include <hip/hip_runtime.h>
 
 #include "layers.h"
@@ -30,6 +32,41 @@ struct SsmArgs {
   int t, heads, vdim, groups, state, q, chunks;
   bool fresh;
 };
+
+// A thread takes four channels (V) of ROWS_CONV rows, the taps' rows sliding through registers; any channel count otherwise.
+constexpr int ROWS_CONV = 8;
+template <int TAPS>
+__global__ void __launch_bounds__(256) conv_silu_rows4_kernel(const float* __restrict__ x, size_t x_stride, const float* __restrict__ taps, const float* __restrict__ bias,
+                                                              const float* __restrict__ ring, long long pos, int t, int channels, float* __restrict__ dst, size_t dst_stride) {
+  const int c = (blockIdx.x * 256 + threadIdx.x) * 4, i0 = blockIdx.y * ROWS_CONV;
+  if (c >= channels) return;
+  auto row = [&](int r) -> f32x4_t {
+    if (r >= 0) return r < t ? *reinterpret_cast<const f32x4_t*>(x + (size_t)r * x_stride + c) : f32x4_t{0.f, 0.f, 0.f, 0.f};
+    if (pos + r >= 0) return *reinterpret_cast<const f32x4_t*>(ring + (size_t)((pos + r) % TAPS) * channels + c);
+    return f32x4_t{0.f, 0.f, 0.f, 0.f};
+  };
+  float w[4][TAPS];
+#pragma unroll
+  for (int e = 0; e < 4; ++e)
+#pragma unroll
+    for (int j = 0; j < TAPS; ++j) w[e][j] = taps[(size_t)(c + e) * TAPS + j];
+  const f32x4_t b = bias ? *reinterpret_cast<const f32x4_t*>(bias + c) : f32x4_t{0.f, 0.f, 0.f, 0.f};
+  f32x4_t in[ROWS_CONV + TAPS - 1];
+#pragma unroll
+  for (int j = 0; j < ROWS_CONV + TAPS - 1; ++j) in[j] = row(i0 - (TAPS - 1) + j);
+#pragma unroll
+  for (int i = 0; i < ROWS_CONV; ++i) {
+    if (i0 + i >= t) break;
+    f32x4_t v = b;
+#pragma unroll
+    for (int j = 0; j < TAPS; ++j)
+#pragma unroll
+      for (int e = 0; e < 4; ++e) v[e] += w[e][j] * in[i + j][e];
+#pragma unroll
+    for (int e = 0; e < 4; ++e) v[e] = silu_f(v[e]);
+    *reinterpret_cast<f32x4_t*>(dst + (size_t)(i0 + i) * dst_stride + c) = v;
+  }
+}
 
 __global__ void __launch_bounds__(256) conv_silu_rows_kernel(const float* __restrict__ x, size_t x_stride, const float* __restrict__ taps, const float* __restrict__ bias,
                                                              int n_taps, const float* __restrict__ ring, long long pos, int t, int channels, float* __restrict__ dst,
@@ -57,66 +94,159 @@ __global__ void __launch_bounds__(256) conv_ring_store_kernel(const float* __res
   ring[(size_t)((pos + i) % n_taps) * channels + c] = x[(size_t)i * x_stride + c];
 }
 
-// cum[i] = A_i and d[i] for the chunk's rows, rows past the end with d = 0 and the last A.  The first wave scans (q <= 64).
+// cum[i] = A_i and d[i] for the chunk's rows, rows past the end with d = 0 and the last A.  One wave (q <= 64).
 __device__ __forceinline__ void chunk_decays(const SsmArgs& a, int h, int row0, float* cum, float* d) {
-  if (threadIdx.x < 64) {
-    const int i = threadIdx.x;
-    float dv = 0.f;
-    if (i < a.q && row0 + i < a.t) dv = softplus_f(a.dt[(size_t)(row0 + i) * a.dt_stride + h] + a.dt_bias[h]);
-    float s = -expf(a.a_log[h]) * dv;
-    for (int k = 1; k < 64; k <<= 1) {
-      const float o = __shfl_up(s, k, 64);
-      if (i >= k) s += o;
-    }
-    if (i < a.q) cum[i] = s, d[i] = dv;
+  const int i = threadIdx.x & 63;
+  float dv = 0.f;
+  if (i < a.q && row0 + i < a.t) dv = softplus_f(a.dt[(size_t)(row0 + i) * a.dt_stride + h] + a.dt_bias[h]);
+  float s = -expf(a.a_log[h]) * dv;
+  for (int k = 1; k < 64; k <<= 1) {
+    const float o = __shfl_up(s, k, 64);
+    if (i >= k) s += o;
   }
-  __syncthreads();
+  cum[i] = s, d[i] = dv;
 }
 
 __device__ __forceinline__ f32x4_t mfma16(float x, float y, f32x4_t acc) { return __builtin_amdgcn_mfma_f32_16x16x4f32(x, y, acc, 0, 0, 0); }
 
-constexpr int PB = 64;  // columns of vdim per workgroup
+constexpr int PB = 64, PS = PB + 4;  // columns of vdim at a time, and the stride of their rows in LDS
 
 __device__ __host__ inline int pad16(int v) { return (v + 15) & ~15; }
-// row strides of LDS tiles: 4 mod 64 or a multiple of 16 plus 4, so that 16 rows x 4 neighbours spread over the banks
+// row stride of LDS tiles of `state` columns: a multiple of 16 plus 4, so that 16 rows x 4 neighbours spread over the banks
 __device__ __host__ inline int row_n(int state) { return pad16(state) + 4; }
 
-__global__ void __launch_bounds__(256) ssm_chunk_state_kernel(SsmArgs a) {
-  extern __shared__ float lds[];
-  const int q = a.q, chunk = blockIdx.x, h = blockIdx.y, p0 = blockIdx.z * PB, row0 = chunk * q;
-  const int pw = min(PB, a.vdim - p0), N = a.state, ns = row_n(N), ps = PB + 4, inner = a.heads * a.vdim, g = h / (a.heads / a.groups);
-  float* cum = lds;
-  float* d = lds + 64;
-  float* Bs = lds + 128;      // [q][ns]
-  float* Xs = Bs + q * ns;    // [q][ps]
-  chunk_decays(a, h, row0, cum, d);
-  const float end = cum[q - 1];
-  const int np = pad16(N);
-  for (int e = threadIdx.x; e < q * np; e += 256) {
-    const int i = e / np, n = e % np;
-    float v = 0.f;
-    if (row0 + i < a.t && n < N) v = a.xbc[(size_t)(row0 + i) * a.xbc_stride + inner + (size_t)g * N + n] * (d[i] * expf(end - cum[i]));
-    Bs[i * ns + n] = v;
-  }
-  for (int e = threadIdx.x; e < q * PB; e += 256) {
-    const int i = e / PB, p = e % PB;
-    Xs[i * ps + p] = row0 + i < a.t && p < pw ? a.xbc[(size_t)(row0 + i) * a.xbc_stride + (size_t)h * a.vdim + p0 + p] : 0.f;
-  }
-  __syncthreads();
-  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, j = lane & 15, kg = lane >> 4;
-  const int tn = np / 16, tp = pad16(pw) / 16;
-  float* out = a.chunk_s + ((size_t)chunk * a.heads + h) * N * a.vdim;
-  for (int tile = wave; tile < tn * tp; tile += 4) {
-    const int n0 = (tile / tp) * 16, c0 = (tile % tp) * 16;
-    f32x4_t acc = {0.f, 0.f, 0.f, 0.f};
-    for (int k = kg; k < q; k += 4) acc = mfma16(Bs[k * ns + n0 + j], Xs[k * ps + c0 + j], acc);
+// `rows` x `cols` (cols <= 4 * width4) of a row-major matrix, zeros outside, through registers: N4 runs of four per thread.
+template <int N4, bool VEC>
+struct TileRegs {
+  f32x4_t v[N4];
+  __device__ void load(const float* src, size_t stride, int rows, int cols, int width4, int total) {
 #pragma unroll
-    for (int e = 0; e < 4; ++e) {
-      const int n = n0 + 4 * kg + e;
-      if (n < N && c0 + j < pw) out[(size_t)n * a.vdim + p0 + c0 + j] = acc[e];
+    for (int u = 0; u < N4; ++u) {
+      const int e = threadIdx.x + u * 256, r = e / width4, c = (e - r * width4) * 4;
+      v[u] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+      if (e >= total || r >= rows) continue;
+      const float* p = src + (size_t)r * stride + c;
+      if (VEC) {
+        if (c < cols) v[u] = *reinterpret_cast<const f32x4_t*>(p);
+      } else {
+#pragma unroll
+        for (int i = 0; i < 4; ++i)
+          if (c + i < cols) v[u][i] = p[i];
+      }
     }
   }
-  if (blockIdx.z == 0 && threadIdx.x == 0) a.decay[(size_t)chunk * a.heads + h] = expf(end);
+  // scale (may be null): row r times scale[r]
+  __device__ void store(float* lds, int ld, int width4, int total, const float* scale = nullptr) const {
+#pragma unroll
+    for (int u = 0; u < N4; ++u) {
+      const int e = threadIdx.x + u * 256, r = e / width4, c = (e - r * width4) * 4;
+      if (e >= total) continue;
+      f32x4_t w = v[u];
+      if (scale) w *= scale[r];
+      *reinterpret_cast<f32x4_t*>(lds + r * ld + c) = w;
+    }
+  }
+};
+template <bool VEC>
+__device__ __forceinline__ void tile_to_lds(float* lds, int ld, const float* src, size_t stride, int rows, int cols, int width4, int total) {
+  for (int base = 0; base < total; base += 256 * 4) {  // four loads per thread on their way at a time
+    f32x4_t v[4];
+#pragma unroll
+    for (int u = 0; u < 4; ++u) {
+      const int e = base + threadIdx.x + u * 256, r = e / width4, c = (e - r * width4) * 4;
+      v[u] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+      if (e >= total || r >= rows) continue;
+      const float* p = src + (size_t)r * stride + c;
+      if (VEC) {
+        if (c < cols) v[u] = *reinterpret_cast<const f32x4_t*>(p);
+      } else {
+#pragma unroll
+        for (int i = 0; i < 4; ++i)
+          if (c + i < cols) v[u][i] = p[i];
+      }
+    }
+#pragma unroll
+    for (int u = 0; u < 4; ++u) {
+      const int e = base + threadIdx.x + u * 256, r = e / width4, c = (e - r * width4) * 4;
+      if (e < total) *reinterpret_cast<f32x4_t*>(lds + r * ld + c) = v[u];
+    }
+  }
+}
+
+// What a workgroup walks: heads h0 .. h0 + n of a group, each in blocks of PB columns.
+struct HeadWalk {
+  int g, h0, items, blocks;
+  __device__ HeadWalk(const SsmArgs& a) {
+    const int per = a.heads / a.groups, each = (per + (int)gridDim.z - 1) / (int)gridDim.z;
+    g = blockIdx.y;
+    blocks = (a.vdim + PB - 1) / PB;
+    const int first = (int)blockIdx.z * each, last = min(per, first + each);
+    h0 = g * per + first;
+    items = max(0, last - first) * blocks;
+  }
+  __device__ int head(int i) const { return h0 + i / blocks; }
+  __device__ int col(int i) const { return i % blocks * PB; }
+};
+
+template <bool VEC>
+__global__ void __launch_bounds__(256) ssm_chunk_state_kernel(SsmArgs a) {
+  extern __shared__ __attribute__((aligned(16))) float lds[];
+  const int q = a.q, chunk = blockIdx.x, row0 = chunk * q, rows = min(q, a.t - row0), N = a.state, ns = row_n(N), np = pad16(N), inner = a.heads * a.vdim;
+  const HeadWalk hw(a);
+  float* cum = lds;
+  float* d = lds + 64;
+  float* wgt = lds + 128;
+  float* Bs = lds + 192;      // [q][ns]
+  float* Xs = Bs + q * ns;    // [q][PS]
+  const float* xbc0 = a.xbc + (size_t)row0 * a.xbc_stride;
+  tile_to_lds<VEC>(Bs, ns, xbc0 + inner + (size_t)hw.g * N, a.xbc_stride, rows, N, np / 4, q * np / 4);
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, j = lane & 15, kg = lane >> 4, tn = np / 16, xt = q * PB / 4;
+  TileRegs<4, VEC> x;
+  auto fetch = [&](int i) { x.load(xbc0 + (size_t)hw.head(i) * a.vdim + hw.col(i), a.xbc_stride, rows, min(PB, a.vdim - hw.col(i)), PB / 4, xt); };
+  if (hw.items) fetch(0);
+  for (int it = 0; it < hw.items; ++it) {
+    const int h = hw.head(it), p0 = hw.col(it), pw = min(PB, a.vdim - p0);
+    __syncthreads();
+    if (wave == 0) {
+      chunk_decays(a, h, row0, cum, d);
+      __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "workgroup");  // one wave's own LDS writes, read back below
+      __builtin_amdgcn_wave_barrier();
+      if (lane < q) wgt[lane] = d[lane] * expf(cum[q - 1] - cum[lane]);
+      if (lane == 0 && p0 == 0) a.decay[(size_t)chunk * a.heads + h] = expf(cum[q - 1]);
+    }
+    __syncthreads();
+    x.store(Xs, PS, PB / 4, xt, wgt);
+    if (it + 1 < hw.items) fetch(it + 1);
+    __syncthreads();
+    float* out = a.chunk_s + ((size_t)chunk * a.heads + h) * N * a.vdim + p0;
+    for (int n_tile = wave * 2; n_tile < tn; n_tile += 8) {  // two row tiles by four column tiles at a time
+      const int n0 = n_tile * 16, n1 = min(n_tile + 1, tn - 1) * 16;
+      f32x4_t acc[2][4];
+#pragma unroll
+      for (int u = 0; u < 4; ++u) acc[0][u] = acc[1][u] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+#pragma unroll 4
+      for (int k = kg; k < q; k += 4) {
+        const float b0 = Bs[k * ns + n0 + j], b1 = Bs[k * ns + n1 + j];
+#pragma unroll
+        for (int u = 0; u < 4; ++u) {
+          const float xv = Xs[k * PS + u * 16 + j];
+          acc[0][u] = mfma16(b0, xv, acc[0][u]);
+          acc[1][u] = mfma16(b1, xv, acc[1][u]);
+        }
+      }
+#pragma unroll
+      for (int v = 0; v < 2; ++v) {
+        if (v == 1 && n_tile + 1 >= tn) break;
+#pragma unroll
+        for (int u = 0; u < 4; ++u)
+#pragma unroll
+          for (int e = 0; e < 4; ++e) {
+            const int n = (v ? n1 : n0) + 4 * kg + e;
+            if (n < N && u * 16 + j < pw) out[(size_t)n * a.vdim + u * 16 + j] = acc[v][u][e];
+          }
+      }
+    }
+  }
 }
 
 __global__ void __launch_bounds__(256) ssm_chunk_scan_kernel(SsmArgs a) {
@@ -133,61 +263,98 @@ __global__ void __launch_bounds__(256) ssm_chunk_scan_kernel(SsmArgs a) {
   a.s[h * per + e] = s;
 }
 
+template <bool VEC>
 __global__ void __launch_bounds__(256) ssm_chunk_out_kernel(SsmArgs a) {
-  extern __shared__ float lds[];
-  const int q = a.q, chunk = blockIdx.x, h = blockIdx.y, p0 = blockIdx.z * PB, row0 = chunk * q;
-  const int pw = min(PB, a.vdim - p0), N = a.state, ns = row_n(N), ps = PB + 4, ms = q + 4, inner = a.heads * a.vdim, g = h / (a.heads / a.groups);
+  extern __shared__ __attribute__((aligned(16))) float lds[];
+  const int q = a.q, chunk = blockIdx.x, row0 = chunk * q, rows = min(q, a.t - row0), N = a.state, ns = row_n(N), np = pad16(N), gs = q + 4, inner = a.heads * a.vdim;
+  const HeadWalk hw(a);
   float* cum = lds;
   float* d = lds + 64;
-  float* Bs = lds + 128;      // [q][ns]
-  float* Cs = Bs + q * ns;    // [q][ns]
-  float* Xs = Cs + q * ns;    // [q][ps]
-  float* Ms = Xs + q * ps;    // [q][ms]
-  chunk_decays(a, h, row0, cum, d);
-  const int np = pad16(N);
-  for (int e = threadIdx.x; e < q * np; e += 256) {
-    const int i = e / np, n = e % np;
-    float b = 0.f, c = 0.f;
-    if (row0 + i < a.t && n < N) {
-      const float* row = a.xbc + (size_t)(row0 + i) * a.xbc_stride + inner + (size_t)g * N + n;
-      b = row[0];
-      c = row[(size_t)a.groups * N];
-    }
-    Bs[i * ns + n] = b;
-    Cs[i * ns + n] = c;
-  }
-  for (int e = threadIdx.x; e < q * PB; e += 256) {
-    const int i = e / PB, p = e % PB;
-    Xs[i * ps + p] = row0 + i < a.t && p < pw ? a.xbc[(size_t)(row0 + i) * a.xbc_stride + (size_t)h * a.vdim + p0 + p] : 0.f;
-  }
+  float* Cs = lds + 128;      // [q][ns]
+  float* Gs = Cs + q * ns;    // [q][gs]: C_i . B_j
+  float* Bs = Gs + q * gs;    // [q][ns], then
+  float* Xs = Bs;             // [q][PS]
+  float* Ss = Xs + q * PS;    // [np][PS]
+  const float* xbc0 = a.xbc + (size_t)row0 * a.xbc_stride;
+  tile_to_lds<VEC>(Bs, ns, xbc0 + inner + (size_t)hw.g * N, a.xbc_stride, rows, N, np / 4, q * np / 4);
+  tile_to_lds<VEC>(Cs, ns, xbc0 + inner + (size_t)(a.groups + hw.g) * N, a.xbc_stride, rows, N, np / 4, q * np / 4);
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, j = lane & 15, kg = lane >> 4, tq = q / 16, i0 = wave * 16, xt = q * PB / 4, st = np * PB / 4;
+  TileRegs<4, VEC> x;
+  TileRegs<8, VEC> s;
+  auto fetch = [&](int i) {
+    const int pw = min(PB, a.vdim - hw.col(i));
+    x.load(xbc0 + (size_t)hw.head(i) * a.vdim + hw.col(i), a.xbc_stride, rows, pw, PB / 4, xt);
+    s.load(a.chunk_s + ((size_t)chunk * a.heads + hw.head(i)) * N * a.vdim + hw.col(i), a.vdim, N, pw, PB / 4, st);
+  };
+  if (hw.items) fetch(0);
   __syncthreads();
-  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, j = lane & 15, kg = lane >> 4, tq = q / 16;
-  for (int tile = wave; tile < tq * tq; tile += 4) {
-    const int i0 = (tile / tq) * 16, j0 = (tile % tq) * 16;
-    f32x4_t acc = {0.f, 0.f, 0.f, 0.f};
-    if (j0 <= i0)
-      for (int k = kg; k < np; k += 4) acc = mfma16(Cs[(i0 + j) * ns + k], Bs[(j0 + j) * ns + k], acc);
+  if (wave < tq) {
+    f32x4_t acc[4];
 #pragma unroll
-    for (int e = 0; e < 4; ++e) {
-      const int i = i0 + 4 * kg + e, jj = j0 + j;
-      Ms[i * ms + jj] = jj <= i ? acc[e] * expf(cum[i] - cum[jj]) * d[jj] : 0.f;
+    for (int u = 0; u < 4; ++u) acc[u] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+#pragma unroll 2
+    for (int k = 4 * kg; k < np; k += 16) {  // k four elements per lane at a time: 16-byte reads
+      const f32x4_t c = *reinterpret_cast<const f32x4_t*>(Cs + (i0 + j) * ns + k);
+#pragma unroll
+      for (int u = 0; u < 4; ++u) {
+        if (u > wave) break;  // columns past the row tile are not used
+        const f32x4_t b = *reinterpret_cast<const f32x4_t*>(Bs + (u * 16 + j) * ns + k);
+        acc[u] = mfma16(c.x, b.x, acc[u]);
+        acc[u] = mfma16(c.y, b.y, acc[u]);
+        acc[u] = mfma16(c.z, b.z, acc[u]);
+        acc[u] = mfma16(c.w, b.w, acc[u]);
+      }
     }
+#pragma unroll
+    for (int u = 0; u < 4; ++u)
+      if (u < tq)
+#pragma unroll
+        for (int e = 0; e < 4; ++e) Gs[(i0 + 4 * kg + e) * gs + u * 16 + j] = acc[u][e];
   }
-  __syncthreads();
-  const int tp = pad16(pw) / 16;
-  const float* S = a.chunk_s + ((size_t)chunk * a.heads + h) * N * a.vdim + p0;
-  for (int tile = wave; tile < tq * tp; tile += 4) {
-    const int i0 = (tile / tp) * 16, c0 = (tile % tp) * 16;
-    f32x4_t acc = {0.f, 0.f, 0.f, 0.f}, from_s = {0.f, 0.f, 0.f, 0.f};
-    for (int k = kg; k < i0 + 16; k += 4) acc = mfma16(Ms[(i0 + j) * ms + k], Xs[k * ps + c0 + j], acc);
-    const bool col_ok = c0 + j < pw;
-    for (int k = kg; k < np; k += 4) from_s = mfma16(Cs[(i0 + j) * ns + k], col_ok && k < N ? S[(size_t)k * a.vdim + c0 + j] : 0.f, from_s);
-    if (!col_ok) continue;
+  for (int it = 0; it < hw.items; ++it) {
+    const int h = hw.head(it), p0 = hw.col(it), pw = min(PB, a.vdim - p0);
+    __syncthreads();
+    x.store(Xs, PS, PB / 4, xt);
+    s.store(Ss, PS, PB / 4, st);
+    for (int base = 2048; base < st; base += 2048) {  // states of more than 128 rows: the rest without prefetch
+      const int r0 = base / (PB / 4);
+      tile_to_lds<VEC>(Ss + r0 * PS, PS, a.chunk_s + (((size_t)chunk * a.heads + h) * N + r0) * a.vdim + p0, a.vdim, N - r0, pw, PB / 4, min(2048, st - base));
+    }
+    if (wave == 0) chunk_decays(a, h, row0, cum, d);
+    __syncthreads();
+    if (it + 1 < hw.items) fetch(it + 1);
+    if (wave >= tq) continue;  // q < 64: the waves without rows only move data
+    f32x4_t in_chunk[4], from_s[4];
+#pragma unroll
+    for (int u = 0; u < 4; ++u) in_chunk[u] = from_s[u] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+    const float ci = cum[i0 + j];
+#pragma unroll 4
+    for (int k = kg; k < i0 + 16; k += 4) {
+      const float m = k <= i0 + j ? Gs[(i0 + j) * gs + k] * expf(ci - cum[k]) * d[k] : 0.f;
+#pragma unroll
+      for (int u = 0; u < 4; ++u) in_chunk[u] = mfma16(m, Xs[k * PS + u * 16 + j], in_chunk[u]);
+    }
+#pragma unroll 2
+    for (int k = 4 * kg; k < np; k += 16) {
+      const f32x4_t c = *reinterpret_cast<const f32x4_t*>(Cs + (i0 + j) * ns + k);
+#pragma unroll
+      for (int u = 0; u < 4; ++u) {
+        from_s[u] = mfma16(c.x, Ss[k * PS + u * 16 + j], from_s[u]);
+        from_s[u] = mfma16(c.y, Ss[(k + 1) * PS + u * 16 + j], from_s[u]);
+        from_s[u] = mfma16(c.z, Ss[(k + 2) * PS + u * 16 + j], from_s[u]);
+        from_s[u] = mfma16(c.w, Ss[(k + 3) * PS + u * 16 + j], from_s[u]);
+      }
+    }
+    const float skip = a.skip[h];
 #pragma unroll
     for (int e = 0; e < 4; ++e) {
       const int i = i0 + 4 * kg + e;
-      if (row0 + i < a.t)
-        a.dst[(size_t)(row0 + i) * a.dst_stride + (size_t)h * a.vdim + p0 + c0 + j] = acc[e] + expf(cum[i]) * from_s[e] + a.skip[h] * Xs[i * ps + c0 + j];
+      const float decay = expf(cum[i]);
+      if (i >= rows) continue;
+#pragma unroll
+      for (int u = 0; u < 4; ++u)
+        if (u * 16 + j < pw)
+          a.dst[(size_t)(row0 + i) * a.dst_stride + (size_t)h * a.vdim + p0 + u * 16 + j] = in_chunk[u][e] + decay * from_s[u][e] + skip * Xs[i * PS + u * 16 + j];
     }
   }
 }
@@ -195,7 +362,7 @@ __global__ void __launch_bounds__(256) ssm_chunk_out_kernel(SsmArgs a) {
 // One position in one launch.  A workgroup takes a head and 16 of its columns: it convolves those columns and the head's B and
 // C rows (again in every workgroup: a few hundred channels), then 16 threads per column walk the state.  The ring's slot of this
 // position is one no tap of this position reads, so the rows go in while other workgroups still convolve.
-constexpr int STEP_COLS = 16;
+constexpr int STEP_COLS = 16, STEP_ROWS = 8;
 struct SsmStepArgs {
   const float* xbc;  // this position's inputs of the convolution
   const float* dt;
@@ -228,6 +395,11 @@ __global__ void __launch_bounds__(256) ssm_step_kernel(SsmStepArgs a) {
   const int h = blockIdx.x, p0 = blockIdx.y * STEP_COLS, inner = a.heads * a.vdim, N = a.state, per = a.heads / a.groups, g = h / per;
   const bool first = h % per == 0 && blockIdx.y == 0;  // stores the group's B and C rows
   float* slot = a.ring + (size_t)(a.pos % a.n_taps) * a.channels;
+  const int col = threadIdx.x & 15, ng = threadIdx.x >> 4, p = p0 + col;
+  float* S = a.s + (size_t)h * N * a.vdim + p;
+  float held[STEP_ROWS];  // the first of the state's rows, asked for before anything else
+#pragma unroll
+  for (int u = 0; u < STEP_ROWS; ++u) held[u] = a.pos && p < a.vdim && ng + 16 * u < N ? S[(size_t)(ng + 16 * u) * a.vdim] : 0.f;
   for (int i = threadIdx.x; i < 2 * N; i += 256) {
     const int c = inner + (i < N ? 0 : a.groups * N) + g * N + (i < N ? i : i - N);
     lds[i] = conv_one(a, c);
@@ -239,13 +411,19 @@ __global__ void __launch_bounds__(256) ssm_step_kernel(SsmStepArgs a) {
     slot[c] = a.xbc[c];
   }
   __syncthreads();
-  const int col = threadIdx.x & 15, ng = threadIdx.x >> 4, p = p0 + col;
   const float d = softplus_f(a.dt[h] + a.dt_bias[h]), keep = expf(-expf(a.a_log[h]) * d);
   float y = 0.f;
   if (p < a.vdim) {
     const float dx = d * xs[col];
-    float* S = a.s + (size_t)h * N * a.vdim + p;
-    for (int n = ng; n < N; n += 16) {
+#pragma unroll
+    for (int u = 0; u < STEP_ROWS; ++u) {
+      const int n = ng + 16 * u;
+      if (n >= N) break;
+      const float v = keep * held[u] + dx * B[n];
+      S[(size_t)n * a.vdim] = v;
+      y += v * C[n];
+    }
+    for (int n = ng + 16 * STEP_ROWS; n < N; n += 16) {
       float v = dx * B[n];
       if (a.pos) v += keep * S[(size_t)n * a.vdim];
       S[(size_t)n * a.vdim] = v;
@@ -262,7 +440,11 @@ __global__ void __launch_bounds__(256) ssm_step_kernel(SsmStepArgs a) {
   }
 }
 
-size_t chunk_lds_bytes(int q, int state) { return (size_t)(128 + 2 * q * row_n(state) + q * (PB + 4) + q * (q + 4)) * sizeof(float); }
+size_t state_lds_bytes(int q, int state) { return (size_t)(192 + q * row_n(state) + q * PS) * sizeof(float); }
+size_t out_lds_bytes(int q, int state) {
+  const size_t b = (size_t)q * row_n(state), xs = (size_t)(q + pad16(state)) * PS;
+  return (128 + (size_t)q * row_n(state) + (size_t)q * (q + 4) + (b > xs ? b : xs)) * sizeof(float);
+}
 
 }  // namespace
 
@@ -278,6 +460,14 @@ extern "C" int ughip_conv_silu_rows(ughip_device* dev, ughip_view x, const ughip
   if (int rc = check_view(dev, dst, t, channels, UGHIP_F32, "conv_silu_rows dst")) return rc;
   if (t == 0 || channels == 0) return UGHIP_OK;
   if (int rc = device_activate(dev)) return rc;
+  auto a16 = [](const void* p) { return (reinterpret_cast<uintptr_t>(p) & 15) == 0; };
+  if (n_taps == 4 && channels % 4 == 0 && x.stride % 4 == 0 && dst.stride % 4 == 0 && a16(view_ptr<float>(x)) && a16(view_ptr<float>(dst)) && t / ROWS_CONV < 65535) {
+    const dim3 g4((unsigned)((channels / 4 + 255) / 256), (unsigned)((t + ROWS_CONV - 1) / ROWS_CONV));
+    conv_silu_rows4_kernel<4><<<g4, 256, 0, dev->stream>>>(view_ptr<float>(x), x.stride, buf_ptr<float>(taps), buf_ptr<float>(bias), buf_ptr<float>(ring), (long long)pos,
+                                                           (int)t, (int)channels, view_ptr<float>(dst), dst.stride);
+    UGHIP_HIPCHK(hipGetLastError());
+    return UGHIP_OK;
+  }
   const dim3 grid((unsigned)((channels + 255) / 256), (unsigned)(t < 16384 ? t : 16384));
   conv_silu_rows_kernel<<<grid, 256, 0, dev->stream>>>(view_ptr<float>(x), x.stride, buf_ptr<float>(taps), buf_ptr<float>(bias), (int)n_taps, buf_ptr<float>(ring),
                                                        (long long)pos, (int)t, (int)channels, view_ptr<float>(dst), dst.stride);
@@ -311,25 +501,35 @@ extern "C" int ughip_ssm_rows(ughip_device* dev, ughip_view xbc, ughip_view dt, 
   if (int rc = check_view(dev, dst, t, heads * vdim, UGHIP_F32, "ssm_rows dst")) return rc;
   if (t == 0) return UGHIP_OK;
   int q = 64;
-  while (q > 16 && (chunk_lds_bytes(q, (int)state) > 160 * 1024 || (size_t)(q / 2) >= t)) q /= 2;
-  const size_t lds = chunk_lds_bytes(q, (int)state);
-  if (lds > 160 * 1024) return set_error(UGHIP_ERR_UNSUPPORTED, "ssm_rows: a state of %zu rows does not fit LDS", state);
+  while (q > 16 && (out_lds_bytes(q, (int)state) > 160 * 1024 || (size_t)(q / 2) >= t)) q /= 2;
+  if (out_lds_bytes(q, (int)state) > 160 * 1024 || state_lds_bytes(q, (int)state) > 160 * 1024) return set_error(UGHIP_ERR_UNSUPPORTED, "ssm_rows: a state of %zu rows does not fit LDS", state);
   if (int rc = device_activate(dev)) return rc;
-  const size_t chunks = (t + q - 1) / q, per = state * vdim, decay_bytes = (chunks * heads * sizeof(float) + 255) & ~(size_t)255;
+  const size_t chunks = (t + q - 1) / q, elems = state * vdim, decay_bytes = (chunks * heads * sizeof(float) + 255) & ~(size_t)255;
   void* ws = nullptr;
-  if (int rc = rows_scratch(dev, decay_bytes + chunks * heads * per * sizeof(float), &ws)) return rc;
+  if (int rc = rows_scratch(dev, decay_bytes + chunks * heads * elems * sizeof(float), &ws)) return rc;
   SsmArgs a{view_ptr<float>(xbc), view_ptr<float>(dt), buf_ptr<float>(dt_bias), buf_ptr<float>(a_log), buf_ptr<float>(skip), static_cast<float*>(s->ptr),
             reinterpret_cast<float*>(static_cast<char*>(ws) + decay_bytes), static_cast<float*>(ws), view_ptr<float>(dst), xbc.stride, dt.stride, dst.stride,
             (int)t, (int)heads, (int)vdim, (int)groups, (int)state, q, (int)chunks, pos == 0};
-  const dim3 grid((unsigned)chunks, (unsigned)heads, (unsigned)((vdim + PB - 1) / PB));
+  // a group's heads share a workgroup unless the chip would stay empty
+  const size_t per = heads / groups;
+  size_t share = (512 + chunks * groups - 1) / (chunks * groups);
+  if (share > per) share = per;
+  const dim3 grid((unsigned)chunks, (unsigned)groups, (unsigned)share);
+  const bool vec = vdim % 4 == 0 && state % 4 == 0 && xbc.stride % 4 == 0 && (reinterpret_cast<uintptr_t>(a.xbc) & 15) == 0;
   static const hipError_t attr = [] {
-    hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(ssm_chunk_state_kernel), hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
-    return e != hipSuccess ? e : hipFuncSetAttribute(reinterpret_cast<const void*>(ssm_chunk_out_kernel), hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
+    hipError_t e = hipSuccess;
+    for (const void* f : {reinterpret_cast<const void*>(ssm_chunk_state_kernel<true>), reinterpret_cast<const void*>(ssm_chunk_state_kernel<false>),
+                          reinterpret_cast<const void*>(ssm_chunk_out_kernel<true>), reinterpret_cast<const void*>(ssm_chunk_out_kernel<false>)})
+      if (e == hipSuccess) e = hipFuncSetAttribute(f, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
+    return e;
   }();
   UGHIP_HIPCHK(attr);
-  ssm_chunk_state_kernel<<<grid, 256, lds, dev->stream>>>(a);
-  ssm_chunk_scan_kernel<<<dim3((unsigned)((per + 255) / 256), (unsigned)heads), 256, 0, dev->stream>>>(a);
-  ssm_chunk_out_kernel<<<grid, 256, lds, dev->stream>>>(a);
+  const size_t lds_s = state_lds_bytes(q, (int)state), lds_o = out_lds_bytes(q, (int)state);
+  if (vec) ssm_chunk_state_kernel<true><<<grid, 256, lds_s, dev->stream>>>(a);
+  else ssm_chunk_state_kernel<false><<<grid, 256, lds_s, dev->stream>>>(a);
+  ssm_chunk_scan_kernel<<<dim3((unsigned)((elems + 255) / 256), (unsigned)heads), 256, 0, dev->stream>>>(a);
+  if (vec) ssm_chunk_out_kernel<true><<<grid, 256, lds_o, dev->stream>>>(a);
+  else ssm_chunk_out_kernel<false><<<grid, 256, lds_o, dev->stream>>>(a);
   UGHIP_HIPCHK(hipGetLastError());
   return UGHIP_OK;
 }
