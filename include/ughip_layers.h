@@ -128,7 +128,7 @@ int ughip_group_rows(ughip_device* dev, const ughip_slice* ids, size_t m, size_t
  *     result is one run of n columns per chosen expert, top n in all;
  *   route == 2: ids and weights are read, x holds one row of k per chosen expert (top k values), and the result is the weighted
  *     sum of the experts' products: n columns.
- * k (route 2: top k) <= 16000. */
+ * The input row, every expert's part rounded up to a multiple of 512, has at most 16384 elements. */
 typedef struct ughip_row_step {
   const ughip_slice* x;
   size_t x_offset;

@@ -136,7 +136,7 @@ struct RowStep {
   size_t norm_groups = 1, gate_offset = 0;
   float eps = 0;
 };
-constexpr size_t kRowStepMax = 16000;  // elements of the row a folded product meets
+constexpr size_t kRowStepMax = 16000;  // elements of the row a folded product meets (an expert's part counts in runs of 512)
 
 // `pending` joins x first; keep_x: the joined row lies in front of the result (which starts at *at).
 LB row_step(const Rows& x, const Stream* pending, size_t width, const RowStep& r, size_t* at, bool keep_x = true) {
@@ -434,7 +434,7 @@ struct MoeFeedForward : FeedForward {
     gate_up = ld.stacked(gs, width), down = ld.stacked(ds, ff);
   }
   void run(StepContext& c, Stream& s) const override {
-    if (c.fused && std::max(width, top * ff) <= kRowStepMax && top <= 64) return run_step(c, s);
+    if (c.fused && std::max(width, top * ((ff + 511) / 512 * 512)) <= kRowStepMax && top <= 64) return run_step(c, s);
     settle(c, s);
     const size_t t = c.t, E = experts, tp = top, w = width, f = ff, gc = count, kp = keep, pairs = t * tp;
     const int mode = product_mode(gate_up);

@@ -419,7 +419,7 @@ __global__ void __launch_bounds__(256) gemm_dma4(MMArgs p, int tiles_m, int tile
         if constexpr (ROWS == 2) {
           const floatx4 u = acc[i][j + NC] + bu;
 #pragma unroll
-          for (int e = 0; e < 4; ++e) v[e] = v[e] / (1.f + __expf(-v[e])) * u[e];
+          for (int e = 0; e < 4; ++e) v[e] = v[e] * __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(-1.4426950408889634f * v[e])) * u[e];
         }
         const size_t at = (size_t)(m0 + row) * rw.dst_stride + col;
         if (rw.dst_bf16) *reinterpret_cast<u32x2*>(static_cast<T*>(rw.dst) + at) = __builtin_bit_cast(u32x2, __builtin_convertvector(v, bf16x4));
@@ -656,17 +656,17 @@ bool gemm_dma_rows_supported(const MMArgs& p, const DmaRows& r, bool swiglu, int
 }
 
 int gemm_dma_rows_pick(const MMArgs& p, const DmaRows& r, bool swiglu) {
-  int best = 0;
-  double best_us = 0;
-  MMArgs q = p;
-  const size_t groups = r.groups ? r.groups : 1;
-  q.M = (int)((p.M + groups - 1) / groups);  // rows as if they were spread evenly
-  for (int tile : {256, 128, 64}) {
-    if (!gemm_dma_rows_supported(p, r, swiglu, tile)) continue;
-    const double us = gemm_dma_cost_us(q, groups, tile);
-    if (!best || us < best_us * 0.97) best = tile, best_us = us;
+  if (long long s; tune_get(TUNE_GEMM_SHAPE, &s)) {  // tuning aid, as for gemm_dma_pick
+    const int forced = s == 3 ? 256 : s == 4 ? 128 : s == 5 ? 64 : 0;
+    return forced && gemm_dma_rows_supported(p, r, swiglu, forced) ? forced : 0;
   }
-  return best;
+  // Measured on bf16 rows with K around 2048 (products of a prompt of 2048 positions, dense and by expert): the largest tile
+  // wherever it numbers most of the chip (47 GFLOP over 16 experts 116 us against 139-152), the smallest elsewhere (2048 x 2048 x
+  // 4096: 32 us against 37 and 51); the middle one was never the fastest.
+  const size_t groups = r.groups ? r.groups : 1, m = (p.M + groups - 1) / groups;  // rows as if they were spread evenly
+  const size_t tiles = groups * ((m + 255) / 256) * ((p.N + 255) / 256);
+  if (tiles >= 200 && m > 128 && gemm_dma_rows_supported(p, r, swiglu, 256)) return 256;
+  return gemm_dma_rows_supported(p, r, swiglu, 64) ? 64 : 0;
 }
 
 hipError_t gemm_dma_launch_rows(hipStream_t stream, const MMArgs& p, const DmaRows& r, bool swiglu, int tile) {

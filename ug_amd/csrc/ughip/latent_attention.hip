@@ -70,6 +70,7 @@ struct PackArgs {
   void* kp;
   size_t q_stride;
   int t, pos, heads, dim, rot, rank, q_rows, k_rows;
+  bool q_vec;  // a head's query starts on 16 bytes
 };
 
 template <typename T>
@@ -93,6 +94,16 @@ __global__ void __launch_bounds__(256) latent_pack_kernel(PackArgs a) {
     const float* qr = is_q ? a.q + (size_t)r * a.q_stride + (size_t)head * (a.dim + a.rot) : nullptr;
     const T* kr = static_cast<const T*>(a.k) + (size_t)r * a.heads * a.dim + (size_t)head * a.dim;
     const float* rr = a.cache + (size_t)r * (a.rank + a.rot) + a.rank;
+    if (a.dim % 8 == 0 && !is_q && c < a.dim) {  // a whole piece of a head's own key
+      __builtin_memcpy(v, __builtin_assume_aligned(kr + c, 16), 16);
+    } else if (a.dim % 8 == 0 && is_q && c < a.dim && a.q_vec) {
+#pragma unroll
+      for (int e = 0; e < E; e += 4) {
+        const f32x4_t f = *reinterpret_cast<const f32x4_t*>(qr + c + e);
+#pragma unroll
+        for (int i = 0; i < 4; ++i) v[e + i] = to_elem<T>(f[i]);
+      }
+    } else
 #pragma unroll
     for (int e = 0; e < E; ++e) {
       const int d = c + e;
@@ -443,7 +454,29 @@ __device__ __forceinline__ void load_rows(float* lds, int ld, int Lp, int n, con
   }
 }
 
-template <int NT>  // 16-column tiles of the result per wave
+// A tile of SK cache rows through registers: NL 16-byte pieces per thread.
+template <int NL>
+struct CacheTile {
+  f32x4_t v[NL];
+  __device__ void load(const float* src, int L, int l4, int left) {
+#pragma unroll
+    for (int u = 0; u < NL; ++u) {
+      const int x = threadIdx.x + u * 256, r = x / l4, c = (x - r * l4) * 4;
+      v[u] = r < left && r < SK && c < L ? *reinterpret_cast<const f32x4_t*>(src + (size_t)r * L + c) : f32x4_t{0.f, 0.f, 0.f, 0.f};
+    }
+  }
+  __device__ void store(float* lds, int ld, int l4) const {
+#pragma unroll
+    for (int u = 0; u < NL; ++u) {
+      const int x = threadIdx.x + u * 256, r = x / l4, c = (x - r * l4) * 4;
+      if (r < SK) *reinterpret_cast<f32x4_t*>(lds + r * ld + c) = v[u];
+    }
+  }
+};
+
+// NT: 16-column tiles of the result per wave; NL > 0: rows of L % 4 == 0 elements in NL pieces per thread, the next tile on its way
+// while this one is multiplied
+template <int NT, int NL>
 __global__ void __launch_bounds__(256) latent_split_kernel(SplitArgs a) {
   extern __shared__ __attribute__((aligned(16))) float sl[];
   const int ld = split_row(a.L), Lp = (a.L + 15) & ~15;
@@ -456,15 +489,22 @@ __global__ void __launch_bounds__(256) latent_split_kernel(SplitArgs a) {
   float* arow = lrow + 16;
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, j = lane & 15, g = lane >> 4;
   const int r0 = blockIdx.x * 16, split = blockIdx.y;
+  const int k_begin = split * a.tiles_per_split * SK, k_stop = min(a.keys, k_begin + a.tiles_per_split * SK);
+  CacheTile<NL ? NL : 1> ahead;
+  if constexpr (NL != 0) ahead.load(a.cache + (size_t)k_begin * a.L, a.L, Lp / 4, k_stop - k_begin);
   load_rows(Qs, ld, Lp, 16, a.qa + (size_t)r0 * a.L, a.L, a.rows - r0);
   if (threadIdx.x < 16) mrow[threadIdx.x] = -INFINITY, lrow[threadIdx.x] = 0.f;
   f32x4_t acc[NT];
 #pragma unroll
   for (int i = 0; i < NT; ++i) acc[i] = f32x4_t{0.f, 0.f, 0.f, 0.f};
-  const int k_begin = split * a.tiles_per_split * SK, k_stop = min(a.keys, k_begin + a.tiles_per_split * SK);
   for (int k0 = k_begin; k0 < k_stop; k0 += SK) {
     __syncthreads();
-    load_rows(Ks, ld, Lp, SK, a.cache + (size_t)k0 * a.L, a.L, k_stop - k0);
+    if constexpr (NL != 0) {
+      ahead.store(Ks, ld, Lp / 4);
+      if (k0 + SK < k_stop) ahead.load(a.cache + (size_t)(k0 + SK) * a.L, a.L, Lp / 4, k_stop - k0 - SK);
+    } else {
+      load_rows(Ks, ld, Lp, SK, a.cache + (size_t)k0 * a.L, a.L, k_stop - k0);
+    }
     __syncthreads();
     {  // wave: 16 keys (wave % 2), every other run of 16 elements (wave / 2)
       f32x4_t s = {0.f, 0.f, 0.f, 0.f};
@@ -545,6 +585,14 @@ __global__ void __launch_bounds__(256) latent_merge_kernel(const float* __restri
   __shared__ float fac[SPLITS_MAX];
   const int h = blockIdx.x, i = blockIdx.y, v0 = blockIdx.z * MERGE_V, row = i * heads + h;
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  f32x4_t held[MERGE_V / 4][2];  // the first 512 elements of the wave's matrix rows, asked for before anything else
+#pragma unroll
+  for (int u = 0; u < MERGE_V / 4; ++u)
+#pragma unroll
+    for (int b = 0; b < 2; ++b) {
+      const int v = v0 + wave + 4 * u, c = b * 256 + lane * 4;
+      held[u][b] = v < vdim && c < rank ? load4<V4>(w + ((size_t)h * vdim + v) * rank + c, rank - c) : f32x4_t{0.f, 0.f, 0.f, 0.f};
+    }
   if (wave == 0) {
     const float m = lane < splits ? ml[((size_t)lane * rows + row) * 2] : -INFINITY, l = lane < splits ? ml[((size_t)lane * rows + row) * 2 + 1] : 0.f;
     float top = m;
@@ -571,13 +619,13 @@ __global__ void __launch_bounds__(256) latent_merge_kernel(const float* __restri
     const WT* wr = w + ((size_t)h * vdim + v) * rank;
     float s = 0.f;
     for (int c = lane * 4; c < rank; c += 256) {
-      const f32x4_t a = load4<V4>(wr + c, rank - c), b = *reinterpret_cast<const f32x4_t*>(lat + c);
+      const f32x4_t a = c < 256 ? held[u][0] : c < 512 ? held[u][1] : load4<V4>(wr + c, rank - c), b = *reinterpret_cast<const f32x4_t*>(lat + c);
       s += a.x * b.x;
       s += a.y * b.y;
       s += a.z * b.z;
       s += a.w * b.w;
     }
-    for (int d = 32; d; d >>= 1) s += __shfl_xor(s, d, 64);
+    s = wave_sum(s);
     if (lane == 0) dst[(size_t)i * dst_stride + (size_t)h * vdim + v] = s;
   }
 }
@@ -637,6 +685,7 @@ extern "C" int ughip_latent_attention_rows(ughip_device* dev, ughip_view q, cons
   PackArgs pk{};
   pk.q = view_ptr<float>(q), pk.k = k->ptr, pk.cache = buf_ptr<float>(cache), pk.cos = buf_ptr<float>(cos), pk.sin = buf_ptr<float>(sin), pk.q_stride = q.stride;
   pk.t = (int)t, pk.pos = (int)pos, pk.heads = (int)heads, pk.dim = (int)dim, pk.rot = (int)rot, pk.rank = (int)rank;
+  pk.q_vec = (dim + rot) % 4 == 0 && q.stride % 4 == 0 && (reinterpret_cast<uintptr_t>(pk.q) & 15) == 0;
   return k->dtype == UGHIP_BF16 ? launch_rows_any<uint16_t>(dev, a, pk) : launch_rows_any<float>(dev, a, pk);
 }
 
@@ -689,18 +738,18 @@ extern "C" int ughip_latent_attention_absorbed(ughip_device* dev, ughip_view q, 
   UGHIP_HIPCHK(hipGetLastError());
   const dim3 g2((unsigned)row_blocks, (unsigned)splits);
   const size_t lds = split_lds_bytes((int)L);
-  static const hipError_t attr = [] {
-    hipError_t e = hipSuccess;
-    for (const void* f : {reinterpret_cast<const void*>(latent_split_kernel<2>), reinterpret_cast<const void*>(latent_split_kernel<4>),
-                          reinterpret_cast<const void*>(latent_split_kernel<8>), reinterpret_cast<const void*>(latent_split_kernel<16>)})
-      if (e == hipSuccess) e = hipFuncSetAttribute(f, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
-    return e;
-  }();
-  UGHIP_HIPCHK(attr);
-  if (rank <= 128) latent_split_kernel<2><<<g2, 256, lds, dev->stream>>>(a);
-  else if (rank <= 256) latent_split_kernel<4><<<g2, 256, lds, dev->stream>>>(a);
-  else if (rank <= 512) latent_split_kernel<8><<<g2, 256, lds, dev->stream>>>(a);
-  else latent_split_kernel<16><<<g2, 256, lds, dev->stream>>>(a);
+  auto split_go = [&](auto kernel) {
+    if (lds > 64 * 1024)
+      if (hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(kernel), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds); e != hipSuccess) return e;
+    kernel<<<g2, 256, lds, dev->stream>>>(a);
+    return hipSuccess;
+  };
+  const size_t pieces = (size_t)SK * ((L + 15) & ~(size_t)15) / 4;  // 16-byte pieces of a tile
+  const int nl = L % 4 ? 0 : pieces <= 6 * 256 ? 6 : pieces <= 12 * 256 ? 12 : pieces <= 20 * 256 ? 20 : 0;
+  if (rank <= 128) UGHIP_HIPCHK(nl == 6 ? split_go(latent_split_kernel<2, 6>) : split_go(latent_split_kernel<2, 0>));
+  else if (rank <= 256) UGHIP_HIPCHK(nl && nl <= 12 ? split_go(latent_split_kernel<4, 12>) : split_go(latent_split_kernel<4, 0>));
+  else if (rank <= 512) UGHIP_HIPCHK(nl ? split_go(latent_split_kernel<8, 20>) : split_go(latent_split_kernel<8, 0>));
+  else UGHIP_HIPCHK(split_go(latent_split_kernel<16, 0>));
   UGHIP_HIPCHK(hipGetLastError());
   const dim3 g3((unsigned)heads, (unsigned)t, (unsigned)((vdim + MERGE_V - 1) / MERGE_V));
   const size_t lds3 = ((rank + 255) & ~(size_t)255) * sizeof(float);

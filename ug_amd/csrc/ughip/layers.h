@@ -6,6 +6,7 @@
 
 #include "internal.h"
 #include "ughip_layers.h"
+#include "wave_ops.h"
 
 namespace ughip {
 
@@ -38,7 +39,8 @@ inline const T* buf_ptr(const ughip_slice* s) {
 }
 
 __device__ __forceinline__ float bf16_to_f32(uint16_t v) { return __uint_as_float((uint32_t)v << 16); }
-__device__ __forceinline__ float silu_f(float z) { return z / (1.f + expf(-z)); }
+// z / (1 + exp(-z)) with the exponential as a power of two and a reciprocal: a few units of the last place
+__device__ __forceinline__ float silu_f(float z) { return z * __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(-1.4426950408889634f * z)); }
 __device__ __forceinline__ float softplus_f(float z) { return z > 20.f ? z + log1pf(expf(-z)) : log1pf(expf(z)); }
 __device__ __forceinline__ float gelu_tanh_f(float z) {
   return 0.5f * z * (1.f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z)));
@@ -48,7 +50,7 @@ __device__ __forceinline__ float gelu_tanh_f(float z) {
 // be used again after the next barrier of the caller.
 template <int WAVES>
 __device__ __forceinline__ float block_sum(float v, float* red) {
-  for (int d = 32; d; d >>= 1) v += __shfl_xor(v, d, 64);
+  v = wave_sum(v);
   if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = v;
   __syncthreads();
   float s = 0.f;

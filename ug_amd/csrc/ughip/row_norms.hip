@@ -102,6 +102,39 @@ int check_result(const ughip_device* dev, const ughip_view& v, size_t m, size_t 
   return UGHIP_OK;
 }
 
+// The same for parts of up to 4096 elements, a multiple of 4, held in registers.
+__global__ void __launch_bounds__(256) gated_rms_norm4_kernel(const float* __restrict__ y, size_t y_stride, const float* __restrict__ z, size_t z_stride,
+                                                              const float* __restrict__ w, float eps, void* __restrict__ dst, size_t dst_stride, bool dst_bf16, int part) {
+  __shared__ float red[4];
+  const size_t i = blockIdx.x, c0 = (size_t)blockIdx.y * part;
+  f32x4_t g[4];
+  float ss = 0.f;
+#pragma unroll
+  for (int u = 0; u < 4; ++u) {
+    const int c = (u * 256 + (int)threadIdx.x) * 4;
+    g[u] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+    if (c >= part) continue;
+    g[u] = *reinterpret_cast<const f32x4_t*>(y + i * y_stride + c0 + c);
+    if (z) {
+      const f32x4_t q = *reinterpret_cast<const f32x4_t*>(z + i * z_stride + c0 + c);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) g[u][e] *= silu_f(q[e]);
+    }
+    ss += g[u].x * g[u].x + g[u].y * g[u].y + g[u].z * g[u].z + g[u].w * g[u].w;
+  }
+  ss = block_sum<4>(ss, red);
+  const float inv = 1.f / sqrtf(ss / (float)part + eps);
+#pragma unroll
+  for (int u = 0; u < 4; ++u) {
+    const int c = (u * 256 + (int)threadIdx.x) * 4;
+    if (c >= part) continue;
+    const f32x4_t v = g[u] * inv * *reinterpret_cast<const f32x4_t*>(w + c0 + c);
+    const size_t at = i * dst_stride + c0 + c;
+    if (dst_bf16) *reinterpret_cast<ushort4*>(static_cast<uint16_t*>(dst) + at) = make_ushort4(bf16_rne(v.x), bf16_rne(v.y), bf16_rne(v.z), bf16_rne(v.w));
+    else *reinterpret_cast<f32x4_t*>(static_cast<float*>(dst) + at) = v;
+  }
+}
+
 constexpr size_t ROW_MAX = 16000;  // the row and the reduction fit the 64 KiB a launch gets without asking
 
 }  // namespace
@@ -169,6 +202,13 @@ extern "C" int ughip_gated_rms_norm_rows(ughip_device* dev, ughip_view y, ughip_
   if (m == 0 || n == 0) return UGHIP_OK;
   if (int rc = device_activate(dev)) return rc;
   const size_t part = n / groups;
+  auto a16 = [](const void* q) { return (reinterpret_cast<uintptr_t>(q) & 15) == 0; };
+  if (part % 4 == 0 && part <= 4096 && y.stride % 4 == 0 && (!z.s || z.stride % 4 == 0) && dst.stride % 4 == 0 && a16(view_ptr<float>(y)) && a16(view_ptr<float>(z)) && a16(d)) {
+    gated_rms_norm4_kernel<<<dim3((unsigned)m, (unsigned)groups), 256, 0, dev->stream>>>(view_ptr<float>(y), y.stride, view_ptr<float>(z), z.stride, buf_ptr<float>(w), eps, d,
+                                                                                         dst.stride, bf16, (int)part);
+    UGHIP_HIPCHK(hipGetLastError());
+    return UGHIP_OK;
+  }
   gated_rms_norm_kernel<<<dim3((unsigned)m, (unsigned)groups), 256, part * sizeof(float), dev->stream>>>(view_ptr<float>(y), y.stride, view_ptr<float>(z), z.stride,
                                                                                                         buf_ptr<float>(w), eps, d, dst.stride, bf16, (int)part);
   UGHIP_HIPCHK(hipGetLastError());

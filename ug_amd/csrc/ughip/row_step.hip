@@ -1,10 +1,12 @@
 // Products of one row with their neighbours folded in (ughip_product_row): a decode step of the layers in ughip_layers.h.
 //
 // A workgroup of four waves takes 4 R columns, R per wave.  It asks for everything the input row is made of (PV 16-byte pieces per
-// thread and vector), then every wave for the first PRE runs of 512 elements of its matrix rows (eight elements per lane and run);
+// thread and vector), then every wave for the first NB batches of four runs of 512 elements of its matrix rows (eight elements per
+// lane and run);
 // the row -- residual add with the norm of the sublayer in front, gate, norm -- is made in LDS in the shadow of the matrix, and
-// every wave multiplies.  The input row costs a few cache reads per workgroup and spares the launches that would make it; the
-// first workgroup stores the new residual.  PV = 0: rows of any length and alignment, element by element.
+// every wave multiplies, asking for batch b + NB where batch b was.  The input row costs a few cache reads per workgroup and spares the launches that would make it; the
+// first workgroup stores the new residual.  PLAIN: the row is x as it is (or, routed, times the experts' weights).  PV = 0: rows of any
+// length and alignment, element by element.
 #include <hip/hip_runtime.h>
 
 #include "layers.h"
@@ -27,7 +29,7 @@ struct RowArgs {
   const void* table;
   const int* ids;
   size_t table_stride, table_col, w_group;
-  float eps;
+  float eps, inv_k;
   int n, k, cols, norm_groups, table_rows, segs;
   bool table_bf16;
   const float* logits;
@@ -36,7 +38,7 @@ struct RowArgs {
   float* route_weights;
 };
 
-constexpr int RUN = 512;
+constexpr int RUN = 512, PRE = 4;
 
 template <typename WT>
 struct Eight;
@@ -90,24 +92,33 @@ struct Eight<float> {
   }
 };
 
-// R columns of NM matrices per wave; VEC: rows are 16-byte aligned and a multiple of 8 long.  ROUTE as in ughip_row_step.
-template <typename WT, int R, int NM, int ROUTE, bool VEC, int PRE, int PV>
+// R columns of NM matrices per wave; VEC: rows are 16-byte aligned and a multiple of 8 long.  ROUTE as in ughip_row_step: with 2 a
+// column's row is the chosen experts' rows one after the other, each from a batch of its own on.
+template <typename WT, int R, int NM, int ROUTE, bool VEC, int NB, int PV, bool PLAIN>
 __global__ void __launch_bounds__(256) row_step_kernel(RowArgs a) {
-  extern __shared__ __attribute__((aligned(16))) float in[];  // the row, then ROUTE 1: logits and the choice's work space
+  extern __shared__ __attribute__((aligned(16))) float in[];  // the row (segments `padded` apart), then ROUTE 1: logits and work space
   __shared__ float red[4][4];
+  __shared__ float part_sum[4 * (PV ? PV : 1)];
   __shared__ int s_ids[64];
+  __shared__ float s_wts[64];
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
-  const int total = ROUTE == 2 ? a.segs * a.k : a.k;  // elements of the input row
-  const int padded = (total + RUN - 1) / RUN * RUN;
+  const int padded = (a.k + RUN - 1) / RUN * RUN, bps = (padded / RUN + PRE - 1) / PRE, batches = (ROUTE == 2 ? a.segs : 1) * bps;
   const int col0 = (blockIdx.x * 4 + wave) * R;
   constexpr int NP = PV ? PV : 1;
   const f32x4_t zero = {0.f, 0.f, 0.f, 0.f};
+  const int total = (ROUTE == 2 ? a.segs : 1) * a.k;
   f32x4_t px[NP], py[NP], pyn[NP], pn[NP];  // x, y or the gate, and the two norms' weights
-  if constexpr (PV != 0) {
+  if constexpr (PV != 0 && PLAIN) {
 #pragma unroll
     for (int u = 0; u < PV; ++u) {
       const int i = (u * 256 + (int)threadIdx.x) * 4;
-      const bool ok = i < total;  // a multiple of 4
+      px[u] = i < total ? *reinterpret_cast<const f32x4_t*>(a.x + i) : zero;
+    }
+  } else if constexpr (PV != 0) {
+#pragma unroll
+    for (int u = 0; u < PV; ++u) {
+      const int i = (u * 256 + (int)threadIdx.x) * 4;
+      const bool ok = i < a.k;  // a multiple of 4
       px[u] = ok ? *reinterpret_cast<const f32x4_t*>(a.x + i) : zero;
       py[u] = ok && (a.y || a.gate) ? *reinterpret_cast<const f32x4_t*>((a.y ? a.y : a.gate) + i) : zero;
       pyn[u] = ok && a.y ? *reinterpret_cast<const f32x4_t*>(a.y_norm + i) : zero;
@@ -132,6 +143,7 @@ __global__ void __launch_bounds__(256) row_step_kernel(RowArgs a) {
     if (threadIdx.x < (unsigned)a.segs) {
       const int e = a.route_ids[threadIdx.x];
       s_ids[threadIdx.x] = e >= 0 && e < a.route.experts ? e : 0;
+      s_wts[threadIdx.x] = a.route_weights[threadIdx.x];
     }
     __syncthreads();
   }
@@ -150,40 +162,55 @@ __global__ void __launch_bounds__(256) row_step_kernel(RowArgs a) {
     rows[0][r] = static_cast<const WT*>(a.w) + at;
     if (NM == 2) rows[NM - 1][r] = static_cast<const WT*>(a.w) + at + (size_t)a.n * a.k;  // gate rows, then up rows
   }
-  // eight elements from `kk` on of a row (ROUTE 2: of the segments' rows one after the other)
-  auto fetch = [&](Eight<WT>& e, const WT* row, bool ok, int kk) {
-    e.clear();
-    if (!ok || kk >= total) return;
-    if constexpr (ROUTE == 2) {
-      if constexpr (VEC) {
-        const int j = kk / a.k;
-        e.load(row + (size_t)s_ids[j] * a.w_group + (kk - j * a.k));
-      } else {
-        WT t[8];
+  Eight<WT> held[NB][NM][R][PRE];
+  int fj = 0, fc = 0;  // the next batch to ask for: segment and batch inside it
+  auto fetch = [&](Eight<WT>(&to)[NM][R][PRE]) {
+    const size_t seg = ROUTE == 2 && fj < a.segs ? (size_t)s_ids[fj] * a.w_group : 0;
+    const bool more = ROUTE == 2 ? fj < a.segs : fc < bps;
 #pragma unroll
-        for (int i = 0; i < 8; ++i) {
-          const int q = kk + i, j = q < total ? q / a.k : 0;
-          t[i] = q < total ? row[(size_t)s_ids[j] * a.w_group + (q - j * a.k)] : WT(0);
+    for (int c = 0; c < PRE; ++c) {
+      const int kk = (fc * PRE + c) * RUN + lane * 8;
+#pragma unroll
+      for (int r = 0; r < R; ++r)
+#pragma unroll
+        for (int m = 0; m < NM; ++m) {
+          Eight<WT>& e = to[m][r][c];
+          e.clear();
+          if (!more || !live[r] || kk >= a.k) continue;
+          if constexpr (VEC) e.load(rows[m][r] + seg + kk);
+          else e.load_some(rows[m][r] + seg + kk, a.k - kk);
         }
-        e.load_some(t, 8);
-      }
-    } else {
-      if constexpr (VEC) e.load(row + kk);
-      else e.load_some(row + kk, total - kk);
     }
+    if (ROUTE == 2 && fc + 1 == bps) ++fj, fc = 0;
+    else ++fc;
   };
-  Eight<WT> pre[NM][R][PRE];
 #pragma unroll
-  for (int c = 0; c < PRE; ++c)
-#pragma unroll
-    for (int r = 0; r < R; ++r)
-#pragma unroll
-      for (int m = 0; m < NM; ++m) fetch(pre[m][r][c], rows[m][r], live[r], c * RUN + lane * 8);
+  for (int b = 0; b < NB; ++b) fetch(held[b]);
   __builtin_amdgcn_sched_barrier(0);
 
   // the input row
   float ss = 0.f;
-  if constexpr (PV != 0) {
+  if constexpr (PV != 0 && PLAIN) {
+#pragma unroll
+    for (int u = 0; u < PV; ++u) {
+      const int i = (u * 256 + (int)threadIdx.x) * 4;
+      if constexpr (ROUTE == 2) {
+        // (i + 1/2) / k is never within a rounding of a whole number
+        const int j = (int)(((float)i + 0.5f) * a.inv_k);
+        if (i < total) *reinterpret_cast<f32x4_t*>(in + j * padded + (i - j * a.k)) = px[u] * s_wts[j];
+      } else {
+        if (i < padded) *reinterpret_cast<f32x4_t*>(in + i) = px[u];
+      }
+    }
+    if constexpr (ROUTE == 2)
+      for (int j = 0; j < a.segs; ++j)
+        for (int i = a.k + (int)threadIdx.x; i < padded; i += 256) in[j * padded + i] = 0.f;
+  } else if constexpr (ROUTE == 2) {
+    for (int j = 0; j < a.segs; ++j) {
+      const float w = s_wts[j];
+      for (int i = threadIdx.x; i < padded; i += 256) in[j * padded + i] = i < a.k ? a.x[j * a.k + i] * w : 0.f;
+    }
+  } else if constexpr (PV != 0) {
     auto square = [](const f32x4_t& v) { return v.x * v.x + v.y * v.y + v.z * v.z + v.w * v.w; };
     if (a.y) {
 #pragma unroll
@@ -194,20 +221,13 @@ __global__ void __launch_bounds__(256) row_step_kernel(RowArgs a) {
       for (int u = 0; u < PV; ++u) {
         px[u] = px[u] + py[u] * inv * pyn[u];
         const int i = (u * 256 + (int)threadIdx.x) * 4;
-        if (a.x_out && blockIdx.x == 0 && i < total) *reinterpret_cast<f32x4_t*>(a.x_out + i) = px[u];
+        if (a.x_out && blockIdx.x == 0 && i < a.k) *reinterpret_cast<f32x4_t*>(a.x_out + i) = px[u];
       }
     } else if (a.gate) {
 #pragma unroll
       for (int u = 0; u < PV; ++u)
 #pragma unroll
         for (int e = 0; e < 4; ++e) px[u][e] *= silu_f(py[u][e]);
-    }
-    if (ROUTE == 2) {
-#pragma unroll
-      for (int u = 0; u < PV; ++u) {
-        const int i = (u * 256 + (int)threadIdx.x) * 4;
-        if (i < total) px[u] *= a.route_weights[i / a.k];  // a.k is a multiple of 4
-      }
     }
     if (a.norm && a.norm_groups == 1) {
       ss = 0.f;
@@ -217,6 +237,22 @@ __global__ void __launch_bounds__(256) row_step_kernel(RowArgs a) {
       const float inv = 1.f / sqrtf(ss / (float)a.k + a.eps);
 #pragma unroll
       for (int u = 0; u < PV; ++u) px[u] = px[u] * inv * pn[u];
+    } else if (a.norm) {
+      // parts of whole runs of 256 elements (the host checks): one wave's pieces each
+      const int runs = a.k / a.norm_groups / 256;
+#pragma unroll
+      for (int u = 0; u < PV; ++u) {
+        const float s = wave_sum(square(px[u]));
+        if (lane == 0) part_sum[u * 4 + wave] = s;
+      }
+      __syncthreads();
+#pragma unroll
+      for (int u = 0; u < PV; ++u) {
+        const int first = (u * 4 + wave) / runs * runs;
+        float s = 0.f;
+        for (int i = 0; i < runs && first + i < 4 * PV; ++i) s += part_sum[first + i];
+        px[u] = px[u] * (1.f / sqrtf(s / (float)(runs * 256) + a.eps)) * pn[u];
+      }
     }
 #pragma unroll
     for (int u = 0; u < PV; ++u) {
@@ -226,10 +262,9 @@ __global__ void __launch_bounds__(256) row_step_kernel(RowArgs a) {
   } else {
     for (int i = threadIdx.x; i < padded; i += 256) {
       float v = 0.f;
-      if (i < total) {
+      if (i < a.k) {
         v = a.y ? a.y[i] : a.x[i];
         if (a.gate) v *= silu_f(a.gate[i]);
-        if (ROUTE == 2) v *= a.route_weights[i / a.k];
       }
       in[i] = v;  // read back by the same thread until the last barrier
       ss += v * v;
@@ -238,7 +273,7 @@ __global__ void __launch_bounds__(256) row_step_kernel(RowArgs a) {
       ss = block_sum<4>(ss, red[0]);
       const float inv = 1.f / sqrtf(ss / (float)a.k + a.eps);
       ss = 0.f;
-      for (int i = threadIdx.x; i < total; i += 256) {
+      for (int i = threadIdx.x; i < a.k; i += 256) {
         const float v = a.x[i] + in[i] * inv * a.y_norm[i];
         in[i] = v;
         ss += v * v;
@@ -248,18 +283,17 @@ __global__ void __launch_bounds__(256) row_step_kernel(RowArgs a) {
     if (a.norm && a.norm_groups == 1) {
       ss = block_sum<4>(ss, red[1]);
       const float inv = 1.f / sqrtf(ss / (float)a.k + a.eps);
-      for (int i = threadIdx.x; i < total; i += 256) in[i] *= inv * a.norm[i];
-    }
-  }
-  if (a.norm && a.norm_groups > 1) {
-    const int part = a.k / a.norm_groups;
-    __syncthreads();  // a part is summed by one wave
-    for (int g = wave; g < a.norm_groups; g += 4) {
-      float s = 0.f;
-      for (int i = lane; i < part; i += 64) s += in[g * part + i] * in[g * part + i];
-      for (int d = 32; d; d >>= 1) s += __shfl_xor(s, d, 64);
-      const float inv = 1.f / sqrtf(s / (float)part + a.eps);
-      for (int i = lane; i < part; i += 64) in[g * part + i] *= inv * a.norm[g * part + i];
+      for (int i = threadIdx.x; i < a.k; i += 256) in[i] *= inv * a.norm[i];
+    } else if (a.norm) {
+      const int part = a.k / a.norm_groups;
+      __syncthreads();  // a part is summed by one wave
+      for (int g = wave; g < a.norm_groups; g += 4) {
+        float s = 0.f;
+        for (int i = lane; i < part; i += 64) s += in[g * part + i] * in[g * part + i];
+        s = wave_sum(s);
+        const float inv = 1.f / sqrtf(s / (float)part + a.eps);
+        for (int i = lane; i < part; i += 64) in[g * part + i] *= inv * a.norm[g * part + i];
+      }
     }
   }
   __syncthreads();
@@ -269,38 +303,36 @@ __global__ void __launch_bounds__(256) row_step_kernel(RowArgs a) {
   for (int m = 0; m < NM; ++m)
 #pragma unroll
     for (int r = 0; r < R; ++r) acc[m][r] = 0.f;
-  const int runs = padded / RUN;
-#pragma unroll
-  for (int c = 0; c < PRE; ++c) {
-    if (c >= runs) break;
-    const f32x4_t xa = *reinterpret_cast<const f32x4_t*>(in + c * RUN + lane * 8), xb = *reinterpret_cast<const f32x4_t*>(in + c * RUN + lane * 8 + 4);
-#pragma unroll
-    for (int r = 0; r < R; ++r)
-#pragma unroll
-      for (int m = 0; m < NM; ++m) acc[m][r] = pre[m][r][c].dot(xa, xb, acc[m][r]);
-  }
-  for (int c0 = PRE; c0 < runs; c0 += PRE) {
-#pragma unroll
-    for (int c = 0; c < PRE; ++c)
-#pragma unroll
-      for (int r = 0; r < R; ++r)
-#pragma unroll
-        for (int m = 0; m < NM; ++m) fetch(pre[m][r][c], rows[m][r], live[r], (c0 + c) * RUN + lane * 8);
+  int dj = 0, dc = 0;  // the batch to multiply
+  auto multiply = [&](const Eight<WT>(&from)[NM][R][PRE]) {
+    const float* row = in + dj * padded + dc * PRE * RUN + lane * 8;
+    const int left = padded / RUN - dc * PRE;
 #pragma unroll
     for (int c = 0; c < PRE; ++c) {
-      if (c0 + c >= runs) break;
-      const f32x4_t xa = *reinterpret_cast<const f32x4_t*>(in + (c0 + c) * RUN + lane * 8), xb = *reinterpret_cast<const f32x4_t*>(in + (c0 + c) * RUN + lane * 8 + 4);
+      if (c < left) {
+        const f32x4_t xa = *reinterpret_cast<const f32x4_t*>(row + c * RUN), xb = *reinterpret_cast<const f32x4_t*>(row + c * RUN + 4);
 #pragma unroll
-      for (int r = 0; r < R; ++r)
+        for (int r = 0; r < R; ++r)
 #pragma unroll
-        for (int m = 0; m < NM; ++m) acc[m][r] = pre[m][r][c].dot(xa, xb, acc[m][r]);
+          for (int m = 0; m < NM; ++m) acc[m][r] = from[m][r][c].dot(xa, xb, acc[m][r]);
+      }
+    }
+    if (ROUTE == 2 && dc + 1 == bps) ++dj, dc = 0;
+    else ++dc;
+  };
+  for (int b0 = 0; b0 < batches; b0 += NB) {
+#pragma unroll
+    for (int b = 0; b < NB; ++b) {
+      if (b0 + b < batches) {
+        multiply(held[b]);
+        if (b0 + b + NB < batches) fetch(held[b]);
+      }
     }
   }
 #pragma unroll
   for (int r = 0; r < R; ++r) {
 #pragma unroll
-    for (int m = 0; m < NM; ++m)
-      for (int d = 32; d; d >>= 1) acc[m][r] += __shfl_xor(acc[m][r], d, 64);
+    for (int m = 0; m < NM; ++m) acc[m][r] = wave_sum(acc[m][r]);
     if (lane != 0 || !live[r]) continue;
     const int col = col0 + r;
     float v = acc[0][r];
@@ -322,11 +354,11 @@ __global__ void __launch_bounds__(256) row_step_kernel(RowArgs a) {
   }
 }
 
-template <typename WT, int R, int NM, int ROUTE, bool VEC, int PRE, int PV>
+template <typename WT, int R, int NM, int ROUTE, bool VEC, int NB, int PV, bool PLAIN>
 hipError_t launch_one(hipStream_t st, const RowArgs& a, size_t lds) {
   const unsigned grid = (unsigned)((a.cols + 4 * R - 1) / (4 * R));
-  auto kernel = row_step_kernel<WT, R, NM, ROUTE, VEC, PRE, PV>;
-  if (lds > 64 * 1024)
+  auto kernel = row_step_kernel<WT, R, NM, ROUTE, VEC, NB, PV, PLAIN>;
+  if (lds > 60 * 1024)
     if (hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(kernel), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds); e != hipSuccess) return e;
   kernel<<<grid, 256, lds, st>>>(a);
   return hipGetLastError();
@@ -335,13 +367,18 @@ hipError_t launch_one(hipStream_t st, const RowArgs& a, size_t lds) {
 // pieces: the input row is read 16 bytes at a time
 template <typename WT, int R, int NM, int ROUTE>
 hipError_t launch_vec(hipStream_t st, const RowArgs& a, size_t lds, bool vec, bool pieces) {
+  if (!vec) return launch_one<WT, R, NM, ROUTE, false, 1, 0, false>(st, a, lds);
   const int total = (ROUTE == 2 ? a.segs : 1) * a.k;
-  if (!vec) return launch_one<WT, R, NM, ROUTE, false, 4, 0>(st, a, lds);
-  if (!pieces || total > 8192) return launch_one<WT, R, NM, ROUTE, true, 4, 0>(st, a, lds);
-  constexpr bool ROOM = R * NM * sizeof(WT) <= 4;  // registers for twelve runs of every row
-  if (total <= 2048) return launch_one<WT, R, NM, ROUTE, true, 4, 2>(st, a, lds);
-  if (total <= 4096) return launch_one<WT, R, NM, ROUTE, true, ROOM ? 8 : 4, 4>(st, a, lds);
-  return launch_one<WT, R, NM, ROUTE, true, ROOM ? 12 : 4, 8>(st, a, lds);
+  if (pieces && !a.y && !a.gate && !a.norm && total <= 8192) {
+    if constexpr (ROUTE != 2)
+      if (total <= 2048) return launch_one<WT, R, NM, ROUTE, true, 1, 2, true>(st, a, lds);
+    return launch_one<WT, R, NM, ROUTE, true, 2, 8, true>(st, a, lds);
+  }
+  if constexpr (ROUTE != 2) {
+    if (pieces && a.k <= 2048) return launch_one<WT, R, NM, ROUTE, true, 1, 2, false>(st, a, lds);
+    if (pieces && a.k <= 4096) return launch_one<WT, R, NM, ROUTE, true, 2, 4, false>(st, a, lds);
+  }
+  return launch_one<WT, R, NM, ROUTE, true, 2, 0, false>(st, a, lds);
 }
 
 template <typename WT, int NM, int ROUTE>
@@ -370,7 +407,7 @@ extern "C" int ughip_product_row(ughip_device* dev, const ughip_row_step* p) {
   if (p->act < UGHIP_ACT_NONE || p->act > UGHIP_ACT_GELU_MUL || p->route < 0 || p->route > 2) return set_error(UGHIP_ERR_INVALID, "%s: act %d, route %d", what, p->act, p->route);
   if (p->n == 0) return UGHIP_OK;
   const size_t segs = p->route == 2 ? p->top : 1, total = segs * p->k;
-  if (p->k == 0 || p->k > ROW_MAX || segs == 0 || segs > 64 || total > ROW_MAX) return set_error(UGHIP_ERR_UNSUPPORTED, "%s: rows of %zu elements, up to %zu are supported", what, total, ROW_MAX);
+  if (p->k == 0 || p->k > ROW_MAX || segs == 0 || segs > 64 || segs * ((p->k + RUN - 1) / RUN * RUN) > 32 * RUN) return set_error(UGHIP_ERR_UNSUPPORTED, "%s: %zu rows of %zu elements, up to %zu in all (in runs of %d) are supported", what, segs, p->k, (size_t)32 * RUN, RUN);
   if (p->n > 0x7fffffffull / 128) return set_error(UGHIP_ERR_INVALID, "%s: shape too large", what);
   if (p->w->dtype != UGHIP_F32 && p->w->dtype != UGHIP_BF16) return set_error(UGHIP_ERR_UNSUPPORTED, "%s: matrices are F32 or BF16", what);
   const size_t mats = p->route ? p->experts : 1, w_rows = p->act == UGHIP_ACT_SWIGLU ? 2 * p->n : p->n;
@@ -432,8 +469,8 @@ extern "C" int ughip_product_row(ughip_device* dev, const ughip_row_step* p) {
     a.table = p->table->ptr, a.table_bf16 = p->table->dtype == UGHIP_BF16, a.table_rows = (int)p->table_rows;
     a.table_stride = p->table_stride, a.table_col = p->table_col, a.ids = buf_ptr<int>(p->ids);
   }
-  a.w_group = w_rows * p->k, a.eps = p->eps, a.n = (int)p->n, a.k = (int)p->k, a.cols = (int)cols, a.segs = (int)segs;
-  size_t lds = (total + RUN - 1) / RUN * RUN * sizeof(float);
+  a.w_group = w_rows * p->k, a.eps = p->eps, a.inv_k = 1.f / (float)p->k, a.n = (int)p->n, a.k = (int)p->k, a.cols = (int)cols, a.segs = (int)segs;
+  size_t lds = segs * ((p->k + RUN - 1) / RUN * RUN) * sizeof(float);
   if (p->route) {
     a.route = RouteArgs{buf_ptr<float>(p->correction), (int)p->experts, (int)p->groups, (int)p->keep, (int)p->top};
     a.route_ids = static_cast<int*>(p->route_ids->ptr), a.route_weights = static_cast<float*>(p->route_weights->ptr);
@@ -444,7 +481,7 @@ extern "C" int ughip_product_row(ughip_device* dev, const ughip_row_step* p) {
   }
   const bool vec = p->k % 8 == 0 && (reinterpret_cast<uintptr_t>(a.w) & 15) == 0;
   auto a16 = [](const void* q) { return (reinterpret_cast<uintptr_t>(q) & 15) == 0; };
-  const bool pieces = p->k % 4 == 0 && a16(a.x) && a16(a.y) && a16(a.gate) && a16(a.x_out);
+  const bool pieces = p->k % 4 == 0 && (!p->norm || norm_groups == 1 || (p->k / norm_groups) % 256 == 0) && a16(a.x) && a16(a.y) && a16(a.gate) && a16(a.x_out);
   UGHIP_HIPCHK(p->w->dtype == UGHIP_BF16 ? launch_any<uint16_t>(dev->stream, a, p->route, p->act == UGHIP_ACT_SWIGLU, lds, vec, pieces)
                                          : launch_any<float>(dev->stream, a, p->route, p->act == UGHIP_ACT_SWIGLU, lds, vec, pieces));
   return UGHIP_OK;

@@ -169,24 +169,31 @@ __global__ void __launch_bounds__(256) rows_product_kernel(ProductArgs a) {
 #pragma unroll
       for (int e = 0; e < 16; ++e) acc[i][j][e] = 0.f;
 
-  Raw<CT, XT> xr[XC];
-  Raw<CT, WT> wr[WC];
+  // steps on their way in registers: the small tile's are short, one would not cover the way from memory
+  constexpr int DEPTH = MI * NI == 1 ? 3 : 1;
+  Raw<CT, XT> xr[DEPTH][XC];
+  Raw<CT, WT> wr[DEPTH][WC];
   const int ck = (tid & 7) * CE;
-  auto fetch = [&](int k0) {
+  auto fetch = [&](int d, int k0) {
 #pragma unroll
-    for (int i = 0; i < XC; ++i) xr[i] = load_chunk<CT, XT, VEC>(xrow[i], k0 + ck, a.k, xok[i]);
+    for (int i = 0; i < XC; ++i) xr[d][i] = load_chunk<CT, XT, VEC>(xrow[i], k0 + ck, a.k, xok[i]);
 #pragma unroll
-    for (int i = 0; i < WC; ++i) wr[i] = load_chunk<CT, WT, VEC>(wrow[i], k0 + ck, a.k, wok[i]);
+    for (int i = 0; i < WC; ++i) wr[d][i] = load_chunk<CT, WT, VEC>(wrow[i], k0 + ck, a.k, wok[i]);
   };
-  fetch(0);
   const int steps = (a.k + KE - 1) / KE;
-  for (int s = 0; s < steps; ++s) {
+#pragma unroll
+  for (int d = 0; d < DEPTH; ++d) fetch(d, d * KE);  // (past the end: zeros)
+  for (int s0 = 0; s0 < steps; s0 += DEPTH)
+#pragma unroll
+   for (int d = 0; d < DEPTH; ++d) {
+    const int s = s0 + d;
+    if (s >= steps) break;
     char* buf = lds[s & 1];
 #pragma unroll
-    for (int i = 0; i < XC; ++i) *reinterpret_cast<u32x4_t*>(buf + ((tid >> 3) + 32 * i) * ROW_BYTES + (tid & 7) * 16) = xr[i].pack();
+    for (int i = 0; i < XC; ++i) *reinterpret_cast<u32x4_t*>(buf + ((tid >> 3) + 32 * i) * ROW_BYTES + (tid & 7) * 16) = xr[d][i].pack();
 #pragma unroll
-    for (int i = 0; i < WC; ++i) *reinterpret_cast<u32x4_t*>(buf + (BM + (tid >> 3) + 32 * i) * ROW_BYTES + (tid & 7) * 16) = wr[i].pack();
-    if (s + 1 < steps) fetch((s + 1) * KE);
+    for (int i = 0; i < WC; ++i) *reinterpret_cast<u32x4_t*>(buf + (BM + (tid >> 3) + 32 * i) * ROW_BYTES + (tid & 7) * 16) = wr[d][i].pack();
+    if (s + DEPTH < steps) fetch(d, (s + DEPTH) * KE);
     __syncthreads();  // (one barrier a step: the buffer written two steps from now is read before the next barrier)
     const char* xa = buf + (wm * 32 * MI + (lane & 31)) * ROW_BYTES + (lane >> 5) * 16;
     const char* wa = buf + (BM + wn * 32 * NI + (lane & 31)) * ROW_BYTES + (lane >> 5) * 16;
@@ -202,7 +209,7 @@ __global__ void __launch_bounds__(256) rows_product_kernel(ProductArgs a) {
 #pragma unroll
         for (int j = 0; j < NI; ++j) mfma_chunk<CT>(fx[i], fw[j], acc[i][j]);
     }
-  }
+   }
 
   // element e of an accumulator: row 8 (e / 4) + 4 (lane / 32) + e % 4, column lane % 32
 #pragma unroll
