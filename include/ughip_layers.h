@@ -32,7 +32,8 @@ int ughip_gather_rows(ughip_device* dev, const ughip_slice* table, size_t table_
 /* ---- products of rows ---------------------------------------------------------------------------------------------------
  * dst = act(x w^T + bias), any m, n, k.  `product`:
  *   UGHIP_PRODUCT_F32   x and w F32, the f32 matrix pipe;
- *   UGHIP_PRODUCT_BF16  x and w rounded to (or stored as) bf16, the bf16 matrix pipe, f32 accumulation.
+ *   UGHIP_PRODUCT_BF16  x and w rounded to (or stored as) bf16, the bf16 matrix pipe, f32 accumulation.  (2 .. 128 dense F32 rows
+ *                       against a BF16 matrix of regular sizes keep their F32 values: the kernels of ughip_linear_rows.)
  * x, w and dst may each be F32 or BF16 (F32 only for UGHIP_PRODUCT_F32).  BF16 rows and matrices of regular sizes take the
  * one-wave-per-SIMD kernel of ughip_matmul, the rest one that takes any size (ughip_last_kernel names it).
  * `act`:

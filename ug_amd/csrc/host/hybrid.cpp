@@ -47,6 +47,10 @@ LB scratch(DType dtype, size_t n, const DevicePtr& dev) {
   return lb;
 }
 
+// From kHalfRows positions on the stream is kept as bf16 rows too, for the products of bf16 matrices; plain products of up to
+// kFewRows positions are better off with the f32 rows (they share their K among workgroups).
+constexpr size_t kHalfRows = 33, kFewRows = 128;
+
 struct Product {
   LB w, bias;  // UGHIP_ACT_SWIGLU: gate rows then up rows
   size_t n = 0, k = 0;
@@ -124,10 +128,11 @@ void settle(StepContext& c, Stream& s) {
 
 // A product of the (settled) stream's rows, in the form the step's products read.
 LB stream_product(const StepContext& c, const Stream& s, const Product& p, DType out_type = DType::F32) {
-  if (s.x16.valid()) return product_rows({s.x16, 0, c.width}, c.t, p, s.x.lb, out_type);
+  if (s.x16.valid() && (c.t > kFewRows || p.act == UGHIP_ACT_SWIGLU)) return product_rows({s.x16, 0, c.width}, c.t, p, s.x.lb, out_type);
   return product_rows(s.x, c.t, p, LB(), out_type);
 }
-DType half_type(const StepContext& c) { return c.half_rows ? DType::BF16 : DType::F32; }
+// What a producer of rows that only a product reads writes.
+DType half_type(const StepContext& c) { return c.half_rows && c.t > kFewRows ? DType::BF16 : DType::F32; }
 
 // One position: a product of one row with what stands in front of it folded in (ughip_product_row).
 struct RowStep {
@@ -182,9 +187,6 @@ LB stream_step(StepContext& c, Stream& s, RowStep r, size_t* at) {
   }
   return out;
 }
-
-// From this many positions on, products of bf16 matrices read rows that their producers wrote as bf16.
-constexpr size_t kHalfRows = 96;
 
 // ---- loading --------------------------------------------------------------------------------------------------------------
 struct Loader {

@@ -64,6 +64,10 @@ int rows_scratch(ughip_device* dev, size_t bytes, void** out);
 bool rows_add_product_reads_planes(ughip_device* dev, const ughip_slice* w, const void* x, const void* residual, const void* dst, size_t m, size_t n, size_t k, int product);
 int rows_add_product_from(ughip_device* dev, const char* what, const float* x, const uint16_t* planes, const ughip_slice* w, const float* residual, float* dst, size_t m,
                           size_t n, size_t k, int product);
+// dst [m, n] = x w^T on dense f32 rows and a BF16 matrix through the kernels of ughip_linear_rows: up to 32 rows on the f32 pipe, up to
+// 128 as three bf16 terms.  false: not their shapes (nothing is launched).
+bool few_rows_product_fits(const ughip_slice* w, const float* x, const float* dst, size_t m, size_t n, size_t k);
+int few_rows_product(ughip_device* dev, const char* what, const float* x, const ughip_slice* w, float* dst, size_t m, size_t n, size_t k);
 const char* dtype_name(int dt);
 
 // Tuning switches (tile / split / kernel-family overrides for measurements and tests).  The table is filled once per

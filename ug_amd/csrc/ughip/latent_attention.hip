@@ -507,15 +507,17 @@ __global__ void __launch_bounds__(256) latent_split_kernel(SplitArgs a) {
     }
     __syncthreads();
     {  // wave: 16 keys (wave % 2), every other run of 16 elements (wave / 2)
-      f32x4_t s = {0.f, 0.f, 0.f, 0.f};
+      f32x4_t s = {0.f, 0.f, 0.f, 0.f}, s2 = s;  // two chains
       const int kb = (wave & 1) * 16;
+#pragma unroll 3
       for (int c = (wave >> 1) * 16; c < Lp; c += 32) {
         const f32x4_t x = *reinterpret_cast<const f32x4_t*>(Qs + j * ld + c + 4 * g), y = *reinterpret_cast<const f32x4_t*>(Ks + (kb + j) * ld + c + 4 * g);
         s = __builtin_amdgcn_mfma_f32_16x16x4f32(x.x, y.x, s, 0, 0, 0);
-        s = __builtin_amdgcn_mfma_f32_16x16x4f32(x.y, y.y, s, 0, 0, 0);
+        s2 = __builtin_amdgcn_mfma_f32_16x16x4f32(x.y, y.y, s2, 0, 0, 0);
         s = __builtin_amdgcn_mfma_f32_16x16x4f32(x.z, y.z, s, 0, 0, 0);
-        s = __builtin_amdgcn_mfma_f32_16x16x4f32(x.w, y.w, s, 0, 0, 0);
+        s2 = __builtin_amdgcn_mfma_f32_16x16x4f32(x.w, y.w, s2, 0, 0, 0);
       }
+      s += s2;
 #pragma unroll
       for (int e = 0; e < 4; ++e) Sp[((wave >> 1) * 16 + 4 * g + e) * S_ROW + kb + j] = s[e];
     }
@@ -583,6 +585,7 @@ __global__ void __launch_bounds__(256) latent_merge_kernel(const float* __restri
                                                            size_t dst_stride, int rows, int splits, int heads, int rank, int vdim) {
   extern __shared__ __attribute__((aligned(16))) float lat[];  // [rank], zeros up to a multiple of 256
   __shared__ float fac[SPLITS_MAX];
+  __shared__ f32x4_t part[256];
   const int h = blockIdx.x, i = blockIdx.y, v0 = blockIdx.z * MERGE_V, row = i * heads + h;
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   f32x4_t held[MERGE_V / 4][2];  // the first 512 elements of the wave's matrix rows, asked for before anything else
@@ -603,13 +606,32 @@ __global__ void __launch_bounds__(256) latent_merge_kernel(const float* __restri
     fac[lane] = f / sum;
   }
   __syncthreads();
-  for (int c = threadIdx.x; c < ((rank + 255) & ~255); c += 256) {
-    float v = 0.f;
-    if (c < rank) {
-#pragma unroll 8
-      for (int s = 0; s < splits; ++s) v += fac[s] * acc[((size_t)s * rows + row) * rank + c];
+  const int padded = (rank + 255) & ~255;
+  const float* mine = acc + (size_t)row * rank;
+  const size_t step = (size_t)rows * rank;
+  if (V4 && rank <= 1024) {
+    // four columns per thread, the splits dealt to as many threads per column as there are
+    const int nc = padded / 4, share = 256 / nc, c = (threadIdx.x % nc) * 4, g = threadIdx.x / nc;  // nc: 64, 128, 192 or 256
+    f32x4_t v = {0.f, 0.f, 0.f, 0.f};
+    if (c < rank && g < share) {
+#pragma unroll 16
+      for (int s = g; s < splits; s += share) v += *reinterpret_cast<const f32x4_t*>(mine + s * step + c) * fac[s];
     }
-    lat[c] = v;
+    part[threadIdx.x] = v;
+    __syncthreads();
+    if (g == 0) {
+      for (int k = 1; k < share; ++k) v += part[k * nc + threadIdx.x];
+      *reinterpret_cast<f32x4_t*>(lat + c) = v;
+    }
+  } else {
+    for (int c = threadIdx.x; c < padded; c += 256) {
+      float v = 0.f;
+      if (c < rank) {
+#pragma unroll 16
+        for (int s = 0; s < splits; ++s) v += fac[s] * mine[s * step + c];
+      }
+      lat[c] = v;
+    }
   }
   __syncthreads();
 #pragma unroll

@@ -1096,4 +1096,14 @@ int rows_add_product_from(ughip_device* dev, const char* what, const float* x, c
   return linear_rows_core(dev, what, x, w, residual, dst, m, n, k, GemmEpilogue::ADD, product, &ar);
 }
 
+bool few_rows_product_fits(const ughip_slice* w, const float* x, const float* dst, size_t m, size_t n, size_t k) {
+  if (w->dtype != UGHIP_BF16 || m < 2 || m > 128 || k % 64 != 0 || n % 8 != 0 || n == 0 || n > 0x7fffffffull || k > 0x7fffffffull / 3) return false;
+  const bool x3 = m > 32;
+  return gemm_tiled_supported(x3 ? UGHIP_BF16 : UGHIP_F32, rows_args(x, w->ptr, const_cast<float*>(dst), m, n, k, x3), 1, !x3);
+}
+
+int few_rows_product(ughip_device* dev, const char* what, const float* x, const ughip_slice* w, float* dst, size_t m, size_t n, size_t k) {
+  return linear_rows_core(dev, what, x, w, nullptr, dst, m, n, k, GemmEpilogue::NONE, m > 32 ? UGHIP_PRODUCT_BF16X3 : UGHIP_PRODUCT_F32, nullptr);
+}
+
 }  // namespace ughip

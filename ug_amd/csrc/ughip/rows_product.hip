@@ -337,6 +337,10 @@ extern "C" int ughip_product_rows(ughip_device* dev, const ughip_product* p) {
   a.row_index = buf_ptr<int>(p->row_index), a.group_end = buf_ptr<int>(p->group_end), a.groups = (int)p->groups, a.x_rows = (int)x_rows;
   const bool vec = p->k % 8 == 0 && (p->x.stride * xs) % 16 == 0 && (w_stride * (p->w->dtype == UGHIP_BF16 ? 2 : 4)) % 16 == 0 && aligned16(a.x) && aligned16(a.w);
   const bool xb = p->x.s->dtype == UGHIP_BF16, wb = p->w->dtype == UGHIP_BF16;
+  // few dense rows: products that share their K among workgroups
+  if (!f32 && !xb && wb && !a.dst_bf16 && p->act == UGHIP_ACT_NONE && !a.bias && !a.groups && p->x.stride == p->k && p->dst.stride == p->n && w_stride == p->k &&
+      few_rows_product_fits(p->w, static_cast<const float*>(a.x), static_cast<const float*>(a.dst), p->m, p->n, p->k))
+    return few_rows_product(dev, what, static_cast<const float*>(a.x), p->w, static_cast<float*>(a.dst), p->m, p->n, p->k);
   if (xb && wb && p->act != UGHIP_ACT_GELU_MUL && p->m >= DMA_ROWS_MIN) {
     MMArgs q;
     q.a = a.x, q.b = a.w, q.c = nullptr;

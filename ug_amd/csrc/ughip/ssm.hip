@@ -3,6 +3,7 @@
 //   S_t = exp(a_t) S_{t-1} + d_t B_t x_t^T,   y_t = S_t^T C_t + skip x_t,   a_t = -exp(a_log) d_t, d_t = softplus(dt_t + bias)
 //
 // Several positions run in chunks of Q.  With A_i = a_1 + .. + a_i inside a chunk:
+//   ssm_chunk_decays  d_i and A_i
 //   ssm_chunk_state   what a chunk adds to the state: sum_j B_j (exp(A_Q - A_j) d_j x_j)^T
 //   ssm_chunk_scan    the state in front of every chunk, S <- exp(A_Q) S + that, in place              (elementwise, chunks in order)
 //   ssm_chunk_out     y_i = sum_{j <= i} exp(A_i - A_j) d_j (C_i . B_j) x_j + exp(A_i) S^T C_i + skip x_i
@@ -26,7 +27,8 @@ struct SsmArgs {
   const float* skip;
   float* s;        // [heads, state, vdim]
   float* chunk_s;  // [chunks, heads, state, vdim]
-  float* decay;    // [chunks, heads]: exp(A_Q)
+  float* cum;      // [chunks, heads, 64]: A_i, and
+  float* step;     // d_i (0 past the last row, where A_i stays)
   float* dst;
   size_t xbc_stride, dt_stride, dst_stride;
   int t, heads, vdim, groups, state, q, chunks;
@@ -94,9 +96,10 @@ __global__ void __launch_bounds__(256) conv_ring_store_kernel(const float* __res
   ring[(size_t)((pos + i) % n_taps) * channels + c] = x[(size_t)i * x_stride + c];
 }
 
-// cum[i] = A_i and d[i] for the chunk's rows, rows past the end with d = 0 and the last A.  One wave (q <= 64).
-__device__ __forceinline__ void chunk_decays(const SsmArgs& a, int h, int row0, float* cum, float* d) {
-  const int i = threadIdx.x & 63;
+// One wave per chunk and head (q <= 64).
+__global__ void __launch_bounds__(256) ssm_chunk_decays_kernel(SsmArgs a) {
+  const int i = threadIdx.x & 63, h = blockIdx.y * 4 + (threadIdx.x >> 6), row0 = blockIdx.x * a.q;
+  if (h >= a.heads) return;
   float dv = 0.f;
   if (i < a.q && row0 + i < a.t) dv = softplus_f(a.dt[(size_t)(row0 + i) * a.dt_stride + h] + a.dt_bias[h]);
   float s = -expf(a.a_log[h]) * dv;
@@ -104,7 +107,8 @@ __device__ __forceinline__ void chunk_decays(const SsmArgs& a, int h, int row0, 
     const float o = __shfl_up(s, k, 64);
     if (i >= k) s += o;
   }
-  cum[i] = s, d[i] = dv;
+  const size_t at = ((size_t)blockIdx.x * a.heads + h) * 64 + i;
+  a.cum[at] = s, a.step[at] = dv;
 }
 
 __device__ __forceinline__ f32x4_t mfma16(float x, float y, f32x4_t acc) { return __builtin_amdgcn_mfma_f32_16x16x4f32(x, y, acc, 0, 0, 0); }
@@ -193,27 +197,26 @@ __global__ void __launch_bounds__(256) ssm_chunk_state_kernel(SsmArgs a) {
   extern __shared__ __attribute__((aligned(16))) float lds[];
   const int q = a.q, chunk = blockIdx.x, row0 = chunk * q, rows = min(q, a.t - row0), N = a.state, ns = row_n(N), np = pad16(N), inner = a.heads * a.vdim;
   const HeadWalk hw(a);
-  float* cum = lds;
-  float* d = lds + 64;
-  float* wgt = lds + 128;
-  float* Bs = lds + 192;      // [q][ns]
+  float* wgt = lds;
+  float* Bs = lds + 64;       // [q][ns]
   float* Xs = Bs + q * ns;    // [q][PS]
   const float* xbc0 = a.xbc + (size_t)row0 * a.xbc_stride;
   tile_to_lds<VEC>(Bs, ns, xbc0 + inner + (size_t)hw.g * N, a.xbc_stride, rows, N, np / 4, q * np / 4);
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, j = lane & 15, kg = lane >> 4, tn = np / 16, xt = q * PB / 4;
   TileRegs<4, VEC> x;
-  auto fetch = [&](int i) { x.load(xbc0 + (size_t)hw.head(i) * a.vdim + hw.col(i), a.xbc_stride, rows, min(PB, a.vdim - hw.col(i)), PB / 4, xt); };
+  float weight = 0.f;  // of row `lane` (first wave)
+  auto fetch = [&](int i) {
+    x.load(xbc0 + (size_t)hw.head(i) * a.vdim + hw.col(i), a.xbc_stride, rows, min(PB, a.vdim - hw.col(i)), PB / 4, xt);
+    if (wave == 0) {
+      const size_t at = ((size_t)chunk * a.heads + hw.head(i)) * 64;
+      weight = a.step[at + lane] * expf(a.cum[at + 63] - a.cum[at + lane]);
+    }
+  };
   if (hw.items) fetch(0);
   for (int it = 0; it < hw.items; ++it) {
     const int h = hw.head(it), p0 = hw.col(it), pw = min(PB, a.vdim - p0);
     __syncthreads();
-    if (wave == 0) {
-      chunk_decays(a, h, row0, cum, d);
-      __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "workgroup");  // one wave's own LDS writes, read back below
-      __builtin_amdgcn_wave_barrier();
-      if (lane < q) wgt[lane] = d[lane] * expf(cum[q - 1] - cum[lane]);
-      if (lane == 0 && p0 == 0) a.decay[(size_t)chunk * a.heads + h] = expf(cum[q - 1]);
-    }
+    if (wave == 0) wgt[lane] = weight;
     __syncthreads();
     x.store(Xs, PS, PB / 4, xt, wgt);
     if (it + 1 < hw.items) fetch(it + 1);
@@ -258,7 +261,7 @@ __global__ void __launch_bounds__(256) ssm_chunk_scan_kernel(SsmArgs a) {
     float* at = a.chunk_s + ((size_t)c * a.heads + h) * per + e;
     const float add = *at;
     *at = s;
-    s = a.decay[(size_t)c * a.heads + h] * s + add;
+    s = expf(a.cum[((size_t)c * a.heads + h) * 64 + 63]) * s + add;
   }
   a.s[h * per + e] = s;
 }
@@ -276,13 +279,25 @@ __global__ void __launch_bounds__(256) ssm_chunk_out_kernel(SsmArgs a) {
   float* Xs = Bs;             // [q][PS]
   float* Ss = Xs + q * PS;    // [np][PS]
   const float* xbc0 = a.xbc + (size_t)row0 * a.xbc_stride;
-  tile_to_lds<VEC>(Bs, ns, xbc0 + inner + (size_t)hw.g * N, a.xbc_stride, rows, N, np / 4, q * np / 4);
-  tile_to_lds<VEC>(Cs, ns, xbc0 + inner + (size_t)(a.groups + hw.g) * N, a.xbc_stride, rows, N, np / 4, q * np / 4);
+  const float *b_src = xbc0 + inner + (size_t)hw.g * N, *c_src = xbc0 + inner + (size_t)(a.groups + hw.g) * N;
+  const int bt = q * np / 4;
+  if (bt <= 8 * 256) {
+    TileRegs<8, VEC> b, c;  // both on their way at once
+    b.load(b_src, a.xbc_stride, rows, N, np / 4, bt);
+    c.load(c_src, a.xbc_stride, rows, N, np / 4, bt);
+    b.store(Bs, ns, np / 4, bt);
+    c.store(Cs, ns, np / 4, bt);
+  } else {
+    tile_to_lds<VEC>(Bs, ns, b_src, a.xbc_stride, rows, N, np / 4, bt);
+    tile_to_lds<VEC>(Cs, ns, c_src, a.xbc_stride, rows, N, np / 4, bt);
+  }
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, j = lane & 15, kg = lane >> 4, tq = q / 16, i0 = wave * 16, xt = q * PB / 4, st = np * PB / 4;
   TileRegs<4, VEC> x;
   TileRegs<8, VEC> s;
+  float decays = 0.f;  // A of row `lane` (first wave), d of it (second)
   auto fetch = [&](int i) {
     const int pw = min(PB, a.vdim - hw.col(i));
+    if (wave < 2) decays = (wave ? a.step : a.cum)[((size_t)chunk * a.heads + hw.head(i)) * 64 + lane];
     x.load(xbc0 + (size_t)hw.head(i) * a.vdim + hw.col(i), a.xbc_stride, rows, pw, PB / 4, xt);
     s.load(a.chunk_s + ((size_t)chunk * a.heads + hw.head(i)) * N * a.vdim + hw.col(i), a.vdim, N, pw, PB / 4, st);
   };
@@ -320,7 +335,7 @@ __global__ void __launch_bounds__(256) ssm_chunk_out_kernel(SsmArgs a) {
       const int r0 = base / (PB / 4);
       tile_to_lds<VEC>(Ss + r0 * PS, PS, a.chunk_s + (((size_t)chunk * a.heads + h) * N + r0) * a.vdim + p0, a.vdim, N - r0, pw, PB / 4, min(2048, st - base));
     }
-    if (wave == 0) chunk_decays(a, h, row0, cum, d);
+    if (wave < 2) (wave ? d : cum)[lane] = decays;
     __syncthreads();
     if (it + 1 < hw.items) fetch(it + 1);
     if (wave >= tq) continue;  // q < 64: the waves without rows only move data
@@ -440,7 +455,7 @@ __global__ void __launch_bounds__(256) ssm_step_kernel(SsmStepArgs a) {
   }
 }
 
-size_t state_lds_bytes(int q, int state) { return (size_t)(192 + q * row_n(state) + q * PS) * sizeof(float); }
+size_t state_lds_bytes(int q, int state) { return (size_t)(64 + q * row_n(state) + q * PS) * sizeof(float); }
 size_t out_lds_bytes(int q, int state) {
   const size_t b = (size_t)q * row_n(state), xs = (size_t)(q + pad16(state)) * PS;
   return (128 + (size_t)q * row_n(state) + (size_t)q * (q + 4) + (b > xs ? b : xs)) * sizeof(float);
@@ -504,11 +519,11 @@ extern "C" int ughip_ssm_rows(ughip_device* dev, ughip_view xbc, ughip_view dt, 
   while (q > 16 && (out_lds_bytes(q, (int)state) > 160 * 1024 || (size_t)(q / 2) >= t)) q /= 2;
   if (out_lds_bytes(q, (int)state) > 160 * 1024 || state_lds_bytes(q, (int)state) > 160 * 1024) return set_error(UGHIP_ERR_UNSUPPORTED, "ssm_rows: a state of %zu rows does not fit LDS", state);
   if (int rc = device_activate(dev)) return rc;
-  const size_t chunks = (t + q - 1) / q, elems = state * vdim, decay_bytes = (chunks * heads * sizeof(float) + 255) & ~(size_t)255;
+  const size_t chunks = (t + q - 1) / q, elems = state * vdim, n_decay = chunks * heads * 64;
   void* ws = nullptr;
-  if (int rc = rows_scratch(dev, decay_bytes + chunks * heads * elems * sizeof(float), &ws)) return rc;
+  if (int rc = rows_scratch(dev, (2 * n_decay + chunks * heads * elems) * sizeof(float), &ws)) return rc;
   SsmArgs a{view_ptr<float>(xbc), view_ptr<float>(dt), buf_ptr<float>(dt_bias), buf_ptr<float>(a_log), buf_ptr<float>(skip), static_cast<float*>(s->ptr),
-            reinterpret_cast<float*>(static_cast<char*>(ws) + decay_bytes), static_cast<float*>(ws), view_ptr<float>(dst), xbc.stride, dt.stride, dst.stride,
+            static_cast<float*>(ws) + 2 * n_decay, static_cast<float*>(ws), static_cast<float*>(ws) + n_decay, view_ptr<float>(dst), xbc.stride, dt.stride, dst.stride,
             (int)t, (int)heads, (int)vdim, (int)groups, (int)state, q, (int)chunks, pos == 0};
   // a group's heads share a workgroup unless the chip would stay empty
   const size_t per = heads / groups;
@@ -525,6 +540,7 @@ extern "C" int ughip_ssm_rows(ughip_device* dev, ughip_view xbc, ughip_view dt, 
   }();
   UGHIP_HIPCHK(attr);
   const size_t lds_s = state_lds_bytes(q, (int)state), lds_o = out_lds_bytes(q, (int)state);
+  ssm_chunk_decays_kernel<<<dim3((unsigned)chunks, (unsigned)((heads + 3) / 4)), 256, 0, dev->stream>>>(a);
   if (vec) ssm_chunk_state_kernel<true><<<grid, 256, lds_s, dev->stream>>>(a);
   else ssm_chunk_state_kernel<false><<<grid, 256, lds_s, dev->stream>>>(a);
   ssm_chunk_scan_kernel<<<dim3((unsigned)((elems + 255) / 256), (unsigned)heads), 256, 0, dev->stream>>>(a);
