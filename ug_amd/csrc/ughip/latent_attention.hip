@@ -187,21 +187,20 @@ __global__ void __launch_bounds__(256) latent_rows_kernel(RowsArgs a) {
     for (int u = 0; u < NK; ++u) kr[u] = *reinterpret_cast<const u32x4_t*>(k_head + (size_t)k0 * DQ * sizeof(T) + (threadIdx.x + u * 256) * 16);
 #pragma unroll
     for (int u = 0; u < NV; ++u) {
-      const int x = threadIdx.x + u * 256, vc = x / VC, kp = k0 + x % VC * E;
-      u32x4_t chunk = {0, 0, 0, 0};
-      if (vc < a.vdim && kp < s_all) {
-        const T* p = v_head + (size_t)vc * a.v_stride + kp;
-        if (kp + E <= s_all) {
-          chunk = *reinterpret_cast<const u32x4_t*>(p);  // rows are padded to whole tiles and 16-byte aligned
-        } else {  // values past the last position were never written
-          T v[E];
-#pragma unroll
-          for (int e = 0; e < E; ++e) v[e] = kp + e < s_all ? p[e] : T(0);
-          __builtin_memcpy(&chunk, v, 16);
-        }
-      }
-      vr[u] = chunk;
+      // rows are padded to whole tiles and 16-byte aligned; every lane loads (no branches between loads)
+      const int x = threadIdx.x + u * 256, vc = x / VC;
+      vr[u] = *reinterpret_cast<const u32x4_t*>(v_head + (size_t)(vc < a.vdim ? vc : 0) * a.v_stride + k0 + x % VC * E);
     }
+  };
+  // what of a piece of values is none: columns past the last one, positions past the last one (never written)
+  auto value_piece = [&](const u32x4_t& piece, int vc, int kp) {
+    T v[E];
+    __builtin_memcpy(v, &piece, 16);
+#pragma unroll
+    for (int e = 0; e < E; ++e) v[e] = vc < a.vdim && kp + e < s_all ? v[e] : T(0);
+    u32x4_t out;
+    __builtin_memcpy(&out, v, 16);
+    return out;
   };
   if (AHEAD) fetch(0);
   for (int k0 = 0; k0 < keys; k0 += KT) {
@@ -215,7 +214,8 @@ __global__ void __launch_bounds__(256) latent_rows_kernel(RowsArgs a) {
 #pragma unroll
     for (int u = 0; u < NV; ++u) {
       const int x = threadIdx.x + u * 256;
-      *reinterpret_cast<u32x4_t*>(Vs + x / VC * V_ROW + x % VC * 16) = vr[u];
+      const bool whole = k0 + KT <= s_all && DV == a.vdim;
+      *reinterpret_cast<u32x4_t*>(Vs + x / VC * V_ROW + x % VC * 16) = whole ? vr[u] : value_piece(vr[u], x / VC, k0 + x % VC * E);
     }
     __syncthreads();
     if (AHEAD && k0 + KT < keys) fetch(k0 + KT);
@@ -458,18 +458,21 @@ __device__ __forceinline__ void load_rows(float* lds, int ld, int Lp, int n, con
 template <int NL>
 struct CacheTile {
   f32x4_t v[NL];
+  int rows;
   __device__ void load(const float* src, int L, int l4, int left) {
+    rows = left;
 #pragma unroll
     for (int u = 0; u < NL; ++u) {
       const int x = threadIdx.x + u * 256, r = x / l4, c = (x - r * l4) * 4;
-      v[u] = r < left && r < SK && c < L ? *reinterpret_cast<const f32x4_t*>(src + (size_t)r * L + c) : f32x4_t{0.f, 0.f, 0.f, 0.f};
+      const bool ok = r < left && r < SK && c < L;
+      v[u] = *reinterpret_cast<const f32x4_t*>(src + (ok ? (size_t)r * L + c : 0));  // every lane loads: no branches between loads
     }
   }
-  __device__ void store(float* lds, int ld, int l4) const {
+  __device__ void store(float* lds, int ld, int L, int l4) const {
 #pragma unroll
     for (int u = 0; u < NL; ++u) {
       const int x = threadIdx.x + u * 256, r = x / l4, c = (x - r * l4) * 4;
-      if (r < SK) *reinterpret_cast<f32x4_t*>(lds + r * ld + c) = v[u];
+      if (r < SK) *reinterpret_cast<f32x4_t*>(lds + r * ld + c) = r < rows && c < L ? v[u] : f32x4_t{0.f, 0.f, 0.f, 0.f};
     }
   }
 };
@@ -500,7 +503,7 @@ __global__ void __launch_bounds__(256) latent_split_kernel(SplitArgs a) {
   for (int k0 = k_begin; k0 < k_stop; k0 += SK) {
     __syncthreads();
     if constexpr (NL != 0) {
-      ahead.store(Ks, ld, Lp / 4);
+      ahead.store(Ks, ld, a.L, Lp / 4);
       if (k0 + SK < k_stop) ahead.load(a.cache + (size_t)(k0 + SK) * a.L, a.L, Lp / 4, k_stop - k0 - SK);
     } else {
       load_rows(Ks, ld, Lp, SK, a.cache + (size_t)k0 * a.L, a.L, k_stop - k0);

@@ -165,8 +165,8 @@ __global__ void __launch_bounds__(256) row_step_kernel(RowArgs a) {
   Eight<WT> held[NB][NM][R][PRE];
   int fj = 0, fc = 0;  // the next batch to ask for: segment and batch inside it
   auto fetch = [&](Eight<WT>(&to)[NM][R][PRE]) {
-    const size_t seg = ROUTE == 2 && fj < a.segs ? (size_t)s_ids[fj] * a.w_group : 0;
-    const bool more = ROUTE == 2 ? fj < a.segs : fc < bps;
+    if (ROUTE == 2 ? fj >= a.segs : fc >= bps) return;  // the same for the whole workgroup
+    const size_t seg = ROUTE == 2 ? (size_t)s_ids[fj] * a.w_group : 0;
 #pragma unroll
     for (int c = 0; c < PRE; ++c) {
       const int kk = (fc * PRE + c) * RUN + lane * 8;
@@ -175,10 +175,10 @@ __global__ void __launch_bounds__(256) row_step_kernel(RowArgs a) {
 #pragma unroll
         for (int m = 0; m < NM; ++m) {
           Eight<WT>& e = to[m][r][c];
-          e.clear();
-          if (!more || !live[r] || kk >= a.k) continue;
-          if constexpr (VEC) e.load(rows[m][r] + seg + kk);
-          else e.load_some(rows[m][r] + seg + kk, a.k - kk);
+          // every lane loads (past the row's end: its first elements, which meet zeros): with branches around loads the compiler
+          // waits for all of them at once
+          if constexpr (VEC) e.load(rows[m][r] + seg + (kk < a.k ? kk : 0));
+          else e.load_some(rows[m][r] + seg + kk, live[r] ? a.k - kk : 0);
         }
     }
     if (ROUTE == 2 && fc + 1 == bps) ++fj, fc = 0;

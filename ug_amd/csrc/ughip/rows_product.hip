@@ -2,9 +2,9 @@
 // x / w / result as F32 or BF16, bias, SwiGLU or gated-lookup epilogues, and the grouped form (rows sorted by expert, a
 // matrix per group, rows of x gathered on their way in).
 //
-// A workgroup of four waves (2 x 2) takes a 64 MI x 64 NI tile.  A K step is 128 bytes of every row in LDS: 64 bf16 or 32
-// floats, in eight 16-byte chunks; rows are 144 bytes apart, which spreads the 16-byte reads of 32 consecutive rows over all
-// banks.  Two LDS buffers: while one step is multiplied the next one's elements are in flight to registers.  Whatever type
+// A workgroup of four waves (2 x 2) takes a 64 MI x 64 NI tile.  A K step is 128 bytes of every row in LDS (256 for the smallest
+// tile), in 16-byte chunks; rows are 16 bytes further apart than they are long, which spreads the 16-byte reads of consecutive
+// rows over all banks.  Two LDS buffers: while one step is multiplied the next ones' elements are in flight to registers.  Whatever type
 // the operands are stored in, they are converted between registers and LDS; the products are v_mfma_f32_32x32x16_bf16 or, for
 // F32, four v_mfma_f32_32x32x2_f32 per chunk (k taken chunk by chunk: lanes 0-31 the even, lanes 32-63 the odd one).
 #include <hip/hip_runtime.h>
@@ -40,15 +40,15 @@ struct ProductArgs {
   int groups, x_rows;
 };
 
-constexpr int ROW_BYTES = 144, CHUNKS = 8;
-
 // One 16-byte LDS chunk's worth of a row, as it is stored: 8 elements for bf16 products, 4 for f32 ones.
 template <typename CT, typename ST>
 struct Raw;
 template <>
 struct Raw<__bf16, float> {
   f32x4_t a, b;
+  bool ok;
   __device__ u32x4_t pack() const {
+    if (!ok) return u32x4_t{0, 0, 0, 0};
     const f32x8 v = {a.x, a.y, a.z, a.w, b.x, b.y, b.z, b.w};
     return __builtin_bit_cast(u32x4_t, __builtin_convertvector(v, bf16x8));
   }
@@ -56,30 +56,35 @@ struct Raw<__bf16, float> {
 template <>
 struct Raw<__bf16, uint16_t> {
   u32x4_t a;
-  __device__ u32x4_t pack() const { return a; }
+  bool ok;
+  __device__ u32x4_t pack() const { return ok ? a : u32x4_t{0, 0, 0, 0}; }
 };
 template <>
 struct Raw<float, float> {
   f32x4_t a;
-  __device__ u32x4_t pack() const { return __builtin_bit_cast(u32x4_t, a); }
+  bool ok;
+  __device__ u32x4_t pack() const { return ok ? __builtin_bit_cast(u32x4_t, a) : u32x4_t{0, 0, 0, 0}; }
 };
 
 template <typename CT, typename ST, bool VEC>
 __device__ __forceinline__ Raw<CT, ST> load_chunk(const ST* row, int k0, int k, bool ok) {
   constexpr int E = sizeof(CT) == 2 ? 8 : 4;
   Raw<CT, ST> r;
-  if constexpr (VEC) {  // k is a multiple of 8 and rows are 16-byte aligned: a chunk is inside or outside as a whole
-    ok = ok && k0 < k;
-    if constexpr (sizeof(CT) == 2 && sizeof(ST) == 4) {
-      r.a = ok ? *reinterpret_cast<const f32x4_t*>(row + k0) : f32x4_t{0.f, 0.f, 0.f, 0.f};
-      r.b = ok ? *reinterpret_cast<const f32x4_t*>(row + k0 + 4) : f32x4_t{0.f, 0.f, 0.f, 0.f};
-    } else if constexpr (sizeof(ST) == 4) {
-      r.a = ok ? *reinterpret_cast<const f32x4_t*>(row + k0) : f32x4_t{0.f, 0.f, 0.f, 0.f};
+  if constexpr (VEC) {
+    // k is a multiple of 8 and rows are 16-byte aligned: a chunk is inside or outside as a whole.  Every lane loads (its row's
+    // first elements where there is nothing of its own; pack() makes that zeros): with branches around loads the compiler waits for
+    // all of them at once.
+    r.ok = ok && k0 < k;
+    const ST* p = row + (k0 < k ? k0 : 0);
+    if constexpr (sizeof(ST) == 4) {
+      r.a = *reinterpret_cast<const f32x4_t*>(p);
+      if constexpr (sizeof(CT) == 2) r.b = *reinterpret_cast<const f32x4_t*>(p + 4);
     } else {
-      r.a = ok ? *reinterpret_cast<const u32x4_t*>(row + k0) : u32x4_t{0, 0, 0, 0};
+      r.a = *reinterpret_cast<const u32x4_t*>(p);
     }
   } else {
     ST v[E];
+    r.ok = true;
 #pragma unroll
     for (int i = 0; i < E; ++i) v[i] = ok && k0 + i < k ? row[k0 + i] : ST(0);
     if constexpr (sizeof(CT) == 2 && sizeof(ST) == 4) {
@@ -109,7 +114,11 @@ __device__ __forceinline__ void mfma_chunk(const u32x4_t& a, const u32x4_t& b, f
 
 template <typename CT, typename XT, typename WT, int MI, int NI, int ACT, bool VEC>
 __global__ void __launch_bounds__(256) rows_product_kernel(ProductArgs a) {
-  constexpr int BM = 64 * MI, BN = 64 * NI, XC = BM / 32, WC = BN / 32, KE = sizeof(CT) == 2 ? 64 : 32, CE = KE / CHUNKS;
+  constexpr int BM = 64 * MI, BN = 64 * NI;
+  // 16-byte chunks of a row per K step (the small tile's steps are twice as long: it has little to do between two barriers), rows in
+  // LDS 16 bytes further apart than they are long, rows a pass of the workgroup covers
+  constexpr int CHUNKS = MI * NI == 1 ? 16 : 8, ROW_BYTES = CHUNKS * 16 + 16, CSH = CHUNKS == 16 ? 4 : 3, RP = 256 / CHUNKS;
+  constexpr int XC = BM / RP, WC = BN / RP, CE = sizeof(CT) == 2 ? 8 : 4, KE = CHUNKS * CE;
   constexpr int COLS = ACT == UGHIP_ACT_SWIGLU ? BN / 2 : BN;  // result columns of a tile
   __shared__ __attribute__((aligned(16))) char lds[2][(BM + BN) * ROW_BYTES];
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, wm = wave >> 1, wn = wave & 1;
@@ -138,7 +147,7 @@ __global__ void __launch_bounds__(256) rows_product_kernel(ProductArgs a) {
   bool wok[WC];
 #pragma unroll
   for (int i = 0; i < XC; ++i) {
-    const int r = m0 + (tid >> 3) + 32 * i;
+    const int r = m0 + (tid >> CSH) + RP * i;
     xok[i] = r < m_end;
     int src = xok[i] ? r : 0;
     if (a.row_index && xok[i]) {
@@ -150,7 +159,7 @@ __global__ void __launch_bounds__(256) rows_product_kernel(ProductArgs a) {
   }
 #pragma unroll
   for (int i = 0; i < WC; ++i) {
-    const int rb = (tid >> 3) + 32 * i;
+    const int rb = (tid >> CSH) + RP * i;
     int col, up = 0;
     if (ACT == UGHIP_ACT_SWIGLU) {  // LDS rows: 32 gate columns, the same 32 of up, the next 32 gate columns, ...
       col = n0 + (rb >> 6) * 32 + (rb & 31);
@@ -170,10 +179,10 @@ __global__ void __launch_bounds__(256) rows_product_kernel(ProductArgs a) {
       for (int e = 0; e < 16; ++e) acc[i][j][e] = 0.f;
 
   // steps on their way in registers: the small tile's are short, one would not cover the way from memory
-  constexpr int DEPTH = MI * NI == 1 ? 3 : 1;
+  constexpr int DEPTH = MI * NI == 1 ? 2 : 1;
   Raw<CT, XT> xr[DEPTH][XC];
   Raw<CT, WT> wr[DEPTH][WC];
-  const int ck = (tid & 7) * CE;
+  const int ck = (tid & (CHUNKS - 1)) * CE;
   auto fetch = [&](int d, int k0) {
 #pragma unroll
     for (int i = 0; i < XC; ++i) xr[d][i] = load_chunk<CT, XT, VEC>(xrow[i], k0 + ck, a.k, xok[i]);
@@ -190,9 +199,9 @@ __global__ void __launch_bounds__(256) rows_product_kernel(ProductArgs a) {
     if (s >= steps) break;
     char* buf = lds[s & 1];
 #pragma unroll
-    for (int i = 0; i < XC; ++i) *reinterpret_cast<u32x4_t*>(buf + ((tid >> 3) + 32 * i) * ROW_BYTES + (tid & 7) * 16) = xr[d][i].pack();
+    for (int i = 0; i < XC; ++i) *reinterpret_cast<u32x4_t*>(buf + ((tid >> CSH) + RP * i) * ROW_BYTES + (tid & (CHUNKS - 1)) * 16) = xr[d][i].pack();
 #pragma unroll
-    for (int i = 0; i < WC; ++i) *reinterpret_cast<u32x4_t*>(buf + (BM + (tid >> 3) + 32 * i) * ROW_BYTES + (tid & 7) * 16) = wr[d][i].pack();
+    for (int i = 0; i < WC; ++i) *reinterpret_cast<u32x4_t*>(buf + (BM + (tid >> CSH) + RP * i) * ROW_BYTES + (tid & (CHUNKS - 1)) * 16) = wr[d][i].pack();
     if (s + DEPTH < steps) fetch(d, (s + DEPTH) * KE);
     __syncthreads();  // (one barrier a step: the buffer written two steps from now is read before the next barrier)
     const char* xa = buf + (wm * 32 * MI + (lane & 31)) * ROW_BYTES + (lane >> 5) * 16;
@@ -212,11 +221,27 @@ __global__ void __launch_bounds__(256) rows_product_kernel(ProductArgs a) {
    }
 
   // element e of an accumulator: row 8 (e / 4) + 4 (lane / 32) + e % 4, column lane % 32
+  auto row_of = [&](int i, int e) { return m0 + wm * 32 * MI + i * 32 + 8 * (e >> 2) + 4 * (lane >> 5) + (e & 3); };
 #pragma unroll
-  for (int i = 0; i < MI; ++i)
+  for (int i = 0; i < MI; ++i) {
+    float factor[16][NI];  // what the gates of these rows multiply: the rows' tokens first, then all of their table elements
+    if constexpr (ACT == UGHIP_ACT_GELU_MUL) {
+      int id[16];
+#pragma unroll
+      for (int e = 0; e < 16; ++e) id[e] = a.ids[min(row_of(i, e), a.m - 1)];
+#pragma unroll
+      for (int e = 0; e < 16; ++e)
+#pragma unroll
+        for (int j = 0; j < NI; ++j) {
+          const bool there = id[e] >= 0 && id[e] < a.table_rows;
+          const size_t at = (size_t)(there ? id[e] : 0) * a.table_stride + a.table_col + min(n0 + wn * 32 * NI + j * 32 + (lane & 31), a.n - 1);
+          const float t = a.table_bf16 ? bf16_to_f32(static_cast<const uint16_t*>(a.table)[at]) : static_cast<const float*>(a.table)[at];
+          factor[e][j] = there ? t : __uint_as_float(0x7fc00000u);
+        }
+    }
 #pragma unroll
     for (int e = 0; e < 16; ++e) {
-      const int r = m0 + wm * 32 * MI + i * 32 + 8 * (e >> 2) + 4 * (lane >> 5) + (e & 3);
+      const int r = row_of(i, e);
       if (r >= m_end) continue;
 #pragma unroll
       for (int j = 0; j < (ACT == UGHIP_ACT_SWIGLU ? 1 : NI); ++j) {
@@ -229,20 +254,13 @@ __global__ void __launch_bounds__(256) rows_product_kernel(ProductArgs a) {
           if (a.bias) u += a.bias[a.n + col];
           v = silu_f(v) * u;
         }
-        if constexpr (ACT == UGHIP_ACT_GELU_MUL) {
-          const int id = a.ids[r];
-          float t = __uint_as_float(0x7fc00000u);
-          if (id >= 0 && id < a.table_rows) {
-            const size_t at = (size_t)id * a.table_stride + a.table_col + col;
-            t = a.table_bf16 ? bf16_to_f32(static_cast<const uint16_t*>(a.table)[at]) : static_cast<const float*>(a.table)[at];
-          }
-          v = gelu_tanh_f(v) * t;
-        }
+        if constexpr (ACT == UGHIP_ACT_GELU_MUL) v = gelu_tanh_f(v) * factor[e][j];
         const size_t at = (size_t)r * a.dst_stride + col;
         if (a.dst_bf16) static_cast<uint16_t*>(a.dst)[at] = bf16_rne(v);
         else static_cast<float*>(a.dst)[at] = v;
       }
     }
+  }
 }
 
 template <typename CT, typename XT, typename WT, int MI, int NI, int ACT>

@@ -123,19 +123,21 @@ __device__ __host__ inline int row_n(int state) { return pad16(state) + 4; }
 template <int N4, bool VEC>
 struct TileRegs {
   f32x4_t v[N4];
+  int n_rows, n_cols;
   __device__ void load(const float* src, size_t stride, int rows, int cols, int width4, int total) {
+    n_rows = rows, n_cols = cols;
 #pragma unroll
     for (int u = 0; u < N4; ++u) {
       const int e = threadIdx.x + u * 256, r = e / width4, c = (e - r * width4) * 4;
-      v[u] = f32x4_t{0.f, 0.f, 0.f, 0.f};
-      if (e >= total || r >= rows) continue;
-      const float* p = src + (size_t)r * stride + c;
-      if (VEC) {
-        if (c < cols) v[u] = *reinterpret_cast<const f32x4_t*>(p);
+      const bool ok = e < total && r < rows;
+      const float* p = src + (size_t)(ok ? r : 0) * stride;
+      if (VEC) {  // every lane loads (store() drops what is not there): with branches around loads the compiler waits for all of them at once
+        v[u] = *reinterpret_cast<const f32x4_t*>(p + (c < cols ? c : 0));
       } else {
+        v[u] = f32x4_t{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
         for (int i = 0; i < 4; ++i)
-          if (c + i < cols) v[u][i] = p[i];
+          if (ok && c + i < cols) v[u][i] = p[c + i];
       }
     }
   }
@@ -146,6 +148,7 @@ struct TileRegs {
       const int e = threadIdx.x + u * 256, r = e / width4, c = (e - r * width4) * 4;
       if (e >= total) continue;
       f32x4_t w = v[u];
+      if (VEC && (r >= n_rows || c >= n_cols)) w = f32x4_t{0.f, 0.f, 0.f, 0.f};
       if (scale) w *= scale[r];
       *reinterpret_cast<f32x4_t*>(lds + r * ld + c) = w;
     }
