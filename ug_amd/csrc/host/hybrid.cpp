@@ -240,6 +240,7 @@ struct LatentAttention : Mixer {
   std::shared_ptr<RopeTables> rope;
   LB down;  // [dq; dkv], or dq alone
   LB dq_norm, kv_norm, uq, uk, uv, o;
+  static constexpr size_t kAbsorbMax = 736;
   // Steps of up to this many positions attend to the latents themselves instead of expanding all of them into keys and values.
   size_t absorb_up_to;
 
@@ -258,7 +259,8 @@ struct LatentAttention : Mixer {
     uv = ld.matrix(p + "uv", {heads * vdim, rank});
     o = ld.matrix(p + "o", {width, heads * vdim});
     absorb_up_to = std::max<size_t>(1, (dim + vdim) / 4);
-    if (dim + rot > 256 || vdim > 256) absorb_up_to = (size_t)-1;  // sizes the expanded kernel is not built for
+    if (rank + rot > kAbsorbMax) absorb_up_to = 0;  // rows too long for the absorbed kernel
+    else if (dim + rot > 256 || vdim > 256) absorb_up_to = (size_t)-1;  // sizes the expanded kernel is not built for
   }
 
   MixerState new_state(size_t capacity) const override {

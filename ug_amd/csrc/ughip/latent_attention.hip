@@ -425,95 +425,84 @@ struct SplitArgs {
   int rows, heads, pos, keys, rank, L, tiles_per_split;
 };
 
-constexpr int SK = 32, S_ROW = SK + 4;
+constexpr int SK = 32, S_ROW = SK + 4, SPLIT_WAVES = 16, SPLIT_PARTS = SPLIT_WAVES / 2;
 __host__ __device__ inline int split_row(int L) { return ((L + 15) & ~15) + 4; }
-inline size_t split_lds_bytes(int L) { return ((size_t)(SK + 16) * split_row(L) + 3 * 16 * S_ROW + 48) * sizeof(float); }
+inline size_t split_lds_bytes(int L) { return ((size_t)(SK + 16) * split_row(L) + SPLIT_PARTS * 16 * S_ROW + 48) * sizeof(float); }
 
-// n rows of L floats (rows from `left` on and columns from L on are zeros) to LDS, eight 16-byte loads per thread on their way at once.
-__device__ __forceinline__ void load_rows(float* lds, int ld, int Lp, int n, const float* src, int L, int left) {
-  if (L % 4 == 0) {
-    const int l4 = Lp / 4, total = n * l4;
-    for (int base = 0; base < total; base += 8 * 256) {
-      f32x4_t v[8];
-#pragma unroll
-      for (int u = 0; u < 8; ++u) {
-        const int x = base + threadIdx.x + u * 256, r = x / l4, c = (x - r * l4) * 4;
-        v[u] = x < total && r < left && c < L ? *reinterpret_cast<const f32x4_t*>(src + (size_t)r * L + c) : f32x4_t{0.f, 0.f, 0.f, 0.f};
-      }
-#pragma unroll
-      for (int u = 0; u < 8; ++u) {
-        const int x = base + threadIdx.x + u * 256, r = x / l4, c = (x - r * l4) * 4;
-        if (x < total) *reinterpret_cast<f32x4_t*>(lds + r * ld + c) = v[u];
-      }
-    }
-  } else {
-    for (int x = threadIdx.x; x < n * Lp; x += 256) {
-      const int r = x / Lp, c = x % Lp;
-      lds[r * ld + c] = r < left && c < L ? src[(size_t)r * L + c] : 0.f;
-    }
-  }
-}
-
-// A tile of SK cache rows through registers: NL 16-byte pieces per thread.
-template <int NL>
-struct CacheTile {
-  f32x4_t v[NL];
+// N rows of L floats (rows from `left` on and columns from L on are zeros) through registers to LDS, a row per wave and turn.
+// NC > 0: rows of L % 4 == 0 elements in NC pieces of 16 bytes per lane, all on their way at once.
+template <int N, int NC>
+struct RowsAhead {
+  static constexpr int TURNS = N / SPLIT_WAVES;
+  f32x4_t v[TURNS][NC ? NC : 1];
+  const float* from;
   int rows;
-  __device__ void load(const float* src, int L, int l4, int left) {
-    rows = left;
+  __device__ void load(const float* src, int L, int left) {
+    from = src, rows = left;
+    if constexpr (NC != 0) {
+      const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
 #pragma unroll
-    for (int u = 0; u < NL; ++u) {
-      const int x = threadIdx.x + u * 256, r = x / l4, c = (x - r * l4) * 4;
-      const bool ok = r < left && r < SK && c < L;
-      v[u] = *reinterpret_cast<const f32x4_t*>(src + (ok ? (size_t)r * L + c : 0));  // every lane loads: no branches between loads
+      for (int u = 0; u < TURNS; ++u)
+#pragma unroll
+        for (int b = 0; b < NC; ++b) {
+          const int r = wave + u * SPLIT_WAVES, c = b * 256 + lane * 4;
+          v[u][b] = *reinterpret_cast<const f32x4_t*>(src + (r < left && c < L ? (size_t)r * L + c : 0));  // every lane loads: no branches between loads
+        }
     }
   }
-  __device__ void store(float* lds, int ld, int L, int l4) const {
+  __device__ void store(float* lds, int ld, int L, int Lp) const {
+    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
 #pragma unroll
-    for (int u = 0; u < NL; ++u) {
-      const int x = threadIdx.x + u * 256, r = x / l4, c = (x - r * l4) * 4;
-      if (r < SK) *reinterpret_cast<f32x4_t*>(lds + r * ld + c) = r < rows && c < L ? v[u] : f32x4_t{0.f, 0.f, 0.f, 0.f};
+    for (int u = 0; u < TURNS; ++u) {
+      const int r = wave + u * SPLIT_WAVES;
+      if constexpr (NC != 0) {
+#pragma unroll
+        for (int b = 0; b < NC; ++b) {
+          const int c = b * 256 + lane * 4;
+          if (c < Lp) *reinterpret_cast<f32x4_t*>(lds + r * ld + c) = r < rows && c < L ? v[u][b] : f32x4_t{0.f, 0.f, 0.f, 0.f};
+        }
+      } else {
+        for (int c = lane; c < Lp; c += 64) lds[r * ld + c] = r < rows && c < L ? from[(size_t)r * L + c] : 0.f;
+      }
     }
   }
 };
 
-// NT: 16-column tiles of the result per wave; NL > 0: rows of L % 4 == 0 elements in NL pieces per thread, the next tile on its way
-// while this one is multiplied
-template <int NT, int NL>
-__global__ void __launch_bounds__(256) latent_split_kernel(SplitArgs a) {
+// NT: 16-column tiles of the result per wave; NC as in RowsAhead, the next tile on its way while this one is multiplied
+template <int NT, int NC>
+__global__ void __launch_bounds__(64 * SPLIT_WAVES) latent_split_kernel(SplitArgs a) {
   extern __shared__ __attribute__((aligned(16))) float sl[];
   const int ld = split_row(a.L), Lp = (a.L + 15) & ~15;
   float* Ks = sl;                     // [SK][ld]
   float* Qs = Ks + SK * ld;           // [16][ld]
-  float* Sp = Qs + 16 * ld;           // [2][16][S_ROW] halves of the scores
-  float* Ps = Sp + 2 * 16 * S_ROW;    // [16][S_ROW]
-  float* mrow = Ps + 16 * S_ROW;      // running maximum, sum, and this tile's factor
+  float* Sp = Qs + 16 * ld;           // [SPLIT_PARTS][16][S_ROW] parts of the scores
+  float* Ps = Sp;                     // [16][S_ROW] weights, in place of the first part
+  float* mrow = Sp + SPLIT_PARTS * 16 * S_ROW;  // running maximum, sum, and this tile's factor
   float* lrow = mrow + 16;
   float* arow = lrow + 16;
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, j = lane & 15, g = lane >> 4;
   const int r0 = blockIdx.x * 16, split = blockIdx.y;
   const int k_begin = split * a.tiles_per_split * SK, k_stop = min(a.keys, k_begin + a.tiles_per_split * SK);
-  CacheTile<NL ? NL : 1> ahead;
-  if constexpr (NL != 0) ahead.load(a.cache + (size_t)k_begin * a.L, a.L, Lp / 4, k_stop - k_begin);
-  load_rows(Qs, ld, Lp, 16, a.qa + (size_t)r0 * a.L, a.L, a.rows - r0);
+  RowsAhead<SK, NC> ahead;
+  {
+    RowsAhead<16, NC> queries;
+    queries.load(a.qa + (size_t)r0 * a.L, a.L, a.rows - r0);
+    ahead.load(a.cache + (size_t)k_begin * a.L, a.L, k_stop - k_begin);
+    queries.store(Qs, ld, a.L, Lp);
+  }
   if (threadIdx.x < 16) mrow[threadIdx.x] = -INFINITY, lrow[threadIdx.x] = 0.f;
   f32x4_t acc[NT];
 #pragma unroll
   for (int i = 0; i < NT; ++i) acc[i] = f32x4_t{0.f, 0.f, 0.f, 0.f};
   for (int k0 = k_begin; k0 < k_stop; k0 += SK) {
     __syncthreads();
-    if constexpr (NL != 0) {
-      ahead.store(Ks, ld, a.L, Lp / 4);
-      if (k0 + SK < k_stop) ahead.load(a.cache + (size_t)(k0 + SK) * a.L, a.L, Lp / 4, k_stop - k0 - SK);
-    } else {
-      load_rows(Ks, ld, Lp, SK, a.cache + (size_t)k0 * a.L, a.L, k_stop - k0);
-    }
+    ahead.store(Ks, ld, a.L, Lp);
+    if (k0 + SK < k_stop) ahead.load(a.cache + (size_t)(k0 + SK) * a.L, a.L, k_stop - k0 - SK);
     __syncthreads();
-    {  // wave: 16 keys (wave % 2), every other run of 16 elements (wave / 2)
+    {  // wave: 16 keys (wave % 2), every SPLIT_PARTS-th run of 16 elements (from wave / 2)
       f32x4_t s = {0.f, 0.f, 0.f, 0.f}, s2 = s;  // two chains
       const int kb = (wave & 1) * 16;
-#pragma unroll 3
-      for (int c = (wave >> 1) * 16; c < Lp; c += 32) {
+      for (int c = (wave >> 1) * 16; c < Lp; c += 16 * SPLIT_PARTS) {
         const f32x4_t x = *reinterpret_cast<const f32x4_t*>(Qs + j * ld + c + 4 * g), y = *reinterpret_cast<const f32x4_t*>(Ks + (kb + j) * ld + c + 4 * g);
         s = __builtin_amdgcn_mfma_f32_16x16x4f32(x.x, y.x, s, 0, 0, 0);
         s2 = __builtin_amdgcn_mfma_f32_16x16x4f32(x.y, y.y, s2, 0, 0, 0);
@@ -525,9 +514,11 @@ __global__ void __launch_bounds__(256) latent_split_kernel(SplitArgs a) {
       for (int e = 0; e < 4; ++e) Sp[((wave >> 1) * 16 + 4 * g + e) * S_ROW + kb + j] = s[e];
     }
     __syncthreads();
-    {  // row 4 wave + g, keys j and j + 16
+    if (wave < 4) {  // row 4 wave + g, keys j and j + 16
       const int r = 4 * wave + g, limit = a.pos + (r0 + r) / a.heads;
-      float s0 = Sp[r * S_ROW + j] + Sp[(16 + r) * S_ROW + j], s1 = Sp[r * S_ROW + j + 16] + Sp[(16 + r) * S_ROW + j + 16];
+      float s0 = 0.f, s1 = 0.f;
+#pragma unroll
+      for (int x = 0; x < SPLIT_PARTS; ++x) s0 += Sp[(x * 16 + r) * S_ROW + j], s1 += Sp[(x * 16 + r) * S_ROW + j + 16];
       if (k0 + j > limit || k0 + j >= k_stop) s0 = -INFINITY;
       if (k0 + j + 16 > limit || k0 + j + 16 >= k_stop) s1 = -INFINITY;
       float top = fmaxf(s0, s1);
@@ -555,7 +546,7 @@ __global__ void __launch_bounds__(256) latent_split_kernel(SplitArgs a) {
     for (int kk = 0; kk < SK / 4; ++kk) pf[kk] = Ps[j * S_ROW + 4 * kk + g];
 #pragma unroll
     for (int i = 0; i < NT; ++i) {
-      const int c0 = (wave + 4 * i) * 16;
+      const int c0 = (wave + SPLIT_WAVES * i) * 16;
       if (c0 >= a.rank) continue;  // uniform over the wave (columns up to Lp exist in LDS)
 #pragma unroll
       for (int e = 0; e < 4; ++e) acc[i][e] *= al[e];
@@ -566,7 +557,7 @@ __global__ void __launch_bounds__(256) latent_split_kernel(SplitArgs a) {
   __syncthreads();
 #pragma unroll
   for (int i = 0; i < NT; ++i) {
-    const int c = (wave + 4 * i) * 16 + j;
+    const int c = (wave + SPLIT_WAVES * i) * 16 + j;
     if (c >= a.rank) continue;
 #pragma unroll
     for (int e = 0; e < 4; ++e) {
@@ -582,31 +573,37 @@ __global__ void __launch_bounds__(256) latent_split_kernel(SplitArgs a) {
 }
 
 // The parts of one (position, head) added up, then 16 elements of the head's result through the values' up-projection.
-constexpr int MERGE_V = 16, SPLITS_MAX = 64;
+constexpr int MERGE_V = 16, MERGE_WAVES = 16, MERGE_THREADS = 64 * MERGE_WAVES, SPLITS_MAX = 128;
 template <typename WT, bool V4>
-__global__ void __launch_bounds__(256) latent_merge_kernel(const float* __restrict__ acc, const float* __restrict__ ml, const WT* __restrict__ w, float* __restrict__ dst,
+__global__ void __launch_bounds__(MERGE_THREADS) latent_merge_kernel(const float* __restrict__ acc, const float* __restrict__ ml, const WT* __restrict__ w, float* __restrict__ dst,
                                                            size_t dst_stride, int rows, int splits, int heads, int rank, int vdim) {
   extern __shared__ __attribute__((aligned(16))) float lat[];  // [rank], zeros up to a multiple of 256
   __shared__ float fac[SPLITS_MAX];
-  __shared__ f32x4_t part[256];
+  __shared__ f32x4_t part[MERGE_THREADS];
   const int h = blockIdx.x, i = blockIdx.y, v0 = blockIdx.z * MERGE_V, row = i * heads + h;
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
-  f32x4_t held[MERGE_V / 4][2];  // the first 512 elements of the wave's matrix rows, asked for before anything else
+  f32x4_t held[MERGE_V / MERGE_WAVES][2];  // the first 512 elements of the wave's matrix rows, asked for before anything else
 #pragma unroll
-  for (int u = 0; u < MERGE_V / 4; ++u)
+  for (int u = 0; u < MERGE_V / MERGE_WAVES; ++u)
 #pragma unroll
     for (int b = 0; b < 2; ++b) {
-      const int v = v0 + wave + 4 * u, c = b * 256 + lane * 4;
+      const int v = v0 + wave + MERGE_WAVES * u, c = b * 256 + lane * 4;
       held[u][b] = v < vdim && c < rank ? load4<V4>(w + ((size_t)h * vdim + v) * rank + c, rank - c) : f32x4_t{0.f, 0.f, 0.f, 0.f};
     }
   if (wave == 0) {
-    const float m = lane < splits ? ml[((size_t)lane * rows + row) * 2] : -INFINITY, l = lane < splits ? ml[((size_t)lane * rows + row) * 2 + 1] : 0.f;
-    float top = m;
+    float m[SPLITS_MAX / 64], l[SPLITS_MAX / 64], top = -INFINITY, sum = 0.f;
+#pragma unroll
+    for (int u = 0; u < SPLITS_MAX / 64; ++u) {
+      const int s = lane + 64 * u;
+      m[u] = s < splits ? ml[((size_t)s * rows + row) * 2] : -INFINITY, l[u] = s < splits ? ml[((size_t)s * rows + row) * 2 + 1] : 0.f;
+      top = fmaxf(top, m[u]);
+    }
     for (int d = 32; d; d >>= 1) top = fmaxf(top, __shfl_xor(top, d, 64));
-    const float f = expf(m - top);
-    float sum = f * l;
+#pragma unroll
+    for (int u = 0; u < SPLITS_MAX / 64; ++u) m[u] = expf(m[u] - top), sum += m[u] * l[u];
     for (int d = 32; d; d >>= 1) sum += __shfl_xor(sum, d, 64);
-    fac[lane] = f / sum;
+#pragma unroll
+    for (int u = 0; u < SPLITS_MAX / 64; ++u) fac[lane + 64 * u] = m[u] / sum;
   }
   __syncthreads();
   const int padded = (rank + 255) & ~255;
@@ -614,7 +611,7 @@ __global__ void __launch_bounds__(256) latent_merge_kernel(const float* __restri
   const size_t step = (size_t)rows * rank;
   if (V4 && rank <= 1024) {
     // four columns per thread, the splits dealt to as many threads per column as there are
-    const int nc = padded / 4, share = 256 / nc, c = (threadIdx.x % nc) * 4, g = threadIdx.x / nc;  // nc: 64, 128, 192 or 256
+    const int nc = padded / 4, share = MERGE_THREADS / nc, c = (threadIdx.x % nc) * 4, g = threadIdx.x / nc;  // nc: 64, 128, 192 or 256; a share of 4 to 16
     f32x4_t v = {0.f, 0.f, 0.f, 0.f};
     if (c < rank && g < share) {
 #pragma unroll 16
@@ -627,7 +624,7 @@ __global__ void __launch_bounds__(256) latent_merge_kernel(const float* __restri
       *reinterpret_cast<f32x4_t*>(lat + c) = v;
     }
   } else {
-    for (int c = threadIdx.x; c < padded; c += 256) {
+    for (int c = threadIdx.x; c < padded; c += MERGE_THREADS) {
       float v = 0.f;
       if (c < rank) {
 #pragma unroll 16
@@ -638,8 +635,8 @@ __global__ void __launch_bounds__(256) latent_merge_kernel(const float* __restri
   }
   __syncthreads();
 #pragma unroll
-  for (int u = 0; u < MERGE_V / 4; ++u) {
-    const int v = v0 + wave + 4 * u;
+  for (int u = 0; u < MERGE_V / MERGE_WAVES; ++u) {
+    const int v = v0 + wave + MERGE_WAVES * u;
     if (v >= vdim) break;
     const WT* wr = w + ((size_t)h * vdim + v) * rank;
     float s = 0.f;
@@ -766,21 +763,23 @@ extern "C" int ughip_latent_attention_absorbed(ughip_device* dev, ughip_view q, 
   auto split_go = [&](auto kernel) {
     if (lds > 64 * 1024)
       if (hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(kernel), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds); e != hipSuccess) return e;
-    kernel<<<g2, 256, lds, dev->stream>>>(a);
+    kernel<<<g2, 64 * SPLIT_WAVES, lds, dev->stream>>>(a);
     return hipSuccess;
   };
-  const size_t pieces = (size_t)SK * ((L + 15) & ~(size_t)15) / 4;  // 16-byte pieces of a tile
-  const int nl = L % 4 ? 0 : pieces <= 6 * 256 ? 6 : pieces <= 12 * 256 ? 12 : pieces <= 20 * 256 ? 20 : 0;
-  if (rank <= 128) UGHIP_HIPCHK(nl == 6 ? split_go(latent_split_kernel<2, 6>) : split_go(latent_split_kernel<2, 0>));
-  else if (rank <= 256) UGHIP_HIPCHK(nl && nl <= 12 ? split_go(latent_split_kernel<4, 12>) : split_go(latent_split_kernel<4, 0>));
-  else if (rank <= 512) UGHIP_HIPCHK(nl ? split_go(latent_split_kernel<8, 20>) : split_go(latent_split_kernel<8, 0>));
-  else UGHIP_HIPCHK(split_go(latent_split_kernel<16, 0>));
+  auto split_any = [&](auto nc) {
+    constexpr int NC = decltype(nc)::value;
+    return rank <= 256 ? split_go(latent_split_kernel<1, NC>) : rank <= 512 ? split_go(latent_split_kernel<2, NC>) : split_go(latent_split_kernel<4, NC>);
+  };
+  using std::integral_constant;
+  const size_t nc = L % 4 ? 0 : (((L + 15) & ~(size_t)15) + 255) / 256;  // at most 3: the rows' bytes in LDS are limited above
+  UGHIP_HIPCHK(nc == 0 ? split_any(integral_constant<int, 0>{}) : nc == 1 ? split_any(integral_constant<int, 1>{}) : nc == 2 ? split_any(integral_constant<int, 2>{})
+                                                                                                                           : split_any(integral_constant<int, 3>{}));
   UGHIP_HIPCHK(hipGetLastError());
   const dim3 g3((unsigned)heads, (unsigned)t, (unsigned)((vdim + MERGE_V - 1) / MERGE_V));
   const size_t lds3 = ((rank + 255) & ~(size_t)255) * sizeof(float);
   auto merge = [&](auto* w, auto vec) {
     latent_merge_kernel<std::remove_const_t<std::remove_pointer_t<decltype(w)>>, decltype(vec)::value>
-        <<<g3, 256, lds3, dev->stream>>>(a.acc, a.ml, w, view_ptr<float>(dst), dst.stride, (int)rows, (int)splits, (int)heads, (int)rank, (int)vdim);
+        <<<g3, MERGE_THREADS, lds3, dev->stream>>>(a.acc, a.ml, w, view_ptr<float>(dst), dst.stride, (int)rows, (int)splits, (int)heads, (int)rank, (int)vdim);
   };
   if (bf && v4) merge(buf_ptr<uint16_t>(w_uv), std::true_type{});
   else if (bf) merge(buf_ptr<uint16_t>(w_uv), std::false_type{});
