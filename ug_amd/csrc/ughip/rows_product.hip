@@ -190,8 +190,38 @@ __global__ void __launch_bounds__(256) rows_product_kernel(ProductArgs a) {
     for (int i = 0; i < WC; ++i) wr[d][i] = load_chunk<CT, WT, VEC>(wrow[i], k0 + ck, a.k, wok[i]);
   };
   const int steps = (a.k + KE - 1) / KE;
+  // element e of an accumulator: row 8 (e / 4) + 4 (lane / 32) + e % 4, column lane % 32
+  auto row_of = [&](int i, int e) { return m0 + wm * 32 * MI + i * 32 + 8 * (e >> 2) + 4 * (lane >> 5) + (e & 3); };
+  // what the gates of the rows multiply, asked for here so that the way to the table's scattered rows is over by the end: the rows'
+  // tokens first, then all of their table elements
+  constexpr bool GATE = ACT == UGHIP_ACT_GELU_MUL;
+  int id[GATE ? MI : 1][16];
+  uint32_t factor[GATE ? MI : 1][16][NI];  // bits
+  bool there[GATE ? MI : 1][16];
+  if constexpr (GATE) {
+#pragma unroll
+    for (int i = 0; i < MI; ++i)
+#pragma unroll
+      for (int e = 0; e < 16; ++e) id[i][e] = a.ids[min(row_of(i, e), a.m - 1)];
+  }
 #pragma unroll
   for (int d = 0; d < DEPTH; ++d) fetch(d, d * KE);  // (past the end: zeros)
+  if constexpr (GATE) {
+    auto ask = [&](auto* table) {  // (one branch on the table's type around all of the loads)
+#pragma unroll
+      for (int i = 0; i < MI; ++i)
+#pragma unroll
+        for (int e = 0; e < 16; ++e)
+#pragma unroll
+          for (int j = 0; j < NI; ++j) {
+            there[i][e] = id[i][e] >= 0 && id[i][e] < a.table_rows;
+            const size_t at = (size_t)(there[i][e] ? id[i][e] : 0) * a.table_stride + a.table_col + min(n0 + wn * 32 * NI + j * 32 + (lane & 31), a.n - 1);
+            factor[i][e][j] = table[at];
+          }
+    };
+    if (a.table_bf16) ask(static_cast<const uint16_t*>(a.table));
+    else ask(static_cast<const uint32_t*>(a.table));
+  }
   for (int s0 = 0; s0 < steps; s0 += DEPTH)
 #pragma unroll
    for (int d = 0; d < DEPTH; ++d) {
@@ -202,43 +232,33 @@ __global__ void __launch_bounds__(256) rows_product_kernel(ProductArgs a) {
     for (int i = 0; i < XC; ++i) *reinterpret_cast<u32x4_t*>(buf + ((tid >> CSH) + RP * i) * ROW_BYTES + (tid & (CHUNKS - 1)) * 16) = xr[d][i].pack();
 #pragma unroll
     for (int i = 0; i < WC; ++i) *reinterpret_cast<u32x4_t*>(buf + (BM + (tid >> CSH) + RP * i) * ROW_BYTES + (tid & (CHUNKS - 1)) * 16) = wr[d][i].pack();
-    if (s + DEPTH < steps) fetch(d, (s + DEPTH) * KE);
+    if (DEPTH > 1 || s + 1 < steps) fetch(d, (s + DEPTH) * KE);  // (without a branch, so that the next step's loads can be waited for alone)
     __syncthreads();  // (one barrier a step: the buffer written two steps from now is read before the next barrier)
     const char* xa = buf + (wm * 32 * MI + (lane & 31)) * ROW_BYTES + (lane >> 5) * 16;
     const char* wa = buf + (BM + wn * 32 * NI + (lane & 31)) * ROW_BYTES + (lane >> 5) * 16;
+    // fragments of BATCH pairs of chunks at once: a small tile's products do not cover the way from LDS one by one
+    constexpr int BATCH = MI * NI == 1 ? CHUNKS / 4 : 1;
 #pragma unroll
-    for (int c = 0; c < CHUNKS / 2; ++c) {
-      u32x4_t fx[MI], fw[NI];
+    for (int c0 = 0; c0 < CHUNKS / 2; c0 += BATCH) {
+      u32x4_t fx[BATCH][MI], fw[BATCH][NI];
 #pragma unroll
-      for (int i = 0; i < MI; ++i) fx[i] = *reinterpret_cast<const u32x4_t*>(xa + i * 32 * ROW_BYTES + c * 32);
+      for (int c = 0; c < BATCH; ++c) {
 #pragma unroll
-      for (int j = 0; j < NI; ++j) fw[j] = *reinterpret_cast<const u32x4_t*>(wa + j * 32 * ROW_BYTES + c * 32);
+        for (int i = 0; i < MI; ++i) fx[c][i] = *reinterpret_cast<const u32x4_t*>(xa + i * 32 * ROW_BYTES + (c0 + c) * 32);
 #pragma unroll
-      for (int i = 0; i < MI; ++i)
+        for (int j = 0; j < NI; ++j) fw[c][j] = *reinterpret_cast<const u32x4_t*>(wa + j * 32 * ROW_BYTES + (c0 + c) * 32);
+      }
 #pragma unroll
-        for (int j = 0; j < NI; ++j) mfma_chunk<CT>(fx[i], fw[j], acc[i][j]);
+      for (int c = 0; c < BATCH; ++c)
+#pragma unroll
+        for (int i = 0; i < MI; ++i)
+#pragma unroll
+          for (int j = 0; j < NI; ++j) mfma_chunk<CT>(fx[c][i], fw[c][j], acc[i][j]);
     }
    }
 
-  // element e of an accumulator: row 8 (e / 4) + 4 (lane / 32) + e % 4, column lane % 32
-  auto row_of = [&](int i, int e) { return m0 + wm * 32 * MI + i * 32 + 8 * (e >> 2) + 4 * (lane >> 5) + (e & 3); };
 #pragma unroll
   for (int i = 0; i < MI; ++i) {
-    float factor[16][NI];  // what the gates of these rows multiply: the rows' tokens first, then all of their table elements
-    if constexpr (ACT == UGHIP_ACT_GELU_MUL) {
-      int id[16];
-#pragma unroll
-      for (int e = 0; e < 16; ++e) id[e] = a.ids[min(row_of(i, e), a.m - 1)];
-#pragma unroll
-      for (int e = 0; e < 16; ++e)
-#pragma unroll
-        for (int j = 0; j < NI; ++j) {
-          const bool there = id[e] >= 0 && id[e] < a.table_rows;
-          const size_t at = (size_t)(there ? id[e] : 0) * a.table_stride + a.table_col + min(n0 + wn * 32 * NI + j * 32 + (lane & 31), a.n - 1);
-          const float t = a.table_bf16 ? bf16_to_f32(static_cast<const uint16_t*>(a.table)[at]) : static_cast<const float*>(a.table)[at];
-          factor[e][j] = there ? t : __uint_as_float(0x7fc00000u);
-        }
-    }
 #pragma unroll
     for (int e = 0; e < 16; ++e) {
       const int r = row_of(i, e);
@@ -254,7 +274,7 @@ __global__ void __launch_bounds__(256) rows_product_kernel(ProductArgs a) {
           if (a.bias) u += a.bias[a.n + col];
           v = silu_f(v) * u;
         }
-        if constexpr (ACT == UGHIP_ACT_GELU_MUL) v = gelu_tanh_f(v) * factor[e][j];
+        if constexpr (ACT == UGHIP_ACT_GELU_MUL) v = gelu_tanh_f(v) * __uint_as_float(!there[i][e] ? 0x7fc00000u : a.table_bf16 ? factor[i][e][j] << 16 : factor[i][e][j]);
         const size_t at = (size_t)r * a.dst_stride + col;
         if (a.dst_bf16) static_cast<uint16_t*>(a.dst)[at] = bf16_rne(v);
         else static_cast<float*>(a.dst)[at] = v;
