@@ -11,94 +11,15 @@ import pytest
 import hybrid_models as hm
 import plain_hybrid as ph
 import ug_amd
+from gpu_calls import BF16, F32, GELU_MUL, NONE, SWIGLU, Gpu, Product, RowStep, View, Z, close, get, p, rand, view
 from ug_amd import rng
 
 pytestmark = pytest.mark.gpu
 
 ROOT = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
-F32, BF16 = 0, 2                       # UGHIP_PRODUCT_*
-NONE, SWIGLU, GELU_MUL = 0, 1, 2       # UGHIP_ACT_*
-Z = C.c_size_t
-
-
-class View(C.Structure):
-    _fields_ = [("s", C.c_void_p), ("offset", Z), ("stride", Z)]
-
-
-class Product(C.Structure):
-    _fields_ = [("x", View), ("dst", View), ("w", C.c_void_p), ("bias", C.c_void_p), ("w_stride", Z), ("m", Z), ("n", Z), ("k", Z), ("product", C.c_int), ("act", C.c_int),
-                ("table", C.c_void_p), ("ids", C.c_void_p), ("table_rows", Z), ("table_stride", Z), ("table_col", Z), ("row_index", C.c_void_p), ("group_end", C.c_void_p),
-                ("groups", Z), ("x_rows", Z)]
-
-
-class RowStep(C.Structure):
-    _fields_ = [("x", C.c_void_p), ("x_offset", Z), ("y", C.c_void_p), ("y_norm", C.c_void_p), ("gate", C.c_void_p), ("norm", C.c_void_p), ("y_offset", Z), ("gate_offset", Z),
-                ("norm_groups", Z), ("eps", C.c_float), ("act", C.c_int), ("route", C.c_int), ("keep_x", C.c_int), ("w", C.c_void_p), ("bias", C.c_void_p), ("n", Z), ("k", Z),
-                ("table", C.c_void_p), ("ids", C.c_void_p), ("table_rows", Z), ("table_stride", Z), ("table_col", Z), ("logits", C.c_void_p), ("correction", C.c_void_p),
-                ("logits_offset", Z), ("experts", Z), ("groups", Z), ("keep", Z), ("top", Z), ("route_ids", C.c_void_p), ("route_weights", C.c_void_p), ("dst", C.c_void_p),
-                ("dst_offset", Z), ("x_out", Z)]
-
-
-class Gpu:
-    """Calls into libughip.so on slices of numpy arrays."""
-
-    def __init__(self, dev):
-        self.dev, self.lib = dev, ug_amd.ughip_lib()
-
-    def up(self, a, bf16=False):
-        a = np.ascontiguousarray(a)
-        if a.dtype.kind == "i":
-            return self.dev.slice_from(a.astype(np.int32).ravel())
-        a = a.astype(np.float32).ravel()
-        if bf16:
-            s = self.dev.allocate_uninit(ug_amd.BF16, a.size)
-            s.copy_host_to_device(rng.to_bf16_bits(a), ug_amd.BF16)
-            return s
-        return self.dev.slice_from(a)
-
-    def out(self, n, bf16=False):
-        s = self.dev.allocate_uninit(ug_amd.BF16 if bf16 else ug_amd.F32, n)
-        s.copy_host_to_device(np.full(n, 0x7fc0, np.uint16) if bf16 else np.full(n, np.nan, np.float32), ug_amd.BF16 if bf16 else ug_amd.F32)
-        return s
-
-    def ints(self, n):
-        return self.dev.slice_from(np.full(n, -7, np.int32))
-
-    def call(self, name, *args):
-        fn = getattr(self.lib, name)
-        fn.restype = C.c_int
-        assert fn(C.c_void_p(self.dev.raw_hip()), *args) == 0, self.lib.ughip_last_error().decode()
-
-
-def p(s):
-    return C.c_void_p(s.raw()) if s is not None else None
-
-
-def view(s, offset, stride):
-    return View(s.raw() if s is not None else None, offset, stride)
-
-
-def get(s, shape):
-    v = s.to_vec()
-    return (rng.from_bf16_bits(v) if s.dtype == ug_amd.BF16 else v).reshape(shape).astype(np.float64)
-
-
 @pytest.fixture
 def gpu(hip):
     return Gpu(hip)
-
-
-def rand(seed, *shape, std=1.0):
-    """bf16 values, so that both product modes see the same operands."""
-    return rng.bf16_round(rng.normal(seed, int(np.prod(shape)), std)).reshape(shape).astype(np.float64)
-
-
-def close(got, want, tol, rel=0.0):
-    """Within tol times the root mean square of `want`, plus rel times the element (a result rounded to bf16)."""
-    scale = np.sqrt(np.mean(want ** 2)) + 1e-30
-    assert np.all(np.isfinite(got)), "not finite"
-    worst = np.max(np.abs(got - want) - rel * np.abs(want)) / scale
-    assert worst <= tol, (worst, tol)
 
 
 def product(gpu, x, w, n, k, mode, act=NONE, bias=None, out_bf16=False, x_bf16=False, table=None, ids=None, col=0, row_index=None, group_end=None, groups=0, m=None):
@@ -232,13 +153,13 @@ def test_norms_of_rows(gpu):
     x, y, w = rand(1, m, n), rand(2, m * 3, n), rand(3, n)
     sx, sy, sw, dst, half = gpu.up(x), gpu.up(y), gpu.up(w), gpu.out(m * n), gpu.out(m * n, bf16=True)
     none = View(None, 0, 0)
-    gpu.call("ughip_add_rms_norm_rows", view(sx, 0, n), view(sy, n, 2 * n), None, None, Z(0), Z(0), p(sw), C.c_float(eps), view(dst, 0, n), p(half), Z(m), Z(n))
+    gpu.call("ughip_add_rms_norm_rows", view(sx, 0, n), view(sy, n, 2 * n), None, None, Z(0), Z(0), p(sw), C.c_float(eps), none, view(dst, 0, n), None, p(half), Z(m), Z(n))
     want = x + ph.rms(y.reshape(-1)[n:][: (2 * m - 1) * n].reshape(-1, n)[::2], eps) * w
     close(get(dst, (m, n)), want, 3e-6)
     close(get(half, (m, n)), want, 3e-6, rel=2.0 ** -8)
     slots, weights = np.stack([np.arange(m) * 3 % 27, np.arange(m) + 11], axis=1), rand(4, m, 2)
     ss, sw2 = gpu.up(slots), gpu.up(weights)
-    gpu.call("ughip_add_rms_norm_rows", none, view(sy, 0, n), p(ss), p(sw2), Z(2), Z(m * 3), p(sw), C.c_float(eps), view(dst, 0, n), None, Z(m), Z(n))
+    gpu.call("ughip_add_rms_norm_rows", none, view(sy, 0, n), p(ss), p(sw2), Z(2), Z(m * 3), p(sw), C.c_float(eps), none, view(dst, 0, n), None, None, Z(m), Z(n))
     close(get(dst, (m, n)), ph.rms((weights[:, :, None] * y[slots]).sum(1), eps) * w, 3e-6)
     for parts, cols in ((1, n), (5, n), (2, 128)):
         z = rand(5, m, cols)

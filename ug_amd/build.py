@@ -33,7 +33,7 @@ def _run(cmd):
 
 
 UGHIP_SOURCES = ("runtime.cpp", "lower_hip.cpp", "llama_ops.hip", "matmul.hip", "gemm_tiled.hip", "gemm_dma.hip", "gemm_dma_f32.hip", "rows_x3.hip", "attention.hip", "fused_linear.hip", "convert.hip",
-                 "rows_product.hip", "row_step.hip", "row_norms.hip", "latent_attention.hip", "ssm.hip", "moe.hip")
+                 "rows_product.hip", "row_step.hip", "row_norms.hip", "latent_attention.hip", "grouped_attention.hip", "ssm.hip", "delta.hip", "moe.hip")
 
 
 def build_ughip(only_changed=False):
@@ -63,7 +63,7 @@ def build_ughip(only_changed=False):
 
 def build_host():
     src = os.path.join(CSRC, "host")
-    files = [os.path.join(src, f) for f in ("ug/lower_op.cpp", "ug/lazy_buffer.cpp", "ug/schedule.cpp", "ug/safetensors.cpp", "hip_device.cpp", "llama.cpp", "hybrid.cpp", "decoder.cpp", "capi.cpp")]
+    files = [os.path.join(src, f) for f in ("ug/lower_op.cpp", "ug/lazy_buffer.cpp", "ug/schedule.cpp", "ug/safetensors.cpp", "hip_device.cpp", "llama.cpp", "hybrid_ops.cpp", "hybrid.cpp", "grouped_attention.cpp", "channel_delta.cpp", "decoder.cpp", "capi.cpp")]
     _run(["g++", "-std=c++17", "-O2", "-fPIC", "-shared", "-Wall", "-I" + INC, "-I" + src] + files +
          ["-L" + LIB, "-lughip", "-Wl,-rpath,$ORIGIN", "-lpthread", "-o", os.path.join(LIB, "libug_host.so")])
 

@@ -32,7 +32,9 @@ std::unique_ptr<Decoder> build_llama(const Json& c, WeightSource& w, Precision p
   return m;
 }
 
-std::unique_ptr<Decoder> build_hybrid(const Json& c, WeightSource& w, Precision precision, const DevicePtr& dev) { return std::make_unique<HybridModel>(c, w, precision, dev); }
+DecoderBuilder hybrid(const HybridDesign& (*design)()) {
+  return [design](const Json& c, WeightSource& w, Precision precision, const DevicePtr& dev) { return std::make_unique<HybridModel>(design(), c, w, precision, dev); };
+}
 
 std::string read_file(const std::string& path) {
   std::ifstream f(path, std::ios::binary);
@@ -45,7 +47,7 @@ std::string read_file(const std::string& path) {
 }  // namespace
 
 std::map<std::string, DecoderBuilder>& decoder_registry() {
-  static std::map<std::string, DecoderBuilder> r = {{"Tanolorn", build_hybrid}, {"LlamaForCausalLM", build_llama}, {"llama", build_llama}};
+  static std::map<std::string, DecoderBuilder> r = {{"Tanolorn", hybrid(tanolorn_design)}, {"Tugelorn", hybrid(tugelorn_design)}, {"LlamaForCausalLM", build_llama}, {"llama", build_llama}};
   return r;
 }
 

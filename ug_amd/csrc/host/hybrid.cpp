@@ -2,235 +2,14 @@
 
 #include <algorithm>
 #include <cmath>
-#include <mutex>
 
-#include "hip_device.h"
-#include "ughip_layers.h"
+#include "hybrid_ops.h"
 
 namespace ug_llama {
 
 using namespace ug;
 
 namespace {
-
-// ---- ops ------------------------------------------------------------------------------------------------------------------
-// A schedule item over `args` (buffers may repeat: each reaches the item once), its result a new buffer of `shape`.  Arguments
-// may be written as well (caches, states, scratch): they are stores that only this model's ops touch, in the order the data
-// dependences between those ops give.
-using HipCall = std::function<int(ughip_device*, const std::vector<ughip_slice*>&, ughip_slice*)>;
-LB hip_op(const char* what, const std::vector<LB>& args, const std::vector<size_t>& shape, HipCall call, DType dtype = DType::F32) {
-  HipDevice* hd = dynamic_cast<HipDevice*>(args[0].device().get());
-  if (!hd) bail(std::string(what) + ": this model runs on the hip device only");
-  ughip_device* dev = hd->raw();
-  std::vector<LB> unique;
-  std::vector<size_t> index;
-  for (const LB& a : args) {
-    size_t i = 0;
-    while (i < unique.size() && unique[i].data().get() != a.data().get()) ++i;
-    if (i == unique.size()) unique.push_back(a);
-    index.push_back(i);
-  }
-  const std::string name = what;
-  auto f = [=, n = unique.size()](const std::vector<Slice*>& vs) {
-    if (vs.size() != n + 1) bail(name + ": unexpected number of slices");
-    std::vector<ughip_slice*> in;
-    in.reserve(index.size());
-    for (size_t i : index) in.push_back(hip_raw_slice(*vs[i]));
-    if (call(dev, in, hip_raw_slice(*vs[n]))) bail(name + ": " + ughip_last_error());
-  };
-  return LB::custom(f, unique, Shape(shape), dtype, args[0].device());
-}
-
-LB scratch(DType dtype, size_t n, const DevicePtr& dev) {
-  LB lb = LB::alloc_uninit(dtype, Shape({n}), dev);
-  lb.maybe_allocate_uninit();
-  return lb;
-}
-
-// From kHalfRows positions on the stream is kept as bf16 rows too, for the products of bf16 matrices; plain products of up to
-// kFewRows positions are better off with the f32 rows (they share their K among workgroups).
-constexpr size_t kHalfRows = 33, kFewRows = 128;
-
-struct Product {
-  LB w, bias;  // UGHIP_ACT_SWIGLU: gate rows then up rows
-  size_t n = 0, k = 0;
-  int act = UGHIP_ACT_NONE;
-  LB table, ids;
-  size_t table_rows = 0, table_stride = 0, table_col = 0;
-};
-int product_mode(const LB& w) { return w.dtype() == DType::BF16 ? (int)UGHIP_PRODUCT_BF16 : (int)UGHIP_PRODUCT_F32; }
-
-// `after`: a buffer whose op has to run first (x is scratch that it wrote).
-LB product_rows(const Rows& x, size_t m, const Product& p, const LB& after = LB(), DType out_type = DType::F32) {
-  std::vector<LB> args = {x.lb, p.w};
-  auto add = [&](const LB& lb) {
-    if (!lb.valid()) return (size_t)0;
-    args.push_back(lb);
-    return args.size() - 1;
-  };
-  const size_t b = add(p.bias), tb = add(p.table), ids = add(p.ids);
-  add(after);
-  const size_t off = x.offset, stride = x.stride, n = p.n, k = p.k, trows = p.table_rows, tstride = p.table_stride, tcol = p.table_col;
-  const int act = p.act, mode = product_mode(p.w);
-  return hip_op("product_rows", args, {m, n}, [=](ughip_device* d, const std::vector<ughip_slice*>& in, ughip_slice* out) {
-    ughip_product q{};
-    q.x = {in[0], off, stride};
-    q.dst = {out, 0, n};
-    q.w = in[1];
-    if (b) q.bias = in[b];
-    if (tb) q.table = in[tb], q.ids = in[ids];
-    q.m = m, q.n = n, q.k = k, q.product = mode, q.act = act;
-    q.table_rows = trows, q.table_stride = tstride, q.table_col = tcol;
-    return ughip_product_rows(d, &q);
-  }, out_type);
-}
-
-LB norm_rows(const Rows& y, size_t m, size_t n, const LB& w, float eps, DType out_type = DType::F32) {
-  const size_t off = y.offset, stride = y.stride;
-  return hip_op("norm_rows", {y.lb, w}, {m, n}, [=](ughip_device* d, const std::vector<ughip_slice*>& in, ughip_slice* out) {
-    return ughip_add_rms_norm_rows(d, {nullptr, 0, 0}, {in[0], off, stride}, nullptr, nullptr, 0, 0, in[1], eps, {out, 0, n}, nullptr, m, n);
-  }, out_type);
-}
-
-// copy (may be invalid): scratch that receives the rows as bf16
-LB gather_rows(const LB& table, size_t rows, size_t stride, size_t col, size_t cols, const LB& ids, size_t m, const LB& copy = LB()) {
-  std::vector<LB> args = {table, ids};
-  const bool twice = copy.valid();
-  if (twice) args.push_back(copy);
-  return hip_op("gather_rows", args, {m, cols}, [=](ughip_device* d, const std::vector<ughip_slice*>& in, ughip_slice* out) {
-    if (twice)
-      if (int rc = ughip_gather_rows(d, in[0], rows, stride, col, cols, in[1], m, {in[2], 0, cols})) return rc;
-    return ughip_gather_rows(d, in[0], rows, stride, col, cols, in[1], m, {out, 0, cols});
-  });
-}
-
-// The pending output joins the residual: s.x is a plain [t, width] buffer afterwards.
-void settle(StepContext& c, Stream& s) {
-  if (!s.norm.valid()) return;
-  const Rows x = s.x, y = s.y;
-  const size_t t = c.t, n = c.width, top = s.top, y_rows = s.y_rows;
-  const float eps = c.eps;
-  std::vector<LB> args = {x.lb, y.lb, s.norm};
-  if (top) args.push_back(s.slots), args.push_back(s.weights);
-  s.x16 = c.half_rows ? scratch(DType::BF16, t * n, c.dev) : LB();
-  const size_t copy = s.x16.valid() ? args.size() : 0;
-  if (copy) args.push_back(s.x16);
-  LB out = hip_op("add_norm", args, {t, n}, [=](ughip_device* d, const std::vector<ughip_slice*>& in, ughip_slice* dst) {
-    return ughip_add_rms_norm_rows(d, {in[0], x.offset, x.stride}, {in[1], y.offset, y.stride}, top ? in[3] : nullptr, top ? in[4] : nullptr, top, y_rows, in[2], eps,
-                                   {dst, 0, n}, copy ? in[copy] : nullptr, t, n);
-  });
-  s.x = {out, 0, n};
-  s.y = Rows();
-  s.norm = LB();
-  s.slots = s.weights = LB();
-  s.top = s.y_rows = 0;
-}
-
-// A product of the (settled) stream's rows, in the form the step's products read.
-LB stream_product(const StepContext& c, const Stream& s, const Product& p, DType out_type = DType::F32) {
-  if (s.x16.valid() && (c.t > kFewRows || p.act == UGHIP_ACT_SWIGLU)) return product_rows({s.x16, 0, c.width}, c.t, p, s.x.lb, out_type);
-  return product_rows(s.x, c.t, p, LB(), out_type);
-}
-// What a producer of rows that only a product reads writes.
-DType half_type(const StepContext& c) { return c.half_rows && c.t > kFewRows ? DType::BF16 : DType::F32; }
-
-// One position: a product of one row with what stands in front of it folded in (ughip_product_row).
-struct RowStep {
-  Product p;
-  LB norm, gate;  // v = x * silu(gate), then normed over `norm_groups` parts
-  size_t norm_groups = 1, gate_offset = 0;
-  float eps = 0;
-};
-constexpr size_t kRowStepMax = 16000;  // elements of the row a folded product meets (an expert's part counts in runs of 512)
-
-// `pending` joins x first; keep_x: the joined row lies in front of the result (which starts at *at).
-LB row_step(const Rows& x, const Stream* pending, size_t width, const RowStep& r, size_t* at, bool keep_x = true) {
-  const bool join = pending && pending->norm.valid();
-  std::vector<LB> args = {x.lb, r.p.w};
-  auto add = [&](const LB& lb) {
-    if (!lb.valid()) return (size_t)0;
-    args.push_back(lb);
-    return args.size() - 1;
-  };
-  const size_t b = add(r.p.bias), tb = add(r.p.table), ids = add(r.p.ids), nm = add(r.norm), gt = add(r.gate);
-  const size_t y = join ? add(pending->y.lb) : 0, yn = join ? add(pending->norm) : 0, y_off = join ? pending->y.offset : 0, off = x.offset;
-  const Product pr = r.p;  // (the buffers inside keep their owners alive as the arguments do)
-  const size_t ng = r.norm_groups, g_off = r.gate_offset, base = join && keep_x ? width : 0;
-  const float eps = r.eps;
-  const size_t n = pr.n, k = pr.k, trows = pr.table_rows, tstride = pr.table_stride, tcol = pr.table_col;
-  const int act = pr.act;
-  *at = base;
-  return hip_op("row_step", args, {1, base + n}, [=](ughip_device* d, const std::vector<ughip_slice*>& in, ughip_slice* out) {
-    ughip_row_step q{};
-    q.x = in[0], q.x_offset = off, q.w = in[1];
-    if (y) q.y = in[y], q.y_offset = y_off, q.y_norm = in[yn], q.keep_x = base != 0;
-    if (b) q.bias = in[b];
-    if (tb) q.table = in[tb], q.ids = in[ids];
-    if (nm) q.norm = in[nm], q.norm_groups = ng;
-    if (gt) q.gate = in[gt], q.gate_offset = g_off;
-    q.eps = eps, q.act = act, q.n = n, q.k = k;
-    q.table_rows = trows, q.table_stride = tstride, q.table_col = tcol;
-    q.dst = out, q.dst_offset = base, q.x_out = 0;
-    return ughip_product_row(d, &q);
-  });
-}
-
-// A product of the stream's row; what was pending joins the residual on the way, which then lies in front of the result.
-LB stream_step(StepContext& c, Stream& s, RowStep r, size_t* at) {
-  if (s.top) settle(c, s);
-  r.eps = c.eps;
-  LB out = row_step(s.x, &s, c.width, r, at);
-  if (s.norm.valid()) {
-    s.x = {out, 0, c.width};
-    s.y = Rows();
-    s.norm = LB();
-  }
-  return out;
-}
-
-// ---- loading --------------------------------------------------------------------------------------------------------------
-struct Loader {
-  WeightSource& w;
-  Precision precision;
-  const DevicePtr& dev;
-  LB vec(const std::string& name, size_t n, float plus = 0.f) const {
-    std::vector<float> v = w.get(name, {n});
-    if (plus != 0.f)
-      for (float& e : v) e += plus;
-    return LB::copy(v.data(), DType::F32, n, Shape({n}), dev);
-  }
-  LB stacked_vec(const std::vector<std::pair<std::string, size_t>>& parts) const {
-    std::vector<float> all;
-    for (const auto& p : parts) {
-      std::vector<float> v = w.get(p.first, {p.second});
-      all.insert(all.end(), v.begin(), v.end());
-    }
-    return LB::copy(all.data(), DType::F32, all.size(), Shape({all.size()}), dev);
-  }
-  LB f32(const std::string& name, const std::vector<size_t>& shape) const { return w.load(name, shape, dev); }
-  // a matrix (or several by rows) in the dtype the products of this model read
-  LB matrix(const std::string& name, const std::vector<size_t>& shape) const { return stored(w.load(name, shape, dev)); }
-  LB stacked(const std::vector<std::pair<std::string, size_t>>& parts, size_t k) const {
-    size_t rows = 0;
-    for (const auto& p : parts) rows += p.second;
-    std::vector<float> all;
-    all.reserve(rows * k);
-    for (const auto& p : parts) {
-      std::vector<float> v = w.get(p.first, {p.second, k});
-      all.insert(all.end(), v.begin(), v.end());
-    }
-    return stored(LB::copy(all.data(), DType::F32, all.size(), Shape({rows, k}), dev));
-  }
-
- private:
-  LB stored(const LB& lb) const {
-    if (precision == Precision::F32) return lb;
-    LB n = lb.cast(DType::BF16);
-    n.realize();
-    n.detach();
-    return n;
-  }
-};
 
 // ---- latent attention -----------------------------------------------------------------------------------------------------
 struct LatentAttention : Mixer {
@@ -269,12 +48,12 @@ struct LatentAttention : Mixer {
     return st;
   }
 
-  void run(StepContext& c, Stream& s, size_t layer) const override {
+  void run(StepContext& c, Stream& s, size_t run) const override {
     const bool own = kv_from < 0;
     const size_t t = c.t, pos = c.pos, cap = c.capacity, H = heads, d = dim, r = rot, v = vdim, rk = rank, qr = q_rank, all = pos + t;
     const size_t wide = qr + (own ? rk + r : 0), trows = rope->rows;
     const float e = eps, sc = scale;
-    const LB cache = c.state->layers[own ? layer : (size_t)kv_from].buffers[0];
+    const LB cache = c.state->layers[own ? run : (size_t)kv_from].buffers[0];
     const bool fused = c.fused && t <= absorb_up_to && std::max({width, qr, H * v}) <= kRowStepMax;
     LB low, q;
     size_t low_at = 0, none;
@@ -363,10 +142,10 @@ struct Mamba2 : Mixer {
     return MixerState{{scratch(DType::F32, heads * state * vdim, in.device()), scratch(DType::F32, taps * channels(), in.device())}};
   }
 
-  void run(StepContext& c, Stream& s, size_t layer) const override {
+  void run(StepContext& c, Stream& s, size_t run) const override {
     const size_t t = c.t, pos = c.pos, I = inner(), ch = channels(), H = heads, vd = vdim, N = state, G = groups, nt = taps, wide = I + ch + H, ng = norm_groups;
     const float e = eps;
-    const LB S = c.state->layers[layer].buffers[0], ring = c.state->layers[layer].buffers[1];
+    const LB S = c.state->layers[run].buffers[0], ring = c.state->layers[run].buffers[1];
     if (c.fused && std::max(width, I) <= kRowStepMax && N <= 4096) {
       size_t at, none;
       LB p = stream_step(c, s, {{in, LB(), wide, width}}, &at);
@@ -398,20 +177,27 @@ struct Mamba2 : Mixer {
 struct DenseFeedForward : FeedForward {
   size_t ff, width;
   LB gate_up, gate_up_b, down, down_b;
-  DenseFeedForward(const Json& m, const std::string& p, const Loader& ld, size_t width_) : width(width_) {
-    ff = m.size_at("ff");
-    gate_up = ld.stacked({{p + "gate", ff}, {p + "up", ff}}, width), gate_up_b = ld.stacked_vec({{p + "gate.b", ff}, {p + "up.b", ff}});
-    down = ld.matrix(p + "down", {width, ff}), down_b = ld.vec(p + "down.b", width);
+  int act;
+  Glu glu;
+  // act: UGHIP_ACT_SWIGLU, or UGHIP_ACT_GLU as `glu` says
+  DenseFeedForward(const PartBuild& b, bool bias, int act_, const Glu& glu_) : width(b.width), act(act_), glu(glu_) {
+    const std::string& p = b.prefix;
+    ff = b.config.size_at("ff");
+    gate_up = b.ld.stacked({{p + "gate", ff}, {p + "up", ff}}, width);
+    down = b.ld.matrix(p + "down", {width, ff});
+    if (bias) gate_up_b = b.ld.stacked_vec({{p + "gate.b", ff}, {p + "up.b", ff}}), down_b = b.ld.vec(p + "down.b", width);
   }
   void run(StepContext& c, Stream& s) const override {
-    const Product first{gate_up, gate_up_b, ff, width, UGHIP_ACT_SWIGLU}, second{down, down_b, width, ff};
+    Product first{gate_up, gate_up_b, ff, width, act};
+    first.glu = glu;
+    const Product second{down, down_b, width, ff};
     if (c.fused && std::max(width, ff) <= kRowStepMax) {
       size_t at, none;
       LB a = stream_step(c, s, {first}, &at);
       s.y = {row_step({a, at, ff}, nullptr, 0, {second}, &none), 0, width};
       return;
     }
-    settle(c, s);
+    settle(c, s, true);
     LB a = stream_product(c, s, first, half_type(c));
     s.y = {product_rows({a, 0, ff}, c.t, second), 0, width};
   }
@@ -506,7 +292,7 @@ void RopeTables::ensure(size_t n) {
   const size_t half = dims_ / 2;
   std::vector<float> c(n * half), s(n * half);
   for (size_t i = 0; i < half; ++i) {
-    const double f = std::pow(base_, -2.0 * (double)i / (double)dims_);
+    const double f = std::pow(base_, -2.0 * (double)i / (double)dims_) / factor_;
     for (size_t p = 0; p < n; ++p) {
       const double a = (double)p * f;
       c[p * half + i] = (float)std::cos(a);
@@ -518,10 +304,64 @@ void RopeTables::ensure(size_t n) {
   rows = n;
 }
 
+void QueryFactors::ensure(size_t n) {
+  if (n <= rows) return;
+  std::vector<float> v(n);
+  for (size_t p = 0; p < n; ++p) v[p] = (float)(1.0 + coef_ * std::log(std::floor((double)(p + 1) / every_) + 1.0));
+  values = LB::copy(v.data(), DType::F32, n, Shape({n}), dev_);
+  rows = n;
+}
+
+// ---- designs ----------------------------------------------------------------------------------------------------------------
+const HybridDesign& tanolorn_design() {
+  static const HybridDesign design = [] {
+    HybridDesign d;
+    d.norm_base = 1.f;
+    d.mixers["latent_attention"] = [](const PartBuild& b) -> std::unique_ptr<Mixer> {
+      const Json &m = b.config, &rot = m.at("rot");
+      const size_t dims = rot.size_at("dims");
+      if (dims != m.size_at("rot_dim") || dims == 0 || dims % 2) bail("configuration: layer " + std::to_string(b.index) + " rotates " + std::to_string(dims) + " elements");
+      if (m.find("kv_from")) {
+        const size_t from = m.size_at("kv_from");
+        const std::vector<Json>& all = b.layers.arr;
+        if (from >= b.index || all[from].str_at("type") != "latent_attention" || all[from].at("mixer").find("kv_from") ||
+            all[from].at("mixer").size_at("kv_rank") != m.size_at("kv_rank") || all[from].at("mixer").size_at("rot_dim") != dims)
+          bail("configuration: layer " + std::to_string(b.index) + " reads the latents of layer " + std::to_string(from) + ", which has none that fit");
+      }
+      return std::make_unique<LatentAttention>(m, b.prefix, b.ld, b.width, b.eps, b.rope(rot.num_at("base"), dims, 1.0));
+    };
+    d.mixers["mamba2"] = [](const PartBuild& b) { return std::make_unique<Mamba2>(b.config, b.prefix, b.ld, b.width, b.eps); };
+    d.mlps["dense"] = [](const PartBuild& b) { return std::make_unique<DenseFeedForward>(b, true, (int)UGHIP_ACT_SWIGLU, Glu()); };
+    d.mlps["moe"] = [](const PartBuild& b) { return std::make_unique<MoeFeedForward>(b.config, b.prefix, b.ld, b.width); };
+    return d;
+  }();
+  return design;
+}
+
+const HybridDesign& tugelorn_design() {
+  static const HybridDesign design = [] {
+    HybridDesign d;
+    d.norm_ahead = true;
+    d.residual_mult = "residual_mult";
+    d.mixers["attention"] = [](const PartBuild& b) { return make_grouped_attention(b, false, true, true, false); };
+    d.mixers["attention_2"] = [](const PartBuild& b) { return make_grouped_attention(b, true, false, false, true); };
+    d.mixers["channel_delta"] = make_channel_delta;
+    d.mlps["dense"] = [](const PartBuild& b) {
+      const double limit = b.config.num_at("limit");
+      if (!(limit > 0)) bail("configuration: a feed-forward with the limit " + std::to_string(limit));
+      return std::make_unique<DenseFeedForward>(b, false, (int)UGHIP_ACT_GLU, Glu{1.702f, 1.f, (float)limit});
+    };
+    return d;
+  }();
+  return design;
+}
+
 // ---- the model ------------------------------------------------------------------------------------------------------------
-HybridModel::HybridModel(const Json& cfg, WeightSource& weights, Precision precision, const DevicePtr& dev) : dev_(dev), ops_(hip_ops()), precision_(precision) {
+HybridModel::HybridModel(const HybridDesign& design, const Json& cfg, WeightSource& weights, Precision precision, const DevicePtr& dev)
+    : dev_(dev), ops_(hip_ops()), precision_(precision), norm_ahead_(design.norm_ahead) {
   vocab_ = cfg.size_at("vocab"), width_ = cfg.size_at("width");
   eps_ = (float)cfg.at("norm").num_at("eps");
+  const float mult = design.residual_mult ? (float)cfg.num_at(design.residual_mult) : 1.f;
   const Json& list = cfg.at("layers");
   if (list.kind != Json::Arr) bail("configuration: 'layers' is not a list");
   const size_t n_layers = list.arr.size();
@@ -530,39 +370,37 @@ HybridModel::HybridModel(const Json& cfg, WeightSource& weights, Precision preci
   Loader ld{weights, precision, dev};
   embed_ = ld.matrix("embed", {vocab_, width_});
   if (side_dim_) side_embed_ = ld.matrix("side.embed", {vocab_, n_layers * side_dim_});
-  std::map<std::pair<double, size_t>, std::shared_ptr<RopeTables>> tables;
-  // norms are stored around zero: the weight is 1 + what the file holds
-  auto norm = [&](const std::string& name) { return ld.vec(name, width_, 1.f); };
+  std::map<std::vector<double>, std::shared_ptr<RopeTables>> ropes;
+  std::map<std::vector<double>, std::shared_ptr<QueryFactors>> factors;
+  auto rope = [&](double base, size_t dims, double factor) {
+    std::shared_ptr<RopeTables>& tb = ropes[{base, (double)dims, factor}];
+    if (!tb) tables_.push_back(tb = std::make_shared<RopeTables>(base, dims, factor, dev));
+    return tb;
+  };
+  auto query_factors = [&](double coef, double every) {
+    std::shared_ptr<QueryFactors>& tb = factors[{coef, every}];
+    if (!tb) tables_.push_back(tb = std::make_shared<QueryFactors>(coef, every, dev));
+    return tb;
+  };
+  auto norm = [&](const std::string& name, float times = 1.f) { return ld.vec(name, width_, design.norm_base, times); };
+  const char* behind = norm_ahead_ ? "b" : "";
   for (size_t i = 0; i < n_layers; ++i) {
     const Json& lc = list.arr[i];
-    const Json& m = lc.at("mixer");
     const std::string p = "l" + std::to_string(i) + ".", type = lc.str_at("type");
+    auto part = [&](const Json& config, const char* name) { return PartBuild{list, i, config, p + name, ld, width_, eps_, rope, query_factors}; };
     Layer l;
-    if (type == "latent_attention") {
-      const Json& rot = m.at("rot");
-      const size_t dims = rot.size_at("dims");
-      if (dims != m.size_at("rot_dim") || dims == 0 || dims % 2) bail("configuration: layer " + std::to_string(i) + " rotates " + std::to_string(dims) + " elements");
-      std::shared_ptr<RopeTables>& tb = tables[{rot.num_at("base"), dims}];
-      if (!tb) tables_.push_back(tb = std::make_shared<RopeTables>(rot.num_at("base"), dims, dev));
-      if (m.find("kv_from")) {
-        const size_t from = m.size_at("kv_from");
-        if (from >= i || list.arr[from].str_at("type") != "latent_attention" || list.arr[from].at("mixer").find("kv_from") ||
-            list.arr[from].at("mixer").size_at("kv_rank") != m.size_at("kv_rank") || list.arr[from].at("mixer").size_at("rot_dim") != dims)
-          bail("configuration: layer " + std::to_string(i) + " reads the latents of layer " + std::to_string(from) + ", which has none that fit");
-      }
-      l.mixer = std::make_unique<LatentAttention>(m, p + "mix.", ld, width_, eps_, tb);
-    } else if (type == "mamba2") {
-      l.mixer = std::make_unique<Mamba2>(m, p + "mix.", ld, width_, eps_);
-    } else {
-      bail("configuration: unknown mixer '" + type + "'");
-    }
-    l.norm1 = norm(p + "norm1");
+    const auto mixer = design.mixers.find(type);
+    if (mixer == design.mixers.end()) bail("configuration: unknown mixer '" + type + "'");
+    l.mixer = mixer->second(part(lc.at("mixer"), "mix."));
+    if (norm_ahead_) l.ahead1 = norm(p + "norm1");
+    l.norm1 = norm(p + "norm1" + behind, mult);
     if (const Json* mlp = lc.find("mlp")) {
       const std::string kind = mlp->str_at("kind");
-      if (kind == "dense") l.mlp = std::make_unique<DenseFeedForward>(*mlp, p + "mlp.", ld, width_);
-      else if (kind == "moe") l.mlp = std::make_unique<MoeFeedForward>(*mlp, p + "mlp.", ld, width_);
-      else bail("configuration: unknown feed-forward '" + kind + "'");
-      l.norm2 = norm(p + "norm2");
+      const auto ff = design.mlps.find(kind);
+      if (ff == design.mlps.end()) bail("configuration: unknown feed-forward '" + kind + "'");
+      l.mlp = ff->second(part(*mlp, "mlp."));
+      if (norm_ahead_) l.ahead2 = norm(p + "norm2");
+      l.norm2 = norm(p + "norm2" + behind, mult);
     }
     if (side_dim_) {
       l.side_gate = ld.matrix(p + "side.gate", {side_dim_, width_});
@@ -573,13 +411,23 @@ HybridModel::HybridModel(const Json& cfg, WeightSource& weights, Precision preci
   }
   final_norm_ = norm("final.norm");
   head_ = ld.matrix("head", {vocab_, width_});
+  size_t start = 0, stop = 0, times = 1;
+  if (const Json* loop = cfg.find("loop")) {
+    start = loop->size_at("start"), stop = loop->size_at("stop"), times = loop->size_at("times");
+    if (start > stop || stop > n_layers || times == 0)
+      bail("configuration: layers " + std::to_string(start) + " .. " + std::to_string(stop) + " of " + std::to_string(n_layers) + " run " + std::to_string(times) + " times");
+  }
+  for (size_t i = 0; i < start; ++i) runs_.push_back({i, false});
+  for (size_t pass = 0; pass < times; ++pass)
+    for (size_t i = start; i < stop; ++i) runs_.push_back({i, pass > 0 && i == start});
+  for (size_t i = stop; i < n_layers; ++i) runs_.push_back({i, false});
 }
 
 std::unique_ptr<DecoderState> HybridModel::new_state(size_t max_tokens) const {
   auto st = std::make_unique<HybridState>();
   st->capacity = std::max<size_t>(1, max_tokens);
   for (const auto& t : tables_) t->ensure(st->capacity);
-  for (const Layer& l : layers_) st->layers.push_back(l.mixer->new_state(st->capacity));
+  for (const Run& r : runs_) st->layers.push_back(layers_[r.layer].mixer->new_state(st->capacity));
   return st;
 }
 
@@ -602,24 +450,34 @@ void HybridModel::side(StepContext& c, Stream& s, const Layer& l, size_t index) 
 
 LB HybridModel::step(const LB& tokens, const LB&, DecoderState& state, const LB* rows, const std::function<void(const LB&)>* after_layer) const {
   HybridState* st = dynamic_cast<HybridState*>(&state);
-  if (!st || st->layers.size() != layers_.size()) bail("this step needs a state of the same model");
+  if (!st || st->layers.size() != runs_.size()) bail("this step needs a state of the same model");
   const size_t t = tokens.elem_count();
   if (t == 0) bail("a step without tokens");
   if (st->len + t > st->capacity) bail("a sequence of " + std::to_string(st->len) + " + " + std::to_string(t) + " positions exceeds its capacity of " + std::to_string(st->capacity));
-  StepContext c{dev_, tokens, t, st->len, st->capacity, width_, eps_, st, precision_ == Precision::BF16 && t >= kHalfRows, t == 1 && !switch_on(SW_NO_FUSED_STEP)};
+  StepContext c{dev_, tokens, t, st->len, st->capacity, width_, eps_, st, precision_ == Precision::BF16 && t >= kHalfRows, t == 1 && !switch_on(SW_NO_FUSED_STEP), norm_ahead_};
   Stream s;
-  if (c.half_rows) s.x16 = scratch(DType::BF16, t * width_, dev_);
+  if (c.half_rows && !norm_ahead_) s.x16 = scratch(DType::BF16, t * width_, dev_);
   s.x = {gather_rows(embed_, vocab_, width_, 0, width_, tokens, t, s.x16), 0, width_};
-  for (size_t i = 0; i < layers_.size(); ++i) {
-    const Layer& l = layers_[i];
-    l.mixer->run(c, s, i);
+  const Rows embedded = s.x;
+  // a sublayer, with the norm in front of it where there is one
+  auto sublayer = [&](const LB& ahead, auto&& run) {
+    s.ahead = ahead;
+    run();
+    s.ahead = s.h = s.h_by = LB();
+  };
+  for (size_t i = 0; i < runs_.size(); ++i) {
+    const Layer& l = layers_[runs_[i].layer];
+    if (runs_[i].again) s.extra = embedded;
+    sublayer(l.ahead1, [&] { l.mixer->run(c, s, i); });
     s.norm = l.norm1;
     if (l.mlp) {
-      l.mlp->run(c, s);
+      sublayer(l.ahead2, [&] { l.mlp->run(c, s); });
       s.norm = l.norm2;
     }
-    if (side_dim_) side(c, s, l, i);
+    if (side_dim_) side(c, s, l, runs_[i].layer);
     if (after_layer) {
+      // (the next layer's norm goes with it where nothing else comes first)
+      if (!c.fused && i + 1 < runs_.size() && !runs_[i + 1].again) s.ahead = layers_[runs_[i + 1].layer].ahead1;
       settle(c, s);
       (*after_layer)(s.x.lb);
     }

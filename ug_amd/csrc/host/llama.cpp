@@ -735,6 +735,7 @@ struct SafetensorsWeights : WeightSource {
   ug::MmapedSafetensors st;
   explicit SafetensorsWeights(const std::vector<std::string>& paths)
       : st(paths.size() == 1 ? ug::MmapedSafetensors::open(paths[0]) : ug::MmapedSafetensors::multi(paths)) {}
+  std::vector<size_t> shape_of(const std::string& name, const std::vector<size_t>&) override { return st.get(name).shape; }
   void check_shape(const std::string& name, const std::vector<size_t>& got, const std::vector<size_t>& want) {
     if (got != want) bail("unexpected shape for " + name + ": " + Shape(got).str() + ", expected " + Shape(want).str());
   }

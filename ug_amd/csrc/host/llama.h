@@ -138,6 +138,8 @@ struct Config {
 struct WeightSource {
   virtual ~WeightSource() = default;
   virtual std::vector<float> get(const std::string& name, const std::vector<size_t>& shape) = 0;
+  // The shape a tensor is stored with; `fallback` where the source makes tensors of any shape.
+  virtual std::vector<size_t> shape_of(const std::string&, const std::vector<size_t>& fallback) { return fallback; }
   // The tensor as an f32 buffer on `dev`; the default uploads what get() returns.
   virtual LB load(const std::string& name, const std::vector<size_t>& shape, const ug::DevicePtr& dev);
 };

@@ -1,0 +1,233 @@
+// Attention of many positions over keys and values in memory, the scores never leaving registers; shared by the kinds of attention
+// that bring their operands into this form.
+//   A wave owns 32 queries, a workgroup 128; keys come in tiles of 64 through LDS.  The scores are computed transposed, S^T = K Q^T
+//   (32 x 32 tiles), which leaves lane l with query l % 32 as its column: the running maximum and sum are one exchange with lane
+//   l ^ 32, and the weights sit where the second product, O^T = V^T P^T, wants its right operand (the order in which keys take
+//   part in it is the order the accumulator layout gives; V is read in the same order).  Values come transposed for that.
+//   bf16 operands: v_mfma_f32_32x32x16_bf16, a weight as two bf16 terms (16 bits of it); f32: v_mfma_f32_32x32x2_f32.
+#pragma once
+#include <hip/hip_runtime.h>
+
+#include "bf16_split.h"
+#include "layers.h"
+
+namespace ughip {
+namespace {  // every file that launches the kernel has its own
+
+typedef float f32x16 __attribute__((ext_vector_type(16)));
+typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
+
+// q [heads][q_rows][DQ], k [kv_heads][k_rows][DQ], v [kv_heads vdim][v_stride] (one row per value element, position along it); zeros
+// past a query's and a key's last element and past the last query.
+struct AttRowsArgs {
+  const void* q;
+  const void* k;
+  const void* v;
+  void* dst;
+  size_t v_stride, dst_stride;
+  int t, pos, vdim, q_rows, k_rows;
+  int kv_heads;  // key head of query head h: h / (heads / kv_heads)
+  int window;    // > 0: a position sees itself and the window - 1 positions in front of it
+  float scale2;  // scale * log2(e): the weights are powers of two
+  bool dst_bf16;
+};
+
+template <typename T>
+__device__ __forceinline__ T to_elem(float v) {
+  if constexpr (sizeof(T) == 2) return bf16_rne(v);
+  else return v;
+}
+
+template <typename T>
+__device__ __forceinline__ void mfma_chunk(const u32x4_t& a, const u32x4_t& b, f32x16& acc) {
+  if constexpr (sizeof(T) == 2) {
+    acc = __builtin_amdgcn_mfma_f32_32x32x16_bf16(__builtin_bit_cast(bf16x8, a), __builtin_bit_cast(bf16x8, b), acc, 0, 0, 0);
+  } else {
+    const f32x4_t x = __builtin_bit_cast(f32x4_t, a), y = __builtin_bit_cast(f32x4_t, b);
+    acc = __builtin_amdgcn_mfma_f32_32x32x2f32(x.x, y.x, acc, 0, 0, 0);
+    acc = __builtin_amdgcn_mfma_f32_32x32x2f32(x.y, y.y, acc, 0, 0, 0);
+    acc = __builtin_amdgcn_mfma_f32_32x32x2f32(x.z, y.z, acc, 0, 0, 0);
+    acc = __builtin_amdgcn_mfma_f32_32x32x2f32(x.w, y.w, acc, 0, 0, 0);
+  }
+}
+
+constexpr int ATT_KT = 64, ATT_QT = 128;
+template <typename T, int DQ, int DV>
+constexpr int attention_rows_lds_bytes() {
+  return ATT_KT * (DQ * (int)sizeof(T) + 16) + DV * (ATT_KT * (int)sizeof(T) + 16);
+}
+
+// DQ >= dim + rot and DV >= vdim, the surplus is zeros.  T: uint16_t (bf16) or float.
+template <typename T, int DQ, int DV>
+__global__ void __launch_bounds__(256) attention_rows_kernel(AttRowsArgs a) {
+  constexpr int E = 16 / sizeof(T), QC = DQ / E, K_ROW = DQ * sizeof(T) + 16, V_ROW = ATT_KT * sizeof(T) + 16, VC = ATT_KT / E;
+  constexpr int NK = ATT_KT * QC / 256, NV = DV * VC / 256;  // 16-byte pieces of a tile per thread
+  constexpr bool AHEAD = NK + NV <= 16;                   // the next tile waits in registers while this one is multiplied
+  static_assert(ATT_KT * QC % 256 == 0 && DV * VC % 256 == 0, "whole pieces per thread");
+  extern __shared__ __attribute__((aligned(16))) char lds[];
+  char* Ks = lds;                // [ATT_KT][DQ]
+  char* Vs = lds + ATT_KT * K_ROW;   // [DV][ATT_KT]
+  // consecutive workgroups (dealt round robin to the chip's eight parts) take different key heads: those that share one meet in a cache
+  const int per = gridDim.x / a.kv_heads, kv = blockIdx.x % a.kv_heads, head = kv * per + blockIdx.x / a.kv_heads;
+  const int qb = gridDim.y - 1 - blockIdx.y;  // the longest rows first
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, col = lane & 31, hf = lane >> 5;
+  const int i_mine = qb * ATT_QT + wave * 32 + col, p_mine = a.pos + min(i_mine, a.t - 1);
+  // the wave's queries as the right operand of S^T: chunk 2 c + hf of query `col` (rows up to q_rows exist, zeros past t)
+  u32x4_t qf[QC / 2];
+  {
+    const char* qr = static_cast<const char*>(a.q) + ((size_t)head * a.q_rows + i_mine) * DQ * sizeof(T) + hf * 16;
+#pragma unroll
+    for (int c = 0; c < QC / 2; ++c) qf[c] = *reinterpret_cast<const u32x4_t*>(qr + c * 32);
+  }
+  f32x16 o[DV / 32];
+#pragma unroll
+  for (int i = 0; i < DV / 32; ++i)
+#pragma unroll
+    for (int e = 0; e < 16; ++e) o[i][e] = 0.f;
+  float mx = -INFINITY, sum = 0.f;
+  const int s_all = a.pos + a.t, last_q = min(a.t, (qb + 1) * ATT_QT), keys = a.pos + last_q, first_p = a.pos + qb * ATT_QT + wave * 32;
+  const int k_begin = a.window ? max(0, a.pos + qb * ATT_QT - a.window + 1) / ATT_KT * ATT_KT : 0, oldest = a.window ? p_mine - a.window : -1;  // keys > oldest are seen
+  const char* k_head = static_cast<const char*>(a.k) + (size_t)kv * a.k_rows * DQ * sizeof(T);
+  const T* v_head = static_cast<const T*>(a.v) + (size_t)kv * a.vdim * a.v_stride;
+  u32x4_t kr[NK], vr[NV];
+  auto fetch = [&](int k0) {
+#pragma unroll
+    for (int u = 0; u < NK; ++u) kr[u] = *reinterpret_cast<const u32x4_t*>(k_head + (size_t)k0 * DQ * sizeof(T) + (threadIdx.x + u * 256) * 16);
+#pragma unroll
+    for (int u = 0; u < NV; ++u) {
+      // rows are padded to whole tiles and 16-byte aligned; every lane loads (no branches between loads)
+      const int x = threadIdx.x + u * 256, vc = x / VC;
+      vr[u] = *reinterpret_cast<const u32x4_t*>(v_head + (size_t)(vc < a.vdim ? vc : 0) * a.v_stride + k0 + x % VC * E);
+    }
+  };
+  // what of a piece of values is none: columns past the last one, positions past the last one (never written)
+  auto value_piece = [&](const u32x4_t& piece, int vc, int kp) {
+    T v[E];
+    __builtin_memcpy(v, &piece, 16);
+#pragma unroll
+    for (int e = 0; e < E; ++e) v[e] = vc < a.vdim && kp + e < s_all ? v[e] : T(0);
+    u32x4_t out;
+    __builtin_memcpy(&out, v, 16);
+    return out;
+  };
+  if (AHEAD) fetch(k_begin);
+  for (int k0 = k_begin; k0 < keys; k0 += ATT_KT) {
+    __syncthreads();
+    if (!AHEAD) fetch(k0);
+#pragma unroll
+    for (int u = 0; u < NK; ++u) {
+      const int x = threadIdx.x + u * 256;
+      *reinterpret_cast<u32x4_t*>(Ks + x / QC * K_ROW + x % QC * 16) = kr[u];
+    }
+#pragma unroll
+    for (int u = 0; u < NV; ++u) {
+      const int x = threadIdx.x + u * 256;
+      const bool whole = k0 + ATT_KT <= s_all && DV == a.vdim;
+      *reinterpret_cast<u32x4_t*>(Vs + x / VC * V_ROW + x % VC * 16) = whole ? vr[u] : value_piece(vr[u], x / VC, k0 + x % VC * E);
+    }
+    __syncthreads();
+    if (AHEAD && k0 + ATT_KT < keys) fetch(k0 + ATT_KT);
+    if (k0 > first_p + 31 || (a.window && k0 + ATT_KT - 1 <= first_p - a.window)) continue;  // nothing in this tile is visible to the wave's queries
+    f32x16 s[2];
+#pragma unroll
+    for (int b = 0; b < 2; ++b)
+#pragma unroll
+      for (int e = 0; e < 16; ++e) s[b][e] = 0.f;
+#pragma unroll
+    for (int c = 0; c < QC / 2; ++c)
+#pragma unroll
+      for (int b = 0; b < 2; ++b) mfma_chunk<T>(*reinterpret_cast<const u32x4_t*>(Ks + (b * 32 + col) * K_ROW + hf * 16 + c * 32), qf[c], s[b]);
+    // element e of s[b]: key k0 + 32 b + 8 (e / 4) + 4 hf + e % 4, query `col`
+    float top = mx;
+    if (k0 + ATT_KT - 1 > first_p || (a.window && k0 <= first_p + 31 - a.window)) {  // some keys of the tile are not visible to some of the wave's queries
+#pragma unroll
+      for (int b = 0; b < 2; ++b)
+#pragma unroll
+        for (int e = 0; e < 16; ++e) {
+          const int key = k0 + 32 * b + 8 * (e >> 2) + 4 * hf + (e & 3);
+          s[b][e] = key <= p_mine && key > oldest ? s[b][e] * a.scale2 : -INFINITY;
+        }
+    } else {
+#pragma unroll
+      for (int b = 0; b < 2; ++b)
+#pragma unroll
+        for (int e = 0; e < 16; ++e) s[b][e] *= a.scale2;
+    }
+#pragma unroll
+    for (int b = 0; b < 2; ++b)
+#pragma unroll
+      for (int e = 0; e < 16; ++e) top = fmaxf(top, s[b][e]);
+    top = fmaxf(top, __shfl_xor(top, 32, 64));
+    if (__any(top > mx)) {
+      const float alpha = top > mx ? exp2f(mx - top) : 1.f;  // (a lane whose query has seen nothing yet: both are -infinity)
+      sum *= alpha;
+#pragma unroll
+      for (int i = 0; i < DV / 32; ++i)
+#pragma unroll
+        for (int e = 0; e < 16; ++e) o[i][e] *= alpha;
+      mx = top;
+    }
+    const float base = mx == -INFINITY ? 0.f : mx;
+    float part = 0.f;
+#pragma unroll
+    for (int b = 0; b < 2; ++b)
+#pragma unroll
+      for (int e = 0; e < 16; ++e) {
+        s[b][e] = __builtin_amdgcn_exp2f(s[b][e] - base);
+        part += s[b][e];
+      }
+    sum += part + __shfl_xor(part, 32, 64);
+#pragma unroll
+    for (int b = 0; b < 2; ++b) {
+      if constexpr (sizeof(T) == 2) {
+#pragma unroll
+        for (int u = 0; u < 2; ++u) {
+          bf16x8 hi, lo;
+#pragma unroll
+          for (int e = 0; e < 8; ++e) {
+            hi[e] = (__bf16)s[b][8 * u + e];
+            lo[e] = (__bf16)(s[b][8 * u + e] - (float)hi[e]);
+          }
+          bf16x8 vf[DV / 32];
+#pragma unroll
+          for (int i = 0; i < DV / 32; ++i) {
+            const char* p = Vs + (i * 32 + col) * V_ROW + (b * 32 + 16 * u + 4 * hf) * 2;
+            const uint2 v0 = *reinterpret_cast<const uint2*>(p), v1 = *reinterpret_cast<const uint2*>(p + 16);
+            vf[i] = __builtin_bit_cast(bf16x8, u32x4_t{v0.x, v0.y, v1.x, v1.y});
+          }
+#pragma unroll
+          for (int i = 0; i < DV / 32; ++i) o[i] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(vf[i], hi, o[i], 0, 0, 0);
+#pragma unroll
+          for (int i = 0; i < DV / 32; ++i) o[i] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(vf[i], lo, o[i], 0, 0, 0);
+        }
+      } else {
+#pragma unroll
+        for (int u = 0; u < 4; ++u)
+#pragma unroll
+          for (int i = 0; i < DV / 32; ++i) {
+            const f32x4_t v = *reinterpret_cast<const f32x4_t*>(Vs + (i * 32 + col) * V_ROW + (b * 32 + 8 * u + 4 * hf) * 4);
+            o[i] = __builtin_amdgcn_mfma_f32_32x32x2f32(v.x, s[b][4 * u], o[i], 0, 0, 0);
+            o[i] = __builtin_amdgcn_mfma_f32_32x32x2f32(v.y, s[b][4 * u + 1], o[i], 0, 0, 0);
+            o[i] = __builtin_amdgcn_mfma_f32_32x32x2f32(v.z, s[b][4 * u + 2], o[i], 0, 0, 0);
+            o[i] = __builtin_amdgcn_mfma_f32_32x32x2f32(v.w, s[b][4 * u + 3], o[i], 0, 0, 0);
+          }
+      }
+    }
+  }
+  if (i_mine >= a.t) return;
+  const float inv = 1.f / sum;
+  const size_t at = (size_t)i_mine * a.dst_stride + (size_t)head * a.vdim;
+#pragma unroll
+  for (int i = 0; i < DV / 32; ++i)
+#pragma unroll
+    for (int e = 0; e < 16; ++e) {
+      const int vc = i * 32 + 8 * (e >> 2) + 4 * hf + (e & 3);
+      if (vc < a.vdim) {
+        if (a.dst_bf16) static_cast<uint16_t*>(a.dst)[at + vc] = bf16_rne(o[i][e] * inv);
+        else static_cast<float*>(a.dst)[at + vc] = o[i][e] * inv;
+      }
+    }
+}
+
+}  // namespace
+}  // namespace ughip

@@ -72,7 +72,8 @@ void gemm_tiled_name(int dtype, const MMArgs& p, size_t batch, bool rhs_bf16, co
 
 // The same kernel for rows that meet a matrix per group and leave through an epilogue (ughip_product_rows): bf16 rows (gathered by
 // row_index when given) against [n, k]-major bf16 matrices, `groups` of them w_group elements apart with the rows sorted by group
-// (group_end), or one (groups 0).  swiglu: the matrices are [2 n_out, k], gate rows then up rows, the result silu(gate) * up.
+// (group_end), or one (groups 0).  swiglu: the matrices are [2 n_out, k], gate rows then up rows, the result silu(gate) * up (or the
+// gated unit that the last three fields describe).
 // p: a, a_rs, b, b_cs (k), M rows, N matrix rows (2 n_out with swiglu), K; p.c is not used.
 struct DmaRows {
   const int* row_index = nullptr;
@@ -82,6 +83,7 @@ struct DmaRows {
   long long w_group = 0, dst_stride = 0;
   int groups = 0, x_rows = 0, n_out = 0;
   bool dst_bf16 = false;
+  float glu_alpha = 1.f, glu_shift = 0.f, glu_limit = 0.f;  // the gated unit with swiglu: gate * sigmoid(alpha gate) * (up + shift), both limited (limit > 0)
 };
 bool gemm_dma_rows_supported(const MMArgs& p, const DmaRows& r, bool swiglu, int tile);
 int gemm_dma_rows_pick(const MMArgs& p, const DmaRows& r, bool swiglu);  // a tile code, 0: no tile takes it

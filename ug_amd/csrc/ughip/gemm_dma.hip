@@ -417,9 +417,16 @@ __global__ void __launch_bounds__(256) gemm_dma4(MMArgs p, int tiles_m, int tile
         if (row > m_last) continue;
         floatx4 v = acc[i][j] + b;
         if constexpr (ROWS == 2) {
-          const floatx4 u = acc[i][j + NC] + bu;
+          floatx4 u = acc[i][j + NC] + bu;
+          if (rw.glu_limit > 0.f) {
 #pragma unroll
-          for (int e = 0; e < 4; ++e) v[e] = v[e] * __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(-1.4426950408889634f * v[e])) * u[e];
+            for (int e = 0; e < 4; ++e) {
+              v[e] = v[e] > rw.glu_limit ? rw.glu_limit : v[e];
+              u[e] = u[e] > rw.glu_limit ? rw.glu_limit : u[e] < -rw.glu_limit ? -rw.glu_limit : u[e];
+            }
+          }
+#pragma unroll
+          for (int e = 0; e < 4; ++e) v[e] = v[e] * __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(-1.4426950408889634f * rw.glu_alpha * v[e])) * (u[e] + rw.glu_shift);
         }
         const size_t at = (size_t)(m0 + row) * rw.dst_stride + col;
         if (rw.dst_bf16) *reinterpret_cast<u32x2*>(static_cast<T*>(rw.dst) + at) = __builtin_bit_cast(u32x2, __builtin_convertvector(v, bf16x4));

@@ -1,12 +1,7 @@
 // Attention over latents (ughip_layers.h): the cache of a layer is one row per position, [normed latent (rank) | rotated key part
 // (rot)], shared by all heads.
 //
-// Many positions (latent_rows_kernel): keys and values are expanded by products before, and the scores never leave registers.
-//   A wave owns 32 queries, a workgroup 128; keys come in tiles of 64 through LDS.  The scores are computed transposed, S^T = K Q^T
-//   (32 x 32 tiles), which leaves lane l with query l % 32 as its column: the running maximum and sum are one exchange with lane
-//   l ^ 32, and the weights sit where the second product, O^T = V^T P^T, wants its right operand (the order in which keys take
-//   part in it is the order the accumulator layout gives; V is read in the same order).  Values come transposed for that.
-//   bf16 operands: v_mfma_f32_32x32x16_bf16, a weight as two bf16 terms (16 bits of it); f32: v_mfma_f32_32x32x2_f32.
+// Many positions: keys and values are expanded by products before, the kernel of attention_rows.h does the rest.
 // Few positions (absorb, split, merge): the up-projection of the keys is folded into the query, that of the values into the
 //   result, so that a head's keys and values are both the cache rows as they are.  16 (position, head) pairs per workgroup against
 //   tiles of 32 cache rows in LDS, v_mfma_f32_16x16x4_f32; the cache is split over workgroups, a last launch adds the parts up.
@@ -14,15 +9,13 @@
 
 #include <type_traits>
 
+#include "attention_rows.h"
 #include "bf16_split.h"
 #include "layers.h"
 
 using namespace ughip;
 
 namespace {
-
-typedef float f32x16 __attribute__((ext_vector_type(16)));
-typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
 
 // element e of a rotated part of `rot` elements at a table row: pairs (i, i + rot / 2)
 __device__ __forceinline__ float rotated(const float* part, int e, int rot, const float* cos, const float* sin) {
@@ -73,12 +66,6 @@ struct PackArgs {
   bool q_vec;  // a head's query starts on 16 bytes
 };
 
-template <typename T>
-__device__ __forceinline__ T to_elem(float v) {
-  if constexpr (sizeof(T) == 2) return bf16_rne(v);
-  else return v;
-}
-
 // The operands of the scores as the kernel below reads them: [heads][rows][DQ], queries rotated, keys with the shared rotated part
 // behind each head's own, zeros past the last element and the last position.  A thread makes 16 bytes.
 template <typename T, int DQ>
@@ -122,226 +109,28 @@ __global__ void __launch_bounds__(256) latent_pack_kernel(PackArgs a) {
   *reinterpret_cast<u32x4_t*>(out) = chunk;
 }
 
-struct RowsArgs {
-  const void* q;  // packed
-  const void* k;
-  const void* v;
-  void* dst;
-  size_t v_stride, dst_stride;
-  int t, pos, vdim, q_rows, k_rows;
-  float scale2;  // scale * log2(e): the weights are powers of two
-  bool dst_bf16;
-};
-
-template <typename T>
-__device__ __forceinline__ void mfma_chunk(const u32x4_t& a, const u32x4_t& b, f32x16& acc) {
-  if constexpr (sizeof(T) == 2) {
-    acc = __builtin_amdgcn_mfma_f32_32x32x16_bf16(__builtin_bit_cast(bf16x8, a), __builtin_bit_cast(bf16x8, b), acc, 0, 0, 0);
-  } else {
-    const f32x4_t x = __builtin_bit_cast(f32x4_t, a), y = __builtin_bit_cast(f32x4_t, b);
-    acc = __builtin_amdgcn_mfma_f32_32x32x2f32(x.x, y.x, acc, 0, 0, 0);
-    acc = __builtin_amdgcn_mfma_f32_32x32x2f32(x.y, y.y, acc, 0, 0, 0);
-    acc = __builtin_amdgcn_mfma_f32_32x32x2f32(x.z, y.z, acc, 0, 0, 0);
-    acc = __builtin_amdgcn_mfma_f32_32x32x2f32(x.w, y.w, acc, 0, 0, 0);
-  }
-}
-
-constexpr int KT = 64, QT = 128;
 template <typename T, int DQ, int DV>
-constexpr int rows_lds_bytes() {
-  return KT * (DQ * (int)sizeof(T) + 16) + DV * (KT * (int)sizeof(T) + 16);
-}
-
-// DQ >= dim + rot and DV >= vdim, the surplus is zeros.  T: uint16_t (bf16) or float.
-template <typename T, int DQ, int DV>
-__global__ void __launch_bounds__(256) latent_rows_kernel(RowsArgs a) {
-  constexpr int E = 16 / sizeof(T), QC = DQ / E, K_ROW = DQ * sizeof(T) + 16, V_ROW = KT * sizeof(T) + 16, VC = KT / E;
-  constexpr int NK = KT * QC / 256, NV = DV * VC / 256;  // 16-byte pieces of a tile per thread
-  constexpr bool AHEAD = NK + NV <= 16;                   // the next tile waits in registers while this one is multiplied
-  static_assert(KT * QC % 256 == 0 && DV * VC % 256 == 0, "whole pieces per thread");
-  extern __shared__ __attribute__((aligned(16))) char lds[];
-  char* Ks = lds;                // [KT][DQ]
-  char* Vs = lds + KT * K_ROW;   // [DV][KT]
-  const int head = blockIdx.x, qb = gridDim.y - 1 - blockIdx.y;  // the longest rows first
-  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, col = lane & 31, hf = lane >> 5;
-  const int i_mine = qb * QT + wave * 32 + col, p_mine = a.pos + min(i_mine, a.t - 1);
-  // the wave's queries as the right operand of S^T: chunk 2 c + hf of query `col` (rows up to q_rows exist, zeros past t)
-  u32x4_t qf[QC / 2];
-  {
-    const char* qr = static_cast<const char*>(a.q) + ((size_t)head * a.q_rows + i_mine) * DQ * sizeof(T) + hf * 16;
-#pragma unroll
-    for (int c = 0; c < QC / 2; ++c) qf[c] = *reinterpret_cast<const u32x4_t*>(qr + c * 32);
-  }
-  f32x16 o[DV / 32];
-#pragma unroll
-  for (int i = 0; i < DV / 32; ++i)
-#pragma unroll
-    for (int e = 0; e < 16; ++e) o[i][e] = 0.f;
-  float mx = -INFINITY, sum = 0.f;
-  const int s_all = a.pos + a.t, last_q = min(a.t, (qb + 1) * QT), keys = a.pos + last_q, first_p = a.pos + qb * QT + wave * 32;
-  const char* k_head = static_cast<const char*>(a.k) + (size_t)head * a.k_rows * DQ * sizeof(T);
-  const T* v_head = static_cast<const T*>(a.v) + (size_t)head * a.vdim * a.v_stride;
-  u32x4_t kr[NK], vr[NV];
-  auto fetch = [&](int k0) {
-#pragma unroll
-    for (int u = 0; u < NK; ++u) kr[u] = *reinterpret_cast<const u32x4_t*>(k_head + (size_t)k0 * DQ * sizeof(T) + (threadIdx.x + u * 256) * 16);
-#pragma unroll
-    for (int u = 0; u < NV; ++u) {
-      // rows are padded to whole tiles and 16-byte aligned; every lane loads (no branches between loads)
-      const int x = threadIdx.x + u * 256, vc = x / VC;
-      vr[u] = *reinterpret_cast<const u32x4_t*>(v_head + (size_t)(vc < a.vdim ? vc : 0) * a.v_stride + k0 + x % VC * E);
-    }
-  };
-  // what of a piece of values is none: columns past the last one, positions past the last one (never written)
-  auto value_piece = [&](const u32x4_t& piece, int vc, int kp) {
-    T v[E];
-    __builtin_memcpy(v, &piece, 16);
-#pragma unroll
-    for (int e = 0; e < E; ++e) v[e] = vc < a.vdim && kp + e < s_all ? v[e] : T(0);
-    u32x4_t out;
-    __builtin_memcpy(&out, v, 16);
-    return out;
-  };
-  if (AHEAD) fetch(0);
-  for (int k0 = 0; k0 < keys; k0 += KT) {
-    __syncthreads();
-    if (!AHEAD) fetch(k0);
-#pragma unroll
-    for (int u = 0; u < NK; ++u) {
-      const int x = threadIdx.x + u * 256;
-      *reinterpret_cast<u32x4_t*>(Ks + x / QC * K_ROW + x % QC * 16) = kr[u];
-    }
-#pragma unroll
-    for (int u = 0; u < NV; ++u) {
-      const int x = threadIdx.x + u * 256;
-      const bool whole = k0 + KT <= s_all && DV == a.vdim;
-      *reinterpret_cast<u32x4_t*>(Vs + x / VC * V_ROW + x % VC * 16) = whole ? vr[u] : value_piece(vr[u], x / VC, k0 + x % VC * E);
-    }
-    __syncthreads();
-    if (AHEAD && k0 + KT < keys) fetch(k0 + KT);
-    if (k0 > first_p + 31) continue;  // nothing in this tile is visible to the wave's queries
-    f32x16 s[2];
-#pragma unroll
-    for (int b = 0; b < 2; ++b)
-#pragma unroll
-      for (int e = 0; e < 16; ++e) s[b][e] = 0.f;
-#pragma unroll
-    for (int c = 0; c < QC / 2; ++c)
-#pragma unroll
-      for (int b = 0; b < 2; ++b) mfma_chunk<T>(*reinterpret_cast<const u32x4_t*>(Ks + (b * 32 + col) * K_ROW + hf * 16 + c * 32), qf[c], s[b]);
-    // element e of s[b]: key k0 + 32 b + 8 (e / 4) + 4 hf + e % 4, query `col`
-    float top = mx;
-    if (k0 + KT - 1 > first_p) {  // some keys of the tile lie behind some of the wave's queries
-#pragma unroll
-      for (int b = 0; b < 2; ++b)
-#pragma unroll
-        for (int e = 0; e < 16; ++e) {
-          const int key = k0 + 32 * b + 8 * (e >> 2) + 4 * hf + (e & 3);
-          s[b][e] = key <= p_mine ? s[b][e] * a.scale2 : -INFINITY;
-        }
-    } else {
-#pragma unroll
-      for (int b = 0; b < 2; ++b)
-#pragma unroll
-        for (int e = 0; e < 16; ++e) s[b][e] *= a.scale2;
-    }
-#pragma unroll
-    for (int b = 0; b < 2; ++b)
-#pragma unroll
-      for (int e = 0; e < 16; ++e) top = fmaxf(top, s[b][e]);
-    top = fmaxf(top, __shfl_xor(top, 32, 64));
-    if (__any(top > mx)) {  // (key 0 is visible to everyone: after the first tile top is finite)
-      const float alpha = exp2f(mx - top);
-      sum *= alpha;
-#pragma unroll
-      for (int i = 0; i < DV / 32; ++i)
-#pragma unroll
-        for (int e = 0; e < 16; ++e) o[i][e] *= alpha;
-      mx = top;
-    }
-    float part = 0.f;
-#pragma unroll
-    for (int b = 0; b < 2; ++b)
-#pragma unroll
-      for (int e = 0; e < 16; ++e) {
-        s[b][e] = __builtin_amdgcn_exp2f(s[b][e] - mx);
-        part += s[b][e];
-      }
-    sum += part + __shfl_xor(part, 32, 64);
-#pragma unroll
-    for (int b = 0; b < 2; ++b) {
-      if constexpr (sizeof(T) == 2) {
-#pragma unroll
-        for (int u = 0; u < 2; ++u) {
-          bf16x8 hi, lo;
-#pragma unroll
-          for (int e = 0; e < 8; ++e) {
-            hi[e] = (__bf16)s[b][8 * u + e];
-            lo[e] = (__bf16)(s[b][8 * u + e] - (float)hi[e]);
-          }
-          bf16x8 vf[DV / 32];
-#pragma unroll
-          for (int i = 0; i < DV / 32; ++i) {
-            const char* p = Vs + (i * 32 + col) * V_ROW + (b * 32 + 16 * u + 4 * hf) * 2;
-            const uint2 v0 = *reinterpret_cast<const uint2*>(p), v1 = *reinterpret_cast<const uint2*>(p + 16);
-            vf[i] = __builtin_bit_cast(bf16x8, u32x4_t{v0.x, v0.y, v1.x, v1.y});
-          }
-#pragma unroll
-          for (int i = 0; i < DV / 32; ++i) o[i] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(vf[i], hi, o[i], 0, 0, 0);
-#pragma unroll
-          for (int i = 0; i < DV / 32; ++i) o[i] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(vf[i], lo, o[i], 0, 0, 0);
-        }
-      } else {
-#pragma unroll
-        for (int u = 0; u < 4; ++u)
-#pragma unroll
-          for (int i = 0; i < DV / 32; ++i) {
-            const f32x4_t v = *reinterpret_cast<const f32x4_t*>(Vs + (i * 32 + col) * V_ROW + (b * 32 + 8 * u + 4 * hf) * 4);
-            o[i] = __builtin_amdgcn_mfma_f32_32x32x2f32(v.x, s[b][4 * u], o[i], 0, 0, 0);
-            o[i] = __builtin_amdgcn_mfma_f32_32x32x2f32(v.y, s[b][4 * u + 1], o[i], 0, 0, 0);
-            o[i] = __builtin_amdgcn_mfma_f32_32x32x2f32(v.z, s[b][4 * u + 2], o[i], 0, 0, 0);
-            o[i] = __builtin_amdgcn_mfma_f32_32x32x2f32(v.w, s[b][4 * u + 3], o[i], 0, 0, 0);
-          }
-      }
-    }
-  }
-  if (i_mine >= a.t) return;
-  const float inv = 1.f / sum;
-  const size_t at = (size_t)i_mine * a.dst_stride + (size_t)head * a.vdim;
-#pragma unroll
-  for (int i = 0; i < DV / 32; ++i)
-#pragma unroll
-    for (int e = 0; e < 16; ++e) {
-      const int vc = i * 32 + 8 * (e >> 2) + 4 * hf + (e & 3);
-      if (vc < a.vdim) {
-        if (a.dst_bf16) static_cast<uint16_t*>(a.dst)[at + vc] = bf16_rne(o[i][e] * inv);
-        else static_cast<float*>(a.dst)[at + vc] = o[i][e] * inv;
-      }
-    }
-}
-
-template <typename T, int DQ, int DV>
-int launch_rows(ughip_device* dev, RowsArgs a, PackArgs pk) {
-  constexpr int bytes = rows_lds_bytes<T, DQ, DV>();
+int launch_rows(ughip_device* dev, AttRowsArgs a, PackArgs pk) {
+  constexpr int bytes = attention_rows_lds_bytes<T, DQ, DV>();
   static_assert(bytes <= 160 * 1024, "tile does not fit LDS");
-  static const hipError_t attr = hipFuncSetAttribute(reinterpret_cast<const void*>(latent_rows_kernel<T, DQ, DV>), hipFuncAttributeMaxDynamicSharedMemorySize, bytes);
+  static const hipError_t attr = hipFuncSetAttribute(reinterpret_cast<const void*>(attention_rows_kernel<T, DQ, DV>), hipFuncAttributeMaxDynamicSharedMemorySize, bytes);
   UGHIP_HIPCHK(attr);
-  pk.q_rows = (pk.t + QT - 1) / QT * QT, pk.k_rows = (pk.pos + pk.t + KT - 1) / KT * KT;
+  pk.q_rows = (pk.t + ATT_QT - 1) / ATT_QT * ATT_QT, pk.k_rows = (pk.pos + pk.t + ATT_KT - 1) / ATT_KT * ATT_KT;
   const size_t q_bytes = (size_t)pk.heads * pk.q_rows * DQ * sizeof(T), k_bytes = (size_t)pk.heads * pk.k_rows * DQ * sizeof(T);
   void* ws = nullptr;
   if (int rc = rows_scratch(dev, q_bytes + k_bytes, &ws)) return rc;
   pk.qp = ws, pk.kp = static_cast<char*>(ws) + q_bytes;
-  a.q = pk.qp, a.k = pk.kp, a.q_rows = pk.q_rows, a.k_rows = pk.k_rows;
+  a.q = pk.qp, a.k = pk.kp, a.q_rows = pk.q_rows, a.k_rows = pk.k_rows, a.kv_heads = pk.heads, a.window = 0;
   constexpr int CH = DQ * (int)sizeof(T) / 16;
   const size_t pieces = (size_t)(pk.q_rows + pk.k_rows) * CH;
   latent_pack_kernel<T, DQ><<<dim3((unsigned)((pieces + 255) / 256), (unsigned)pk.heads), 256, 0, dev->stream>>>(pk);
   UGHIP_HIPCHK(hipGetLastError());
-  latent_rows_kernel<T, DQ, DV><<<dim3((unsigned)pk.heads, (unsigned)(pk.q_rows / QT)), 256, bytes, dev->stream>>>(a);
+  attention_rows_kernel<T, DQ, DV><<<dim3((unsigned)pk.heads, (unsigned)(pk.q_rows / ATT_QT)), 256, bytes, dev->stream>>>(a);
   UGHIP_HIPCHK(hipGetLastError());
   return UGHIP_OK;
 }
 template <typename T>
-int launch_rows_any(ughip_device* dev, const RowsArgs& a, const PackArgs& pk) {
+int launch_rows_any(ughip_device* dev, const AttRowsArgs& a, const PackArgs& pk) {
   const int dq = pk.dim + pk.rot;
   if (dq <= 64 && a.vdim <= 64) return launch_rows<T, 64, 64>(dev, a, pk);
   if (dq <= 128 && a.vdim <= 128) return launch_rows<T, 128, 128>(dev, a, pk);
@@ -699,9 +488,9 @@ extern "C" int ughip_latent_attention_rows(ughip_device* dev, ughip_view q, cons
   const bool bf16 = dst.s->dtype == UGHIP_BF16;
   if (!bf16 && dst.s->dtype != UGHIP_F32) return set_error(UGHIP_ERR_UNSUPPORTED, "%s: the result is F32 or BF16", what);
   if (t == 0) return UGHIP_OK;
-  if ((t + QT - 1) / QT > 65535) return set_error(UGHIP_ERR_UNSUPPORTED, "%s: too many positions", what);
+  if ((t + ATT_QT - 1) / ATT_QT > 65535) return set_error(UGHIP_ERR_UNSUPPORTED, "%s: too many positions", what);
   if (int rc = device_activate(dev)) return rc;
-  RowsArgs a{};
+  AttRowsArgs a{};
   a.v = v_t->ptr, a.dst = static_cast<char*>(dst.s->ptr) + dst.offset * (bf16 ? 2 : 4), a.v_stride = v_stride, a.dst_stride = dst.stride;
   a.t = (int)t, a.pos = (int)pos, a.vdim = (int)vdim, a.scale2 = scale * 1.4426950408889634f, a.dst_bf16 = bf16;
   PackArgs pk{};

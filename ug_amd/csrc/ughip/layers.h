@@ -46,6 +46,26 @@ __device__ __forceinline__ float gelu_tanh_f(float z) {
   return 0.5f * z * (1.f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z)));
 }
 
+// A gated linear unit: gate * sigmoid(alpha gate) * (up + shift), the gate cut off above `limit`, up on both sides (limit <= 0:
+// neither).  alpha = 1, shift = 0 without a limit is SwiGLU.
+struct GluForm {
+  float alpha = 1.f, shift = 0.f, limit = 0.f;
+};
+__device__ __forceinline__ float glu_f(float gate, float up, const GluForm& f) {
+  if (f.limit > 0.f) {  // the same for every thread of a launch
+    gate = gate > f.limit ? f.limit : gate;  // (a NaN stays one)
+    up = up > f.limit ? f.limit : up < -f.limit ? -f.limit : up;
+  }
+  return gate * __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(-1.4426950408889634f * f.alpha * gate)) * (up + f.shift);
+}
+// What ughip_product and ughip_row_step say of it.
+inline GluForm glu_form(int act, float alpha, float shift, float limit) {
+  GluForm f;
+  if (act == UGHIP_ACT_GLU) f.alpha = alpha, f.shift = shift, f.limit = limit;
+  return f;
+}
+__device__ __forceinline__ float sigmoid_f(float z) { return __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(-1.4426950408889634f * z)); }
+
 // The sum over a workgroup of 64 * WAVES threads, the same value in every thread; `red` holds WAVES floats and is free to
 // be used again after the next barrier of the caller.
 template <int WAVES>

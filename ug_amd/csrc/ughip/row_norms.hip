@@ -35,21 +35,25 @@ struct AddNormArgs {
   const float* y;
   const float* w;
   void* dst;
-  uint16_t* dst16;
-  size_t x_stride, y_stride, dst_stride;
+  void* copy;
+  const float* extra;
+  const float* next;
+  size_t x_stride, y_stride, dst_stride, extra_stride;
   const int* slots;
   const float* weights;
   int top, y_rows, n;
   float eps;
-  bool dst_bf16;
+  bool dst_bf16, copy_bf16;
 };
 
 __global__ void __launch_bounds__(256) add_rms_norm_kernel(AddNormArgs a) {
   extern __shared__ float row[];
-  __shared__ float red[4];
+  __shared__ float red[2][4];
   const size_t i = blockIdx.x;
   float ss = 0.f;
-  if (a.slots) {
+  if (!a.y) {
+    for (int c = threadIdx.x; c < a.n; c += 256) row[c] = 0.f;
+  } else if (a.slots) {
     for (int c = threadIdx.x; c < a.n; c += 256) {
       float v = 0.f;
       for (int j = 0; j < a.top; ++j) {
@@ -66,13 +70,65 @@ __global__ void __launch_bounds__(256) add_rms_norm_kernel(AddNormArgs a) {
       ss += v * v;
     }
   }
-  ss = block_sum<4>(ss, red);
+  ss = block_sum<4>(ss, red[0]);
   const float inv = 1.f / sqrtf(ss / (float)a.n + a.eps);
+  ss = 0.f;
   for (int c = threadIdx.x; c < a.n; c += 256) {
-    float v = row[c] * inv * a.w[c];  // every thread reads back its own elements
+    float v = a.y ? row[c] * inv * a.w[c] : 0.f;  // every thread reads back its own elements
     if (a.x) v += a.x[i * a.x_stride + c];
+    if (a.extra) v += a.extra[i * a.extra_stride + c];
     put(a.dst, a.dst_bf16, i * a.dst_stride + c, v);
-    if (a.dst16) a.dst16[i * a.n + c] = bf16_rne(v);
+    if (a.next) row[c] = v, ss += v * v;
+    else if (a.copy) put(a.copy, a.copy_bf16, i * a.n + c, v);
+  }
+  if (!a.next) return;
+  ss = block_sum<4>(ss, red[1]);
+  const float inv2 = 1.f / sqrtf(ss / (float)a.n + a.eps);
+  for (int c = threadIdx.x; c < a.n; c += 256) put(a.copy, a.copy_bf16, i * a.n + c, row[c] * inv2 * a.next[c]);
+}
+
+// The same without routed rows for up to 4096 elements, a multiple of 4, held in registers.
+__global__ void __launch_bounds__(256) add_rms_norm4_kernel(AddNormArgs a) {
+  __shared__ float red[2][4];
+  const size_t i = blockIdx.x;
+  f32x4_t v[4], x[4], e[4];
+  const f32x4_t zero = {0.f, 0.f, 0.f, 0.f};
+  float ss = 0.f;
+  auto square = [](const f32x4_t& q) { return q.x * q.x + q.y * q.y + q.z * q.z + q.w * q.w; };
+#pragma unroll
+  for (int u = 0; u < 4; ++u) {
+    const int c = (u * 256 + (int)threadIdx.x) * 4;
+    const bool ok = c < a.n;
+    v[u] = ok && a.y ? *reinterpret_cast<const f32x4_t*>(a.y + i * a.y_stride + c) : zero;
+    x[u] = ok && a.x ? *reinterpret_cast<const f32x4_t*>(a.x + i * a.x_stride + c) : zero;
+    e[u] = ok && a.extra ? *reinterpret_cast<const f32x4_t*>(a.extra + i * a.extra_stride + c) : zero;
+  }
+#pragma unroll
+  for (int u = 0; u < 4; ++u) ss += square(v[u]);
+  ss = block_sum<4>(ss, red[0]);
+  const float inv = 1.f / sqrtf(ss / (float)a.n + a.eps);
+  auto put4 = [](void* dst, bool bf16, size_t at, const f32x4_t& q) {
+    if (bf16) *reinterpret_cast<ushort4*>(static_cast<uint16_t*>(dst) + at) = make_ushort4(bf16_rne(q.x), bf16_rne(q.y), bf16_rne(q.z), bf16_rne(q.w));
+    else *reinterpret_cast<f32x4_t*>(static_cast<float*>(dst) + at) = q;
+  };
+  ss = 0.f;
+#pragma unroll
+  for (int u = 0; u < 4; ++u) {
+    const int c = (u * 256 + (int)threadIdx.x) * 4;
+    if (c >= a.n) continue;
+    if (a.y) v[u] = v[u] * inv * *reinterpret_cast<const f32x4_t*>(a.w + c) + x[u] + e[u];
+    else v[u] = x[u] + e[u];
+    put4(a.dst, a.dst_bf16, i * a.dst_stride + c, v[u]);
+    if (a.copy && !a.next) put4(a.copy, a.copy_bf16, i * a.n + c, v[u]);
+    ss += square(v[u]);
+  }
+  if (!a.next) return;
+  ss = block_sum<4>(ss, red[1]);
+  const float inv2 = 1.f / sqrtf(ss / (float)a.n + a.eps);
+#pragma unroll
+  for (int u = 0; u < 4; ++u) {
+    const int c = (u * 256 + (int)threadIdx.x) * 4;
+    if (c < a.n) put4(a.copy, a.copy_bf16, i * a.n + c, v[u] * inv2 * *reinterpret_cast<const f32x4_t*>(a.next + c));
   }
 }
 
@@ -162,27 +218,44 @@ extern "C" int ughip_gather_rows(ughip_device* dev, const ughip_slice* table, si
 }
 
 extern "C" int ughip_add_rms_norm_rows(ughip_device* dev, ughip_view x, ughip_view y, const ughip_slice* slots, const ughip_slice* weights, size_t top, size_t y_rows,
-                                       const ughip_slice* w, float eps, ughip_view dst, ughip_slice* dst_bf16, size_t m, size_t n) {
+                                       const ughip_slice* w, float eps, ughip_view extra, ughip_view dst, const ughip_slice* next, ughip_slice* copy, size_t m, size_t n) {
   if (!dev) return set_error(UGHIP_ERR_INVALID, "add_rms_norm_rows: null device");
   if (n > ROW_MAX) return set_error(UGHIP_ERR_UNSUPPORTED, "add_rms_norm_rows: rows of %zu elements, up to %zu are supported", n, ROW_MAX);
   if (x.s)
     if (int rc = check_view(dev, x, m, n, UGHIP_F32, "add_rms_norm_rows x")) return rc;
-  if (int rc = check_view(dev, y, slots ? y_rows : m, n, UGHIP_F32, "add_rms_norm_rows y")) return rc;
+  if (y.s)
+    if (int rc = check_view(dev, y, slots ? y_rows : m, n, UGHIP_F32, "add_rms_norm_rows y")) return rc;
+  if (extra.s)
+    if (int rc = check_view(dev, extra, m, n, UGHIP_F32, "add_rms_norm_rows extra")) return rc;
+  if (!y.s && (!x.s || slots)) return set_error(UGHIP_ERR_INVALID, "add_rms_norm_rows: neither rows to norm nor rows to add to");
   if (slots) {
     if (top == 0 || top > 4096) return set_error(UGHIP_ERR_INVALID, "add_rms_norm_rows: top %zu", top);
     if (int rc = check_buf(dev, slots, m * top, UGHIP_I32, "add_rms_norm_rows slots")) return rc;
     if (int rc = check_buf(dev, weights, m * top, UGHIP_F32, "add_rms_norm_rows weights")) return rc;
   }
-  if (int rc = check_buf(dev, w, n, UGHIP_F32, "add_rms_norm_rows w")) return rc;
+  if (y.s)
+    if (int rc = check_buf(dev, w, n, UGHIP_F32, "add_rms_norm_rows w")) return rc;
+  if (next) {
+    if (!copy) return set_error(UGHIP_ERR_INVALID, "add_rms_norm_rows: a second norm without a place for it");
+    if (int rc = check_buf(dev, next, n, UGHIP_F32, "add_rms_norm_rows next")) return rc;
+  }
   void* d;
   bool bf16;
   if (int rc = check_result(dev, dst, m, n, "add_rms_norm_rows dst", &d, &bf16)) return rc;
-  if (dst_bf16)
-    if (int rc = check_buf(dev, dst_bf16, m * n, UGHIP_BF16, "add_rms_norm_rows bf16 rows")) return rc;
+  void* copy_at = nullptr;
+  bool copy_bf16 = false;
+  if (copy)
+    if (int rc = check_result(dev, ughip_view{copy, 0, n}, m, n, "add_rms_norm_rows copy", &copy_at, &copy_bf16)) return rc;
   if (m == 0 || n == 0) return UGHIP_OK;
   if (int rc = device_activate(dev)) return rc;
-  AddNormArgs a{view_ptr<float>(x), view_ptr<float>(y), buf_ptr<float>(w), d, dst_bf16 ? static_cast<uint16_t*>(dst_bf16->ptr) : nullptr, x.stride, y.stride, dst.stride, buf_ptr<int>(slots), buf_ptr<float>(weights),
-                (int)top, (int)y_rows, (int)n, eps, bf16};
+  AddNormArgs a{view_ptr<float>(x), view_ptr<float>(y), buf_ptr<float>(w), d, copy_at, view_ptr<float>(extra), buf_ptr<float>(next), x.stride, y.stride, dst.stride, extra.stride,
+                buf_ptr<int>(slots), buf_ptr<float>(weights), (int)top, (int)y_rows, (int)n, eps, bf16, copy_bf16};
+  auto rows4 = [](const void* q, size_t stride) { return (reinterpret_cast<uintptr_t>(q) & 15) == 0 && (!q || stride % 4 == 0); };
+  if (!slots && n % 4 == 0 && n <= 4096 && rows4(a.x, a.x_stride) && rows4(a.y, a.y_stride) && rows4(a.extra, a.extra_stride) && rows4(d, a.dst_stride)) {
+    add_rms_norm4_kernel<<<(unsigned)m, 256, 0, dev->stream>>>(a);
+    UGHIP_HIPCHK(hipGetLastError());
+    return UGHIP_OK;
+  }
   add_rms_norm_kernel<<<(unsigned)m, 256, n * sizeof(float), dev->stream>>>(a);
   UGHIP_HIPCHK(hipGetLastError());
   return UGHIP_OK;

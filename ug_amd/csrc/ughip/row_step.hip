@@ -29,9 +29,11 @@ struct RowArgs {
   const void* table;
   const int* ids;
   size_t table_stride, table_col, w_group;
+  const float* extra;  // joins x too
+  GluForm glu;
   float eps, inv_k;
   int n, k, cols, norm_groups, table_rows, segs;
-  bool table_bf16;
+  bool table_bf16, gate_after;
   const float* logits;
   RouteArgs route;
   int* route_ids;
@@ -107,7 +109,7 @@ __global__ void __launch_bounds__(256) row_step_kernel(RowArgs a) {
   constexpr int NP = PV ? PV : 1;
   const f32x4_t zero = {0.f, 0.f, 0.f, 0.f};
   const int total = (ROUTE == 2 ? a.segs : 1) * a.k;
-  f32x4_t px[NP], py[NP], pyn[NP], pn[NP];  // x, y or the gate, and the two norms' weights
+  f32x4_t px[NP], py[NP], pyn[NP], pn[NP], pe[NP];  // x, y or the gate, the two norms' weights, and what joins x besides
   if constexpr (PV != 0 && PLAIN) {
 #pragma unroll
     for (int u = 0; u < PV; ++u) {
@@ -123,6 +125,7 @@ __global__ void __launch_bounds__(256) row_step_kernel(RowArgs a) {
       py[u] = ok && (a.y || a.gate) ? *reinterpret_cast<const f32x4_t*>((a.y ? a.y : a.gate) + i) : zero;
       pyn[u] = ok && a.y ? *reinterpret_cast<const f32x4_t*>(a.y_norm + i) : zero;
       pn[u] = ok && a.norm ? *reinterpret_cast<const f32x4_t*>(a.norm + i) : zero;
+      pe[u] = ok && a.extra ? *reinterpret_cast<const f32x4_t*>(a.extra + i) : zero;
     }
   }
   if constexpr (ROUTE == 1) {  // which experts' matrices: before anything of them can be asked for
@@ -219,11 +222,11 @@ __global__ void __launch_bounds__(256) row_step_kernel(RowArgs a) {
       const float inv = 1.f / sqrtf(ss / (float)a.k + a.eps);
 #pragma unroll
       for (int u = 0; u < PV; ++u) {
-        px[u] = px[u] + py[u] * inv * pyn[u];
+        px[u] = px[u] + py[u] * inv * pyn[u] + pe[u];
         const int i = (u * 256 + (int)threadIdx.x) * 4;
         if (a.x_out && blockIdx.x == 0 && i < a.k) *reinterpret_cast<f32x4_t*>(a.x_out + i) = px[u];
       }
-    } else if (a.gate) {
+    } else if (a.gate && !a.gate_after) {
 #pragma unroll
       for (int u = 0; u < PV; ++u)
 #pragma unroll
@@ -237,6 +240,15 @@ __global__ void __launch_bounds__(256) row_step_kernel(RowArgs a) {
       const float inv = 1.f / sqrtf(ss / (float)a.k + a.eps);
 #pragma unroll
       for (int u = 0; u < PV; ++u) px[u] = px[u] * inv * pn[u];
+    } else if (a.norm && a.k < 256 * a.norm_groups) {
+      // parts inside a wave's piece: 4, 8, .. or 128 elements (the host checks)
+      const int part = a.k / a.norm_groups;
+#pragma unroll
+      for (int u = 0; u < PV; ++u) {
+        float s = square(px[u]);
+        for (int d = part >> 3; d; d >>= 1) s += __shfl_xor(s, d, 64);
+        px[u] = px[u] * (1.f / sqrtf(s / (float)part + a.eps)) * pn[u];
+      }
     } else if (a.norm) {
       // parts of whole runs of 256 elements (the host checks): one wave's pieces each
       const int runs = a.k / a.norm_groups / 256;
@@ -254,6 +266,12 @@ __global__ void __launch_bounds__(256) row_step_kernel(RowArgs a) {
         px[u] = px[u] * (1.f / sqrtf(s / (float)(runs * 256) + a.eps)) * pn[u];
       }
     }
+    if (a.gate && a.gate_after) {
+#pragma unroll
+      for (int u = 0; u < PV; ++u)
+#pragma unroll
+        for (int e = 0; e < 4; ++e) px[u][e] *= sigmoid_f(py[u][e]);
+    }
 #pragma unroll
     for (int u = 0; u < PV; ++u) {
       const int i = (u * 256 + (int)threadIdx.x) * 4;
@@ -264,7 +282,7 @@ __global__ void __launch_bounds__(256) row_step_kernel(RowArgs a) {
       float v = 0.f;
       if (i < a.k) {
         v = a.y ? a.y[i] : a.x[i];
-        if (a.gate) v *= silu_f(a.gate[i]);
+        if (a.gate && !a.gate_after) v *= silu_f(a.gate[i]);
       }
       in[i] = v;  // read back by the same thread until the last barrier
       ss += v * v;
@@ -274,7 +292,7 @@ __global__ void __launch_bounds__(256) row_step_kernel(RowArgs a) {
       const float inv = 1.f / sqrtf(ss / (float)a.k + a.eps);
       ss = 0.f;
       for (int i = threadIdx.x; i < a.k; i += 256) {
-        const float v = a.x[i] + in[i] * inv * a.y_norm[i];
+        const float v = a.x[i] + in[i] * inv * a.y_norm[i] + (a.extra ? a.extra[i] : 0.f);
         in[i] = v;
         ss += v * v;
         if (a.x_out && blockIdx.x == 0) a.x_out[i] = v;
@@ -294,6 +312,10 @@ __global__ void __launch_bounds__(256) row_step_kernel(RowArgs a) {
         const float inv = 1.f / sqrtf(s / (float)part + a.eps);
         for (int i = lane; i < part; i += 64) in[g * part + i] *= inv * a.norm[g * part + i];
       }
+    }
+    if (a.gate && a.gate_after) {
+      __syncthreads();
+      for (int i = threadIdx.x; i < a.k; i += 256) in[i] *= sigmoid_f(a.gate[i]);
     }
   }
   __syncthreads();
@@ -340,7 +362,7 @@ __global__ void __launch_bounds__(256) row_step_kernel(RowArgs a) {
     if (NM == 2) {
       float u = acc[NM - 1][r];
       if (a.bias) u += a.bias[a.n + col];
-      v = silu_f(v) * u;
+      v = glu_f(v, u, a.glu);
     } else if (a.table) {
       const int id = a.ids[0];
       float t = __uint_as_float(0x7fc00000u);
@@ -404,17 +426,18 @@ constexpr size_t ROW_MAX = 16000;
 extern "C" int ughip_product_row(ughip_device* dev, const ughip_row_step* p) {
   const char* what = "product_row";
   if (!dev || !p || !p->w || !p->x || !p->dst) return set_error(UGHIP_ERR_INVALID, "%s: null argument", what);
-  if (p->act < UGHIP_ACT_NONE || p->act > UGHIP_ACT_GELU_MUL || p->route < 0 || p->route > 2) return set_error(UGHIP_ERR_INVALID, "%s: act %d, route %d", what, p->act, p->route);
+  if (p->act < UGHIP_ACT_NONE || p->act > UGHIP_ACT_GLU || p->route < 0 || p->route > 2) return set_error(UGHIP_ERR_INVALID, "%s: act %d, route %d", what, p->act, p->route);
   if (p->n == 0) return UGHIP_OK;
   const size_t segs = p->route == 2 ? p->top : 1, total = segs * p->k;
   if (p->k == 0 || p->k > ROW_MAX || segs == 0 || segs > 64 || segs * ((p->k + RUN - 1) / RUN * RUN) > 32 * RUN) return set_error(UGHIP_ERR_UNSUPPORTED, "%s: %zu rows of %zu elements, up to %zu in all (in runs of %d) are supported", what, segs, p->k, (size_t)32 * RUN, RUN);
   if (p->n > 0x7fffffffull / 128) return set_error(UGHIP_ERR_INVALID, "%s: shape too large", what);
   if (p->w->dtype != UGHIP_F32 && p->w->dtype != UGHIP_BF16) return set_error(UGHIP_ERR_UNSUPPORTED, "%s: matrices are F32 or BF16", what);
-  const size_t mats = p->route ? p->experts : 1, w_rows = p->act == UGHIP_ACT_SWIGLU ? 2 * p->n : p->n;
+  const bool glu = p->act == UGHIP_ACT_SWIGLU || p->act == UGHIP_ACT_GLU;  // gate and up rows
+  const size_t mats = p->route ? p->experts : 1, w_rows = glu ? 2 * p->n : p->n;
   if (p->route) {
     if (int rc = route_check(p->experts, p->groups, p->keep, p->top, what)) return rc;
     if (p->top > 64) return set_error(UGHIP_ERR_UNSUPPORTED, "%s: up to 64 experts per row", what);
-    if (p->bias || (p->route == 1) != (p->act == UGHIP_ACT_SWIGLU) || (p->route == 2 && p->act != UGHIP_ACT_NONE) || p->y || p->norm || p->gate)
+    if (p->bias || (p->route == 1 && !glu) || (p->route == 2 && p->act != UGHIP_ACT_NONE) || p->y || p->norm || p->gate)
       return set_error(UGHIP_ERR_UNSUPPORTED, "%s: routed products are SwiGLU (1) or plain (2), on x as it is", what);
     if (int rc = check_buf(dev, p->route_ids, p->top, UGHIP_I32, "product_row ids")) return rc;
     if (int rc = check_buf(dev, p->route_weights, p->top, UGHIP_F32, "product_row weights")) return rc;
@@ -425,6 +448,11 @@ extern "C" int ughip_product_row(ughip_device* dev, const ughip_row_step* p) {
     if (int rc = row(p->y, p->y_offset, p->k, UGHIP_F32)) return rc;
     if (int rc = row(p->y_norm, 0, p->k, UGHIP_F32)) return rc;
   }
+  if (p->extra) {
+    if (!p->y) return set_error(UGHIP_ERR_INVALID, "%s: extra rows come with y", what);
+    if (int rc = row(p->extra, p->extra_offset, p->k, UGHIP_F32)) return rc;
+  }
+  if (p->gate_after && !p->gate) return set_error(UGHIP_ERR_INVALID, "%s: gate_after without a gate", what);
   if (p->gate)
     if (int rc = row(p->gate, p->gate_offset, p->k, UGHIP_F32)) return rc;
   if (p->gate && p->y) return set_error(UGHIP_ERR_UNSUPPORTED, "%s: a gate or a residual, not both", what);
@@ -442,7 +470,7 @@ extern "C" int ughip_product_row(ughip_device* dev, const ughip_row_step* p) {
     if (!p->y) return set_error(UGHIP_ERR_INVALID, "%s: nothing joins x", what);
     if (int rc = row(p->dst, p->x_out, p->k, UGHIP_F32)) return rc;
   }
-  if (p->dst == p->x || p->dst == p->y || p->dst == p->gate) return set_error(UGHIP_ERR_INVALID, "%s: dst aliases an input", what);
+  if (p->dst == p->x || p->dst == p->y || p->dst == p->gate || (p->extra && p->dst == p->extra)) return set_error(UGHIP_ERR_INVALID, "%s: dst aliases an input", what);
   if (p->act == UGHIP_ACT_GELU_MUL) {
     if (!p->table || (p->table->dtype != UGHIP_F32 && p->table->dtype != UGHIP_BF16)) return set_error(UGHIP_ERR_INVALID, "%s: a gate's table is F32 or BF16", what);
     if (int rc = row(p->table, 0, p->table_rows * p->table_stride, -1)) return rc;
@@ -458,7 +486,9 @@ extern "C" int ughip_product_row(ughip_device* dev, const ughip_row_step* p) {
   RowArgs a{};
   a.x = buf_ptr<float>(p->x) + p->x_offset;
   if (p->y) a.y = buf_ptr<float>(p->y) + p->y_offset, a.y_norm = buf_ptr<float>(p->y_norm);
-  if (p->gate) a.gate = buf_ptr<float>(p->gate) + p->gate_offset;
+  if (p->gate) a.gate = buf_ptr<float>(p->gate) + p->gate_offset, a.gate_after = p->gate_after != 0;
+  if (p->extra) a.extra = buf_ptr<float>(p->extra) + p->extra_offset;
+  a.glu = glu_form(p->act, p->act_alpha, p->act_shift, p->act_limit);
   a.norm = buf_ptr<float>(p->norm), a.norm_groups = (int)norm_groups;
   float* d = static_cast<float*>(p->dst->ptr);
   a.x_out = p->keep_x ? d + p->x_out : nullptr;
@@ -481,8 +511,10 @@ extern "C" int ughip_product_row(ughip_device* dev, const ughip_row_step* p) {
   }
   const bool vec = p->k % 8 == 0 && (reinterpret_cast<uintptr_t>(a.w) & 15) == 0;
   auto a16 = [](const void* q) { return (reinterpret_cast<uintptr_t>(q) & 15) == 0; };
-  const bool pieces = p->k % 4 == 0 && (!p->norm || norm_groups == 1 || (p->k / norm_groups) % 256 == 0) && a16(a.x) && a16(a.y) && a16(a.gate) && a16(a.x_out);
-  UGHIP_HIPCHK(p->w->dtype == UGHIP_BF16 ? launch_any<uint16_t>(dev->stream, a, p->route, p->act == UGHIP_ACT_SWIGLU, lds, vec, pieces)
-                                         : launch_any<float>(dev->stream, a, p->route, p->act == UGHIP_ACT_SWIGLU, lds, vec, pieces));
+  const size_t part = p->k / norm_groups;
+  const bool parts_fit = !p->norm || norm_groups == 1 || part % 256 == 0 || (part >= 4 && part < 256 && (part & (part - 1)) == 0);
+  const bool pieces = p->k % 4 == 0 && parts_fit && a16(a.x) && a16(a.y) && a16(a.gate) && a16(a.x_out) && a16(a.extra);
+  UGHIP_HIPCHK(p->w->dtype == UGHIP_BF16 ? launch_any<uint16_t>(dev->stream, a, p->route, glu, lds, vec, pieces)
+                                         : launch_any<float>(dev->stream, a, p->route, glu, lds, vec, pieces));
   return UGHIP_OK;
 }

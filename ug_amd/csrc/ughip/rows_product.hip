@@ -38,6 +38,7 @@ struct ProductArgs {
   const int* row_index;
   const int* group_end;
   int groups, x_rows;
+  GluForm glu;
 };
 
 // One 16-byte LDS chunk's worth of a row, as it is stored: 8 elements for bf16 products, 4 for f32 ones.
@@ -272,7 +273,7 @@ __global__ void __launch_bounds__(256) rows_product_kernel(ProductArgs a) {
         if constexpr (ACT == UGHIP_ACT_SWIGLU) {
           float u = acc[i][1][e];
           if (a.bias) u += a.bias[a.n + col];
-          v = silu_f(v) * u;
+          v = glu_f(v, u, a.glu);
         }
         if constexpr (ACT == UGHIP_ACT_GELU_MUL) v = gelu_tanh_f(v) * __uint_as_float(!there[i][e] ? 0x7fc00000u : a.table_bf16 ? factor[i][e][j] << 16 : factor[i][e][j]);
         const size_t at = (size_t)r * a.dst_stride + col;
@@ -322,7 +323,9 @@ extern "C" int ughip_product_rows(ughip_device* dev, const ughip_product* p) {
   const char* what = "product_rows";
   if (!dev || !p || !p->w) return set_error(UGHIP_ERR_INVALID, "%s: null argument", what);
   if (p->product != UGHIP_PRODUCT_F32 && p->product != UGHIP_PRODUCT_BF16) return set_error(UGHIP_ERR_INVALID, "%s: unknown product %d", what, p->product);
-  if (p->act < UGHIP_ACT_NONE || p->act > UGHIP_ACT_GELU_MUL) return set_error(UGHIP_ERR_INVALID, "%s: unknown act %d", what, p->act);
+  if (p->act < UGHIP_ACT_NONE || p->act > UGHIP_ACT_GLU) return set_error(UGHIP_ERR_INVALID, "%s: unknown act %d", what, p->act);
+  const bool glu = p->act == UGHIP_ACT_SWIGLU || p->act == UGHIP_ACT_GLU;  // gate and up rows
+  const int act = glu ? (int)UGHIP_ACT_SWIGLU : p->act;
   if (p->m == 0 || p->n == 0) return UGHIP_OK;
   if (p->k == 0) return set_error(UGHIP_ERR_INVALID, "%s: k == 0", what);
   const bool f32 = p->product == UGHIP_PRODUCT_F32;
@@ -333,7 +336,7 @@ extern "C" int ughip_product_rows(ughip_device* dev, const ughip_product* p) {
   if (x_rows == 0) return set_error(UGHIP_ERR_INVALID, "%s: no rows of x", what);
   if (int rc = check_view(dev, p->x, x_rows, p->k, f32 ? UGHIP_F32 : -1, "product_rows x")) return rc;
   const size_t w_stride = p->w_stride ? p->w_stride : p->k;
-  const size_t w_rows = p->act == UGHIP_ACT_SWIGLU ? 2 * p->n : p->n;
+  const size_t w_rows = glu ? 2 * p->n : p->n;
   if (w_stride != p->k && p->groups) return set_error(UGHIP_ERR_UNSUPPORTED, "%s: rows of w %zu elements apart belong to the plain form", what, w_stride);
   if (p->groups) {
     if (int rc = check_buf(dev, p->w, mats * w_rows * p->k, f32 ? UGHIP_F32 : -1, "product_rows w")) return rc;
@@ -373,6 +376,7 @@ extern "C" int ughip_product_rows(ughip_device* dev, const ughip_product* p) {
     a.table_stride = p->table_stride, a.table_col = p->table_col, a.ids = buf_ptr<int>(p->ids);
   }
   a.row_index = buf_ptr<int>(p->row_index), a.group_end = buf_ptr<int>(p->group_end), a.groups = (int)p->groups, a.x_rows = (int)x_rows;
+  a.glu = glu_form(p->act, p->act_alpha, p->act_shift, p->act_limit);
   const bool vec = p->k % 8 == 0 && (p->x.stride * xs) % 16 == 0 && (w_stride * (p->w->dtype == UGHIP_BF16 ? 2 : 4)) % 16 == 0 && aligned16(a.x) && aligned16(a.w);
   const bool xb = p->x.s->dtype == UGHIP_BF16, wb = p->w->dtype == UGHIP_BF16;
   // few dense rows: products that share their K among workgroups
@@ -388,20 +392,20 @@ extern "C" int ughip_product_rows(ughip_device* dev, const ughip_product* p) {
     DmaRows r;
     r.row_index = a.row_index, r.group_end = a.group_end, r.bias = a.bias, r.dst = a.dst, r.w_group = (long long)a.w_group, r.dst_stride = (long long)a.dst_stride;
     r.groups = a.groups, r.x_rows = a.x_rows, r.n_out = a.n, r.dst_bf16 = a.dst_bf16;
-    const bool swiglu = p->act == UGHIP_ACT_SWIGLU;
-    if (const int tile = gemm_dma_rows_pick(q, r, swiglu)) {
-      UGHIP_HIPCHK(gemm_dma_launch_rows(dev->stream, q, r, swiglu, tile));
+    r.glu_alpha = a.glu.alpha, r.glu_shift = a.glu.shift, r.glu_limit = a.glu.limit;
+    if (const int tile = gemm_dma_rows_pick(q, r, glu)) {
+      UGHIP_HIPCHK(gemm_dma_launch_rows(dev->stream, q, r, glu, tile));
       return UGHIP_OK;
     }
   }
   hipError_t e;
-  if (f32) e = launch_types<float, float, float>(dev->stream, a, p->act, vec);
-  else if (xb && wb) e = launch_types<__bf16, uint16_t, uint16_t>(dev->stream, a, p->act, vec);
-  else if (wb) e = launch_types<__bf16, float, uint16_t>(dev->stream, a, p->act, vec);
+  if (f32) e = launch_types<float, float, float>(dev->stream, a, act, vec);
+  else if (xb && wb) e = launch_types<__bf16, uint16_t, uint16_t>(dev->stream, a, act, vec);
+  else if (wb) e = launch_types<__bf16, float, uint16_t>(dev->stream, a, act, vec);
   else if (p->act == UGHIP_ACT_NONE && xb) e = launch_act<__bf16, uint16_t, float, UGHIP_ACT_NONE>(dev->stream, a, vec);
   else if (p->act == UGHIP_ACT_NONE) e = launch_act<__bf16, float, float, UGHIP_ACT_NONE>(dev->stream, a, vec);
   else return set_error(UGHIP_ERR_UNSUPPORTED, "%s: bf16 products with an activation take a BF16 matrix", what);
   UGHIP_HIPCHK(e);
-  note_kernel("rows_product<%s,%s%s>", f32 ? "f32" : "bf16", p->act == UGHIP_ACT_SWIGLU ? "swiglu" : p->act == UGHIP_ACT_GELU_MUL ? "gelu_mul" : "none", p->groups ? ",grouped" : "");
+  note_kernel("rows_product<%s,%s%s>", f32 ? "f32" : "bf16", p->act == UGHIP_ACT_SWIGLU ? "swiglu" : p->act == UGHIP_ACT_GLU ? "glu" : p->act == UGHIP_ACT_GELU_MUL ? "gelu_mul" : "none", p->groups ? ",grouped" : "");
   return UGHIP_OK;
 }

@@ -479,10 +479,13 @@ extern "C" int ughip_conv_silu_rows(ughip_device* dev, ughip_view x, const ughip
   if (t == 0 || channels == 0) return UGHIP_OK;
   if (int rc = device_activate(dev)) return rc;
   auto a16 = [](const void* p) { return (reinterpret_cast<uintptr_t>(p) & 15) == 0; };
-  if (n_taps == 4 && channels % 4 == 0 && x.stride % 4 == 0 && dst.stride % 4 == 0 && a16(view_ptr<float>(x)) && a16(view_ptr<float>(dst)) && t / ROWS_CONV < 65535) {
+  if (n_taps >= 2 && n_taps <= 4 && channels % 4 == 0 && x.stride % 4 == 0 && dst.stride % 4 == 0 && a16(view_ptr<float>(x)) && a16(view_ptr<float>(dst)) && t / ROWS_CONV < 65535) {
     const dim3 g4((unsigned)((channels / 4 + 255) / 256), (unsigned)((t + ROWS_CONV - 1) / ROWS_CONV));
-    conv_silu_rows4_kernel<4><<<g4, 256, 0, dev->stream>>>(view_ptr<float>(x), x.stride, buf_ptr<float>(taps), buf_ptr<float>(bias), buf_ptr<float>(ring), (long long)pos,
-                                                           (int)t, (int)channels, view_ptr<float>(dst), dst.stride);
+    auto go = [&](auto kernel) {
+      kernel<<<g4, 256, 0, dev->stream>>>(view_ptr<float>(x), x.stride, buf_ptr<float>(taps), buf_ptr<float>(bias), buf_ptr<float>(ring), (long long)pos, (int)t, (int)channels,
+                                          view_ptr<float>(dst), dst.stride);
+    };
+    n_taps == 4 ? go(conv_silu_rows4_kernel<4>) : n_taps == 3 ? go(conv_silu_rows4_kernel<3>) : go(conv_silu_rows4_kernel<2>);
     UGHIP_HIPCHK(hipGetLastError());
     return UGHIP_OK;
   }
