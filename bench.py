@@ -1010,16 +1010,29 @@ def hybrid_config(width, layers, heads, q_rank, kv_rank, ssm_heads, ssm_groups, 
     return {"architecture": "Tanolorn", "vocab": 32000, "width": width, "norm": {"eps": 1e-5}, "token_side": {"dim": side}, "layers": out}
 
 
+def tugelorn_config(width, layers, heads, kv_heads, ff):
+    """A Tugelorn of the size a real model's layers have (heads of 128): every second layer is a delta rule, the others take turns
+    between attention over a window of 1024 and over everything."""
+    sizes = {"heads": heads, "kv_heads": kv_heads, "dim": 128, "vdim": 128, "scale": 128 ** -0.5}
+    window = {"type": "attention", "mixer": {**sizes, "mask": {"size": 1024}, "rot": {"base": 10000.0, "dims": 128, "scaling": {"factor": 2.0}}}}
+    full = {"type": "attention_2", "mixer": {**sizes, "q_temp": {"coef": 0.1, "every": 4096}}}
+    delta = {"type": "channel_delta", "mixer": {"heads": heads, "kv_heads": heads, "dim": 128, "vdim": 128, "conv": 4}}
+    return {"architecture": "Tugelorn", "vocab": 32000, "width": width, "norm": {"eps": 1e-5}, "residual_mult": 0.5,
+            "layers": [{**((delta, window, delta, full)[i % 4]), "mlp": {"kind": "dense", "ff": ff, "limit": 7.0}} for i in range(layers)]}
+
+
 def llama_config(width, layers, heads, kv_heads, ff):
     return {"model_type": "llama", "hidden_size": width, "intermediate_size": ff, "max_position_embeddings": 4096, "num_attention_heads": heads, "num_key_value_heads": kv_heads,
             "num_hidden_layers": layers, "rms_norm_eps": 1e-5, "vocab_size": 32000}
 
 
-# width -> the two designs at equal width, depth and (active) feed-forward size
+# width -> the designs at equal width, depth and (active) feed-forward size
 DECODER_SIZES = {
-    "1024": (hybrid_config(1024, 6, 8, 512, 256, 32, 4, 2816, 16, 4, 704, 128), llama_config(1024, 6, 16, 4, 2816)),
-    "2048": (hybrid_config(2048, 6, 16, 768, 512, 64, 8, 5632, 16, 4, 1408, 256), llama_config(2048, 6, 32, 4, 5632)),
-    "4096": (hybrid_config(4096, 3, 32, 1536, 512, 128, 8, 11008, 8, 2, 5504, 256), llama_config(4096, 3, 32, 8, 11008)),
+    "1024": {"tanolorn": hybrid_config(1024, 6, 8, 512, 256, 32, 4, 2816, 16, 4, 704, 128), "tugelorn": tugelorn_config(1024, 6, 8, 2, 2816), "llama": llama_config(1024, 6, 16, 4, 2816)},
+    "2048": {"tanolorn": hybrid_config(2048, 6, 16, 768, 512, 64, 8, 5632, 16, 4, 1408, 256), "tugelorn": tugelorn_config(2048, 6, 16, 4, 5632),
+             "llama": llama_config(2048, 6, 32, 4, 5632)},
+    "4096": {"tanolorn": hybrid_config(4096, 3, 32, 1536, 512, 128, 8, 11008, 8, 2, 5504, 256), "tugelorn": tugelorn_config(4096, 3, 32, 8, 11008),
+             "llama": llama_config(4096, 3, 32, 8, 11008)},
 }
 
 
@@ -1043,13 +1056,13 @@ def decoder_throughput(dev, config, prompts=(128, 512, 2048), n_steps=64):
     return out
 
 
-def decoders(dev, sizes=tuple(DECODER_SIZES)):
-    """Tanolorn beside llama at equal width and depth (random weights, bf16 matrices)."""
+def decoders(dev, sizes=tuple(DECODER_SIZES), models=("tanolorn", "tugelorn", "llama")):
+    """Tanolorn and Tugelorn beside llama at equal width and depth (random weights, bf16 matrices)."""
     dev.set_zero_fill(False)
     out = {}
     for size in sizes:
-        hybrid, llama = DECODER_SIZES[size]
-        out[f"width {size}, {len(hybrid['layers'])} layers"] = {"tanolorn": decoder_throughput(dev, hybrid), "llama": decoder_throughput(dev, llama)}
+        configs = DECODER_SIZES[size]
+        out[f"width {size}, {len(configs['tanolorn']['layers'])} layers"] = {m: decoder_throughput(dev, configs[m]) for m in models}
         print(f"decoders: width {size} done", file=sys.stderr, flush=True)
     dev.set_zero_fill(True)
     return out
@@ -1145,6 +1158,7 @@ def main():
     ap.add_argument("--headline-only", action="store_true", help="only the config-2 kernel: no extras, no llama, no CPU baseline")
     ap.add_argument("--only", choices=["softmax", "bmm", "llama_pieces", "hbm_large", "floors", "safetensors", "cpu", "llama", "decoders"], help="besides the headline, run just this group (profiler runs)")
     ap.add_argument("--decoder-size", action="append", choices=list(DECODER_SIZES), help="with --only decoders: this width only (may be given several times)")
+    ap.add_argument("--decoder-model", action="append", choices=["tanolorn", "tugelorn", "llama"], help="with --only decoders: this model only (may be given several times)")
     ap.add_argument("--no-cpu-baseline", action="store_true")
     ap.add_argument("--sustained-trace", type=float, default=0.0, metavar="SECONDS",
                     help="also run the headline step without a pause for this long and report its rate per 50 ms of elapsed time")
@@ -1219,7 +1233,7 @@ def main():
             line["extras"] = {"error": f"{type(e).__name__}: {e}"}
     if args.only == "decoders":
         try:
-            line.setdefault("extras", {})["decoders"] = decoders(dev, args.decoder_size or tuple(DECODER_SIZES))
+            line.setdefault("extras", {})["decoders"] = decoders(dev, args.decoder_size or tuple(DECODER_SIZES), args.decoder_model or ("tanolorn", "tugelorn", "llama"))
         except Exception as e:  # noqa: BLE001
             line.setdefault("extras", {})["decoders"] = {"error": f"{type(e).__name__}: {e}"}
     if not (args.no_llama or args.headline_only):
