@@ -3,7 +3,8 @@
 //   A wave owns 32 queries, a workgroup 128; keys come in tiles of 64 through LDS.  The scores are computed transposed, S^T = K Q^T
 //   (32 x 32 tiles), which leaves lane l with query l % 32 as its column: the running maximum and sum are one exchange with lane
 //   l ^ 32, and the weights sit where the second product, O^T = V^T P^T, wants its right operand (the order in which keys take
-//   part in it is the order the accumulator layout gives; V is read in the same order).  Values come transposed for that.
+//   part in it is the order the accumulator layout gives; V is read in the same order).  Values come transposed for that.  Two such
+//   groups of waves take turns with the tiles of keys where registers allow it.
 //   bf16 operands: v_mfma_f32_32x32x16_bf16, a weight as two bf16 terms (16 bits of it); f32: v_mfma_f32_32x32x2_f32.
 #pragma once
 #include <hip/hip_runtime.h>
@@ -52,25 +53,37 @@ __device__ __forceinline__ void mfma_chunk(const u32x4_t& a, const u32x4_t& b, f
 }
 
 constexpr int ATT_KT = 64, ATT_QT = 128;
+// Two groups of four waves share the queries and take every second tile of keys, where the registers of two waves per SIMD hold the
+// tiles; their results meet at the end.
+template <typename T, int DQ, int DV>
+constexpr int attention_rows_groups() {
+  return sizeof(T) == 2 && DQ <= 192 && DV <= 128 ? 2 : 1;
+}
+template <typename T, int DQ, int DV>
+constexpr int attention_rows_threads() {
+  return 256 * attention_rows_groups<T, DQ, DV>();
+}
 template <typename T, int DQ, int DV>
 constexpr int attention_rows_lds_bytes() {
-  return ATT_KT * (DQ * (int)sizeof(T) + 16) + DV * (ATT_KT * (int)sizeof(T) + 16);
+  return attention_rows_groups<T, DQ, DV>() * (ATT_KT * (DQ * (int)sizeof(T) + 16) + DV * (ATT_KT * (int)sizeof(T) + 16));
 }
 
 // DQ >= dim + rot and DV >= vdim, the surplus is zeros.  T: uint16_t (bf16) or float.
 template <typename T, int DQ, int DV>
-__global__ void __launch_bounds__(256) attention_rows_kernel(AttRowsArgs a) {
+__global__ void __launch_bounds__((attention_rows_threads<T, DQ, DV>())) attention_rows_kernel(AttRowsArgs a) {
   constexpr int E = 16 / sizeof(T), QC = DQ / E, K_ROW = DQ * sizeof(T) + 16, V_ROW = ATT_KT * sizeof(T) + 16, VC = ATT_KT / E;
   constexpr int NK = ATT_KT * QC / 256, NV = DV * VC / 256;  // 16-byte pieces of a tile per thread
   constexpr bool AHEAD = NK + NV <= 16;                   // the next tile waits in registers while this one is multiplied
   static_assert(ATT_KT * QC % 256 == 0 && DV * VC % 256 == 0, "whole pieces per thread");
   extern __shared__ __attribute__((aligned(16))) char lds[];
-  char* Ks = lds;                // [ATT_KT][DQ]
-  char* Vs = lds + ATT_KT * K_ROW;   // [DV][ATT_KT]
+  constexpr int GROUPS = attention_rows_groups<T, DQ, DV>();
+  const int group = threadIdx.x >> 8, tid = threadIdx.x & 255;
+  char* Ks = lds + group * (ATT_KT * K_ROW + DV * V_ROW);  // [ATT_KT][DQ]
+  char* Vs = Ks + ATT_KT * K_ROW;                          // [DV][ATT_KT]
   // consecutive workgroups (dealt round robin to the chip's eight parts) take different key heads: those that share one meet in a cache
   const int per = gridDim.x / a.kv_heads, kv = blockIdx.x % a.kv_heads, head = kv * per + blockIdx.x / a.kv_heads;
   const int qb = gridDim.y - 1 - blockIdx.y;  // the longest rows first
-  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, col = lane & 31, hf = lane >> 5;
+  const int lane = tid & 63, wave = tid >> 6, col = lane & 31, hf = lane >> 5;
   const int i_mine = qb * ATT_QT + wave * 32 + col, p_mine = a.pos + min(i_mine, a.t - 1);
   // the wave's queries as the right operand of S^T: chunk 2 c + hf of query `col` (rows up to q_rows exist, zeros past t)
   u32x4_t qf[QC / 2];
@@ -92,11 +105,11 @@ __global__ void __launch_bounds__(256) attention_rows_kernel(AttRowsArgs a) {
   u32x4_t kr[NK], vr[NV];
   auto fetch = [&](int k0) {
 #pragma unroll
-    for (int u = 0; u < NK; ++u) kr[u] = *reinterpret_cast<const u32x4_t*>(k_head + (size_t)k0 * DQ * sizeof(T) + (threadIdx.x + u * 256) * 16);
+    for (int u = 0; u < NK; ++u) kr[u] = *reinterpret_cast<const u32x4_t*>(k_head + (size_t)k0 * DQ * sizeof(T) + (tid + u * 256) * 16);
 #pragma unroll
     for (int u = 0; u < NV; ++u) {
       // rows are padded to whole tiles and 16-byte aligned; every lane loads (no branches between loads)
-      const int x = threadIdx.x + u * 256, vc = x / VC;
+      const int x = tid + u * 256, vc = x / VC;
       vr[u] = *reinterpret_cast<const u32x4_t*>(v_head + (size_t)(vc < a.vdim ? vc : 0) * a.v_stride + k0 + x % VC * E);
     }
   };
@@ -110,23 +123,28 @@ __global__ void __launch_bounds__(256) attention_rows_kernel(AttRowsArgs a) {
     __builtin_memcpy(&out, v, 16);
     return out;
   };
-  if (AHEAD) fetch(k_begin);
-  for (int k0 = k_begin; k0 < keys; k0 += ATT_KT) {
+  const int k_mine = k_begin + group * ATT_KT;
+  if (AHEAD && k_mine < keys) fetch(k_mine);
+  for (int k0 = k_mine; k0 - group * ATT_KT < keys; k0 += GROUPS * ATT_KT) {
     __syncthreads();
+    const bool there = GROUPS == 1 || k0 < keys;  // (the last tile of an odd number is the first group's alone)
+    if (there) {
     if (!AHEAD) fetch(k0);
 #pragma unroll
     for (int u = 0; u < NK; ++u) {
-      const int x = threadIdx.x + u * 256;
+      const int x = tid + u * 256;
       *reinterpret_cast<u32x4_t*>(Ks + x / QC * K_ROW + x % QC * 16) = kr[u];
     }
 #pragma unroll
     for (int u = 0; u < NV; ++u) {
-      const int x = threadIdx.x + u * 256;
+      const int x = tid + u * 256;
       const bool whole = k0 + ATT_KT <= s_all && DV == a.vdim;
       *reinterpret_cast<u32x4_t*>(Vs + x / VC * V_ROW + x % VC * 16) = whole ? vr[u] : value_piece(vr[u], x / VC, k0 + x % VC * E);
     }
+    }
     __syncthreads();
-    if (AHEAD && k0 + ATT_KT < keys) fetch(k0 + ATT_KT);
+    if (AHEAD && k0 + GROUPS * ATT_KT < keys) fetch(k0 + GROUPS * ATT_KT);
+    if (!there) continue;
     if (k0 > first_p + 31 || (a.window && k0 + ATT_KT - 1 <= first_p - a.window)) continue;  // nothing in this tile is visible to the wave's queries
     f32x16 s[2];
 #pragma unroll
@@ -213,6 +231,32 @@ __global__ void __launch_bounds__(256) attention_rows_kernel(AttRowsArgs a) {
           }
       }
     }
+  }
+  if constexpr (GROUPS == 2) {
+    constexpr int N = DV / 32 * 4;
+    static_assert(4 * 64 * (N * 16 + 8) <= attention_rows_lds_bytes<T, DQ, DV>(), "a group's results fit where the tiles were");
+    f32x4_t* other = reinterpret_cast<f32x4_t*>(lds) + wave * N * 64 + lane;
+    float* ms = reinterpret_cast<float*>(lds + 4 * 64 * N * 16) + (wave * 64 + lane) * 2;
+    __syncthreads();
+    if (group == 1) {
+#pragma unroll
+      for (int i = 0; i < DV / 32; ++i)
+#pragma unroll
+        for (int q = 0; q < 4; ++q) other[(i * 4 + q) * 64] = f32x4_t{o[i][4 * q], o[i][4 * q + 1], o[i][4 * q + 2], o[i][4 * q + 3]};
+      ms[0] = mx, ms[1] = sum;
+    }
+    __syncthreads();
+    if (group == 1) return;
+    const float m2 = ms[0], s2 = ms[1], top = fmaxf(mx, m2), base = top == -INFINITY ? 0.f : top, f1 = exp2f(mx - base), f2 = exp2f(m2 - base);
+    sum = f1 * sum + f2 * s2;
+#pragma unroll
+    for (int i = 0; i < DV / 32; ++i)
+#pragma unroll
+      for (int q = 0; q < 4; ++q) {
+        const f32x4_t v = other[(i * 4 + q) * 64];
+#pragma unroll
+        for (int e = 0; e < 4; ++e) o[i][4 * q + e] = f1 * o[i][4 * q + e] + f2 * v[e];
+      }
   }
   if (i_mine >= a.t) return;
   const float inv = 1.f / sum;

@@ -10,13 +10,16 @@
 //   delta_scan     (chunks in order)     U = V' - W S, then S'; leaves U and the S in front of every chunk
 //   delta_out      (all chunks at once)  o, normed and gated
 // A quotient G_i / G_j is never taken as one: with strong decays both are too small for f32.  The logarithms are summed inside blocks of
-// 16 rows; between two blocks the quotient is split at the later block's start into two factors <= 1, inside a block every pair has its
-// exponential.
+// 16 rows; between two blocks the quotient is split at the later block's start into two factors <= 1; inside a block it is the product of
+// G_i and 1 / G_j from the block's start as long as the latter stays small, and an exponential per pair otherwise.
+// The triangular system is solved by blocks: the inverses of its diagonal blocks by substitution, the rest as products.
 // The products are v_mfma_f32_16x16x4_f32 (lane l: row or column l % 16, k = l / 16; result element e: row 4 (l / 16) + e, column
 // l % 16).  Four of them take k = 4 (l / 16) + e as element e of a lane's 16 bytes, on both sides: a left operand is then 16 bytes of a
 // row, and a result is a right operand as it is.  That is how the state stays in registers over the scan (every wave holds all
 // channels of 16 columns; what a wave updates of them goes round through LDS), and the layout U and the states are left in.
 #include <hip/hip_runtime.h>
+
+#include <type_traits>
 
 #include "bf16_split.h"
 #include "layers.h"
@@ -89,8 +92,8 @@ __global__ void __launch_bounds__(256) delta_prepare_kernel(DeltaArgs a) {
   float* K = lds;             // [C][ds]
   float* Q = K + C * ds;      // [C][ds]
   float* B = Q + C * ds;      // [C][ds]: log2 of the decays, summed from the start of a block of 16 rows
-  float* At = B + C * ds;     // [C][C + 4]: A transposed
-  float* beta = At + C * (C + 4);
+  float* A = B + C * ds;      // [C][C + 4]: A, then the inverses of I + A in the diagonal blocks
+  float* beta = A + C * (C + 4);
   constexpr int as = C + 4;
   const size_t at = (size_t)chunk * a.heads + h;
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, j = lane & 15, kg = lane >> 4;
@@ -112,7 +115,6 @@ __global__ void __launch_bounds__(256) delta_prepare_kernel(DeltaArgs a) {
     *reinterpret_cast<f32x4_t*>(Q + r * ds + c) = q;
     *reinterpret_cast<f32x4_t*>(B + r * ds + c) = l;
   }
-  for (int e = threadIdx.x; e < C * as / 4; e += 256) *reinterpret_cast<f32x4_t*>(At + 4 * e) = zero;
   if (threadIdx.x < C) beta[threadIdx.x] = (int)threadIdx.x < rows ? exact_sigmoid(a.b[(size_t)(row0 + threadIdx.x) * a.b_stride + h]) : 0.f;
   __syncthreads();
   // unit vectors: 16 lanes per row
@@ -158,13 +160,32 @@ __global__ void __launch_bounds__(256) delta_prepare_kernel(DeltaArgs a) {
 #pragma unroll
         for (int e = 0; e < 4; ++e) {
           const int i = 16 * I + 4 * kg + e;
-          At[(16 * J + j) * as + i] = ak[e] * beta[i];
+          A[i * as + 16 * J + j] = ak[e] * beta[i];
           P[i * C + 16 * J + j] = aq[e];
         }
       }
   }
-  // pairs of the same block: row 16 I + j against rows 16 I + 4 kg ..
+  // pairs of the same block
   for (int I = wave; I < NB; I += 4) {
+    float least = 0.f;
+    for (int c = lane; c < dp; c += 64) least = fminf(least, B[(16 * I + 15) * ds + c]);
+    least = -wave_max(-least);
+    if (least > -64.f) {  // the same for the whole wave
+      f32x4_t ak = zero, aq = zero;
+      for (int c = 4 * kg; c < dp; c += 16) {
+        const f32x4_t l = row4(B, 16 * I + j, c), k = row4(K, 16 * I + j, c), left = exp2_4(l), right = k * exp2_4(-l);
+        ak = mfma16x16(k * left, right, ak);
+        aq = mfma16x16(row4(Q, 16 * I + j, c) * left, right, aq);
+      }
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        const int i = 4 * kg + e, row = 16 * I + i;
+        A[row * as + 16 * I + j] = j < i ? ak[e] * beta[row] : 0.f;
+        P[row * C + 16 * I + j] = j <= i ? aq[e] : 0.f;
+      }
+      continue;
+    }
+    // row 16 I + j against rows 16 I + 4 kg ..
     float ak[4] = {0.f, 0.f, 0.f, 0.f}, aq[4] = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll 2
     for (int c = 0; c < dp; c += 4) {
@@ -184,48 +205,81 @@ __global__ void __launch_bounds__(256) delta_prepare_kernel(DeltaArgs a) {
 #pragma unroll
     for (int x = 0; x < 4; ++x) {
       const int jj = 4 * kg + x;
-      if (jj < j) At[(16 * I + jj) * as + 16 * I + j] = ak[x] * bt;
+      A[(16 * I + j) * as + 16 * I + jj] = jj < j ? ak[x] * bt : 0.f;
       P[(16 * I + j) * C + 16 * I + jj] = jj <= j ? aq[x] : 0.f;
     }
   }
   __syncthreads();
 
-  // (I + A) X = right-hand side, a column per thread: first the channels of beta G K, then the columns of beta V
-  float* W = a.w + at * C * dp;
-  float* V = a.v + at * C * a.vp;
-  for (int col = threadIdx.x; col < dp + a.vp; col += 256) {
-    float x[C];
-    if (col < dp) {
-      float before = 0.f;  // blocks in front of this one
+  // the inverses of the diagonal blocks, a column per lane
+  if (wave < NB && lane < 16) {
+    float* block = A + 16 * wave * as + 16 * wave;
+    float x[16];
+#pragma unroll
+    for (int i = 0; i < 16; ++i) {
+      float v = i == lane ? 1.f : 0.f;
+#pragma unroll
+      for (int m = 0; m < i; ++m) v -= block[i * as + m] * x[m];
+      x[i] = v;
+    }
+#pragma unroll
+    for (int i = 0; i < 16; ++i) block[i * as + lane] = x[i];
+  }
+  __syncthreads();
+  // (I + A) X = right-hand side, 16 columns per wave and turn: first the channels of beta G K, then the columns of beta V
+  {
+    f32x4_t m[NB][NB];
+#pragma unroll
+    for (int I = 0; I < NB; ++I)
+#pragma unroll
+      for (int J = 0; J <= I; ++J) m[I][J] = *reinterpret_cast<const f32x4_t*>(A + (16 * I + j) * as + 16 * J + 4 * kg);
+    const float* values = a.qkv + (size_t)row0 * a.qkv_stride + (size_t)2 * a.kv_heads * d + (size_t)h * a.vdim;
+    const int kt = dp / 16, all = kt + a.vp / 16;
+    f32x4_t ahead[NB];
+    auto fetch = [&](int tile) {
+      if (tile < kt || tile >= all) return;  // uniform over the wave
+      const int c = (tile - kt) * 16 + j;
+      const float* col = values + (c < a.vdim ? c : 0);
+#pragma unroll
+      for (int I = 0; I < NB; ++I)
+#pragma unroll
+        for (int e = 0; e < 4; ++e) ahead[I][e] = col[(size_t)min(16 * I + 4 * kg + e, rows - 1) * a.qkv_stride];
+    };
+    fetch(wave);
+    for (int tile = wave; tile < all; tile += 4) {
+      f32x4_t x[NB];
+      const int c = (tile < kt ? tile : tile - kt) * 16 + j;
+      if (tile < kt) {
+        float before = 0.f;  // blocks in front of this one
+#pragma unroll
+        for (int I = 0; I < NB; ++I) {
+#pragma unroll
+          for (int e = 0; e < 4; ++e) {
+            const int row = 16 * I + 4 * kg + e;
+            x[I][e] = beta[row] * K[row * ds + c] * __builtin_amdgcn_exp2f(before + B[row * ds + c]);
+          }
+          before += B[(16 * I + 15) * ds + c];
+        }
+      } else {
+        const float on = c < a.vdim ? 1.f : 0.f;
+#pragma unroll
+        for (int I = 0; I < NB; ++I)
+#pragma unroll
+          for (int e = 0; e < 4; ++e) x[I][e] = on * beta[16 * I + 4 * kg + e] * ahead[I][e];  // (beta is 0 past the last row)
+      }
+      fetch(tile + 4);
+      float* out = (tile < kt ? a.w + at * C * dp : a.v + at * C * a.vp) + c;
+      const int stride = tile < kt ? dp : a.vp;
 #pragma unroll
       for (int I = 0; I < NB; ++I) {
+        f32x4_t acc = zero;
 #pragma unroll
-        for (int r = 0; r < 16; ++r) x[16 * I + r] = beta[16 * I + r] * K[(16 * I + r) * ds + col] * __builtin_amdgcn_exp2f(before + B[(16 * I + r) * ds + col]);
-        before += B[(16 * I + 15) * ds + col];
-      }
-    } else {
-      const int c = col - dp;
-      const bool ok = c < a.vdim;
-      const float* src = a.qkv + (size_t)row0 * a.qkv_stride + (size_t)2 * a.kv_heads * d + (size_t)h * a.vdim + (ok ? c : 0);
-      const float on = ok ? 1.f : 0.f;
+        for (int J = 0; J < I; ++J) acc = mfma16x16(m[I][J], x[J], acc);
+        x[I] = mfma16x16(m[I][I], x[I] - acc, zero);
 #pragma unroll
-      for (int r = 0; r < C; ++r) x[r] = on * beta[r] * src[(size_t)min(r, rows - 1) * a.qkv_stride];  // (beta is 0 past the last row)
-    }
-#pragma unroll
-    for (int r = 0; r + 1 < C; ++r) {
-      // x[r] is final: its part of the rows below
-#pragma unroll
-      for (int i4 = (r + 1) / 4; i4 < C / 4; ++i4) {
-        const f32x4_t m = *reinterpret_cast<const f32x4_t*>(At + r * as + 4 * i4);
-#pragma unroll
-        for (int e = 0; e < 4; ++e)
-          if (4 * i4 + e > r) x[4 * i4 + e] -= m[e] * x[r];
+        for (int e = 0; e < 4; ++e) out[(size_t)(16 * I + 4 * kg + e) * stride] = x[I][e];
       }
     }
-    float* out = col < dp ? W + col : V + (col - dp);
-    const int stride = col < dp ? dp : a.vp;
-#pragma unroll
-    for (int r = 0; r < C; ++r) out[(size_t)r * stride] = x[r];
   }
   // G q, row by row, and G_C / G k, transposed
   float* QG = a.qg + at * C * dp;
@@ -277,44 +331,45 @@ __global__ void __launch_bounds__(256) delta_scan_kernel(DeltaArgs a) {
     }
     Ss[wave + 4 * m][lane] = mine[m];
   }
-  f32x4_t wf[NT], v0 = zero, kf[MINE][NB], gm[MINE];
+  // what a chunk brings, on its way from two chunks before
+  struct Held {
+    f32x4_t wf[NT], v0, kf[MINE][NB], gm[MINE];
+  } held[2];
   const int ub = NB == 4 ? wave : wave % NB;  // the block of 16 rows whose U the wave makes (with fewer blocks than waves: some twice)
-  auto fetch_w = [&](int chunk) {
-    const size_t at = (size_t)chunk * a.heads + h;
+  auto fetch_w = [&](Held& t, int chunk) {
+    const size_t at = (size_t)min(chunk, a.chunks - 1) * a.heads + h;
     const float* row = a.w + (at * C + 16 * ub + j) * dp + 4 * kg;
 #pragma unroll
-    for (int n = 0; n < NT; ++n) wf[n] = *reinterpret_cast<const f32x4_t*>(row + 16 * n);
+    for (int n = 0; n < NT; ++n) t.wf[n] = *reinterpret_cast<const f32x4_t*>(row + 16 * n);
     const float* v = a.v + (at * C + 16 * ub + 4 * kg) * vp + p0 + j;
 #pragma unroll
-    for (int e = 0; e < 4; ++e) v0[e] = v[e * vp];
+    for (int e = 0; e < 4; ++e) t.v0[e] = v[e * vp];
   };
-  auto fetch_k = [&](int chunk) {
-    const size_t at = (size_t)chunk * a.heads + h;
+  auto fetch_k = [&](Held& t, int chunk) {
+    const size_t at = (size_t)min(chunk, a.chunks - 1) * a.heads + h;
 #pragma unroll
     for (int m = 0; m < MINE; ++m) {
       const int n = wave + 4 * m;
-      gm[m] = *reinterpret_cast<const f32x4_t*>(a.gam + at * dp + 16 * n + 4 * kg);
+      t.gm[m] = *reinterpret_cast<const f32x4_t*>(a.gam + at * dp + 16 * n + 4 * kg);
       const float* row = a.kd + (at * dp + 16 * n + j) * C + 4 * kg;
 #pragma unroll
-      for (int b = 0; b < NB; ++b) kf[m][b] = *reinterpret_cast<const f32x4_t*>(row + 16 * b);
+      for (int b = 0; b < NB; ++b) t.kf[m][b] = *reinterpret_cast<const f32x4_t*>(row + 16 * b);
     }
   };
-  fetch_w(0);
-  fetch_k(0);
+#pragma unroll
+  for (int x = 0; x < 2; ++x) fetch_w(held[x], x), fetch_k(held[x], x);
   __syncthreads();
-#pragma unroll 1
-  for (int chunk = 0; chunk < a.chunks; ++chunk) {
+  auto go = [&](Held& t, int chunk) {
     const size_t at = ((size_t)chunk * a.heads + h) * (vp / 16) + ct;
-    const int next = min(chunk + 1, a.chunks - 1);
     {
       f32x4_t acc[2] = {zero, zero};
 #pragma unroll
-      for (int n = 0; n < NT; ++n) acc[n & 1] = mfma16x16(wf[n], Ss[n][lane], acc[n & 1]);
-      const f32x4_t u = v0 - (acc[0] + acc[1]);
+      for (int n = 0; n < NT; ++n) acc[n & 1] = mfma16x16(t.wf[n], Ss[n][lane], acc[n & 1]);
+      const f32x4_t u = t.v0 - (acc[0] + acc[1]);
       Us[ub][lane] = u;
       *reinterpret_cast<f32x4_t*>(a.u + ((at * NB + ub) * 64 + lane) * 4) = u;
     }
-    fetch_w(next);
+    fetch_w(t, chunk + 2);
     __syncthreads();
     f32x4_t uf[NB];
 #pragma unroll
@@ -322,17 +377,22 @@ __global__ void __launch_bounds__(256) delta_scan_kernel(DeltaArgs a) {
 #pragma unroll
     for (int m = 0; m < MINE; ++m) {
       *reinterpret_cast<f32x4_t*>(a.s0 + ((at * NT + wave + 4 * m) * 64 + lane) * 4) = mine[m];
-      f32x4_t acc = gm[m] * mine[m], acc2 = zero;
+      f32x4_t acc = t.gm[m] * mine[m], acc2 = zero;
 #pragma unroll
       for (int b = 0; b < NB; ++b) {
-        if (b & 1) acc2 = mfma16x16(kf[m][b], uf[b], acc2);
-        else acc = mfma16x16(kf[m][b], uf[b], acc);
+        if (b & 1) acc2 = mfma16x16(t.kf[m][b], uf[b], acc2);
+        else acc = mfma16x16(t.kf[m][b], uf[b], acc);
       }
       mine[m] = acc + acc2;
       Ss[wave + 4 * m][lane] = mine[m];
     }
-    fetch_k(next);
+    fetch_k(t, chunk + 2);
     __syncthreads();
+  };
+#pragma unroll 1
+  for (int chunk = 0; chunk < a.chunks; chunk += 2) {
+    go(held[0], chunk);
+    if (chunk + 1 < a.chunks) go(held[1], chunk + 1);
   }
 #pragma unroll
   for (int m = 0; m < MINE; ++m)
@@ -419,49 +479,82 @@ struct DeltaStepArgs {
   int n_taps, heads, kv_heads, dim, vdim, a_rank, z_rank, channels;
 };
 
+// TAPS > 0: that many, everything asked for at once.
+template <int TAPS>
 __device__ __forceinline__ float conv_one(const DeltaStepArgs& a, int c) {
+  const float* taps = a.taps + (size_t)c * a.n_taps;
+  if constexpr (TAPS > 0) {
+    float w[TAPS], x[TAPS];
+#pragma unroll
+    for (int j = 0; j < TAPS; ++j) {
+      const long long p = a.pos - (TAPS - 1) + j;
+      w[j] = taps[j];
+      x[j] = j + 1 < TAPS ? a.ring[(size_t)((p + TAPS) % TAPS) * a.channels + c] : a.qkv[c];
+    }
+    float v = 0.f;
+#pragma unroll
+    for (int j = 0; j < TAPS; ++j)
+      if (a.pos - (TAPS - 1) + j >= 0) v += w[j] * x[j];
+    return silu_f(v);
+  }
   float v = 0.f;
   for (int j = 0; j + 1 < a.n_taps; ++j) {
     const long long p = a.pos - (a.n_taps - 1) + j;
-    if (p >= 0) v += a.taps[(size_t)c * a.n_taps + j] * a.ring[(size_t)(p % a.n_taps) * a.channels + c];
+    if (p >= 0) v += taps[j] * a.ring[(size_t)(p % a.n_taps) * a.channels + c];
   }
-  return silu_f(v + a.taps[(size_t)c * a.n_taps + a.n_taps - 1] * a.qkv[c]);
+  return silu_f(v + taps[a.n_taps - 1] * a.qkv[c]);
 }
 
-// Eight lanes' part of a row's product with x: pieces of 8 elements (V8: rows of whole aligned pieces), lane l takes every eighth.
+// Eight elements of a matrix row.
+template <typename WT>
+struct Piece8;
+template <>
+struct Piece8<uint16_t> {
+  u32x4_t v;
+  __device__ void load(const uint16_t* p) { v = *reinterpret_cast<const u32x4_t*>(p); }
+  __device__ float dot(const float* x) const {
+    float s = 0.f;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) s += __uint_as_float(v[e] << 16) * x[2 * e] + __uint_as_float(v[e] & 0xffff0000u) * x[2 * e + 1];
+    return s;
+  }
+};
+template <>
+struct Piece8<float> {
+  f32x4_t u, v;
+  __device__ void load(const float* p) { u = *reinterpret_cast<const f32x4_t*>(p), v = *reinterpret_cast<const f32x4_t*>(p + 4); }
+  __device__ float dot(const float* x) const {
+    float s = 0.f;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) s += u[e] * x[e] + v[e] * x[4 + e];
+    return s;
+  }
+};
+// Eight lanes' part of a row's product with x from element k0 on: lane l takes every eighth piece of 8 (V8: rows of whole aligned pieces).
 template <typename WT, bool V8>
-__device__ __forceinline__ float row_part(const WT* row, const float* x, int n, int l) {
+__device__ __forceinline__ float row_part(const WT* row, const float* x, int k0, int n, int l) {
   float s = 0.f;
-  for (int k = l * 8; k < n; k += 64) {
-    float w[8];
-    if constexpr (V8 && sizeof(WT) == 2) {
-      const u32x4_t v = *reinterpret_cast<const u32x4_t*>(row + k);
-#pragma unroll
-      for (int e = 0; e < 4; ++e) w[2 * e] = __uint_as_float(v[e] << 16), w[2 * e + 1] = __uint_as_float(v[e] & 0xffff0000u);
-    } else if constexpr (V8) {
-      const f32x4_t u = *reinterpret_cast<const f32x4_t*>(row + k), v = *reinterpret_cast<const f32x4_t*>(row + k + 4);
-#pragma unroll
-      for (int e = 0; e < 4; ++e) w[e] = u[e], w[4 + e] = v[e];
+  for (int k = k0 + l * 8; k < n; k += 64) {
+    if constexpr (V8) {
+      Piece8<WT> w;
+      w.load(row + k);
+      s += w.dot(x + k);
     } else {
 #pragma unroll
-      for (int e = 0; e < 8; ++e) {
-        w[e] = 0.f;
+      for (int e = 0; e < 8; ++e)
         if (k + e < n) {
-          if constexpr (sizeof(WT) == 2) w[e] = bf16_to_f32(row[k + e]);
-          else w[e] = row[k + e];
+          if constexpr (sizeof(WT) == 2) s += bf16_to_f32(row[k + e]) * x[k + e];
+          else s += row[k + e] * x[k + e];
         }
-      }
     }
-#pragma unroll
-    for (int e = 0; e < 8; ++e)
-      if (V8 || k + e < n) s += w[e] * x[k + e];
   }
   return s;
 }
 
-template <typename WT, bool V8>
+constexpr int ROUNDS = 5, PIECES = 2;  // of the decays' and gates' rows, asked for before anything else: 160 rows of up to 128 elements
+template <typename WT, bool V8, int TAPS>
 __global__ void __launch_bounds__(256) delta_step_kernel(DeltaStepArgs a) {
-  extern __shared__ float lds[];
+  extern __shared__ __attribute__((aligned(16))) float lds[];
   const int d = a.dim, h = blockIdx.x, p0 = blockIdx.y * COLS, per = a.heads / a.kv_heads, g = h / per, gd = a.kv_heads * d;
   float* q = lds;
   float* k = q + d;
@@ -470,25 +563,48 @@ __global__ void __launch_bounds__(256) delta_step_kernel(DeltaStepArgs a) {
   float* z_in = a_in + a.a_rank;
   __shared__ float vs[COLS], part[GROUPS][COLS + 1], scale[2];
   const int tid = threadIdx.x, col = tid & (COLS - 1), grp = tid / COLS, p = p0 + col, lane = tid & 63, wave = tid >> 6;
+  const int mine = min(COLS, a.vdim - p0), l8 = tid & 7, row8 = tid >> 3;
+  // the decays' rows, then the gates'; eight lanes to a row
+  auto row_of = [&](int r) {
+    const bool gate = r >= d;
+    return gate ? static_cast<const WT*>(a.w_z) + (size_t)(h * a.vdim + p0 + r - d) * a.z_rank : static_cast<const WT*>(a.w_a) + (size_t)(h * d + r) * a.a_rank;
+  };
+  Piece8<WT> pre[V8 ? ROUNDS : 1][PIECES];
+  if constexpr (V8) {
+#pragma unroll
+    for (int u = 0; u < ROUNDS; ++u) {
+      const int r = min(row8 + 32 * u, d + mine - 1), n = r >= d ? a.z_rank : a.a_rank;
+#pragma unroll
+      for (int b = 0; b < PIECES; ++b) pre[u][b].load(row_of(r) + (b * 64 + l8 * 8 < n ? b * 64 + l8 * 8 : 0));
+    }
+  }
   float* S = a.s + (size_t)h * d * a.vdim + p;
   const bool there = p < a.vdim;
-  float held[HELD];  // the first of the state's rows, asked for before anything else
+  float held[HELD];  // the first of the state's rows (lanes without a place in it load another's)
+  {
+    const float* Sl = a.s + (size_t)h * d * a.vdim + (there ? p : 0);
 #pragma unroll
-  for (int u = 0; u < HELD; ++u) held[u] = a.pos && there && grp + GROUPS * u < d ? S[(size_t)(grp + GROUPS * u) * a.vdim] : 0.f;
-  for (int i = tid; i < a.a_rank; i += 256) a_in[i] = a.a_in[i];
-  for (int i = tid; i < a.z_rank; i += 256) z_in[i] = a.z_in[i];
+    for (int u = 0; u < HELD; ++u) held[u] = Sl[(size_t)min(grp + GROUPS * u, d - 1) * a.vdim];
+  }
   float* slot = a.ring + (size_t)(a.pos % a.n_taps) * a.channels;
   const bool first = h % per == 0 && blockIdx.y == 0;  // stores the key head's rows
   for (int i = tid; i < 2 * d; i += 256) {
     const int c = (i < d ? 0 : gd - d) + g * d + i;
-    lds[i] = conv_one(a, c);
+    lds[i] = conv_one<TAPS>(a, c);
     if (first) slot[c] = a.qkv[c];
   }
   if (tid < COLS && there) {
     const int c = 2 * gd + h * a.vdim + p;
-    vs[tid] = conv_one(a, c);
+    vs[tid] = conv_one<TAPS>(a, c);
     slot[c] = a.qkv[c];
   }
+  for (int i = tid; i < a.a_rank; i += 256) a_in[i] = a.a_in[i];
+  for (int i = tid; i < a.z_rank; i += 256) z_in[i] = a.z_in[i];
+  if (a.pos == 0) {  // nothing is known of the state's memory
+#pragma unroll
+    for (int u = 0; u < HELD; ++u) held[u] = 0.f;
+  }
+  const float neg = -expf(a.a_log[h]), beta = exact_sigmoid(a.b[h]);
   __syncthreads();
   if (wave < 2) {
     const float* row = wave ? k : q;
@@ -497,20 +613,30 @@ __global__ void __launch_bounds__(256) delta_step_kernel(DeltaStepArgs a) {
     ss = wave_sum(ss);
     if (lane == 0) scale[wave] = 1.f / sqrtf(ss + UNIT_EPS) * (wave ? 1.f : 1.f / sqrtf((float)d));
   }
-  const float neg = -expf(a.a_log[h]);
-  const int mine = min(COLS, a.vdim - p0), l8 = tid & 7;
-  for (int r = tid >> 3; r < d + mine; r += 32) {  // a row's eight lanes stay together
-    const bool gate = r >= d;
-    const int row = gate ? h * a.vdim + p0 + r - d : h * d + r;
-    float s = gate ? row_part<WT, V8>(static_cast<const WT*>(a.w_z) + (size_t)row * a.z_rank, z_in, a.z_rank, l8)
-                   : row_part<WT, V8>(static_cast<const WT*>(a.w_a) + (size_t)row * a.a_rank, a_in, a.a_rank, l8);
+  auto finish = [&](int r, float s) {
     s += __shfl_xor(s, 4, 64);
     s += __shfl_xor(s, 2, 64);
     s += __shfl_xor(s, 1, 64);
-    if (l8 == 0) {
-      if (gate) a.out[(size_t)a.heads * a.vdim + row] = s;
-      else decay[r] = expf(neg * softplus_f(s + a.dt_bias[row]));
+    if (l8 == 0 && r < d + mine) {
+      if (r >= d) a.out[(size_t)a.heads * a.vdim + h * a.vdim + p0 + r - d] = s;
+      else decay[r] = expf(neg * softplus_f(s + a.dt_bias[h * d + r]));
     }
+  };
+  if constexpr (V8) {
+#pragma unroll
+    for (int u = 0; u < ROUNDS; ++u) {
+      const int r = row8 + 32 * u, rr = min(r, d + mine - 1), n = rr >= d ? a.z_rank : a.a_rank;
+      const float* x = rr >= d ? z_in : a_in;
+      float s = 0.f;
+#pragma unroll
+      for (int b = 0; b < PIECES; ++b)
+        if (b * 64 + l8 * 8 < n) s += pre[u][b].dot(x + b * 64 + l8 * 8);
+      finish(r, s + row_part<WT, V8>(row_of(rr), x, PIECES * 64, n, l8));
+    }
+  }
+  for (int r = row8 + (V8 ? 32 * ROUNDS : 0); r < d + mine; r += 32) {  // a row's eight lanes stay together
+    const bool gate = r >= d;
+    finish(r, row_part<WT, V8>(row_of(r), gate ? z_in : a_in, 0, gate ? a.z_rank : a.a_rank, l8));
   }
   __syncthreads();
   const float ks = scale[1], qs = scale[0];
@@ -530,7 +656,7 @@ __global__ void __launch_bounds__(256) delta_step_kernel(DeltaStepArgs a) {
 #pragma unroll
   for (int i = 0; i < GROUPS; ++i) all += part[i][col];
   __syncthreads();
-  const float u_new = there ? exact_sigmoid(a.b[h]) * (vs[col] - all) : 0.f;
+  const float u_new = there ? beta * (vs[col] - all) : 0.f;
   float o = 0.f;
 #pragma unroll
   for (int u = 0; u < HELD; ++u) {
@@ -672,8 +798,13 @@ extern "C" int ughip_delta_step(ughip_device* dev, const ughip_delta* p) {
   const size_t lds = (3 * d + p->a_rank + p->z_rank) * sizeof(float);
   auto go = [&](auto kernel) { kernel<<<dim3((unsigned)H, (unsigned)((vd + COLS - 1) / COLS)), 256, lds, dev->stream>>>(a); };
   const bool bf = p->w_a->dtype == UGHIP_BF16;
-  if (bf) v8 ? go(delta_step_kernel<uint16_t, true>) : go(delta_step_kernel<uint16_t, false>);
-  else v8 ? go(delta_step_kernel<float, true>) : go(delta_step_kernel<float, false>);
+  auto taps = [&](auto type, auto whole) {
+    using WT = decltype(type);
+    constexpr bool V8 = decltype(whole)::value;
+    p->n_taps == 4 ? go(delta_step_kernel<WT, V8, 4>) : p->n_taps == 3 ? go(delta_step_kernel<WT, V8, 3>) : p->n_taps == 2 ? go(delta_step_kernel<WT, V8, 2>) : go(delta_step_kernel<WT, V8, 0>);
+  };
+  if (bf) v8 ? taps(uint16_t(), std::true_type{}) : taps(uint16_t(), std::false_type{});
+  else v8 ? taps(float(), std::true_type{}) : taps(float(), std::false_type{});
   UGHIP_HIPCHK(hipGetLastError());
   return UGHIP_OK;
 }

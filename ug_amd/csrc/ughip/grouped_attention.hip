@@ -29,9 +29,29 @@ struct Turn {
   int rot;
   float mul;
 };
-// elements c .. c + N - 1 (c even) of a head of `dim`, zeros past its end
-template <int N>
+// elements c .. c + N - 1 (c even) of a head of `dim`, zeros past its end; VEC: they are there (or none is) and 16-byte aligned, and a
+// rotated part ends between pieces
+template <int N, bool VEC = false>
 __device__ __forceinline__ void turned(const float* head, int c, int dim, const Turn& t, float (&out)[N]) {
+  if constexpr (VEC) {
+    const bool there = c < dim, turns = t.cos && c < t.rot;
+    float x[N], co[N / 2], si[N / 2];
+#pragma unroll
+    for (int e = 0; e < N; e += 4) __builtin_memcpy(x + e, __builtin_assume_aligned(head + (there ? c : 0) + e, 16), 16);
+    const size_t at = turns ? c >> 1 : 0;
+#pragma unroll
+    for (int e = 0; e < N / 2; e += 2) {
+      co[e] = 1.f, co[e + 1] = 1.f, si[e] = si[e + 1] = 0.f;
+      if (t.cos) __builtin_memcpy(co + e, __builtin_assume_aligned(t.cos + at + e, 8), 8), __builtin_memcpy(si + e, __builtin_assume_aligned(t.sin + at + e, 8), 8);
+    }
+#pragma unroll
+    for (int e = 0; e < N; e += 2) {
+      const float u = there ? x[e] : 0.f, v = there ? x[e + 1] : 0.f, cc = turns ? co[e / 2] : 1.f, ss = turns ? si[e / 2] : 0.f;
+      out[e] = (u * cc - v * ss) * t.mul;
+      out[e + 1] = (v * cc + u * ss) * t.mul;
+    }
+    return;
+  }
 #pragma unroll
   for (int e = 0; e < N; e += 2) {
     const int d = c + e;
@@ -76,7 +96,7 @@ __device__ __forceinline__ Turn turn_of(const GroupedArgs& a, int p, bool query)
 constexpr int VT = 64;  // positions and value elements of a transposed tile
 
 // blockIdx.y: first the query heads (none when q_rows is 0), then the key heads, then blocks of VT value elements of every value head.
-template <typename T, int DQ>
+template <typename T, int DQ, bool VEC>
 __global__ void __launch_bounds__(256) attention_place_kernel(GroupedArgs a) {
   constexpr int E = 16 / sizeof(T), CH = DQ / E;
   __shared__ T tile[VT][VT + 2];
@@ -90,7 +110,7 @@ __global__ void __launch_bounds__(256) attention_place_kernel(GroupedArgs a) {
     u32x4_t piece = {0, 0, 0, 0};
     if (r < a.t) {
       float v[E];
-      turned<E>(a.qkv + (size_t)r * a.row + (size_t)(is_q ? head : a.heads + head) * a.dim, c, a.dim, turn_of(a, a.pos + r, is_q), v);
+      turned<E, VEC>(a.qkv + (size_t)r * a.row + (size_t)(is_q ? head : a.heads + head) * a.dim, c, a.dim, turn_of(a, a.pos + r, is_q), v);
       piece = packed<T>(v);
     }
     T* out = is_q ? static_cast<T*>(a.qp) + ((size_t)head * a.q_rows + r) * DQ + c : static_cast<T*>(a.kc) + ((size_t)head * a.cap + a.pos + r) * DQ + c;
@@ -128,6 +148,7 @@ template <typename T, int DQ, int DV, int NW, bool APPEND>
 __global__ void __launch_bounds__(64 * NW) attention_split_kernel(SplitArgs a) {
   constexpr int E = 16 / sizeof(T), QC = DQ / E, NV = sizeof(T) == 2 ? 2 : 4;  // NV: 16-byte value operands of a tile and 32 value elements
   constexpr bool BF = sizeof(T) == 2;
+  constexpr int Q_ROW = DQ + E;
   extern __shared__ __attribute__((aligned(16))) float parts[];
   const GroupedArgs& g = a.g;
   const int kv = blockIdx.x % g.kv_heads, rb = blockIdx.x / g.kv_heads, split = blockIdx.y, per = g.heads / g.kv_heads;
@@ -159,23 +180,37 @@ __global__ void __launch_bounds__(64 * NW) attention_split_kernel(SplitArgs a) {
   };
   int k0 = (tile0 + split * share + wave) * SK;
   if (k0 < k_stop) fetch(k0);
-  // the queries: chunk 2 c + hf of row `col`
-  u32x4_t qf[QC / 2], ql[BF ? QC / 2 : 1];
-  {
-    const float* head = g.qkv + (size_t)(r_mine / per) * g.row + (size_t)(kv * per + r_mine % per) * g.dim;
-    const Turn turn = turn_of(g, p_mine, true);
-#pragma unroll
-    for (int c = 0; c < QC / 2; ++c) {
-      float v[E];
-      turned<E>(head, (2 * c + hf) * E, g.dim, turn, v);
-      qf[c] = packed<T>(v);
-      if constexpr (BF) {
-        uint16_t e[E];
-        __builtin_memcpy(e, &qf[c], 16);
-#pragma unroll
-        for (int x = 0; x < E; ++x) v[x] -= bf16_to_f32(e[x]);
-        ql[c] = packed<T>(v);
+  // the queries (and the new key and value) through LDS, a pair of elements per thread and turn
+  const int live = r_last + 1 - rb * 32;
+  T* q_hi = reinterpret_cast<T*>(parts);
+  T* q_lo = q_hi + (size_t)live * Q_ROW;  // (bf16 only)
+  T* k_new = q_hi + (size_t)live * Q_ROW * (BF ? 2 : 1);
+  T* v_new = k_new + DQ;
+  for (int x = threadIdx.x; x < (live + (APPEND ? 1 : 0)) * (DQ / 2); x += 64 * NW) {
+    const int r = x / (DQ / 2), d = x % (DQ / 2) * 2, row = min(rb * 32 + r, r_last);
+    const bool query = r < live;
+    const float* head = g.qkv + (size_t)(row / per) * g.row + (size_t)(query ? kv * per + row % per : g.heads + kv) * g.dim;
+    float v[2];
+    turned<2>(head, d, g.dim, turn_of(g, g.pos + row / per, query), v);
+    T* to = query ? q_hi + r * Q_ROW + d : k_new + d;
+    to[0] = to_elem<T>(v[0]), to[1] = to_elem<T>(v[1]);
+    if constexpr (BF) {
+      if (query) {
+        q_lo[r * Q_ROW + d] = to_elem<T>(v[0] - bf16_to_f32(to[0]));
+        q_lo[r * Q_ROW + d + 1] = to_elem<T>(v[1] - bf16_to_f32(to[1]));
       }
+    }
+  }
+  if constexpr (APPEND)
+    for (int v = threadIdx.x; v < DV; v += 64 * NW) v_new[v] = to_elem<T>(v < g.vdim ? g.qkv[(size_t)(g.heads + g.kv_heads) * g.dim + (size_t)kv * g.vdim + v] : 0.f);
+  __syncthreads();
+  const int q_at = (r_mine - rb * 32) * Q_ROW + hf * E;  // chunk 2 c + hf of row `col`: 2 c E further
+  if constexpr (APPEND) {
+    // the workgroup that meets the new key leaves it in the caches
+    if ((tile0 + split * share) * SK <= g.pos && g.pos < k_stop) {
+      T* krow = static_cast<T*>(g.kc) + ((size_t)kv * g.cap + g.pos) * DQ;
+      for (int x = threadIdx.x; x < QC; x += 64 * NW) *reinterpret_cast<u32x4_t*>(krow + x * E) = *reinterpret_cast<const u32x4_t*>(k_new + x * E);
+      for (int v = threadIdx.x; v < g.vdim; v += 64 * NW) static_cast<T*>(g.vc)[((size_t)kv * g.vdim + v) * g.cap + g.pos] = v_new[v];
     }
   }
   f32x16 o[DV / 32];
@@ -187,26 +222,15 @@ __global__ void __launch_bounds__(64 * NW) attention_split_kernel(SplitArgs a) {
   for (; k0 < k_stop; k0 += NW * SK) {
     if constexpr (APPEND) {
       if (k0 + SK > g.pos) {  // the new position's tile
-        T* krow = static_cast<T*>(g.kc) + ((size_t)kv * g.cap + g.pos) * DQ;
-        const float* k_new = g.qkv + (size_t)(g.heads + kv) * g.dim;
-        const Turn turn = turn_of(g, g.pos, false);
         const bool mine = k0 + col == g.pos;
 #pragma unroll
         for (int c = 0; c < QC / 2; ++c) {
-          float v[E];
-          turned<E>(k_new, (2 * c + hf) * E, g.dim, turn, v);
-          const u32x4_t piece = packed<T>(v);
-          if (mine) {
-            kf[c] = piece;
-            *reinterpret_cast<u32x4_t*>(krow + (2 * c + hf) * E) = piece;
-          }
+          const u32x4_t piece = *reinterpret_cast<const u32x4_t*>(k_new + (2 * c + hf) * E);
+          kf[c] = mine ? piece : kf[c];
         }
-        const float* v_new = g.qkv + (size_t)(g.heads + g.kv_heads) * g.dim + (size_t)kv * g.vdim;
 #pragma unroll
         for (int i = 0; i < DV / 32; ++i) {
-          const int v = i * 32 + col;
-          const T now = to_elem<T>(v < g.vdim ? v_new[v] : 0.f);
-          if (hf == 0 && v < g.vdim) static_cast<T*>(g.vc)[((size_t)kv * g.vdim + v) * g.cap + g.pos] = now;
+          const T now = v_new[i * 32 + col];
 #pragma unroll
           for (int u = 0; u < NV; ++u) {
             T e[E];
@@ -235,10 +259,11 @@ __global__ void __launch_bounds__(64 * NW) attention_split_kernel(SplitArgs a) {
     f32x16 s, s2;
 #pragma unroll
     for (int e = 0; e < 16; ++e) s[e] = s2[e] = 0.f;
+    asm volatile("" ::: "memory");  // (the queries' operands are read where they are used: they would not fit the registers)
 #pragma unroll
     for (int c = 0; c < QC / 2; ++c) {
-      mfma_chunk<T>(kf[c], qf[c], s);
-      if constexpr (BF) mfma_chunk<T>(kf[c], ql[c], s2);
+      mfma_chunk<T>(kf[c], *reinterpret_cast<const u32x4_t*>(q_hi + q_at + 2 * c * E), s);
+      if constexpr (BF) mfma_chunk<T>(kf[c], *reinterpret_cast<const u32x4_t*>(q_lo + q_at + 2 * c * E), s2);
     }
     // element e: key k0 + 8 (e / 4) + 4 hf + e % 4, row `col`
     float top = mx;
@@ -288,7 +313,7 @@ __global__ void __launch_bounds__(64 * NW) attention_split_kernel(SplitArgs a) {
     if (k0 + NW * SK < k_stop) fetch(k0 + NW * SK);
   }
   // the waves' parts: [wave][row][DV + 4], then every wave's maximum and sum per row
-  const int live = r_last + 1 - rb * 32;
+  __syncthreads();  // (what was staged there has been read)
   constexpr int P = DV + 4;
   float* ml = parts + (size_t)NW * live * P;
   if (col < live) {
@@ -380,7 +405,10 @@ int place(ughip_device* dev, const GroupedArgs& g) {
   const size_t x = (pieces + 255) / 256 > tiles ? (pieces + 255) / 256 : tiles;
   const int y = (g.q_rows ? g.heads : 0) + g.kv_heads + g.kv_heads * ((g.vdim + VT - 1) / VT);
   if (y > 65535) return set_error(UGHIP_ERR_UNSUPPORTED, "grouped_attention: too many heads");
-  attention_place_kernel<T, DQ><<<dim3((unsigned)x, (unsigned)y), 256, 0, dev->stream>>>(g);
+  auto whole = [](const void* q) { return (reinterpret_cast<uintptr_t>(q) & 15) == 0; };
+  const bool vec = g.dim % 8 == 0 && g.rot % 8 == 0 && g.row % 4 == 0 && whole(g.qkv);
+  if (vec) attention_place_kernel<T, DQ, true><<<dim3((unsigned)x, (unsigned)y), 256, 0, dev->stream>>>(g);
+  else attention_place_kernel<T, DQ, false><<<dim3((unsigned)x, (unsigned)y), 256, 0, dev->stream>>>(g);
   UGHIP_HIPCHK(hipGetLastError());
   return UGHIP_OK;
 }
@@ -395,14 +423,14 @@ int attend_many(ughip_device* dev, GroupedArgs g, AttRowsArgs r) {
   static_assert(bytes <= 160 * 1024, "tile does not fit LDS");
   static const hipError_t attr = hipFuncSetAttribute(reinterpret_cast<const void*>(attention_rows_kernel<T, DQ, DV>), hipFuncAttributeMaxDynamicSharedMemorySize, bytes);
   UGHIP_HIPCHK(attr);
-  attention_rows_kernel<T, DQ, DV><<<dim3((unsigned)g.heads, (unsigned)(g.q_rows / ATT_QT)), 256, bytes, dev->stream>>>(r);
+  attention_rows_kernel<T, DQ, DV><<<dim3((unsigned)g.heads, (unsigned)(g.q_rows / ATT_QT)), attention_rows_threads<T, DQ, DV>(), bytes, dev->stream>>>(r);
   UGHIP_HIPCHK(hipGetLastError());
   return UGHIP_OK;
 }
 
 template <typename T, int DQ, int DV>
 int attend_few(ughip_device* dev, SplitArgs a) {
-  constexpr int NW = DV <= 128 ? 8 : 4;
+  constexpr int NW = DV <= 128 && DQ * sizeof(T) <= 384 ? 8 : 4;
   const GroupedArgs& g = a.g;
   if (g.t > 1)
     if (int rc = place<T, DQ>(dev, g)) return rc;
@@ -424,7 +452,8 @@ int attend_few(ughip_device* dev, SplitArgs a) {
     a.ml = static_cast<float*>(ws), a.acc = a.ml + n_ml;
   }
   const int live = a.rows < 32 ? a.rows : 32;
-  const size_t lds = (size_t)NW * live * (DV + 4 + 2) * sizeof(float);
+  const size_t staged = ((size_t)live * (DQ + 16 / sizeof(T)) * (sizeof(T) == 2 ? 2 : 1) + DQ + DV) * sizeof(T), met = (size_t)NW * live * (DV + 4 + 2) * sizeof(float);
+  const size_t lds = staged > met ? staged : met;
   auto go = [&](auto kernel) {
     if (lds > 60 * 1024)
       if (hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(kernel), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds); e != hipSuccess) return e;

@@ -125,7 +125,7 @@ int launch_rows(ughip_device* dev, AttRowsArgs a, PackArgs pk) {
   const size_t pieces = (size_t)(pk.q_rows + pk.k_rows) * CH;
   latent_pack_kernel<T, DQ><<<dim3((unsigned)((pieces + 255) / 256), (unsigned)pk.heads), 256, 0, dev->stream>>>(pk);
   UGHIP_HIPCHK(hipGetLastError());
-  attention_rows_kernel<T, DQ, DV><<<dim3((unsigned)pk.heads, (unsigned)(pk.q_rows / ATT_QT)), 256, bytes, dev->stream>>>(a);
+  attention_rows_kernel<T, DQ, DV><<<dim3((unsigned)pk.heads, (unsigned)(pk.q_rows / ATT_QT)), attention_rows_threads<T, DQ, DV>(), bytes, dev->stream>>>(a);
   UGHIP_HIPCHK(hipGetLastError());
   return UGHIP_OK;
 }
