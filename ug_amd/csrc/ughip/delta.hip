@@ -38,6 +38,18 @@ __device__ __forceinline__ f32x4_t mfma16x16(const f32x4_t& x, const f32x4_t& y,
   acc = mfma16(x.z, y.z, acc);
   return mfma16(x.w, y.w, acc);
 }
+// acc[i] += x[i] y[i], the chains side by side: a product that waits for the one before it leaves the pipe idle
+template <int N>
+__device__ __forceinline__ void mfma16x16_each(const f32x4_t (&x)[N], const f32x4_t (&y)[N], f32x4_t (&acc)[N]) {
+#pragma unroll
+  for (int e = 0; e < 4; ++e)
+#pragma unroll
+    for (int i = 0; i < N; ++i) acc[i] = mfma16(x[i][e], y[i][e], acc[i]);
+}
+// Where element (row, k) of a left operand lies in its tile, and a tile's lane.
+__device__ __forceinline__ int left_at(int row, int k) { return ((k >> 2) * 16 + row) * 4 + (k & 3); }
+__device__ __forceinline__ float* tile_at(float* tiles, size_t tile, int lane) { return tiles + (tile * 64 + lane) * 4; }
+__device__ __forceinline__ f32x4_t tile_of(const float* tiles, size_t tile, int lane) { return *reinterpret_cast<const f32x4_t*>(tiles + (tile * 64 + lane) * 4); }
 __device__ __forceinline__ float exact_sigmoid(float z) { return 1.f / (1.f + expf(-z)); }
 __device__ __forceinline__ f32x4_t exp2_4(const f32x4_t& v) {
   return f32x4_t{__builtin_amdgcn_exp2f(v.x), __builtin_amdgcn_exp2f(v.y), __builtin_amdgcn_exp2f(v.z), __builtin_amdgcn_exp2f(v.w)};
@@ -57,15 +69,17 @@ struct DeltaArgs {
   int t, heads, kv_heads, dim, vdim, dp, vp, chunks;  // dp: dim rounded up to 64, vp: vdim rounded up to 16
   float eps;
   bool fresh, dst_bf16;
-  // what lies between the launches, per (chunk, head)
-  float* w;      // [C][dp]
-  float* v;      // [C][vp]: V'
-  float* kd;     // [dp][C]: G_C / G k
-  float* qg;     // [C][dp]: G q
-  float* p;      // [C][C], blocks above the diagonal are not there
-  float* gam;    // [dp]: G_C
-  float* s0;     // [vp / 16][dp / 16][64 lanes][4]
-  float* u;      // [vp / 16][C / 16][64 lanes][4]
+  // What lies between the launches, per (chunk, head): tiles of 16 x 16 as the lanes of a wave hold them, 16 bytes each.  Left operands
+  // (lane l: row l % 16, elements 4 (l / 16) .. + 3 of k):
+  float* w;      // [C / 16][dp / 16]: W, rows are positions
+  float* kd;     // [dp / 16][C / 16]: G_C / G k, rows are channels
+  float* qg;     // [C / 16][dp / 16]: G q
+  float* p;      // [C / 16][C / 16]: P, tiles above the diagonal are not there
+  // right operands and results (lane l: column l % 16, rows 4 (l / 16) .. + 3):
+  float* v;      // [vp / 16][C / 16]: V'
+  float* u;      // [vp / 16][C / 16]: U
+  float* s0;     // [vp / 16][dp / 16]: the state in front of the chunk
+  float* gam;    // G_C of every channel
 };
 
 template <int C>
@@ -84,9 +98,13 @@ __device__ __forceinline__ f32x4_t four(const float* p, int left) {
   return v;
 }
 
+template <int C>
+constexpr int prepare_threads() {
+  return C == 64 ? 512 : 256;
+}
 template <int C, bool VEC>
-__global__ void __launch_bounds__(256) delta_prepare_kernel(DeltaArgs a) {
-  constexpr int NB = C / 16;
+__global__ void __launch_bounds__((prepare_threads<C>())) delta_prepare_kernel(DeltaArgs a) {
+  constexpr int NB = C / 16, NT = prepare_threads<C>(), NW = NT / 64;
   extern __shared__ __attribute__((aligned(16))) float lds[];
   const int dp = a.dp, ds = dp + 4, chunk = blockIdx.x, h = blockIdx.y, g = h / (a.heads / a.kv_heads), row0 = chunk * C, rows = min(C, a.t - row0), d = a.dim;
   float* K = lds;             // [C][ds]
@@ -100,7 +118,7 @@ __global__ void __launch_bounds__(256) delta_prepare_kernel(DeltaArgs a) {
   const int d4 = dp / 4;
   const float neg = -expf(a.a_log[h]) * LOG2E;
   const f32x4_t zero = {0.f, 0.f, 0.f, 0.f};
-  for (int e = threadIdx.x; e < C * d4; e += 256) {
+  for (int e = threadIdx.x; e < C * d4; e += NT) {
     const int r = e / d4, c = (e - r * d4) * 4;
     f32x4_t k = zero, q = zero, l = zero;
     if (r < rows && c < d) {
@@ -119,7 +137,7 @@ __global__ void __launch_bounds__(256) delta_prepare_kernel(DeltaArgs a) {
   __syncthreads();
   // unit vectors: 16 lanes per row
   const float q_scale = 1.f / sqrtf((float)d);
-  for (int r = wave * 4 + kg; r < C; r += 16) {
+  for (int r = wave * 4 + kg; r < C; r += 4 * NW) {
 #pragma unroll
     for (int m = 0; m < 2; ++m) {
       float* row = (m ? Q : K) + r * ds;
@@ -132,7 +150,7 @@ __global__ void __launch_bounds__(256) delta_prepare_kernel(DeltaArgs a) {
       for (int c = j * 4; c < dp; c += 64) *reinterpret_cast<f32x4_t*>(row + c) *= f;
     }
   }
-  for (int x = threadIdx.x; x < dp * NB; x += 256) {
+  for (int x = threadIdx.x; x < dp * NB; x += NT) {
     float* col = B + (x / dp) * 16 * ds + x % dp;
     float s = 0.f;
 #pragma unroll
@@ -142,46 +160,62 @@ __global__ void __launch_bounds__(256) delta_prepare_kernel(DeltaArgs a) {
 
   float* P = a.p + at * C * C;
   auto row4 = [&](const float* m, int r, int c) { return *reinterpret_cast<const f32x4_t*>(m + r * ds + c); };
-  // pairs of different blocks
-  {
-    int n = 0;
-    for (int I = 1; I < NB; ++I)
-      for (int J = 0; J < I; ++J, ++n) {
-        if (n % 4 != wave) continue;
-        f32x4_t ak = zero, aq = zero;
-        for (int c = 4 * kg; c < dp; c += 16) {
-          const f32x4_t left = exp2_4(row4(B, 16 * I + j, c));
-          f32x4_t rest = row4(B, 16 * J + 15, c) - row4(B, 16 * J + j, c);
-          for (int M = J + 1; M < I; ++M) rest += row4(B, 16 * M + 15, c);
-          const f32x4_t right = row4(K, 16 * J + j, c) * exp2_4(rest);
-          ak = mfma16x16(row4(K, 16 * I + j, c) * left, right, ak);
-          aq = mfma16x16(row4(Q, 16 * I + j, c) * left, right, aq);
-        }
+  // a pair of blocks per wave and turn, those of a block with itself first
+  for (int n = wave; n < NB * (NB + 1) / 2; n += NW) {
+    int I = n, J = n;
+    if (n >= NB) {
+      I = 1;
+      for (J = n - NB; J >= I; ++I) J -= I;
+    }
+    if (J < I) {
+      f32x4_t acc[4] = {zero, zero, zero, zero};
+      for (int c = 4 * kg; c < dp; c += 32) {
+        f32x4_t x[4], y[4];
 #pragma unroll
-        for (int e = 0; e < 4; ++e) {
-          const int i = 16 * I + 4 * kg + e;
-          A[i * as + 16 * J + j] = ak[e] * beta[i];
-          P[i * C + 16 * J + j] = aq[e];
+        for (int u = 0; u < 2; ++u) {
+          const int cc = c + 16 * u;  // dp is a multiple of 64
+          const f32x4_t left = exp2_4(row4(B, 16 * I + j, cc));
+          f32x4_t rest = row4(B, 16 * J + 15, cc) - row4(B, 16 * J + j, cc);
+          for (int M = J + 1; M < I; ++M) rest += row4(B, 16 * M + 15, cc);
+          y[2 * u] = y[2 * u + 1] = row4(K, 16 * J + j, cc) * exp2_4(rest);
+          x[2 * u] = row4(K, 16 * I + j, cc) * left;
+          x[2 * u + 1] = row4(Q, 16 * I + j, cc) * left;
         }
+        mfma16x16_each(x, y, acc);
       }
-  }
-  // pairs of the same block
-  for (int I = wave; I < NB; I += 4) {
+      const f32x4_t ak = acc[0] + acc[2], aq = acc[1] + acc[3];
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        const int i = 16 * I + 4 * kg + e;
+        A[i * as + 16 * J + j] = ak[e] * beta[i];
+        P[(I * NB + J) * 256 + left_at(4 * kg + e, j)] = aq[e];
+      }
+      continue;
+    }
+
     float least = 0.f;
     for (int c = lane; c < dp; c += 64) least = fminf(least, B[(16 * I + 15) * ds + c]);
     least = -wave_max(-least);
     if (least > -64.f) {  // the same for the whole wave
-      f32x4_t ak = zero, aq = zero;
-      for (int c = 4 * kg; c < dp; c += 16) {
-        const f32x4_t l = row4(B, 16 * I + j, c), k = row4(K, 16 * I + j, c), left = exp2_4(l), right = k * exp2_4(-l);
-        ak = mfma16x16(k * left, right, ak);
-        aq = mfma16x16(row4(Q, 16 * I + j, c) * left, right, aq);
+      f32x4_t acc[4] = {zero, zero, zero, zero};
+      for (int c = 4 * kg; c < dp; c += 32) {
+        f32x4_t x[4], y[4];
+#pragma unroll
+        for (int u = 0; u < 2; ++u) {
+          const int cc = c + 16 * u;
+          const f32x4_t l = row4(B, 16 * I + j, cc), k = row4(K, 16 * I + j, cc), left = exp2_4(l);
+          y[2 * u] = y[2 * u + 1] = k * exp2_4(-l);
+          x[2 * u] = k * left;
+          x[2 * u + 1] = row4(Q, 16 * I + j, cc) * left;
+        }
+        mfma16x16_each(x, y, acc);
       }
+      const f32x4_t ak = acc[0] + acc[2], aq = acc[1] + acc[3];
 #pragma unroll
       for (int e = 0; e < 4; ++e) {
         const int i = 4 * kg + e, row = 16 * I + i;
         A[row * as + 16 * I + j] = j < i ? ak[e] * beta[row] : 0.f;
-        P[row * C + 16 * I + j] = j <= i ? aq[e] : 0.f;
+        P[(I * NB + I) * 256 + left_at(i, j)] = j <= i ? aq[e] : 0.f;
       }
       continue;
     }
@@ -206,7 +240,7 @@ __global__ void __launch_bounds__(256) delta_prepare_kernel(DeltaArgs a) {
     for (int x = 0; x < 4; ++x) {
       const int jj = 4 * kg + x;
       A[(16 * I + j) * as + 16 * I + jj] = jj < j ? ak[x] * bt : 0.f;
-      P[(16 * I + j) * C + 16 * I + jj] = jj <= j ? aq[x] : 0.f;
+      P[(I * NB + I) * 256 + left_at(j, jj)] = jj <= j ? aq[x] : 0.f;
     }
   }
   __syncthreads();
@@ -246,7 +280,7 @@ __global__ void __launch_bounds__(256) delta_prepare_kernel(DeltaArgs a) {
         for (int e = 0; e < 4; ++e) ahead[I][e] = col[(size_t)min(16 * I + 4 * kg + e, rows - 1) * a.qkv_stride];
     };
     fetch(wave);
-    for (int tile = wave; tile < all; tile += 4) {
+    for (int tile = wave; tile < all; tile += NW) {
       f32x4_t x[NB];
       const int c = (tile < kt ? tile : tile - kt) * 16 + j;
       if (tile < kt) {
@@ -267,40 +301,50 @@ __global__ void __launch_bounds__(256) delta_prepare_kernel(DeltaArgs a) {
 #pragma unroll
           for (int e = 0; e < 4; ++e) x[I][e] = on * beta[16 * I + 4 * kg + e] * ahead[I][e];  // (beta is 0 past the last row)
       }
-      fetch(tile + 4);
-      float* out = (tile < kt ? a.w + at * C * dp : a.v + at * C * a.vp) + c;
-      const int stride = tile < kt ? dp : a.vp;
+      fetch(tile + NW);
+      float* W = a.w + at * C * dp;
+      float* V = a.v + at * C * a.vp;
 #pragma unroll
       for (int I = 0; I < NB; ++I) {
-        f32x4_t acc = zero;
+        f32x4_t acc[NB];
 #pragma unroll
-        for (int J = 0; J < I; ++J) acc = mfma16x16(m[I][J], x[J], acc);
-        x[I] = mfma16x16(m[I][I], x[I] - acc, zero);
+        for (int J = 0; J < I; ++J) acc[J] = zero;
 #pragma unroll
-        for (int e = 0; e < 4; ++e) out[(size_t)(16 * I + 4 * kg + e) * stride] = x[I][e];
+        for (int e = 0; e < 4; ++e)
+#pragma unroll
+          for (int J = 0; J < I; ++J) acc[J] = mfma16(m[I][J][e], x[J][e], acc[J]);
+#pragma unroll
+        for (int J = 0; J < I; ++J) x[I] -= acc[J];
+        x[I] = mfma16x16(m[I][I], x[I], zero);
+        if (tile < kt) {
+#pragma unroll
+          for (int e = 0; e < 4; ++e) W[(I * kt + tile) * 256 + left_at(4 * kg + e, j)] = x[I][e];
+        } else {
+          *reinterpret_cast<f32x4_t*>(tile_at(V, (tile - kt) * NB + I, lane)) = x[I];
+        }
       }
     }
   }
-  // G q, row by row, and G_C / G k, transposed
+  // G q, and G_C / G k
   float* QG = a.qg + at * C * dp;
-  for (int e = threadIdx.x; e < C * d4; e += 256) {
-    const int r = e / d4, c = (e - r * d4) * 4;
+  for (int e = threadIdx.x; e < C * d4; e += NT) {
+    const int tile = e / 64, r = tile / (dp / 16) * 16 + (e & 15), c = tile % (dp / 16) * 16 + (e >> 4 & 3) * 4;
     f32x4_t l = row4(B, r, c);
     for (int M = 0; M < r / 16; ++M) l += row4(B, 16 * M + 15, c);
-    *reinterpret_cast<f32x4_t*>(QG + (size_t)r * dp + c) = row4(Q, r, c) * exp2_4(l);
+    *reinterpret_cast<f32x4_t*>(QG + 4 * e) = row4(Q, r, c) * exp2_4(l);
   }
   float* KD = a.kd + at * C * dp;
-  for (int e = threadIdx.x; e < dp * (C / 4); e += 256) {
-    const int c = e % dp, r = e / dp * 4;
+  for (int e = threadIdx.x; e < C * d4; e += NT) {
+    const int tile = e / 64, c = tile / NB * 16 + (e & 15), r = tile % NB * 16 + (e >> 4 & 3) * 4;
     float after = 0.f;
     for (int M = r / 16 + 1; M < NB; ++M) after += B[(16 * M + 15) * ds + c];
     const float end = B[(r | 15) * ds + c];
     f32x4_t v;
 #pragma unroll
     for (int x = 0; x < 4; ++x) v[x] = K[(r + x) * ds + c] * __builtin_amdgcn_exp2f((end - B[(r + x) * ds + c]) + after);
-    *reinterpret_cast<f32x4_t*>(KD + (size_t)c * C + r) = v;
+    *reinterpret_cast<f32x4_t*>(KD + 4 * e) = v;
   }
-  for (int c = threadIdx.x; c < dp; c += 256) {
+  for (int c = threadIdx.x; c < dp; c += NT) {
     float all = 0.f;
 #pragma unroll
     for (int M = 0; M < NB; ++M) all += B[(16 * M + 15) * ds + c];
@@ -336,57 +380,72 @@ __global__ void __launch_bounds__(256) delta_scan_kernel(DeltaArgs a) {
     f32x4_t wf[NT], v0, kf[MINE][NB], gm[MINE];
   } held[2];
   const int ub = NB == 4 ? wave : wave % NB;  // the block of 16 rows whose U the wave makes (with fewer blocks than waves: some twice)
-  auto fetch_w = [&](Held& t, int chunk) {
-    const size_t at = (size_t)min(chunk, a.chunks - 1) * a.heads + h;
-    const float* row = a.w + (at * C + 16 * ub + j) * dp + 4 * kg;
+  // (loads go out between the products: all at once they would wait for each other's turn)
+  auto fetch_w = [&](Held& t, int chunk, int n0, int n1) {
+    const float* w = a.w + ((size_t)min(chunk, a.chunks - 1) * a.heads + h) * C * dp;
 #pragma unroll
-    for (int n = 0; n < NT; ++n) t.wf[n] = *reinterpret_cast<const f32x4_t*>(row + 16 * n);
-    const float* v = a.v + (at * C + 16 * ub + 4 * kg) * vp + p0 + j;
-#pragma unroll
-    for (int e = 0; e < 4; ++e) t.v0[e] = v[e * vp];
+    for (int n = n0; n < n1; ++n) t.wf[n] = tile_of(w, ub * NT + n, lane);
   };
-  auto fetch_k = [&](Held& t, int chunk) {
+  auto fetch_v = [&](Held& t, int chunk) { t.v0 = tile_of(a.v + ((size_t)min(chunk, a.chunks - 1) * a.heads + h) * C * vp, ct * NB + ub, lane); };
+  auto fetch_k = [&](Held& t, int chunk, int m) {
     const size_t at = (size_t)min(chunk, a.chunks - 1) * a.heads + h;
+    const int n = wave + 4 * m;
+    t.gm[m] = *reinterpret_cast<const f32x4_t*>(a.gam + at * dp + 16 * n + 4 * kg);
 #pragma unroll
-    for (int m = 0; m < MINE; ++m) {
-      const int n = wave + 4 * m;
-      t.gm[m] = *reinterpret_cast<const f32x4_t*>(a.gam + at * dp + 16 * n + 4 * kg);
-      const float* row = a.kd + (at * dp + 16 * n + j) * C + 4 * kg;
-#pragma unroll
-      for (int b = 0; b < NB; ++b) t.kf[m][b] = *reinterpret_cast<const f32x4_t*>(row + 16 * b);
-    }
+    for (int b = 0; b < NB; ++b) t.kf[m][b] = tile_of(a.kd + at * C * dp, n * NB + b, lane);
   };
 #pragma unroll
-  for (int x = 0; x < 2; ++x) fetch_w(held[x], x), fetch_k(held[x], x);
+  for (int x = 0; x < 2; ++x) {
+    fetch_w(held[x], x, 0, NT);
+    fetch_v(held[x], x);
+#pragma unroll
+    for (int m = 0; m < MINE; ++m) fetch_k(held[x], x, m);
+  }
   __syncthreads();
   auto go = [&](Held& t, int chunk) {
     const size_t at = ((size_t)chunk * a.heads + h) * (vp / 16) + ct;
     {
-      f32x4_t acc[2] = {zero, zero};
+      f32x4_t acc[4] = {zero, zero, zero, zero};
 #pragma unroll
-      for (int n = 0; n < NT; ++n) acc[n & 1] = mfma16x16(t.wf[n], Ss[n][lane], acc[n & 1]);
-      const f32x4_t u = t.v0 - (acc[0] + acc[1]);
+      for (int n = 0; n < NT; n += 4) {
+        const f32x4_t x[4] = {t.wf[n], t.wf[n + 1], t.wf[n + 2], t.wf[n + 3]}, y[4] = {Ss[n][lane], Ss[n + 1][lane], Ss[n + 2][lane], Ss[n + 3][lane]};
+        mfma16x16_each(x, y, acc);
+        fetch_w(t, chunk + 2, n, n + 4);
+      }
+      const f32x4_t u = t.v0 - ((acc[0] + acc[1]) + (acc[2] + acc[3]));
       Us[ub][lane] = u;
-      *reinterpret_cast<f32x4_t*>(a.u + ((at * NB + ub) * 64 + lane) * 4) = u;
+      *reinterpret_cast<f32x4_t*>(tile_at(a.u, at * NB + ub, lane)) = u;
     }
-    fetch_w(t, chunk + 2);
+    fetch_v(t, chunk + 2);
     __syncthreads();
     f32x4_t uf[NB];
 #pragma unroll
     for (int b = 0; b < NB; ++b) uf[b] = Us[b][lane];
 #pragma unroll
     for (int m = 0; m < MINE; ++m) {
-      *reinterpret_cast<f32x4_t*>(a.s0 + ((at * NT + wave + 4 * m) * 64 + lane) * 4) = mine[m];
-      f32x4_t acc = t.gm[m] * mine[m], acc2 = zero;
-#pragma unroll
-      for (int b = 0; b < NB; ++b) {
-        if (b & 1) acc2 = mfma16x16(t.kf[m][b], uf[b], acc2);
-        else acc = mfma16x16(t.kf[m][b], uf[b], acc);
-      }
-      mine[m] = acc + acc2;
-      Ss[wave + 4 * m][lane] = mine[m];
+      *reinterpret_cast<f32x4_t*>(tile_at(a.s0, at * NT + wave + 4 * m, lane)) = mine[m];
+      mine[m] = t.gm[m] * mine[m];
     }
-    fetch_k(t, chunk + 2);
+#pragma unroll
+    for (int m = 0; m < MINE; m += 2) {  // four chains: two tiles, even and odd blocks
+      const int m2 = m + 1 < MINE ? m + 1 : m;
+      f32x4_t acc[4] = {mine[m], zero, m + 1 < MINE ? mine[m2] : zero, zero};
+#pragma unroll
+      for (int b = 0; b < NB; b += 2) {
+        const int b2 = b + 1 < NB ? b + 1 : b;
+        const f32x4_t x[4] = {t.kf[m][b], b + 1 < NB ? t.kf[m][b2] : zero, m + 1 < MINE ? t.kf[m2][b] : zero, m + 1 < MINE && b + 1 < NB ? t.kf[m2][b2] : zero};
+        const f32x4_t y[4] = {uf[b], uf[b2], uf[b], uf[b2]};
+        mfma16x16_each(x, y, acc);
+      }
+      mine[m] = acc[0] + acc[1];
+      fetch_k(t, chunk + 2, m);
+      if (m + 1 < MINE) {
+        mine[m2] = acc[2] + acc[3];
+        fetch_k(t, chunk + 2, m2);
+      }
+    }
+#pragma unroll
+    for (int m = 0; m < MINE; ++m) Ss[wave + 4 * m][lane] = mine[m];
     __syncthreads();
   };
 #pragma unroll 1
@@ -409,31 +468,40 @@ __global__ void __launch_bounds__(C * 4) delta_out_kernel(DeltaArgs a) {
   constexpr int NB = C / 16;
   constexpr int dp = 16 * NT;
   const int chunk = blockIdx.x, h = blockIdx.y, vt = a.vp / 16, row0 = chunk * C, rows = min(C, a.t - row0);
-  const int lane = threadIdx.x & 63, I = threadIdx.x >> 6, j = lane & 15, kg = lane >> 4;
+  const int lane = threadIdx.x & 63, I = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), j = lane & 15, kg = lane >> 4;
   if (16 * I >= rows) return;
   const size_t at = (size_t)chunk * a.heads + h;
   const f32x4_t zero = {0.f, 0.f, 0.f, 0.f};
   f32x4_t qf[NT], pf[NB], o[NV];
-  const float* q = a.qg + (at * C + 16 * I + j) * dp + 4 * kg;
 #pragma unroll
-  for (int n = 0; n < NT; ++n) qf[n] = *reinterpret_cast<const f32x4_t*>(q + 16 * n);
-  const float* p = a.p + (at * C + 16 * I + j) * C + 4 * kg;
+  for (int n = 0; n < NT; ++n) qf[n] = tile_of(a.qg + at * C * dp, I * NT + n, lane);
 #pragma unroll
-  for (int b = 0; b < NB; ++b) pf[b] = *reinterpret_cast<const f32x4_t*>(p + (b <= I ? 16 * b : 0));
+  for (int b = 0; b < NB; ++b) pf[b] = tile_of(a.p + at * C * C, I * NB + (b <= I ? b : 0), lane);
   float ss[4] = {0.f, 0.f, 0.f, 0.f};
+  f32x4_t sf[2][NT], uf[2][NB];  // a column tile's state and U, on their way one tile ahead
+  auto fetch = [&](int x, int v) {
+    const size_t tile = at * vt + min(v, vt - 1);
+#pragma unroll
+    for (int n = 0; n < NT; ++n) sf[x][n] = tile_of(a.s0, tile * NT + n, lane);
+#pragma unroll
+    for (int b = 0; b < NB; ++b) uf[x][b] = tile_of(a.u, tile * NB + b, lane);
+  };
+  fetch(0, 0);
 #pragma unroll
   for (int v = 0; v < NV; ++v) {
     o[v] = zero;
     if (v >= vt) continue;
-    const float* s = a.s0 + ((at * vt + v) * NT * 64 + lane) * 4;
-    const float* u = a.u + ((at * vt + v) * NB * 64 + lane) * 4;
-    f32x4_t acc[2] = {zero, zero};
+    fetch((v + 1) & 1, v + 1);
+    f32x4_t acc[4] = {zero, zero, zero, zero};
 #pragma unroll
-    for (int n = 0; n < NT; ++n) acc[n & 1] = mfma16x16(qf[n], *reinterpret_cast<const f32x4_t*>(s + n * 256), acc[n & 1]);
+    for (int n = 0; n < NT; n += 4) {
+      const f32x4_t x[4] = {qf[n], qf[n + 1], qf[n + 2], qf[n + 3]}, y[4] = {sf[v & 1][n], sf[v & 1][n + 1], sf[v & 1][n + 2], sf[v & 1][n + 3]};
+      mfma16x16_each(x, y, acc);
+    }
 #pragma unroll
     for (int b = 0; b < NB; ++b)
-      if (b <= I) acc[b & 1] = mfma16x16(pf[b], *reinterpret_cast<const f32x4_t*>(u + b * 256), acc[b & 1]);
-    o[v] = acc[0] + acc[1];  // columns past vdim are zeros
+      if (b <= I) acc[b] = mfma16x16(pf[b], uf[v & 1][b], acc[b]);
+    o[v] = (acc[0] + acc[1]) + (acc[2] + acc[3]);  // columns past vdim are zeros
 #pragma unroll
     for (int e = 0; e < 4; ++e) ss[e] += o[v][e] * o[v][e];
   }
@@ -570,6 +638,8 @@ __global__ void __launch_bounds__(256) delta_step_kernel(DeltaStepArgs a) {
     return gate ? static_cast<const WT*>(a.w_z) + (size_t)(h * a.vdim + p0 + r - d) * a.z_rank : static_cast<const WT*>(a.w_a) + (size_t)(h * d + r) * a.a_rank;
   };
   Piece8<WT> pre[V8 ? ROUNDS : 1][PIECES];
+  const int r_mine = row8 + 32 * l8;  // the row whose decay (or gate) this lane finishes
+  const float bias = a.dt_bias[h * d + min(r_mine, d - 1)];
   if constexpr (V8) {
 #pragma unroll
     for (int u = 0; u < ROUNDS; ++u) {
@@ -586,6 +656,7 @@ __global__ void __launch_bounds__(256) delta_step_kernel(DeltaStepArgs a) {
 #pragma unroll
     for (int u = 0; u < HELD; ++u) held[u] = Sl[(size_t)min(grp + GROUPS * u, d - 1) * a.vdim];
   }
+  __builtin_amdgcn_sched_barrier(0);
   float* slot = a.ring + (size_t)(a.pos % a.n_taps) * a.channels;
   const bool first = h % per == 0 && blockIdx.y == 0;  // stores the key head's rows
   for (int i = tid; i < 2 * d; i += 256) {
@@ -613,30 +684,36 @@ __global__ void __launch_bounds__(256) delta_step_kernel(DeltaStepArgs a) {
     ss = wave_sum(ss);
     if (lane == 0) scale[wave] = 1.f / sqrtf(ss + UNIT_EPS) * (wave ? 1.f : 1.f / sqrtf((float)d));
   }
-  auto finish = [&](int r, float s) {
+  auto over8 = [&](float s) {
     s += __shfl_xor(s, 4, 64);
     s += __shfl_xor(s, 2, 64);
-    s += __shfl_xor(s, 1, 64);
-    if (l8 == 0 && r < d + mine) {
-      if (r >= d) a.out[(size_t)a.heads * a.vdim + h * a.vdim + p0 + r - d] = s;
-      else decay[r] = expf(neg * softplus_f(s + a.dt_bias[h * d + r]));
-    }
+    return s + __shfl_xor(s, 1, 64);
+  };
+  auto finish = [&](int r, float s, float b) {
+    if (r >= d + mine) return;
+    if (r >= d) a.out[(size_t)a.heads * a.vdim + h * a.vdim + p0 + r - d] = s;
+    else decay[r] = expf(neg * softplus_f(s + b));
   };
   if constexpr (V8) {
+    float s_mine = 0.f;
 #pragma unroll
     for (int u = 0; u < ROUNDS; ++u) {
-      const int r = row8 + 32 * u, rr = min(r, d + mine - 1), n = rr >= d ? a.z_rank : a.a_rank;
+      const int rr = min(row8 + 32 * u, d + mine - 1), n = rr >= d ? a.z_rank : a.a_rank;
       const float* x = rr >= d ? z_in : a_in;
       float s = 0.f;
 #pragma unroll
       for (int b = 0; b < PIECES; ++b)
         if (b * 64 + l8 * 8 < n) s += pre[u][b].dot(x + b * 64 + l8 * 8);
-      finish(r, s + row_part<WT, V8>(row_of(rr), x, PIECES * 64, n, l8));
+      if (n > PIECES * 64) s += row_part<WT, V8>(row_of(rr), x, PIECES * 64, n, l8);
+      s = over8(s);
+      if (l8 == u) s_mine = s;
     }
+    if (l8 < ROUNDS) finish(r_mine, s_mine, bias);
   }
   for (int r = row8 + (V8 ? 32 * ROUNDS : 0); r < d + mine; r += 32) {  // a row's eight lanes stay together
     const bool gate = r >= d;
-    finish(r, row_part<WT, V8>(row_of(r), gate ? z_in : a_in, 0, gate ? a.z_rank : a.a_rank, l8));
+    const float s = over8(row_part<WT, V8>(row_of(r), gate ? z_in : a_in, 0, gate ? a.z_rank : a.a_rank, l8));
+    if (l8 == 0) finish(r, s, gate ? 0.f : a.dt_bias[h * d + r]);
   }
   __syncthreads();
   const float ks = scale[1], qs = scale[0];
@@ -700,7 +777,7 @@ int prepare(ughip_device* dev, const DeltaArgs& a) {
   const size_t bytes = prepare_lds_floats<C>(a.dp) * sizeof(float);
   static const hipError_t attr = hipFuncSetAttribute(reinterpret_cast<const void*>(delta_prepare_kernel<C, VEC>), hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
   UGHIP_HIPCHK(attr);
-  delta_prepare_kernel<C, VEC><<<dim3((unsigned)a.chunks, (unsigned)a.heads), 256, bytes, dev->stream>>>(a);
+  delta_prepare_kernel<C, VEC><<<dim3((unsigned)a.chunks, (unsigned)a.heads), prepare_threads<C>(), bytes, dev->stream>>>(a);
   UGHIP_HIPCHK(hipGetLastError());
   return UGHIP_OK;
 }
