@@ -18,7 +18,7 @@ namespace {  // every file that launches the kernel has its own
 typedef float f32x16 __attribute__((ext_vector_type(16)));
 typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
 
-// q [heads][q_rows][DQ], k [kv_heads][k_rows][DQ], v [kv_heads vdim][v_stride] (one row per value element, position along it); zeros
+// Queries come times scale * log2(e): the weights are powers of two of the scores.  q [heads][q_rows][DQ], k [kv_heads][k_rows][DQ], v [kv_heads vdim][v_stride] (one row per value element, position along it); zeros
 // past a query's and a key's last element and past the last query.
 struct AttRowsArgs {
   const void* q;
@@ -29,7 +29,6 @@ struct AttRowsArgs {
   int t, pos, vdim, q_rows, k_rows;
   int kv_heads;  // key head of query head h: h / (heads / kv_heads)
   int window;    // > 0: a position sees itself and the window - 1 positions in front of it
-  float scale2;  // scale * log2(e): the weights are powers of two
   bool dst_bf16;
 };
 
@@ -63,9 +62,18 @@ template <typename T, int DQ, int DV>
 constexpr int attention_rows_threads() {
   return 256 * attention_rows_groups<T, DQ, DV>();
 }
+// A tile's bytes, and whether LDS holds two per group: the next one goes in while this one is multiplied.
+template <typename T, int DQ, int DV>
+constexpr int attention_rows_tile_bytes() {
+  return ATT_KT * (DQ * (int)sizeof(T) + 16) + DV * (ATT_KT * (int)sizeof(T) + 16);
+}
+template <typename T, int DQ, int DV>
+constexpr bool attention_rows_twice() {
+  return 2 * attention_rows_groups<T, DQ, DV>() * attention_rows_tile_bytes<T, DQ, DV>() <= 160 * 1024;
+}
 template <typename T, int DQ, int DV>
 constexpr int attention_rows_lds_bytes() {
-  return attention_rows_groups<T, DQ, DV>() * (ATT_KT * (DQ * (int)sizeof(T) + 16) + DV * (ATT_KT * (int)sizeof(T) + 16));
+  return (attention_rows_twice<T, DQ, DV>() ? 2 : 1) * attention_rows_groups<T, DQ, DV>() * attention_rows_tile_bytes<T, DQ, DV>();
 }
 
 // DQ >= dim + rot and DV >= vdim, the surplus is zeros.  T: uint16_t (bf16) or float.
@@ -78,8 +86,11 @@ __global__ void __launch_bounds__((attention_rows_threads<T, DQ, DV>())) attenti
   extern __shared__ __attribute__((aligned(16))) char lds[];
   constexpr int GROUPS = attention_rows_groups<T, DQ, DV>();
   const int group = threadIdx.x >> 8, tid = threadIdx.x & 255;
-  char* Ks = lds + group * (ATT_KT * K_ROW + DV * V_ROW);  // [ATT_KT][DQ]
-  char* Vs = Ks + ATT_KT * K_ROW;                          // [DV][ATT_KT]
+  constexpr int TILE = attention_rows_tile_bytes<T, DQ, DV>();
+  constexpr bool TWICE = attention_rows_twice<T, DQ, DV>();
+  char* const tiles = lds + group * (TWICE ? 2 : 1) * TILE;
+  char* Ks = tiles;                // [ATT_KT][DQ]
+  char* Vs = Ks + ATT_KT * K_ROW;  // [DV][ATT_KT]
   // consecutive workgroups (dealt round robin to the chip's eight parts) take different key heads: those that share one meet in a cache
   const int per = gridDim.x / a.kv_heads, kv = blockIdx.x % a.kv_heads, head = kv * per + blockIdx.x / a.kv_heads;
   const int qb = gridDim.y - 1 - blockIdx.y;  // the longest rows first
@@ -124,26 +135,48 @@ __global__ void __launch_bounds__((attention_rows_threads<T, DQ, DV>())) attenti
     return out;
   };
   const int k_mine = k_begin + group * ATT_KT;
-  if (AHEAD && k_mine < keys) fetch(k_mine);
-  for (int k0 = k_mine; k0 - group * ATT_KT < keys; k0 += GROUPS * ATT_KT) {
-    __syncthreads();
-    const bool there = GROUPS == 1 || k0 < keys;  // (the last tile of an odd number is the first group's alone)
-    if (there) {
-    if (!AHEAD) fetch(k0);
+  auto place = [&](int k0, char* kt) {
+    char* vt = kt + ATT_KT * K_ROW;
 #pragma unroll
     for (int u = 0; u < NK; ++u) {
       const int x = tid + u * 256;
-      *reinterpret_cast<u32x4_t*>(Ks + x / QC * K_ROW + x % QC * 16) = kr[u];
+      *reinterpret_cast<u32x4_t*>(kt + x / QC * K_ROW + x % QC * 16) = kr[u];
     }
+    const bool whole = k0 + ATT_KT <= s_all && DV == a.vdim;
 #pragma unroll
     for (int u = 0; u < NV; ++u) {
       const int x = tid + u * 256;
-      const bool whole = k0 + ATT_KT <= s_all && DV == a.vdim;
-      *reinterpret_cast<u32x4_t*>(Vs + x / VC * V_ROW + x % VC * 16) = whole ? vr[u] : value_piece(vr[u], x / VC, k0 + x % VC * E);
+      *reinterpret_cast<u32x4_t*>(vt + x / VC * V_ROW + x % VC * 16) = whole ? vr[u] : value_piece(vr[u], x / VC, k0 + x % VC * E);
     }
+  };
+  if (AHEAD && k_mine < keys) fetch(k_mine);
+  if constexpr (TWICE) {
+    if (!AHEAD && k_mine < keys) fetch(k_mine);
+    if (k_mine < keys) place(k_mine, tiles);
+    if (AHEAD && k_mine + GROUPS * ATT_KT < keys) fetch(k_mine + GROUPS * ATT_KT);
+  }
+  for (int k0 = k_mine; k0 - group * ATT_KT < keys; k0 += GROUPS * ATT_KT) {
+    const bool there = GROUPS == 1 || k0 < keys;  // (the last tile of an odd number is the first group's alone)
+    const int k_next = k0 + GROUPS * ATT_KT;
+    if constexpr (TWICE) {
+      __syncthreads();  // (this tile is there, and the one before has been read)
+      if (k_next < keys) {
+        if (!AHEAD) fetch(k_next);
+        place(k_next, tiles + (Ks == tiles ? TILE : 0));
+        if (AHEAD && k_next + GROUPS * ATT_KT < keys) fetch(k_next + GROUPS * ATT_KT);
+      }
+    } else {
+      __syncthreads();
+      if (there) {
+        if (!AHEAD) fetch(k0);
+        place(k0, tiles);
+      }
+      __syncthreads();
+      if (AHEAD && k_next < keys) fetch(k_next);
     }
-    __syncthreads();
-    if (AHEAD && k0 + GROUPS * ATT_KT < keys) fetch(k0 + GROUPS * ATT_KT);
+    const char* const Kc = Ks;
+    const char* const Vc = Vs;
+    if constexpr (TWICE) Ks = Ks == tiles ? tiles + TILE : tiles, Vs = Ks + ATT_KT * K_ROW;
     if (!there) continue;
     if (k0 > first_p + 31 || (a.window && k0 + ATT_KT - 1 <= first_p - a.window)) continue;  // nothing in this tile is visible to the wave's queries
     f32x16 s[2];
@@ -154,7 +187,7 @@ __global__ void __launch_bounds__((attention_rows_threads<T, DQ, DV>())) attenti
 #pragma unroll
     for (int c = 0; c < QC / 2; ++c)
 #pragma unroll
-      for (int b = 0; b < 2; ++b) mfma_chunk<T>(*reinterpret_cast<const u32x4_t*>(Ks + (b * 32 + col) * K_ROW + hf * 16 + c * 32), qf[c], s[b]);
+      for (int b = 0; b < 2; ++b) mfma_chunk<T>(*reinterpret_cast<const u32x4_t*>(Kc + (b * 32 + col) * K_ROW + hf * 16 + c * 32), qf[c], s[b]);
     // element e of s[b]: key k0 + 32 b + 8 (e / 4) + 4 hf + e % 4, query `col`
     float top = mx;
     if (k0 + ATT_KT - 1 > first_p || (a.window && k0 <= first_p + 31 - a.window)) {  // some keys of the tile are not visible to some of the wave's queries
@@ -163,27 +196,24 @@ __global__ void __launch_bounds__((attention_rows_threads<T, DQ, DV>())) attenti
 #pragma unroll
         for (int e = 0; e < 16; ++e) {
           const int key = k0 + 32 * b + 8 * (e >> 2) + 4 * hf + (e & 3);
-          s[b][e] = key <= p_mine && key > oldest ? s[b][e] * a.scale2 : -INFINITY;
+          s[b][e] = key <= p_mine && key > oldest ? s[b][e] : -INFINITY;
         }
-    } else {
-#pragma unroll
-      for (int b = 0; b < 2; ++b)
-#pragma unroll
-        for (int e = 0; e < 16; ++e) s[b][e] *= a.scale2;
     }
 #pragma unroll
     for (int b = 0; b < 2; ++b)
 #pragma unroll
       for (int e = 0; e < 16; ++e) top = fmaxf(top, s[b][e]);
     top = fmaxf(top, __shfl_xor(top, 32, 64));
-    if (__any(top > mx)) {
-      const float alpha = top > mx ? exp2f(mx - top) : 1.f;  // (a lane whose query has seen nothing yet: both are -infinity)
+    // the weights' base follows the maximum only when that has left it well behind: up to 2^8 they lose nothing
+    const bool behind = top > mx + 8.f;
+    if (__any(behind)) {
+      const float alpha = behind ? exp2f(mx - top) : 1.f;
       sum *= alpha;
 #pragma unroll
       for (int i = 0; i < DV / 32; ++i)
 #pragma unroll
         for (int e = 0; e < 16; ++e) o[i][e] *= alpha;
-      mx = top;
+      mx = behind ? top : mx;
     }
     const float base = mx == -INFINITY ? 0.f : mx;
     float part = 0.f;
@@ -209,7 +239,7 @@ __global__ void __launch_bounds__((attention_rows_threads<T, DQ, DV>())) attenti
           bf16x8 vf[DV / 32];
 #pragma unroll
           for (int i = 0; i < DV / 32; ++i) {
-            const char* p = Vs + (i * 32 + col) * V_ROW + (b * 32 + 16 * u + 4 * hf) * 2;
+            const char* p = Vc + (i * 32 + col) * V_ROW + (b * 32 + 16 * u + 4 * hf) * 2;
             const uint2 v0 = *reinterpret_cast<const uint2*>(p), v1 = *reinterpret_cast<const uint2*>(p + 16);
             vf[i] = __builtin_bit_cast(bf16x8, u32x4_t{v0.x, v0.y, v1.x, v1.y});
           }
@@ -223,7 +253,7 @@ __global__ void __launch_bounds__((attention_rows_threads<T, DQ, DV>())) attenti
         for (int u = 0; u < 4; ++u)
 #pragma unroll
           for (int i = 0; i < DV / 32; ++i) {
-            const f32x4_t v = *reinterpret_cast<const f32x4_t*>(Vs + (i * 32 + col) * V_ROW + (b * 32 + 8 * u + 4 * hf) * 4);
+            const f32x4_t v = *reinterpret_cast<const f32x4_t*>(Vc + (i * 32 + col) * V_ROW + (b * 32 + 8 * u + 4 * hf) * 4);
             o[i] = __builtin_amdgcn_mfma_f32_32x32x2f32(v.x, s[b][4 * u], o[i], 0, 0, 0);
             o[i] = __builtin_amdgcn_mfma_f32_32x32x2f32(v.y, s[b][4 * u + 1], o[i], 0, 0, 0);
             o[i] = __builtin_amdgcn_mfma_f32_32x32x2f32(v.z, s[b][4 * u + 2], o[i], 0, 0, 0);

@@ -87,10 +87,11 @@ struct GroupedArgs {
   const float* temp;
   size_t row, cap;
   int t, pos, heads, kv_heads, dim, vdim, rot, q_rows;
+  float scale2;  // scale * log2(e), a part of every query: the weights are powers of two of the scores
 };
 __device__ __forceinline__ Turn turn_of(const GroupedArgs& a, int p, bool query) {
   const size_t at = (size_t)p * (a.rot >> 1);
-  return Turn{a.rot ? a.cos + at : nullptr, a.rot ? a.sin + at : nullptr, a.rot, query && a.temp ? a.temp[p] : 1.f};
+  return Turn{a.rot ? a.cos + at : nullptr, a.rot ? a.sin + at : nullptr, a.rot, query ? (a.temp ? a.temp[p] * a.scale2 : a.scale2) : 1.f};
 }
 
 constexpr int VT = 64;  // positions and value elements of a transposed tile
@@ -138,7 +139,6 @@ struct SplitArgs {
   float* ml;   // [splits][kv_heads rows][2]
   size_t dst_stride;
   int rows, row_blocks, splits, window;  // rows: (position, head) pairs per key head
-  float scale2;
   bool dst_bf16;
 };
 constexpr int SK = 32;
@@ -270,7 +270,7 @@ __global__ void __launch_bounds__(64 * NW) attention_split_kernel(SplitArgs a) {
 #pragma unroll
     for (int e = 0; e < 16; ++e) {
       const int key = k0 + 8 * (e >> 2) + 4 * hf + (e & 3);
-      s[e] = key <= p_mine && key > oldest ? (s[e] + s2[e]) * a.scale2 : -INFINITY;
+      s[e] = key <= p_mine && key > oldest ? s[e] + s2[e] : -INFINITY;
       top = fmaxf(top, s[e]);
     }
     top = fmaxf(top, __shfl_xor(top, 32, 64));
@@ -514,19 +514,19 @@ extern "C" int ughip_grouped_attention(ughip_device* dev, const ughip_attention*
   g.temp = buf_ptr<float>(p->q_factor), g.row = p->qkv.stride, g.cap = rows;
   g.t = (int)p->t, g.pos = (int)p->pos, g.heads = (int)p->heads, g.kv_heads = (int)p->kv_heads, g.dim = (int)p->dim, g.vdim = (int)p->vdim, g.rot = (int)p->rot;
   void* dst = static_cast<char*>(p->dst.s->ptr) + p->dst.offset * (bf16 ? 2 : 4);
-  const float scale2 = p->scale * 1.4426950408889634f;
+  g.scale2 = p->scale * 1.4426950408889634f;
   const Built built = built_for(p->dim, p->vdim);
   const int window = p->window < s ? (int)p->window : 0;  // (one that nothing has left yet is none)
   if (p->t <= FEW) {
     SplitArgs a{};
-    a.g = g, a.dst = dst, a.dst_stride = p->dst.stride, a.window = window, a.scale2 = scale2, a.dst_bf16 = bf16;
+    a.g = g, a.dst = dst, a.dst_stride = p->dst.stride, a.window = window, a.dst_bf16 = bf16;
     return with_sizes(built, [&](auto dq, auto dv) {
       return type == UGHIP_BF16 ? attend_few<uint16_t, decltype(dq)::value, decltype(dv)::value>(dev, a) : attend_few<float, decltype(dq)::value, decltype(dv)::value>(dev, a);
     });
   }
   AttRowsArgs r{};
   r.k = g.kc, r.v = g.vc, r.dst = dst, r.v_stride = rows, r.dst_stride = p->dst.stride, r.t = g.t, r.pos = g.pos, r.vdim = g.vdim, r.kv_heads = g.kv_heads, r.window = window;
-  r.scale2 = scale2, r.dst_bf16 = bf16;
+  r.dst_bf16 = bf16;
   return with_sizes(built, [&](auto dq, auto dv) {
     return type == UGHIP_BF16 ? attend_many<uint16_t, decltype(dq)::value, decltype(dv)::value>(dev, g, r) : attend_many<float, decltype(dq)::value, decltype(dv)::value>(dev, g, r);
   });

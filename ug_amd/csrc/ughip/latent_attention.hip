@@ -63,6 +63,7 @@ struct PackArgs {
   void* kp;
   size_t q_stride;
   int t, pos, heads, dim, rot, rank, q_rows, k_rows;
+  float q_mul;
   bool q_vec;  // a head's query starts on 16 bytes
 };
 
@@ -88,15 +89,15 @@ __global__ void __launch_bounds__(256) latent_pack_kernel(PackArgs a) {
       for (int e = 0; e < E; e += 4) {
         const f32x4_t f = *reinterpret_cast<const f32x4_t*>(qr + c + e);
 #pragma unroll
-        for (int i = 0; i < 4; ++i) v[e + i] = to_elem<T>(f[i]);
+        for (int i = 0; i < 4; ++i) v[e + i] = to_elem<T>(f[i] * a.q_mul);
       }
     } else
 #pragma unroll
     for (int e = 0; e < E; ++e) {
       const int d = c + e;
-      if (d < a.dim) v[e] = is_q ? to_elem<T>(qr[d]) : kr[d];
+      if (d < a.dim) v[e] = is_q ? to_elem<T>(qr[d] * a.q_mul) : kr[d];
       else if (d < a.dim + a.rot)
-        v[e] = to_elem<T>(is_q ? rotated(qr + a.dim, d - a.dim, a.rot, a.cos + (size_t)p * (a.rot / 2), a.sin + (size_t)p * (a.rot / 2)) : rr[d - a.dim]);
+        v[e] = to_elem<T>(is_q ? rotated(qr + a.dim, d - a.dim, a.rot, a.cos + (size_t)p * (a.rot / 2), a.sin + (size_t)p * (a.rot / 2)) * a.q_mul : rr[d - a.dim]);
       else v[e] = T(0);
     }
   } else {
@@ -492,10 +493,11 @@ extern "C" int ughip_latent_attention_rows(ughip_device* dev, ughip_view q, cons
   if (int rc = device_activate(dev)) return rc;
   AttRowsArgs a{};
   a.v = v_t->ptr, a.dst = static_cast<char*>(dst.s->ptr) + dst.offset * (bf16 ? 2 : 4), a.v_stride = v_stride, a.dst_stride = dst.stride;
-  a.t = (int)t, a.pos = (int)pos, a.vdim = (int)vdim, a.scale2 = scale * 1.4426950408889634f, a.dst_bf16 = bf16;
+  a.t = (int)t, a.pos = (int)pos, a.vdim = (int)vdim, a.dst_bf16 = bf16;
   PackArgs pk{};
   pk.q = view_ptr<float>(q), pk.k = k->ptr, pk.cache = buf_ptr<float>(cache), pk.cos = buf_ptr<float>(cos), pk.sin = buf_ptr<float>(sin), pk.q_stride = q.stride;
   pk.t = (int)t, pk.pos = (int)pos, pk.heads = (int)heads, pk.dim = (int)dim, pk.rot = (int)rot, pk.rank = (int)rank;
+  pk.q_mul = scale * 1.4426950408889634f;  // the weights are powers of two
   pk.q_vec = (dim + rot) % 4 == 0 && q.stride % 4 == 0 && (reinterpret_cast<uintptr_t>(pk.q) & 15) == 0;
   return k->dtype == UGHIP_BF16 ? launch_rows_any<uint16_t>(dev, a, pk) : launch_rows_any<float>(dev, a, pk);
 }
