@@ -543,8 +543,9 @@ struct DeltaStepArgs {
   const void* w_z;
   float* s;
   float* out;
-  long long pos;
+  int before, slot;  // positions in front of this one, as far as the taps care; the ring's row of this position
   int n_taps, heads, kv_heads, dim, vdim, a_rank, z_rank, channels;
+  bool fresh;
 };
 
 // TAPS > 0: that many, everything asked for at once.
@@ -555,20 +556,20 @@ __device__ __forceinline__ float conv_one(const DeltaStepArgs& a, int c) {
     float w[TAPS], x[TAPS];
 #pragma unroll
     for (int j = 0; j < TAPS; ++j) {
-      const long long p = a.pos - (TAPS - 1) + j;
+      const int row = a.slot + 1 + j;  // of the position TAPS - 1 - j back
       w[j] = taps[j];
-      x[j] = j + 1 < TAPS ? a.ring[(size_t)((p + TAPS) % TAPS) * a.channels + c] : a.qkv[c];
+      x[j] = j + 1 < TAPS ? a.ring[(size_t)(row < TAPS ? row : row - TAPS) * a.channels + c] : a.qkv[c];
     }
     float v = 0.f;
 #pragma unroll
     for (int j = 0; j < TAPS; ++j)
-      if (a.pos - (TAPS - 1) + j >= 0) v += w[j] * x[j];
+      v += TAPS - 1 - j <= a.before ? w[j] * x[j] : 0.f;
     return silu_f(v);
   }
   float v = 0.f;
   for (int j = 0; j + 1 < a.n_taps; ++j) {
-    const long long p = a.pos - (a.n_taps - 1) + j;
-    if (p >= 0) v += taps[j] * a.ring[(size_t)(p % a.n_taps) * a.channels + c];
+    const int row = a.slot + 1 + j;
+    if (a.n_taps - 1 - j <= a.before) v += taps[j] * a.ring[(size_t)(row < a.n_taps ? row : row - a.n_taps) * a.channels + c];
   }
   return silu_f(v + taps[a.n_taps - 1] * a.qkv[c]);
 }
@@ -657,7 +658,7 @@ __global__ void __launch_bounds__(256) delta_step_kernel(DeltaStepArgs a) {
     for (int u = 0; u < HELD; ++u) held[u] = Sl[(size_t)min(grp + GROUPS * u, d - 1) * a.vdim];
   }
   __builtin_amdgcn_sched_barrier(0);
-  float* slot = a.ring + (size_t)(a.pos % a.n_taps) * a.channels;
+  float* slot = a.ring + (size_t)a.slot * a.channels;
   const bool first = h % per == 0 && blockIdx.y == 0;  // stores the key head's rows
   for (int i = tid; i < 2 * d; i += 256) {
     const int c = (i < d ? 0 : gd - d) + g * d + i;
@@ -671,7 +672,7 @@ __global__ void __launch_bounds__(256) delta_step_kernel(DeltaStepArgs a) {
   }
   for (int i = tid; i < a.a_rank; i += 256) a_in[i] = a.a_in[i];
   for (int i = tid; i < a.z_rank; i += 256) z_in[i] = a.z_in[i];
-  if (a.pos == 0) {  // nothing is known of the state's memory
+  if (a.fresh) {  // nothing is known of the state's memory
 #pragma unroll
     for (int u = 0; u < HELD; ++u) held[u] = 0.f;
   }
@@ -725,7 +726,7 @@ __global__ void __launch_bounds__(256) delta_step_kernel(DeltaStepArgs a) {
     held[u] *= decay[c];
     sk += held[u] * (k[c] * ks);
   }
-  if (there && a.pos)
+  if (there && !a.fresh)
     for (int c = grp + GROUPS * HELD; c < d; c += GROUPS) sk += S[(size_t)c * a.vdim] * decay[c] * (k[c] * ks);
   part[grp][col] = sk;
   __syncthreads();
@@ -746,7 +747,7 @@ __global__ void __launch_bounds__(256) delta_step_kernel(DeltaStepArgs a) {
   if (there)
     for (int c = grp + GROUPS * HELD; c < d; c += GROUPS) {
       float v = k[c] * ks * u_new;
-      if (a.pos) v += S[(size_t)c * a.vdim] * decay[c];
+      if (!a.fresh) v += S[(size_t)c * a.vdim] * decay[c];
       S[(size_t)c * a.vdim] = v;
       o += v * (q[c] * qs);
     }
@@ -869,8 +870,8 @@ extern "C" int ughip_delta_step(ughip_device* dev, const ughip_delta* p) {
   if (int rc = device_activate(dev)) return rc;
   const float* in = buf_ptr<float>(p->p);
   DeltaStepArgs a{in + p->qkv_offset, in + p->b_offset, in + p->a_offset, in + p->z_offset, buf_ptr<float>(p->taps), static_cast<float*>(p->ring->ptr), buf_ptr<float>(p->a_log),
-                  buf_ptr<float>(p->dt_bias), p->w_a->ptr, p->w_z->ptr, static_cast<float*>(p->s->ptr), static_cast<float*>(p->out->ptr) + p->dst_offset, (long long)p->pos,
-                  (int)p->n_taps, (int)H, (int)G, (int)d, (int)vd, (int)p->a_rank, (int)p->z_rank, (int)ch};
+                  buf_ptr<float>(p->dt_bias), p->w_a->ptr, p->w_z->ptr, static_cast<float*>(p->s->ptr), static_cast<float*>(p->out->ptr) + p->dst_offset,
+                  (int)(p->pos < p->n_taps ? p->pos : p->n_taps), (int)(p->pos % p->n_taps), (int)p->n_taps, (int)H, (int)G, (int)d, (int)vd, (int)p->a_rank, (int)p->z_rank, (int)ch, p->pos == 0};
   const bool v8 = p->a_rank % 8 == 0 && p->z_rank % 8 == 0 && (reinterpret_cast<uintptr_t>(a.w_a) & 15) == 0 && (reinterpret_cast<uintptr_t>(a.w_z) & 15) == 0;
   const size_t lds = (3 * d + p->a_rank + p->z_rank) * sizeof(float);
   auto go = [&](auto kernel) { kernel<<<dim3((unsigned)H, (unsigned)((vd + COLS - 1) / COLS)), 256, lds, dev->stream>>>(a); };
