@@ -18,8 +18,9 @@ namespace {  // every file that launches the kernel has its own
 typedef float f32x16 __attribute__((ext_vector_type(16)));
 typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
 
-// Queries come times scale * log2(e): the weights are powers of two of the scores.  q [heads][q_rows][DQ], k [kv_heads][k_rows][DQ], v [kv_heads vdim][v_stride] (one row per value element, position along it); zeros
-// past a query's and a key's last element and past the last query.
+// Queries come times scale * log2(e): the weights are powers of two of the scores.  q [heads][q_rows][DQ], k [kv_heads][k_rows][DQ],
+// v [kv_heads vdim][v_stride] (one row per value element, position along it); zeros past a query's and a key's last element and past
+// the last query.
 struct AttRowsArgs {
   const void* q;
   const void* k;
